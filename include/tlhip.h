@@ -251,9 +251,14 @@ enum tl_mixer_kind {
                                the cache holds the latent and that part only (optionally another layer's, kv_from) */
   TL_MIXER_GDELTA = 3,      /* generalized delta rule: decay and removal rate per key channel,
                                S <- diag(w) S - (a u)(u^T S) + k v^T with the unit key u, o = S^T r */
-  TL_MIXER_LINEAR = 4       /* gated linear attention whose forget gate also decides what is written (no keys):
+  TL_MIXER_LINEAR = 4,      /* gated linear attention whose forget gate also decides what is written (no keys):
                                q = silu(W_q h), f = l + (1 - l) sigmoid(W_f h + b), S <- diag(f) S + (1 - f) v^T, o = S^T q,
                                RMS norm per head with one plain weight [vdim] */
+  TL_MIXER_SSM = 5          /* selective state space with one decay per head and token (Mamba-2's form): z | x | B | C | dt =
+                               W_in h with x [heads][vdim], B and C [kv_heads][dim] (kv_heads = groups of heads that share B
+                               and C, dim = state size), dt [heads]; x, B, C through a causal convolution per channel + bias +
+                               silu (conv_taps); dt <- softplus(dt + dt_bias); S <- exp(-exp(A_log) dt) S + dt B x^T,
+                               y = S^T C + D x; y silu(z), RMS norm in norm_parts equal parts of the row, weights; W_o */
 };
 enum tl_mlp_kind {
   TL_MLP_NONE = 0,
@@ -265,7 +270,8 @@ enum tl_act_kind {
   TL_ACT_NONE = 0,
   TL_ACT_XIELU = 1,         /* z > 0: P z^2 + z / 2; z <= 0: Q (e^z - 1 - z) + z / 2, with P = softplus(p), Q = 1/2 + softplus(q)
                                from the two numbers of the tensor mlp.act */
-  TL_ACT_TANH = 2
+  TL_ACT_TANH = 2,
+  TL_ACT_GELU = 3           /* z Phi(z) = z / 2 (1 + erf(z / sqrt 2)) */
 };
 enum tl_glu_kind {
   TL_GLU_SWISH = 0,         /* g sigmoid(act_alpha g) (u + glu_up_add), g = min(gate, limit), u = clamp(up, -limit, limit) */
@@ -280,7 +286,8 @@ enum tl_norm_kind {
   TL_NORM_RMS_ONE_PLUS = 0, /* y / sqrt(mean(y^2) + eps) * (1 + w) */
   TL_NORM_DYT = 1,          /* tanh(alpha y) * w + b: elementwise, no mean or variance (tensors <name>, <name>.alpha, <name>.b) */
   TL_NORM_LAYER = 2,        /* (y - mean) / sqrt(var + eps) * w + b, var = mean of the squared deviations (tensors <name>, <name>.b) */
-  TL_NORM_RMS = 3           /* y / sqrt(mean(y^2) + eps) * w: plain weights (pre-norm blocks) */
+  TL_NORM_RMS = 3,          /* y / sqrt(mean(y^2) + eps) * w: plain weights (pre-norm blocks) */
+  TL_NORM_LAYER_PLAIN = 4   /* TL_NORM_LAYER without the bias */
 };
 enum tl_attn_weight {
   TL_ATTN_SOFTMAX = 0,      /* weights normalised over the visible keys */
@@ -300,9 +307,11 @@ enum tl_route_kind {
   TL_ROUTE_SOFTMAX_GROUPS = 1, /* scores = softmax over all experts; experts in `route_groups` equal groups of neighbours, a
                                group's score its best expert's, only the best `route_keep` groups can be chosen from;
                                weights = the chosen scores divided by their sum (+ 1e-20) */
-  TL_ROUTE_SIGMOID_GROUPS = 2 /* scores = sigmoid(logits); choice = score + mlp.correction[expert]; a group's rank is the sum of
+  TL_ROUTE_SIGMOID_GROUPS = 2, /* scores = sigmoid(logits); choice = score + mlp.correction[expert]; a group's rank is the sum of
                                its two best choices, experts outside the best `route_keep` groups cannot be chosen; the `top`
                                best choices are taken; weights = their scores (without the correction, not normalised) */
+  TL_ROUTE_SOFTMAX = 3      /* scores = softmax over all experts; the `top` largest; weights = their scores times route_scale (not
+                               renormalised) */
 };
 typedef struct tl_layer_spec {
   int mixer;                /* tl_mixer_kind */
@@ -349,14 +358,16 @@ typedef struct tl_layer_spec {
                                kv_rank, rot_dim and rotation) whose cached latent and rotated key part this layer reads; 0: its own */
   int head_gate;            /* TL_MIXER_LATENT: 1: head n's output is multiplied by sigmoid(W_g h)_n (mix.g, one row per head) */
   float decay_scale;        /* TL_MIXER_GDELTA: decay = exp(-decay_scale * sigmoid(W_w2 tanh(W_w1 h) + w0)); decay_rank = rows of w1 */
-  int act;                  /* TL_MLP_UNIT: tl_act_kind */
+  int act;                  /* TL_MLP_UNIT: tl_act_kind. TL_MLP_MOE: TL_ACT_NONE: the experts are gated units (glu); otherwise an
+                               expert is W_down act(W_up h) (tensors mlp.e<j>.{up,down}) */
   int glu;                  /* tl_glu_kind of the gated units (experts, shared expert, dense unit) */
   /* ---- TL_MIXER_SWA, all zero = none of it ---- */
   int score_maps;           /* 2: differential attention -- q and k hold two maps per head ([map 1 | map 2], dim each) over the
                                same values; o = a1 - lambda a2 with lambda = exp(lq1 . lk1) - exp(lq2 . lk2) + diff_init (tensors
                                mix.lq1 .. mix.lk2 [dim]), then o / rms(o) over vdim (no weight) times (1 - diff_init) */
   float diff_init;
-  int out_gate;             /* 1: the concatenated heads are multiplied by sigmoid(W_g h) (mix.g [heads * vdim][width]) */
+  int out_gate;             /* 1: the concatenated heads are multiplied by sigmoid(W_g h) (mix.g [heads * vdim][width]); also
+                               TL_MIXER_LATENT (instead of head_gate) */
   int qkv_bias;             /* 1: q, k, v = W h + b (mix.q.b, mix.k.b, mix.v.b) */
   int qkv_conv;             /* > 0: taps of a causal convolution over time per channel of q, k, v right after the projection
                                (mix.{q,k,v}.conv [channels][taps], no activation); its last taps - 1 inputs are state */
@@ -371,6 +382,9 @@ typedef struct tl_layer_spec {
           weights_of are the layer's). The first mixer's tensors are then l<i>.mix.left.*, the second's l<i>.mix.right.* ---- */
   const struct tl_layer_spec* side;
   float mix_scale, side_scale;
+  int rot_halves;           /* 1: dimension i turns with dimension i + rot_dims / 2 (0: 2i with 2i + 1); TL_MIXER_LATENT */
+  float route_scale;        /* TL_ROUTE_SOFTMAX: factor on the weights */
+  int norm_parts;           /* TL_MIXER_SSM: equal parts of the row, each normed by its own root mean square */
 } tl_layer_spec;
 typedef struct tl_stack_config {
   int width, vocab, n_layers;
@@ -384,6 +398,11 @@ typedef struct tl_stack_config {
   int canon_taps;           /* > 0 (pre-norm blocks): what a sublayer reads is h + conv(h), a causal convolution over time per
                                channel with so many taps (l<i>.canon1 for the mixer, l<i>.canon2 for the feed-forward,
                                [width][taps], the last column is the current token's); the last taps - 1 inputs are state */
+  int streams;              /* > 0 (pre-norm blocks behind a layer norm): hyper-connections. The residual is so many streams x_s,
+                               all the embedding row at first; sublayer q (1: mixer, 2: feed-forward) reads norm(sum_s in[s] x_s)
+                               and, its output being y, x_t <- sum_s mix[s][t] x_s + residual_mult out[t] y (tensors l<i>.hc<q>.in
+                               and .out [streams], .mix [streams][streams], from x to). The final norm reads the streams' sum */
+  float residual_mult;      /* != 0 (pre-norm blocks behind a layer norm): factor on what a sublayer adds to the residual */
 } tl_stack_config;
 /* the operators such a model is built from, callable on their own (all FP32 in and out, weights bf16 [rows][cols]):
  * Y[T][rows] = X[T][cols] W^T; terms 1 / 3 = MFMA GEMM with bf16-rounded / three-term-split activations, 0 = FP32 GEMV (T = 1) */
@@ -487,13 +506,46 @@ int tl_head_norm(float* o_dev, const float* sub_dev, float sub_coef, const float
 int tl_gated_linear_attention(const float* p_dev, int ld, const float* lower_dev, const float* f_bias_dev, float* state_dev,
                               float* o_dev, float* scratch_dev, int num_tokens, int heads, int dim, int vdim, void* stream);
 
+/* selective state space (TL_MIXER_SSM), token by token in meaning, walked in blocks of tokens on the matrix cores when
+ * num_tokens > 1. xbc [T][ld] = x (heads * vdim) | B (groups * state) | C (groups * state) after convolution and activation;
+ * dt_raw: token t, head h at t * dt_ld + h. dt = softplus(dt_raw + dt_bias), S <- exp(-exp(a_log) dt) S + dt B x^T,
+ * y = S^T C + d x, times silu(z) when z_dev is set (rows z_ld apart). state_dev [heads][state][vdim], updated in place;
+ * y [T][heads * vdim] */
+int tl_state_space(const float* xbc_dev, int ld, const float* dt_raw_dev, int dt_ld, const float* dt_bias_dev,
+                   const float* a_log_dev, const float* d_dev, const float* z_dev, int z_ld, float* state_dev, float* y_dev, int num_tokens, int heads, int groups, int state, int vdim, void* stream);
+/* one token of TL_MIXER_SSM with its convolution: p = z | x | B | C | dt as projected; history [taps - 1][channels] is read, not
+ * written (tl_part_norm shifts it); y [heads * vdim] = (S^T C + d x) silu(z) */
+int tl_state_space_step(const float* p_dev, const void* conv_bf16_dev, const float* conv_bias_dev, int taps,
+                        const float* history_dev, const float* dt_bias_dev, const float* a_log_dev, const float* d_dev,
+                        float* state_dev, float* y_dev, int heads, int groups, int state, int vdim, void* stream);
+/* every row in `parts` equal parts, each divided by its root mean square (eps inside the root), times w [width]; in place.
+ * history_dev (one row only): [taps - 1][channels] loses its oldest row and gains in_dev [channels] */
+int tl_part_norm(float* x_dev, const float* weight_dev, int num_tokens, int width, int parts, float eps, float* history_dev,
+                 const float* in_dev, int taps, int channels, void* stream);
+/* tl_causal_conv with a bias on the convolution's OUTPUT (in front of the activation) */
+int tl_causal_conv_bias(const float* in_dev, int ld_in, int channels, int taps, int num_tokens, const float* out_bias_dev,
+                        const void* w_bf16_dev, float* history_dev, int act, float* out_dev, int ld_out, void* stream);
+/* router (TL_ROUTE_SOFTMAX): ids [T][top] largest score first, weights = scores (softmax over all experts) * scale */
+int tl_moe_route_softmax(const float* x_dev, int num_tokens, int width, const void* w_bf16_dev, int experts, int top,
+                         float scale, int* ids_dev, float* weights_dev, void* stream);
+/* hyper-connections: x [T][streams][width] in place, x_t <- sum_s mix[s * streams + t] x_s + mult out[t] y (y NULL: x as it is);
+ * then, with in_dev, h [T][width] = layer norm (weight, bias optional) of sum_s in[s] x_s; sum_dev (optional) [T][width] = the
+ * streams' sum */
+int tl_hyper_connect(float* x_dev, const float* y_dev, const float* mix_dev, const float* out_dev, float mult, const float* in_dev,
+                     const float* weight_dev, const float* bias_dev, float eps, float* h_dev, float* sum_dev, int num_tokens,
+                     int streams, int width, void* stream);
+/* tl_rotary_heads with dimension i paired with i + rot_dims / 2, no norm */
+int tl_rotary_halves(float* x_dev, int num_tokens, int start_pos, int heads, int dim, int rot_dims, float rot_base,
+                     float rot_factor, float rot_original, float rot_fast, float rot_slow, void* stream);
+
 int tl_model_create_stack(const tl_stack_config* cfg, tl_model** out);
 /* tensors by checkpoint name: embed, embed.norm, final.norm, head, l<i>.norm1, l<i>.norm2, l<i>.mix.{q,k,v,o,q.norm,k.norm,vmix,pb},
  * l<i>.mix.{q,k,v}.conv, l<i>.mix.{b,a1,a2,g1,g2,A_log,dt_bias,norm}, l<i>.mlp.router, l<i>.mlp.router.b,
  * l<i>.mlp.e<j>.{gate,up,down}, l<i>.mlp.shared.{gate,up,down,sg}, l<i>.mlp.{gate,up,down,act,correction}, l<i>.canon{1,2},
  * l<i>.mix.{g,lq1,lk1,lq2,lk2,r1,r2,sink}, l<i>.mix.{q,k,v}.b, l<i>.mix.{f,f.b,lower,a}; with two mixers side by side
  * l<i>.mix.left.* and l<i>.mix.right.*; latent attention
- * l<i>.mix.{dq,dq.norm,uq,dkv,dkv.norm,uk,uv,g,o}; generalized delta rule l<i>.mix.{r,k,v,g,a,a.b,w1,w2,w0,norm,o}; a Dynamic
+ * l<i>.mix.{dq,dq.norm,uq,dkv,dkv.norm,uk,uv,g,o}; state space l<i>.mix.{in,conv,conv.b,dt_bias,A_log,D,norm,o};
+ * hyper-connections l<i>.hc{1,2}.{in,out,mix}; generalized delta rule l<i>.mix.{r,k,v,g,a,a.b,w1,w2,w0,norm,o}; a Dynamic
  * Tanh norm <n> also has <n>.alpha and <n>.b, a layer norm <n>.b. type: TL_BF16 (matrices and vectors) or TL_F32 (vectors). */
 int tl_model_set_tensor_named(tl_model* m, const char* name, int type, const long long* shape, int ndim, const void* host_data);
 /* a prompt, or a portion of one, at positions start_pos..: logits of the token rows listed in rows_host (ascending; NULL: the

@@ -43,13 +43,14 @@ LayerSpec._fields_ = [("mixer", C.c_int), ("heads", C.c_int), ("kv_heads", C.c_i
                 ("glu", C.c_int), ("score_maps", C.c_int), ("diff_init", C.c_float), ("out_gate", C.c_int),
                 ("qkv_bias", C.c_int), ("qkv_conv", C.c_int), ("score_softcap", C.c_float), ("dist_bias", C.c_int),
                 ("decay_per_head", C.c_int), ("side", C.POINTER(LayerSpec)), ("mix_scale", C.c_float),
-                ("side_scale", C.c_float)]
+                ("side_scale", C.c_float), ("rot_halves", C.c_int), ("route_scale", C.c_float), ("norm_parts", C.c_int)]
 
 
 class StackConfig(C.Structure):
     _fields_ = [("width", C.c_int), ("vocab", C.c_int), ("n_layers", C.c_int), ("max_positions", C.c_int),
                 ("norm_eps", C.c_float), ("layers", C.POINTER(LayerSpec)), ("norm", C.c_int), ("embed_norm", C.c_int),
-                ("logit_softcap", C.c_float), ("embed_scale", C.c_float), ("canon_taps", C.c_int)]
+                ("logit_softcap", C.c_float), ("embed_scale", C.c_float), ("canon_taps", C.c_int), ("streams", C.c_int),
+                ("residual_mult", C.c_float)]
 
 
 BF16 = 30
@@ -158,6 +159,15 @@ SIGNATURES = {
     "tl_head_norm": [_fp, _fp, C.c_float, _fp, C.c_int, C.c_int, _fp, C.c_int, C.c_float, C.c_int, C.c_int, C.c_int,
                      C.c_float, _vp],
     "tl_gated_linear_attention": [_fp, C.c_int, _fp, _fp, _fp, _fp, _fp, C.c_int, C.c_int, C.c_int, C.c_int, _vp],
+    "tl_state_space": [_fp, C.c_int, _fp, C.c_int, _fp, _fp, _fp, _fp, C.c_int, _fp, _fp, C.c_int, C.c_int, C.c_int, C.c_int,
+                       C.c_int, _vp],
+    "tl_state_space_step": [_fp, _vp, _fp, C.c_int, _fp, _fp, _fp, _fp, _fp, _fp, C.c_int, C.c_int, C.c_int, C.c_int, _vp],
+    "tl_part_norm": [_fp, _fp, C.c_int, C.c_int, C.c_int, C.c_float, _fp, _fp, C.c_int, C.c_int, _vp],
+    "tl_causal_conv_bias": [_fp, C.c_int, C.c_int, C.c_int, C.c_int, _fp, _vp, _fp, C.c_int, _fp, C.c_int, _vp],
+    "tl_moe_route_softmax": [_fp, C.c_int, C.c_int, _vp, C.c_int, C.c_int, C.c_float, _ip, _fp, _vp],
+    "tl_hyper_connect": [_fp, _fp, _fp, _fp, C.c_float, _fp, _fp, _fp, C.c_float, _fp, _fp, C.c_int, C.c_int, C.c_int, _vp],
+    "tl_rotary_halves": [_fp, C.c_int, C.c_int, C.c_int, C.c_int, C.c_int, C.c_float, C.c_float, C.c_float, C.c_float, C.c_float,
+                         _vp],
     "tl_general_delta": [_fp, C.c_int, _fp, _fp, _fp, C.c_float, _fp, _fp, _fp, C.c_int, C.c_int, C.c_int, _vp],
 }
 

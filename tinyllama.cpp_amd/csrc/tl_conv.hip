@@ -1,6 +1,6 @@
 // tl_conv.hip — a short causal convolution over time on every channel of a row, as layer-list models use it in two places:
 // on what a sublayer reads (out = in + conv(in): add_input) and on projected queries, keys and values right behind their
-// product (with the projection's bias added first, optionally followed by silu). Token t of a call needs the inputs of the
+// product (with the projection's bias added first, or a bias on the result, optionally followed by silu). Token t of a call needs the inputs of the
 // taps - 1 tokens before it; those that precede the call are part of the sequence's state (hist, zeros for an empty sequence),
 // so a prompt may be cut anywhere. Everything is FP32; the weights are the checkpoint's bf16 values widened exactly.
 //
@@ -32,6 +32,7 @@ __global__ __launch_bounds__(256) void conv_kernel(const ConvArgs a) {
     acc += tl_bf2f(w[j]) * u;
     cur = u;
   }
+  if (a.out_bias) acc += a.out_bias[c];
   if (a.act == 1) acc = acc / (1.0f + expf(-acc));
   if (a.add_input) acc += cur;
   a.out[(size_t)t * a.ldo + c] = acc;
@@ -63,6 +64,10 @@ __global__ __launch_bounds__(256) void conv4_kernel(const ConvArgs a) {
     acc.w += tl_bf2f(w[3 * a.taps + j]) * u.w;
     cur = u;
   }
+  if (a.out_bias) {
+    const float4 ob = *reinterpret_cast<const float4*>(a.out_bias + c);
+    acc.x += ob.x, acc.y += ob.y, acc.z += ob.z, acc.w += ob.w;
+  }
   if (a.act == 1) {
     acc.x = acc.x / (1.0f + expf(-acc.x)), acc.y = acc.y / (1.0f + expf(-acc.y));
     acc.z = acc.z / (1.0f + expf(-acc.z)), acc.w = acc.w / (1.0f + expf(-acc.w));
@@ -91,7 +96,7 @@ int tl_launch_causal_conv(const ConvArgs& a, hipStream_t s) {
              "causal_conv: output over input with more than one token");
   TL_REQUIRE(a.act == 0 || a.act == 1, "causal_conv: activation %d", a.act);
   const bool vec = a.T > 1 && (a.C & 3) == 0 && a.ldi == a.C && (a.ldo & 3) == 0 && ((size_t)a.in & 15) == 0 &&
-                   ((size_t)a.out & 15) == 0 && ((size_t)a.hist & 15) == 0 && ((size_t)a.bias & 15) == 0;
+                   ((size_t)a.out & 15) == 0 && ((size_t)a.hist & 15) == 0 && ((size_t)a.bias & 15) == 0 && ((size_t)a.out_bias & 15) == 0;
   if (vec) conv4_kernel<<<dim3((a.C / 4 + 255) / 256, a.T), 256, 0, s>>>(a);
   else conv_kernel<<<dim3((a.C + 255) / 256, a.T), 256, 0, s>>>(a);
   if (a.T > 1 && a.taps > 1) conv_history_rows_kernel<<<(a.C + 255) / 256, 256, 0, s>>>(a);
@@ -113,6 +118,23 @@ extern "C" int tl_causal_conv(const float* in_dev, int ld_in, int channels, int 
   a.hist = history_dev;
   a.act = act;
   a.add_input = add_input;
+  a.out = out_dev;
+  a.ldo = ld_out;
+  return tl_launch_causal_conv(a, static_cast<hipStream_t>(stream));
+}
+
+extern "C" int tl_causal_conv_bias(const float* in_dev, int ld_in, int channels, int taps, int num_tokens, const float* out_bias_dev,
+                                   const void* w_bf16_dev, float* history_dev, int act, float* out_dev, int ld_out, void* stream) {
+  ConvArgs a = {};
+  a.in = in_dev;
+  a.ldi = ld_in;
+  a.C = channels;
+  a.taps = taps;
+  a.T = num_tokens;
+  a.out_bias = out_bias_dev;
+  a.w = static_cast<const uint16_t*>(w_bf16_dev);
+  a.hist = history_dev;
+  a.act = act;
   a.out = out_dev;
   a.ldo = ld_out;
   return tl_launch_causal_conv(a, static_cast<hipStream_t>(stream));

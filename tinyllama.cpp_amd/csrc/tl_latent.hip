@@ -17,9 +17,11 @@
 //   latent_post    per token: the query latent is RMS-normed in place (plain weights); the key/value latent is RMS-normed and,
 //                  with the rotated shared key part behind it, written to row `pos` of the cache.
 //   latent_query   per token and head: the rotated query part goes behind the head's absorbed columns.
-//   head_gate      head n's output times sigmoid(gate_n).
+//   head_gate      head n's output times sigmoid(gate_n);  out_gate: every column of the concatenated heads times its own gate.
 // Norms, angles and the cache are FP32; the angle is formed in double (tl_rotary_sincos).
 #include <math.h>
+
+#include <vector>
 
 #include "tl_stack.h"
 
@@ -40,6 +42,27 @@ __device__ __forceinline__ float group_sum(float v, float* red) {
   float s = 0.0f;
   for (int w = 0; w < (int)(blockDim.x >> 6); ++w) s += red[w];
   return s;
+}
+
+// pair i of a part of rot_dim values, the first rot_dims of which turn by position: (2i, 2i + 1), or with `halves`
+// (i, i + rot_dims / 2); pairs beyond rot_dims / 2 are two neighbours that pass unchanged (a last odd value alone). src may be dst.
+__device__ __forceinline__ void latent_turn(const float* src, float* dst, int i, int rot_dim, int rot_dims, int halves, float mscale,
+                                            const double* freq, int pos) {
+  const int half = rot_dims >> 1;
+  const bool turns = i < half;
+  const int d0 = halves && turns ? i : 2 * i, d1 = halves && turns ? i + half : 2 * i + 1;
+  float u = src[d0], v = d1 < rot_dim ? src[d1] : 0.0f;
+  if (turns) {
+    float sn, cs;
+    tl_rotary_sincos(pos, freq[i], &sn, &cs);
+    sn *= mscale;
+    cs *= mscale;
+    const float nu = u * cs - v * sn, nv = v * cs + u * sn;
+    u = nu;
+    v = nv;
+  }
+  dst[d0] = u;
+  if (d1 < rot_dim) dst[d1] = v;
 }
 
 // grid (T), 256 threads
@@ -63,19 +86,7 @@ __global__ __launch_bounds__(256) void latent_post_kernel(const LatentPostArgs a
   for (int c = tid; c < a.kv_rank; c += 256) out[c] = kv[c] * ki * a.kv_norm[c];
   const float* kr = kv + a.kv_rank;
   float* outr = out + a.kv_rank;
-  for (int i = tid; 2 * i < a.rot_dim; i += 256) {  // pairs (2i, 2i + 1); a last odd dimension passes unchanged
-    const int d0 = 2 * i, d1 = d0 + 1;
-    float u = kr[d0], v = d1 < a.rot_dim ? kr[d1] : 0.0f;
-    if (d1 < a.rot_dims) {
-      float sn, cs;
-      tl_rotary_sincos(pos, a.freq[i], &sn, &cs);
-      const float nu = u * cs - v * sn, nv = v * cs + u * sn;
-      u = nu;
-      v = nv;
-    }
-    outr[d0] = u;
-    if (d1 < a.rot_dim) outr[d1] = v;
-  }
+  for (int i = tid; 2 * i < a.rot_dim; i += 256) latent_turn(kr, outr, i, a.rot_dim, a.rot_dims, a.halves, a.mscale, a.freq, pos);
 }
 
 // grid (T, heads in fours), a wave per (token, head)
@@ -85,19 +96,7 @@ __global__ __launch_bounds__(256) void latent_query_kernel(const LatentQueryArgs
   const int pos = (a.pos_dev ? *a.pos_dev : a.start_pos) + t;
   const float* src = a.q + ((size_t)t * a.heads + n) * a.q_stride + a.q_off;
   float* dst = a.out + ((size_t)t * a.heads + n) * a.out_stride + a.out_off;
-  for (int i = lane; 2 * i < a.rot_dim; i += 64) {
-    const int d0 = 2 * i, d1 = d0 + 1;
-    float u = src[d0], v = d1 < a.rot_dim ? src[d1] : 0.0f;
-    if (d1 < a.rot_dims) {
-      float sn, cs;
-      tl_rotary_sincos(pos, a.freq[i], &sn, &cs);
-      const float nu = u * cs - v * sn, nv = v * cs + u * sn;
-      u = nu;
-      v = nv;
-    }
-    dst[d0] = u;
-    if (d1 < a.rot_dim) dst[d1] = v;
-  }
+  for (int i = lane; 2 * i < a.rot_dim; i += 64) latent_turn(src, dst, i, a.rot_dim, a.rot_dims, a.halves, a.mscale, a.freq, pos);
 }
 
 __global__ __launch_bounds__(256) void latent_spread_kernel(const float* __restrict__ cache, int kv_rank, int rot_dim,
@@ -117,6 +116,28 @@ __global__ __launch_bounds__(256) void head_gate_kernel(float* __restrict__ o, c
   const long long th = i / vdim;  // token * heads + head
   const int t = (int)(th / heads), n = (int)(th % heads);
   o[i] *= 1.0f / (1.0f + expf(-gate[(size_t)t * gate_ld + n]));
+}
+
+__global__ __launch_bounds__(256) void out_gate_kernel(float* __restrict__ o, const float* __restrict__ gate, int gate_ld, int od,
+                                                      long long total) {
+  const long long i = (long long)blockIdx.x * 256 + threadIdx.x;
+  if (i >= total) return;
+  const int t = (int)(i / od), c = (int)(i - (long long)t * od);
+  o[i] *= 1.0f / (1.0f + expf(-gate[(size_t)t * gate_ld + c]));
+}
+
+__global__ __launch_bounds__(256) void out_gate4_kernel(float* __restrict__ o, const float* __restrict__ gate, int gate_ld, int od,
+                                                       long long total) {
+  const long long i = ((long long)blockIdx.x * 256 + threadIdx.x) * 4;
+  if (i >= total) return;
+  const int t = (int)(i / od), c = (int)(i - (long long)t * od);
+  float4 v = *reinterpret_cast<const float4*>(o + i);
+  const float4 g = *reinterpret_cast<const float4*>(gate + (size_t)t * gate_ld + c);
+  v.x *= 1.0f / (1.0f + expf(-g.x));
+  v.y *= 1.0f / (1.0f + expf(-g.y));
+  v.z *= 1.0f / (1.0f + expf(-g.z));
+  v.w *= 1.0f / (1.0f + expf(-g.w));
+  *reinterpret_cast<float4*>(o + i) = v;
 }
 
 }  // namespace
@@ -162,4 +183,40 @@ int tl_launch_head_gate(float* o, const float* gate, int gate_ld, int T, int hea
   head_gate_kernel<<<(unsigned)((total + 255) / 256), 256, 0, s>>>(o, gate, gate_ld, heads, vdim, total);
   TL_HIP(hipGetLastError());
   return 0;
+}
+
+int tl_launch_out_gate(float* o, const float* gate, int gate_ld, int T, int od, hipStream_t s) {
+  TL_REQUIRE(o && gate && T > 0 && od > 0 && gate_ld >= od, "out_gate: bad arguments");
+  const long long total = (long long)T * od;
+  if ((od & 3) == 0 && (gate_ld & 3) == 0 && ((size_t)o & 15) == 0 && ((size_t)gate & 15) == 0)
+    out_gate4_kernel<<<(unsigned)((total / 4 + 255) / 256), 256, 0, s>>>(o, gate, gate_ld, od, total);
+  else
+    out_gate_kernel<<<(unsigned)((total + 255) / 256), 256, 0, s>>>(o, gate, gate_ld, od, total);
+  TL_HIP(hipGetLastError());
+  return 0;
+}
+
+extern "C" int tl_rotary_halves(float* x_dev, int num_tokens, int start_pos, int heads, int dim, int rot_dims, float rot_base,
+                                float rot_factor, float rot_original, float rot_fast, float rot_slow, void* stream) {
+  TL_REQUIRE(x_dev && num_tokens > 0 && heads > 0 && dim > 0 && rot_dims > 0 && rot_dims <= dim && (rot_dims & 1) == 0 && rot_base > 0.0f,
+             "tl_rotary_halves: bad arguments");
+  hipStream_t s = static_cast<hipStream_t>(stream);
+  std::vector<double> f(rot_dims / 2);
+  LatentQueryArgs q = {};
+  tl_rotary_frequencies(rot_dims, rot_base, rot_factor, rot_original, rot_fast, rot_slow, f.data(), &q.mscale);
+  void* ws = nullptr;
+  TL_TRY(tl_scratch(TL_SCRATCH_ROTARY, sizeof(double) * f.size(), &ws));
+  TL_HIP(hipMemcpyAsync(ws, f.data(), sizeof(double) * f.size(), hipMemcpyHostToDevice, s));
+  TL_HIP(hipStreamSynchronize(s));
+  q.q = x_dev;
+  q.out = x_dev;
+  q.q_stride = q.out_stride = dim;
+  q.heads = heads;
+  q.rot_dim = dim;
+  q.rot_dims = rot_dims;
+  q.halves = 1;
+  q.freq = static_cast<const double*>(ws);
+  q.T = num_tokens;
+  q.start_pos = start_pos;
+  return tl_launch_latent_query(q, s);
 }

@@ -45,14 +45,7 @@ __global__ __launch_bounds__(1024) void router_kernel(const RouterArgs a, int ve
   }
   __syncthreads();
   if (wave != 0) return;
-  if (a.kind == TL_ROUTE_SIGMOID_GROUPS)
-    tl_route_select_sigmoid_groups(z, z + a.experts, z + 2 * a.experts, a.corr, a.experts, a.top, a.groups, a.keep,
-                                   a.ids + (size_t)t * a.top, a.wts + (size_t)t * a.top, lane);
-  else if (a.kind == TL_ROUTE_SOFTMAX_GROUPS)
-    tl_route_select_groups(z, z + a.experts, z + 2 * a.experts, a.experts, a.top, a.groups, a.keep, a.ids + (size_t)t * a.top,
-                           a.wts + (size_t)t * a.top, lane);
-  else
-    tl_route_select(z, a.experts, a.top, a.ids + (size_t)t * a.top, a.wts + (size_t)t * a.top, lane);
+  tl_route_token(a, z, t, lane);
 }
 
 __global__ __launch_bounds__(1024) void moe_plan_kernel(const int* __restrict__ ids, int n_slots, int experts,
@@ -103,6 +96,16 @@ __global__ __launch_bounds__(256) void moe_decode_gu_kernel(const MoeDecodeArgs 
   if (lane == 0) a.act[(size_t)j * a.ff + r] = tl_glu_apply(a.glu_kind, gu2[0], gu2[1], shared ? a.slimit : a.limit, a.alpha, a.up_add);
 }
 
+// plain experts: grid (rows of 4 waves over ff / 2, top); a wave owns two neighbouring rows of `up`, whose loads are in flight together
+__global__ __launch_bounds__(256) void moe_decode_up_kernel(const MoeDecodeArgs a, int vec) {
+  const int lane = threadIdx.x & 63, r = (blockIdx.x * 4 + (threadIdx.x >> 6)) * 2, j = blockIdx.y;
+  if (r >= a.ff) return;
+  const unsigned short* up = a.gu + ((size_t)a.ids[j] * a.ff + r) * a.width;
+  float u2[2];
+  tl_wave_dot_rows<2>(up, (size_t)a.width, a.ff - r, a.x, a.width, vec != 0, lane, u2);
+  if (lane < 2 && r + lane < a.ff) a.act[(size_t)j * a.ff + r + lane] = tl_act_apply(a.unit_act, lane ? u2[1] : u2[0], 0.0f, 0.0f);
+}
+
 __global__ __launch_bounds__(256) void moe_decode_down_kernel(const MoeDecodeArgs a, int vec_e, int vec_s) {
   const int lane = threadIdx.x & 63, r = blockIdx.x * 4 + (threadIdx.x >> 6);
   if (r >= a.width) return;
@@ -133,7 +136,7 @@ int tl_launch_router(const RouterArgs& a, hipStream_t s) {
                a.experts / a.groups);
     lds = sizeof(float) * (2 * (size_t)a.experts + a.groups);
   } else {
-    TL_REQUIRE(a.kind == TL_ROUTE_TOP_LOGITS, "router: kind %d", a.kind);
+    TL_REQUIRE(a.kind == TL_ROUTE_TOP_LOGITS || a.kind == TL_ROUTE_SOFTMAX, "router: kind %d", a.kind);
   }
   const int vec = (a.width & 7) == 0 && ((size_t)a.x & 15) == 0 && ((size_t)a.w & 15) == 0;
   // few tokens (the decode step): the experts' rows are latency-bound round trips, so spread them over 16 waves
@@ -171,7 +174,12 @@ int tl_launch_moe_decode(const MoeDecodeArgs& a, hipStream_t s) {
   const int vec_e = al && (a.ff & 7) == 0;
   const int vec_s = vec_e && (a.sff & 7) == 0;
   const int ffmax = a.sgu && a.sff > a.ff ? a.sff : a.ff;
-  moe_decode_gu_kernel<<<dim3((ffmax + 3) / 4, a.top + (a.sgu ? 1 : 0)), 256, 0, s>>>(a, vec_x);
+  if (a.unit_act) {
+    TL_REQUIRE(a.top > 0 && !a.sgu, "moe_decode: plain experts without a shared one");
+    moe_decode_up_kernel<<<dim3((a.ff + 7) / 8, a.top), 256, 0, s>>>(a, vec_x);
+  } else {
+    moe_decode_gu_kernel<<<dim3((ffmax + 3) / 4, a.top + (a.sgu ? 1 : 0)), 256, 0, s>>>(a, vec_x);
+  }
   moe_decode_down_kernel<<<(a.width + 3) / 4, 256, 0, s>>>(a, vec_e, vec_s);
   TL_HIP(hipGetLastError());
   return 0;
@@ -229,5 +237,21 @@ extern "C" int tl_moe_route_sigmoid_groups(const float* x_dev, int num_tokens, i
   a.kind = TL_ROUTE_SIGMOID_GROUPS;
   a.groups = groups;
   a.keep = keep;
+  return tl_launch_router(a, static_cast<hipStream_t>(stream));
+}
+
+extern "C" int tl_moe_route_softmax(const float* x_dev, int num_tokens, int width, const void* w_bf16_dev, int experts, int top,
+                                    float scale, int* ids_dev, float* weights_dev, void* stream) {
+  RouterArgs a = {};
+  a.x = x_dev;
+  a.T = num_tokens;
+  a.width = width;
+  a.experts = experts;
+  a.top = top;
+  a.w = static_cast<const uint16_t*>(w_bf16_dev);
+  a.ids = ids_dev;
+  a.wts = weights_dev;
+  a.kind = TL_ROUTE_SOFTMAX;
+  a.scale = scale;
   return tl_launch_router(a, static_cast<hipStream_t>(stream));
 }

@@ -162,6 +162,21 @@ __global__ __launch_bounds__(1024) void norm_rows_kernel(const float* __restrict
   for (int c = threadIdx.x; c < width; c += blockDim.x) out[(size_t)i * width + c] = row[c] * inv * (w_add + w[c]);
 }
 
+// the router of the feed-forward that reads the finished row in LDS: logits, a wave per expert in turn, then the selection
+__device__ __forceinline__ void route_row(const RouterArgs& r, float* row, int width, int t) {
+  __syncthreads();
+  float* z = row + ((width + 3) & ~3);  // [experts] (+ [experts] keys + [groups] for the group-ranked kinds)
+  const int wave = threadIdx.x >> 6, lane = threadIdx.x & 63, nwaves = blockDim.x >> 6;
+  const bool vec = (width & 7) == 0 && ((size_t)r.w & 15) == 0;
+  for (int e = wave; e < r.experts; e += nwaves) {
+    float sdot;
+    tl_wave_dot_rows<1>(r.w + (size_t)e * width, 0, 1, row, width, vec, lane, &sdot);
+    if (lane == 0) z[e] = sdot + (r.b ? r.b[e] : 0.0f);
+  }
+  __syncthreads();
+  if (wave == 0) tl_route_token(r, z, t, lane);
+}
+
 // pre-norm blocks with an RMS norm: the residual sum and the norm of what reads x next
 __global__ __launch_bounds__(1024) void resid_rms_kernel(const ResidRmsArgs a) {
   extern __shared__ __attribute__((aligned(16))) float row[];
@@ -212,28 +227,7 @@ __global__ __launch_bounds__(1024) void resid_rms_kernel(const ResidRmsArgs a) {
     }
   }
   if (!a.route.w) return;
-  // ---- the router of the feed-forward that reads h: logits over the row in LDS, a wave per expert in turn ----
-  __syncthreads();
-  float* z = row + ((a.width + 3) & ~3);  // [experts] (+ [experts] keys + [groups] for the group-ranked kinds)
-  const int wave = threadIdx.x >> 6, lane = threadIdx.x & 63, nwaves = blockDim.x >> 6;
-  const bool vec = (a.width & 7) == 0 && ((size_t)a.route.w & 15) == 0;
-  for (int e = wave; e < a.route.experts; e += nwaves) {
-    float sdot;
-    tl_wave_dot_rows<1>(a.route.w + (size_t)e * a.width, 0, 1, row, a.width, vec, lane, &sdot);
-    if (lane == 0) z[e] = sdot + (a.route.b ? a.route.b[e] : 0.0f);
-  }
-  __syncthreads();
-  if (wave != 0) return;
-  int* ids = a.route.ids + (size_t)t * a.route.top;
-  float* wts = a.route.wts + (size_t)t * a.route.top;
-  if (a.route.kind == TL_ROUTE_SIGMOID_GROUPS)
-    tl_route_select_sigmoid_groups(z, z + a.route.experts, z + 2 * a.route.experts, a.route.corr, a.route.experts, a.route.top,
-                                   a.route.groups, a.route.keep, ids, wts, lane);
-  else if (a.route.kind == TL_ROUTE_SOFTMAX_GROUPS)
-    tl_route_select_groups(z, z + a.route.experts, z + 2 * a.route.experts, a.route.experts, a.route.top, a.route.groups,
-                           a.route.keep, ids, wts, lane);
-  else
-    tl_route_select(z, a.route.experts, a.route.top, ids, wts, lane);
+  route_row(a.route, row, a.width, t);
 }
 
 constexpr int kMaxRowFloats = 16 * 1024;  // 64 KB of LDS for the staged row
@@ -267,13 +261,13 @@ __global__ __launch_bounds__(1024) void embed_ln_kernel(const unsigned short* __
   float mu, inv;
   if (emb.w) {
     ln_stats(row, width, eps, red, &mu, &inv);
-    for (int c = threadIdx.x; c < width; c += blockDim.x) row[c] = (row[c] - mu) * inv * emb.w[c] + emb.b[c];  // own columns only
+    for (int c = threadIdx.x; c < width; c += blockDim.x) row[c] = (row[c] - mu) * inv * emb.w[c] + (emb.b ? emb.b[c] : 0.0f);  // own columns only
     __syncthreads();
   }
   for (int c = threadIdx.x; c < width; c += blockDim.x) x[(size_t)t * width + c] = row[c];
   if (!next.w) return;
   ln_stats(row, width, eps, red, &mu, &inv);
-  for (int c = threadIdx.x; c < width; c += blockDim.x) h[(size_t)t * width + c] = (row[c] - mu) * inv * next.w[c] + next.b[c];
+  for (int c = threadIdx.x; c < width; c += blockDim.x) h[(size_t)t * width + c] = (row[c] - mu) * inv * next.w[c] + (next.b ? next.b[c] : 0.0f);
 }
 
 __global__ __launch_bounds__(1024) void resid_ln_kernel(float* __restrict__ x, const float* __restrict__ a, int width,
@@ -291,7 +285,7 @@ __global__ __launch_bounds__(1024) void resid_ln_kernel(float* __restrict__ x, c
   __syncthreads();
   float mu, inv;
   ln_stats(row, width, eps, red, &mu, &inv);
-  for (int c = threadIdx.x; c < width; c += blockDim.x) h[(size_t)t * width + c] = (row[c] - mu) * inv * next.w[c] + next.b[c];
+  for (int c = threadIdx.x; c < width; c += blockDim.x) h[(size_t)t * width + c] = (row[c] - mu) * inv * next.w[c] + (next.b ? next.b[c] : 0.0f);
 }
 
 __global__ __launch_bounds__(1024) void ln_rows_kernel(const float* __restrict__ x, int width, const int* __restrict__ rows,
@@ -304,7 +298,143 @@ __global__ __launch_bounds__(1024) void ln_rows_kernel(const float* __restrict__
   __syncthreads();
   float mu, inv;
   ln_stats(row, width, eps, red, &mu, &inv);
-  for (int c = threadIdx.x; c < width; c += blockDim.x) out[(size_t)i * width + c] = (row[c] - mu) * inv * p.w[c] + p.b[c];
+  for (int c = threadIdx.x; c < width; c += blockDim.x) out[(size_t)i * width + c] = (row[c] - mu) * inv * p.w[c] + (p.b ? p.b[c] : 0.0f);
+}
+
+// ---- residual streams: write-back of a sublayer into every stream, the next sublayer's input and its layer norm, one workgroup
+// per token. V columns at a time per thread (16-byte accesses); S streams (0: a.streams of them, at most kMaxStreams) -----------
+constexpr int kMaxStreams = 16;
+
+template <int V>
+struct HyperVec {
+  float v[V];
+  __device__ __forceinline__ void load(const float* p) {
+    if constexpr (V == 4) {
+      const float4 f = *reinterpret_cast<const float4*>(p);
+      v[0] = f.x, v[1] = f.y, v[2] = f.z, v[3] = f.w;
+    } else {
+      v[0] = p[0];
+    }
+  }
+  __device__ __forceinline__ void store(float* p) const {
+    if constexpr (V == 4) *reinterpret_cast<float4*>(p) = make_float4(v[0], v[1], v[2], v[3]);
+    else p[0] = v[0];
+  }
+};
+
+template <int S, int V>
+__global__ __launch_bounds__(1024) void hyper_kernel(const HyperArgs a) {
+  extern __shared__ __attribute__((aligned(16))) float row[];
+  __shared__ float red[kMaxWaves], cf[kMaxStreams * (kMaxStreams + 2)];
+  constexpr int SM = S > 0 ? S : kMaxStreams;
+  const int ns = S > 0 ? S : a.streams, t = blockIdx.x;
+  float* xr = a.x + (size_t)t * ns * a.width;
+  const bool add = a.a || a.slots;
+  // coefficients: mix [from][to] | mult * out [to] | in [from]
+  for (int i = threadIdx.x; i < ns * ns; i += blockDim.x) cf[i] = a.mix ? a.mix[i] : (i / ns == i % ns ? 1.0f : 0.0f);
+  for (int i = threadIdx.x; i < ns; i += blockDim.x) {
+    cf[ns * ns + i] = a.mult * (a.out ? a.out[i] : 1.0f);
+    cf[ns * ns + ns + i] = a.in ? a.in[i] : 1.0f;
+  }
+  __syncthreads();
+  int tok = 0;
+  bool known = true;
+  if (a.table) {
+    tok = a.tokens[t];
+    known = tok >= 0 && tok < a.vocab;
+  }
+  const unsigned short* er = a.table ? a.table + (size_t)(known ? tok : 0) * a.width : nullptr;
+  for (int c = threadIdx.x * V; c < a.width; c += blockDim.x * V) {
+    HyperVec<V> x[SM];
+    if (a.table) {
+#pragma unroll
+      for (int e = 0; e < V; ++e) {
+        const float v = known ? tl_bf2f(er[c + e]) * a.embed_scale : 0.0f;  // (an id outside the table embeds as zeros)
+#pragma unroll
+        for (int s = 0; s < SM; ++s) x[s].v[e] = v;
+      }
+    } else {
+#pragma unroll
+      for (int s = 0; s < SM; ++s)
+        if (s < ns) x[s].load(xr + (size_t)s * a.width + c);
+    }
+    if (add) {
+      HyperVec<V> y;
+#pragma unroll
+      for (int e = 0; e < V; ++e) y.v[e] = 0.0f;
+      if (a.a) y.load(a.a + (size_t)t * a.width + c);
+      if (a.slots) {
+        HyperVec<V> es;
+#pragma unroll
+        for (int e = 0; e < V; ++e) es.v[e] = 0.0f;
+        for (int j = 0; j < a.top; ++j) {
+          HyperVec<V> o;
+          o.load(a.slots + ((size_t)t * a.top + j) * a.width + c);
+          const float w = a.slot_w[t * a.top + j];
+#pragma unroll
+          for (int e = 0; e < V; ++e) es.v[e] += w * o.v[e];
+        }
+#pragma unroll
+        for (int e = 0; e < V; ++e) y.v[e] += es.v[e];
+      }
+      HyperVec<V> n[SM];
+#pragma unroll
+      for (int o = 0; o < SM; ++o) {
+        if (o >= ns) continue;
+#pragma unroll
+        for (int e = 0; e < V; ++e) n[o].v[e] = cf[ns * ns + o] * y.v[e];
+#pragma unroll
+        for (int s = 0; s < SM; ++s) {
+          if (s >= ns) continue;
+          const float m = cf[s * ns + o];
+#pragma unroll
+          for (int e = 0; e < V; ++e) n[o].v[e] += m * x[s].v[e];
+        }
+      }
+#pragma unroll
+      for (int s = 0; s < SM; ++s)
+        if (s < ns) x[s] = n[s];
+    }
+    HyperVec<V> u, sm;
+#pragma unroll
+    for (int e = 0; e < V; ++e) u.v[e] = sm.v[e] = 0.0f;
+#pragma unroll
+    for (int s = 0; s < SM; ++s) {
+      if (s >= ns) continue;
+      if (add || a.table) x[s].store(xr + (size_t)s * a.width + c);
+      const float w = cf[ns * ns + ns + s];
+#pragma unroll
+      for (int e = 0; e < V; ++e) {
+        u.v[e] += w * x[s].v[e];
+        sm.v[e] += x[s].v[e];
+      }
+    }
+    if (a.sum) sm.store(a.sum + (size_t)t * a.width + c);
+    u.store(row + c);
+  }
+  if (!a.next.w) return;
+  __syncthreads();
+  float mu, inv;
+  ln_stats(row, a.width, a.eps, red, &mu, &inv);
+  for (int c = threadIdx.x; c < a.width; c += blockDim.x) {
+    const float v = (row[c] - mu) * inv * a.next.w[c] + (a.next.b ? a.next.b[c] : 0.0f);
+    a.h[(size_t)t * a.width + c] = v;
+    row[c] = v;  // (own columns only) stays for the router below
+  }
+  if (!a.route.w) return;
+  route_row(a.route, row, a.width, t);
+}
+
+template <int V>
+void launch_hyper(const HyperArgs& a, size_t lds, hipStream_t s) {
+  const int th = row_threads(a.T);
+  switch (a.streams) {
+    case 1: hyper_kernel<1, V><<<a.T, th, lds, s>>>(a); break;
+    case 2: hyper_kernel<2, V><<<a.T, th, lds, s>>>(a); break;
+    case 3: hyper_kernel<3, V><<<a.T, th, lds, s>>>(a); break;
+    case 4: hyper_kernel<4, V><<<a.T, th, lds, s>>>(a); break;
+    default: hyper_kernel<0, 1><<<a.T, th, lds, s>>>(a); break;
+  }
 }
 
 __device__ __forceinline__ float dyt_of(float x, float alpha, float w, float b) { return tanhf(alpha * x) * w + b; }
@@ -381,7 +511,7 @@ int tl_launch_embed_ln(const uint16_t* table, int vocab, int width, const int* t
                        const LnParams& next, float eps, float* x, float* h, hipStream_t s) {
   TL_REQUIRE(table && tokens_dev && x && T > 0 && vocab > 0, "embed_ln: bad arguments");
   TL_REQUIRE(width > 0 && width <= kMaxRowFloats, "embed_ln: width %d outside (0, %d]", width, kMaxRowFloats);
-  TL_REQUIRE((!emb.w || emb.b) && (!next.w || (next.b && h)), "embed_ln: a norm without its bias or output");
+  TL_REQUIRE(!next.w || h, "embed_ln: a norm without its output");
   embed_ln_kernel<<<T, row_threads(T), sizeof(float) * width, s>>>(table, vocab, width, tokens_dev, emb, next, eps, x, h);
   TL_HIP(hipGetLastError());
   return 0;
@@ -390,7 +520,7 @@ int tl_launch_embed_ln(const uint16_t* table, int vocab, int width, const int* t
 int tl_launch_resid_ln(float* x, const float* a, int T, int width, const LnParams& next, float eps, float* h, hipStream_t s) {
   TL_REQUIRE(x && a && T > 0, "resid_ln: bad arguments");
   TL_REQUIRE(width > 0 && width <= kMaxRowFloats, "resid_ln: width %d outside (0, %d]", width, kMaxRowFloats);
-  TL_REQUIRE(!next.w || (next.b && h), "resid_ln: a norm without its bias or output");
+  TL_REQUIRE(!next.w || h, "resid_ln: a norm without its output");
   resid_ln_kernel<<<T, row_threads(T), sizeof(float) * width, s>>>(x, a, width, next, eps, h);
   TL_HIP(hipGetLastError());
   return 0;
@@ -398,7 +528,7 @@ int tl_launch_resid_ln(float* x, const float* a, int T, int width, const LnParam
 
 int tl_launch_ln_rows(const float* x, int width, const int* rows_dev, int n, const LnParams& p, float eps, float* out,
                       hipStream_t s) {
-  TL_REQUIRE(x && out && p.w && p.b && n > 0, "ln_rows: bad arguments");
+  TL_REQUIRE(x && out && p.w && n > 0, "ln_rows: bad arguments");
   TL_REQUIRE(width > 0 && width <= kMaxRowFloats, "ln_rows: width %d outside (0, %d]", width, kMaxRowFloats);
   ln_rows_kernel<<<n, row_threads(n), sizeof(float) * width, s>>>(x, width, rows_dev, p, eps, out);
   TL_HIP(hipGetLastError());
@@ -461,7 +591,7 @@ int tl_launch_resid_rms(const ResidRmsArgs& a, hipStream_t s) {
     const RouterArgs& r = a.route;
     TL_REQUIRE(a.w && r.ids && r.wts && r.experts > 0 && r.top > 0 && r.top <= r.experts && !r.gate_w,
                "resid_rms: bad router arguments");
-    TL_REQUIRE(r.kind == TL_ROUTE_TOP_LOGITS || (r.groups > 0 && r.experts % r.groups == 0 && r.keep > 0 && r.keep <= r.groups &&
+    TL_REQUIRE(r.kind == TL_ROUTE_TOP_LOGITS || r.kind == TL_ROUTE_SOFTMAX || (r.groups > 0 && r.experts % r.groups == 0 && r.keep > 0 && r.keep <= r.groups &&
                                                   (long long)r.keep * (r.experts / r.groups) >= r.top),
                "resid_rms: %d experts in %d groups, %d kept, top %d", r.experts, r.groups, r.keep, r.top);
     lds = sizeof(float) * (((a.width + 3) & ~3) + 2 * (size_t)r.experts + (r.groups > 0 ? r.groups : 0));
@@ -491,4 +621,51 @@ extern "C" int tl_resid_rmsnorm(float* x_dev, const float* y_dev, const float* w
   a.w = weight_dev;
   a.eps = eps;
   return tl_launch_resid_norm(a, static_cast<hipStream_t>(stream));
+}
+
+int tl_launch_hyper(const HyperArgs& a, hipStream_t s) {
+  TL_REQUIRE(a.x && a.T > 0 && (a.a || a.slots || a.table || a.sum || a.next.w), "hyper: bad arguments");
+  TL_REQUIRE(a.streams >= 1 && a.streams <= kMaxStreams, "hyper: %d streams outside [1, %d]", a.streams, kMaxStreams);
+  TL_REQUIRE(a.width > 0 && a.width <= kMaxRowFloats, "hyper: width %d outside (0, %d]", a.width, kMaxRowFloats);
+  TL_REQUIRE(!a.slots || (a.slot_w && a.top > 0), "hyper: expert slots without weights");
+  TL_REQUIRE(!a.table || (a.tokens && a.vocab > 0 && !a.a && !a.slots), "hyper: an embedding table without tokens, or with a sublayer's output");
+  TL_REQUIRE(!a.next.w || a.h, "hyper: a norm without its output");
+  size_t lds = sizeof(float) * a.width;
+  if (a.route.w) {
+    const RouterArgs& r = a.route;
+    TL_REQUIRE(a.next.w && r.ids && r.wts && r.experts > 0 && r.top > 0 && r.top <= r.experts && !r.gate_w,
+               "hyper: bad router arguments");
+    TL_REQUIRE(r.kind == TL_ROUTE_TOP_LOGITS || r.kind == TL_ROUTE_SOFTMAX ||
+                   (r.groups > 0 && r.experts % r.groups == 0 && r.keep > 0 && r.keep <= r.groups &&
+                    (long long)r.keep * (r.experts / r.groups) >= r.top),
+               "hyper: %d experts in %d groups, %d kept, top %d", r.experts, r.groups, r.keep, r.top);
+    lds = sizeof(float) * (((a.width + 3) & ~3) + 2 * (size_t)r.experts + (r.groups > 0 ? r.groups : 0));
+    TL_REQUIRE(lds <= 64 * 1024 - 2048, "hyper: width %d + %d experts do not fit the staged row", a.width, r.experts);
+  }
+  const bool v4 = (a.width & 3) == 0 && ((size_t)a.x & 15) == 0 && ((size_t)a.a & 15) == 0 && ((size_t)a.slots & 15) == 0 &&
+                  ((size_t)a.sum & 15) == 0;
+  if (v4) launch_hyper<4>(a, lds, s);
+  else launch_hyper<1>(a, lds, s);
+  TL_HIP(hipGetLastError());
+  return 0;
+}
+
+extern "C" int tl_hyper_connect(float* x_dev, const float* y_dev, const float* mix_dev, const float* out_dev, float mult,
+                                const float* in_dev, const float* weight_dev, const float* bias_dev, float eps, float* h_dev,
+                                float* sum_dev, int num_tokens, int streams, int width, void* stream) {
+  HyperArgs a = {};
+  a.x = x_dev;
+  a.T = num_tokens;
+  a.width = width;
+  a.streams = streams;
+  a.a = y_dev;
+  a.mix = mix_dev;
+  a.out = out_dev;
+  a.mult = mult;
+  a.in = in_dev;
+  if (in_dev) a.next = LnParams{weight_dev, bias_dev};
+  a.eps = eps;
+  a.h = h_dev;
+  a.sum = sum_dev;
+  return tl_launch_hyper(a, static_cast<hipStream_t>(stream));
 }

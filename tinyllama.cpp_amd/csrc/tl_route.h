@@ -4,9 +4,22 @@
 #include <hip/hip_runtime.h>
 #include <math.h>
 
+#include "tlhip.h"
+
 // One wave (all 64 lanes) picks the `top` largest of z[experts] (LDS; overwritten), the lower index among equals, and writes
-// ids[top] (largest first) and wts[top] = the softmax over the chosen logits.
-__device__ __forceinline__ void tl_route_select(float* z, int experts, int top, int* ids, float* wts, int lane) {
+// ids[top] (largest first) and wts[top] = the softmax over the chosen logits; over_all: the softmax over ALL logits, times scale.
+__device__ __forceinline__ void tl_route_select(float* z, int experts, int top, int* ids, float* wts, int lane, bool over_all = false,
+                                                float scale = 1.0f) {
+    float all = 0.0f, top_z = 0.0f;
+    if (over_all) {  // the sum over every expert, before the choices are taken out of z
+      top_z = -INFINITY;
+      for (int e = lane; e < experts; e += 64) top_z = fmaxf(top_z, z[e]);
+#pragma unroll
+      for (int o = 32; o >= 1; o >>= 1) top_z = fmaxf(top_z, __shfl_xor(top_z, o));
+      for (int e = lane; e < experts; e += 64) all += expf(z[e] - top_z);
+#pragma unroll
+      for (int o = 32; o >= 1; o >>= 1) all += __shfl_xor(all, o);
+    }
     // `top` rounds: the lanes scan the experts not yet chosen for the largest logit (lower index wins among equals)
     float mx = 0.0f, denom = 0.0f, mine = 0.0f;
     int my_id = -1;
@@ -46,12 +59,13 @@ __device__ __forceinline__ void tl_route_select(float* z, int experts, int top, 
       __builtin_amdgcn_wave_barrier();
       __builtin_amdgcn_fence(__ATOMIC_ACQUIRE, "wavefront");
     }
+    if (over_all) denom = all;  // (the first choice is the largest logit: mx == top_z)
     if (lane < top && lane < 64) {
       ids[lane] = my_id;
-      wts[lane] = mine / denom;
+      wts[lane] = mine / denom * scale;
     }
     if (top > 64 && lane == 0)
-      for (int j = 64; j < top; ++j) wts[j] /= denom;
+      for (int j = 64; j < top; ++j) wts[j] = wts[j] / denom * scale;
 }
 
 // One wave: scores = softmax(z) over all experts (left in z[]); the experts form `groups` equal groups of neighbours, a
@@ -233,4 +247,18 @@ __device__ __forceinline__ void tl_route_select_sigmoid_groups(float* z, float* 
     }
     wave_sync();
   }
+}
+
+// the selection of a router of any kind (R: RouterArgs) for token t: z [experts] logits in LDS, behind them scratch for the
+// group-ranked kinds ([experts] + [groups])
+template <class R>
+__device__ __forceinline__ void tl_route_token(const R& r, float* z, int t, int lane) {
+  int* ids = r.ids + (size_t)t * r.top;
+  float* wts = r.wts + (size_t)t * r.top;
+  if (r.kind == TL_ROUTE_SIGMOID_GROUPS)
+    tl_route_select_sigmoid_groups(z, z + r.experts, z + 2 * r.experts, r.corr, r.experts, r.top, r.groups, r.keep, ids, wts, lane);
+  else if (r.kind == TL_ROUTE_SOFTMAX_GROUPS)
+    tl_route_select_groups(z, z + r.experts, z + 2 * r.experts, r.experts, r.top, r.groups, r.keep, ids, wts, lane);
+  else
+    tl_route_select(z, r.experts, r.top, ids, wts, lane, r.kind == TL_ROUTE_SOFTMAX, r.kind == TL_ROUTE_SOFTMAX ? r.scale : 1.0f);
 }

@@ -12,7 +12,9 @@
 //                 pre-norm blocks (residual sum + the norm of the sublayer that follows)
 //   tl_rope.hip   rotary positions, per-head unit norm;  tl_delta.hip  two delta-rule recurrences with their preparation
 //   tl_conv.hip   a short causal convolution over time per channel with its history (sublayer inputs; projected q, k, v)
-//   tl_latent.hip latent attention: norms of the latents, the rotated shared key part, cache rows, per-head output gate
+//   tl_latent.hip latent attention: norms of the latents, the rotated shared key part, cache rows, output gates
+//   tl_ssm.hip    selective state space (one decay per head and token): blocks of a prompt on the matrix cores, one-token step,
+//                 RMS norm of a row in equal parts
 #pragma once
 #include "tl_internal.h"
 
@@ -61,6 +63,7 @@ int tl_launch_dense_gemv_heads(const uint16_t* w, int groups, int rows, int cols
 __host__ __device__ inline float tl_act_apply(int act, float z, float p, float q) {
   if (act == TL_ACT_XIELU) return z > 0.0f ? p * z * z + 0.5f * z : q * (expm1f(z) - z) + 0.5f * z;
   if (act == TL_ACT_TANH) return tanhf(z);
+  if (act == TL_ACT_GELU) return 0.5f * z * (1.0f + erff(z * 0.70710678118654752f));
   return z;
 }
 
@@ -156,6 +159,7 @@ struct RouterArgs {
   // kind = TL_ROUTE_SIGMOID_GROUPS: scores = sigmoid(logits), choice = score + corr[expert]; a group ranks by the sum of its two
   // best choices; wts = the chosen experts' scores as they are
   const float* corr;
+  float scale;           // kind = TL_ROUTE_SOFTMAX: wts = softmax over ALL experts of the chosen, times scale
 };
 struct ResidNormArgs {
   float* x;              // [T][width] residual stream, updated in place: x += y / rms(y) * (1 + w)
@@ -227,16 +231,41 @@ int tl_launch_dyt_rows(const float* x, int width, const int* rows_dev, int n, co
 int tl_launch_norm_rows(const float* x, int width, const int* rows_dev, int n, const float* w, float eps, float* out,
                         hipStream_t s, int one_plus = 1);
 
-// ---- layer norm (pre-norm blocks): (x - mean) / sqrt(var + eps) * w + b, statistics in FP32 over the row staged in LDS -------
+// ---- layer norm (pre-norm blocks): (x - mean) / sqrt(var + eps) * w (+ b), statistics in FP32 over the row staged in LDS -------
 struct LnParams {
   const float* w;        // [width] (NULL: no norm asked for)
-  const float* b;        // [width]
+  const float* b;        // optional [width]
 };
 // x[t] = ln(embed[token[t]]; emb) (emb.w == NULL: the plain row); h[t] = ln(x[t]; next) when next.w is set
 int tl_launch_embed_ln(const uint16_t* table, int vocab, int width, const int* tokens_dev, int T, const LnParams& emb,
                        const LnParams& next, float eps, float* x, float* h, hipStream_t s);
 // x[t] += a[t]; h[t] = ln(x[t]; next) when next.w is set (the norm in front of the sublayer that follows)
 int tl_launch_resid_ln(float* x, const float* a, int T, int width, const LnParams& next, float eps, float* h, hipStream_t s);
+// Residual streams (hyper-connections) of pre-norm blocks behind a layer norm; streams == 1 with null mixing weights is the plain
+// residual sum x += mult y. In order: every stream x_s of a token is the scaled embedding row (table set), or as stored; with a
+// sublayer output y (a, slots) x_t <- sum_s mix[s][t] x_s + mult out[t] y; sum <- sum_s x_s; h = ln(sum_s in[s] x_s).
+struct HyperArgs {
+  float* x;              // [T][streams][width]
+  int T, width, streams;
+  const uint16_t* table; // optional: start of a forward pass
+  const int* tokens;
+  int vocab;
+  float embed_scale;
+  const float* a;        // optional [T][width]
+  const float* slots;    // optional [T * top][width] expert outputs, weighted by slot_w
+  const float* slot_w;   // [T * top]
+  int top;
+  const float* mix;      // [streams][streams], from x to (NULL: identity)
+  const float* out;      // [streams] (NULL: ones)
+  float mult;
+  float* sum;            // optional [T][width]
+  const float* in;       // [streams] (NULL: ones)
+  LnParams next;         // next.w == NULL: no norm asked for
+  float eps;
+  float* h;              // [T][width]
+  RouterArgs route;      // optional (route.w): the router of the feed-forward that reads h, as in ResidRmsArgs
+};
+int tl_launch_hyper(const HyperArgs& a, hipStream_t s);
 // out[i] = ln(x[rows[i]]; p)   (rows == NULL: row i)
 int tl_launch_ln_rows(const float* x, int width, const int* rows_dev, int n, const LnParams& p, float eps, float* out,
                       hipStream_t s);
@@ -249,6 +278,7 @@ struct ConvArgs {
   const float* in;       // [T][ldi], channels [0, C)
   int ldi, C, taps, T;
   const float* bias;     // optional [C]
+  const float* out_bias; // optional [C]: added to the convolution's result, in front of the activation
   const uint16_t* w;     // bf16 [C][taps], the last tap is the current token's
   float* hist;           // [taps - 1][C]
   int act;               // 0: none, 1: silu
@@ -266,6 +296,8 @@ struct LatentPostArgs {
   const float* kv_norm;  // plain weights [kv_rank] (NULL: this layer projects no latent of its own; kv_rank columns absent)
   float eps;
   int rot_dims;          // the first rot_dims of the rot_dim part turn, (2i, 2i + 1) by position * freq[i]
+  int halves;            // 1: the pairs are (i, i + rot_dims / 2)
+  float mscale;          // factor on cos and sin
   const double* freq;
   float* cache;          // [max_pos][kv_rank + rot_dim]: row pos = normalised latent | rotated key part
   int T, start_pos;
@@ -278,6 +310,8 @@ struct LatentQueryArgs {
   float* out;            // [T][heads * out_stride]: it goes to column n * out_stride + out_off (may be q itself: in place)
   int out_stride, out_off;
   int heads, rot_dim, rot_dims;
+  int halves;            // as LatentPostArgs
+  float mscale;
   const double* freq;
   int T, start_pos;
   const int* pos_dev;
@@ -286,6 +320,8 @@ int tl_launch_latent_query(const LatentQueryArgs& a, hipStream_t s);
 // keys per head for a prompt chunk: k[p][n * (dim + rot_dim) + dim ..] = the rotated part of cache row p, for every head n and
 // the rows p < P (the plain parts in front come from a product per head over the same rows)
 int tl_launch_latent_spread(const float* cache, int kv_rank, int rot_dim, float* k, int heads, int dim, int P, hipStream_t s);
+// o[t][c] *= sigmoid(gate[t * gate_ld + c]) for the od columns of a token
+int tl_launch_out_gate(float* o, const float* gate, int gate_ld, int T, int od, hipStream_t s);
 // o[t][n][:] *= sigmoid(gate[t * gate_ld + n]) for the heads n of a token; o [T][heads * vdim]
 int tl_launch_head_gate(float* o, const float* gate, int gate_ld, int T, int heads, int vdim, hipStream_t s);
 
@@ -317,6 +353,7 @@ struct MoeDecodeArgs {
   float up_add;          // the gated unit's (u + up_add)
   const float* sgate;    // optional device scalar: factor on the shared expert's output
   int glu_kind;          // tl_glu_kind
+  int unit_act;          // != 0 (a tl_act_kind, no shared expert): plain experts down act(up x), gu = up [experts][ff][width]
 };
 int tl_launch_moe_decode(const MoeDecodeArgs& a, hipStream_t s);
 
@@ -441,6 +478,48 @@ struct GDeltaScanArgs {
   int T, heads, dim, vdim;
 };
 int tl_launch_gdelta_scan(const GDeltaScanArgs& a, hipStream_t s);
+
+// ---- tl_ssm.hip: S <- exp(-exp(a_log) dt) S + dt B x^T, y = S^T C + d x, y silu(z) per head; dt = softplus(raw + dt_bias) -----
+struct SsmScanArgs {
+  const float* xbc;      // [T][ld]: x (heads * vdim) | B (groups * state_n) | C (groups * state_n), convolved and activated
+  int ld;
+  const float* dt_raw;   // token t, head h at t * dt_ld + h
+  int dt_ld;
+  const float *dt_bias, *a_log, *d;  // [heads]
+  const float* z;        // optional, token t at t * z_ld
+  int z_ld;
+  float* state;          // [heads][state_n][vdim]; updated
+  float* y;              // [T][heads * vdim]
+  float* gram;           // scratch, tl_ssm_gram_floats
+  int T, heads, groups, state_n, vdim;
+};
+size_t tl_ssm_gram_floats(int T, int groups);
+int tl_launch_ssm_scan(const SsmScanArgs& a, hipStream_t s);
+// one token with its convolution
+struct SsmStepArgs {
+  const float* p;        // z | x | B | C | dt as projected
+  const uint16_t* conv;  // bf16 [channels][taps], channels = x | B | C; the last tap is the current token's
+  const float* conv_b;   // [channels]
+  int taps;
+  const float* hist;     // [taps - 1][channels], oldest first; not written (PartNormArgs::hist)
+  const float *dt_bias, *a_log, *d;
+  float* state;
+  float* y;              // [heads * vdim]
+  int heads, groups, state_n, vdim;
+};
+int tl_launch_ssm_step(const SsmStepArgs& a, hipStream_t s);
+// every row of x [T][width] in `parts` equal parts, each divided by its root mean square, times w [width]; in place. hist (one
+// row): a convolution's history [taps - 1][channels] drops its oldest row and gains hist_in [channels]
+struct PartNormArgs {
+  float* x;
+  const float* w;
+  int T, width, parts;
+  float eps;
+  float* hist;
+  const float* hist_in;
+  int taps, channels;
+};
+int tl_launch_part_norm(const PartNormArgs& a, hipStream_t s);
 
 // ---- tl_stack.hip: the engine ------------------------------------------------------------------------------------------
 struct TlStack;

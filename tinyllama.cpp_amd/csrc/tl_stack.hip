@@ -23,15 +23,23 @@
 //                         gdelta_pre, gdelta_scan over a per-head state, gated head norm with weights per head; W_o
 //         TL_MIXER_LINEAR gated linear attention: q | f | v = W h in one product; silu, forget gate and what it writes (linear_pre);
 //                         the delta rule's scan without its removal step; RMS norm per head; W_o
+//         TL_MIXER_SSM    z | x | B | C | dt = W h in one product; several tokens: convolution, the blocks' C B^T, the walk over the
+//                         blocks with the state in registers (it applies D, the gate silu(z)), RMS norm in parts; one token: convolution,
+//                         state update and read-out in one launch, then the norm, which also shifts the convolution's history; W_o
 //         TL_MIXER_SWA with its options: two score maps per head over the same values (differential attention: one attention
 //                         launch per map, then (a1 - lambda a2) / rms (1 - diff) sigmoid(gate)), a norm per head and map, biases
 //                         and a causal convolution on q, k, v (tl_conv.hip), capped scores, a logarithmic distance bias, a learned
 //                         sink per head; TL_MIXER_DELTA with one decay per head and direct projections for decay and gate
 //         Two mixers side by side (tl_layer_spec::side): both read the same input, their first products are one product, the
 //                         layer's mixer output is mix_scale * first + side_scale * second
+//         Pre-norm blocks behind a layer norm may keep several residual streams (hyper-connections, tl_stack_config::streams): the
+//                         launch that finishes a sublayer mixes the old streams, adds its output to each, sums the next sublayer's
+//                         input from the new ones and norms it (tl_norm.hip: hyper). Without streams the same launch adds experts'
+//                         outputs and scaled residuals
 //         Pre-norm blocks behind the plain RMS norm (TL_NORM_RMS) may add a causal convolution over time to what each sublayer
 //                         reads (canon_taps); the embedding row may be scaled (embed_scale)
-// Feed-forward  TL_MLP_UNIT  W_down act(W_up h), the activation in the first product's epilogue (pre-norm blocks)
+// Feed-forward  TL_MLP_MOE with an activation: plain experts W_down act(W_up h)
+//               TL_MLP_UNIT  W_down act(W_up h), the activation in the first product's epilogue (pre-norm blocks)
 //               TL_MLP_MOE  router (three kinds, tl_moe.hip) -> top experts (gated units) + optional shared expert, optionally
 //                           gated per token;  TL_MLP_DENSE  one gated unit (it runs where a shared expert would)
 // A layer may use an earlier layer's tensors (weights_of) with a cache or state of its own.
@@ -42,7 +50,8 @@
 // flat by absolute position; a window only bounds what attention reads. Delta layers: S [heads][vdim][dim] and the
 // convolution's last taps - 1 inputs (linear attention: S only; attention with a convolution on q, k, v: that history too;
 // every layer: the histories of the convolutions on what its sublayers read); latent layers with a projection of their
-// own: rows [max_positions][kv_rank + rot_dim]; generalized delta layers: S [heads][dim][dim]. tl_stack_reset gives everything back (one sequence at a time): zeros are the state of
+// own: rows [max_positions][kv_rank + rot_dim]; generalized delta layers: S [heads][dim][dim]; state-space layers: S
+// [heads][state][vdim] and the convolution's history. tl_stack_reset gives everything back (one sequence at a time): zeros are the state of
 // an empty sequence.
 #include <math.h>
 #include <stdio.h>
@@ -97,6 +106,10 @@ struct Layer {
   float *lower = nullptr, *f_bias = nullptr;  // gated linear attention: lower bound and bias of the forget gate
   uint16_t *canon1 = nullptr, *canon2 = nullptr;          // convolutions on what the sublayers read [width][taps]
   float *canon_hist1 = nullptr, *canon_hist2 = nullptr;   // ... and their last taps - 1 inputs (state)
+  // state space: wqkv = in, conv / hist above, dt_bias, a_log, onorm [heads * vdim]
+  float *conv_b = nullptr, *dskip = nullptr;
+  // hyper-connections of the two sublayers: in [streams], out [streams], mix [streams][streams]
+  float *hc_in[2] = {nullptr, nullptr}, *hc_out[2] = {nullptr, nullptr}, *hc_mix[2] = {nullptr, nullptr};
   std::unique_ptr<Layer> side;               // the second mixer of a pair: its mixer fields, tensors and state only
   std::set<std::string> expect, optional;    // tensor names (without the "l<i>." prefix) still missing / accepted and ignored
 };
@@ -135,6 +148,9 @@ struct TlStack {
   float* h = nullptr;       // norm-first blocks: the normalised input both sublayers read
   float *dq = nullptr, *da = nullptr, *dg = nullptr, *dbeta = nullptr, *ddecay = nullptr;  // delta rule
   float *lq = nullptr, *lqa = nullptr;      // latent attention: up-projected queries, absorbed queries
+  float* xs = nullptr;                      // residual streams [chunk][streams][width] (x then holds their sum)
+  float* gram = nullptr;                    // state space: C B^T of a chunk's blocks
+  size_t max_gram = 0;
   float *lk = nullptr, *lv = nullptr;       // ... and, for long chunks, keys / values per head of every row the chunk sees
   int max_lk = 0, max_lv = 0;
   int latent_expand = 64;                   // chunks of at least this many tokens expand (TL_STACK_LATENT_EXPAND; 0: never)
@@ -218,10 +234,10 @@ int setup_mixer(TlStack* st, Layer& L, int i, bool own, int* first_mix) {
   const tl_stack_config* cfg = &st->cfg;
   const tl_layer_spec& sp = L.sp;
   const size_t W = cfg->width;
-  TL_REQUIRE(sp.mixer >= TL_MIXER_SWA && sp.mixer <= TL_MIXER_LINEAR,
+  TL_REQUIRE(sp.mixer >= TL_MIXER_SWA && sp.mixer <= TL_MIXER_SSM,
              "tl_stack_create: layer %d has mixer kind %d; this engine has windowed attention (%d), the gated delta rule (%d), "
-             "latent attention (%d), the generalized delta rule (%d) and gated linear attention (%d)",
-             i, sp.mixer, TL_MIXER_SWA, TL_MIXER_DELTA, TL_MIXER_LATENT, TL_MIXER_GDELTA, TL_MIXER_LINEAR);
+             "latent attention (%d), the generalized delta rule (%d), gated linear attention (%d) and the state space (%d)",
+             i, sp.mixer, TL_MIXER_SWA, TL_MIXER_DELTA, TL_MIXER_LATENT, TL_MIXER_GDELTA, TL_MIXER_LINEAR, TL_MIXER_SSM);
   TL_REQUIRE(sp.heads > 0 && sp.kv_heads > 0 && sp.heads % sp.kv_heads == 0 && sp.dim > 0 && sp.vdim > 0,
              "tl_stack_create: layer %d: %d heads / %d key-value heads / sizes %d, %d", i, sp.heads, sp.kv_heads, sp.dim, sp.vdim);
   if (sp.mixer == TL_MIXER_SWA) {
@@ -314,7 +330,9 @@ int setup_mixer(TlStack* st, Layer& L, int i, bool own, int* first_mix) {
                  "tl_stack_create: layer %d reads the latent cache of layer %d, which is not an earlier latent layer "
                  "with a projection of its own", i, j);
       const tl_layer_spec& o = st->layers[j].sp;
-      TL_REQUIRE(o.kv_rank == sp.kv_rank && o.rot_dim == sp.rot_dim && o.rot_dims == sp.rot_dims && o.rot_base == sp.rot_base,
+      TL_REQUIRE(o.kv_rank == sp.kv_rank && o.rot_dim == sp.rot_dim && o.rot_dims == sp.rot_dims && o.rot_base == sp.rot_base &&
+                     o.rot_halves == sp.rot_halves && o.rot_factor == sp.rot_factor && o.rot_original == sp.rot_original &&
+                     o.rot_fast == sp.rot_fast && o.rot_slow == sp.rot_slow,
                  "tl_stack_create: layer %d and layer %d, whose latent cache it reads, differ in latent size or rotation", i, j);
       L.kv_src = j;
     }
@@ -325,7 +343,8 @@ int setup_mixer(TlStack* st, Layer& L, int i, bool own, int* first_mix) {
     L.vd = 0;
     L.od = sp.heads * sp.vdim;
     L.gate_off = sp.q_rank + L.kd;
-    L.pd = L.gate_off + (sp.head_gate ? sp.heads : 0);
+    TL_REQUIRE(!sp.head_gate || !sp.out_gate, "tl_stack_create: layer %d: a gate per head and one per output column", i);
+    L.pd = L.gate_off + (sp.head_gate ? sp.heads : sp.out_gate ? L.od : 0);
     if (own_kv) st->cache_bytes += sizeof(float) * (size_t)cfg->max_positions * L.kd;
     st->max_lq = L.qd > st->max_lq ? L.qd : st->max_lq;
     st->max_lqa = sp.heads * ah > st->max_lqa ? sp.heads * ah : st->max_lqa;
@@ -334,7 +353,7 @@ int setup_mixer(TlStack* st, Layer& L, int i, bool own, int* first_mix) {
     st->max_od = sp.heads * sp.kv_rank > st->max_od ? sp.heads * sp.kv_rank : st->max_od;  // the weighted latents of all heads
     L.expect.insert({"mix.dq", "mix.dq.norm", "mix.uq", "mix.uk", "mix.uv", "mix.o"});
     if (own_kv) L.expect.insert({"mix.dkv", "mix.dkv.norm"});
-    if (sp.head_gate) L.expect.insert("mix.g");
+    if (sp.head_gate || sp.out_gate) L.expect.insert("mix.g");
     TL_TRY(dev_alloc(st, &L.wuq, (size_t)L.qd * sp.q_rank));
     TL_TRY(dev_alloc(st, &L.wukt, (size_t)sp.heads * sp.kv_rank * sp.dim));
     TL_TRY(dev_alloc(st, &L.wuk, (size_t)sp.heads * sp.kv_rank * sp.dim));
@@ -343,8 +362,7 @@ int setup_mixer(TlStack* st, Layer& L, int i, bool own, int* first_mix) {
     TL_TRY(dev_alloc(st, &L.dkv_norm, sp.kv_rank));
     if (sp.rot_dims > 0) {
       std::vector<double> f(sp.rot_dims / 2);
-      float unused = 1.0f;
-      tl_rotary_frequencies(sp.rot_dims, sp.rot_base, 0.0, 0.0, 0.0, 0.0, f.data(), &unused);
+      tl_rotary_frequencies(sp.rot_dims, sp.rot_base, sp.rot_factor, sp.rot_original, sp.rot_fast, sp.rot_slow, f.data(), &L.mscale);
       TL_TRY(upload_frequencies(st, L, f));
     }
   } else if (sp.mixer == TL_MIXER_GDELTA) {
@@ -363,6 +381,26 @@ int setup_mixer(TlStack* st, Layer& L, int i, bool own, int* first_mix) {
     TL_TRY(dev_alloc(st, &L.w0, hd));
     TL_TRY(dev_alloc(st, &L.a_bias, hd));
     TL_TRY(dev_alloc(st, &L.onorm, hd));
+  } else if (sp.mixer == TL_MIXER_SSM) {
+    TL_REQUIRE(sp.dim <= 512 && sp.conv_taps >= 1 && sp.conv_taps <= 64 && sp.norm_parts > 0 && (sp.heads * sp.vdim) % sp.norm_parts == 0,
+               "tl_stack_create: layer %d: state size %d (at most 512), %d taps, a norm in %d parts of %d", i, sp.dim, sp.conv_taps,
+               sp.norm_parts, sp.heads * sp.vdim);
+    TL_REQUIRE(sp.weights_of == 0 && own, "tl_stack_create: layer %d: a state-space layer owns its tensors", i);
+    L.od = L.vd = sp.heads * sp.vdim;
+    L.qd = L.kd = sp.kv_heads * sp.dim;  // C, B
+    const int ch = L.vd + L.kd + L.qd;   // channels of the convolution: x | B | C
+    L.pd = L.od + ch + sp.heads;         // z | x | B | C | dt
+    st->max_dc = ch > st->max_dc ? ch : st->max_dc;
+    const size_t gr = tl_ssm_gram_floats(st->chunk, sp.kv_heads);
+    st->max_gram = gr > st->max_gram ? gr : st->max_gram;
+    st->cache_bytes += sizeof(float) * ((size_t)sp.heads * sp.vdim * sp.dim + (size_t)(sp.conv_taps - 1) * ch);
+    L.expect.insert({"mix.in", "mix.conv", "mix.conv.b", "mix.dt_bias", "mix.A_log", "mix.D", "mix.norm", "mix.o"});
+    TL_TRY(dev_alloc(st, &L.conv, (size_t)ch * sp.conv_taps));
+    TL_TRY(dev_alloc(st, &L.conv_b, ch));
+    TL_TRY(dev_alloc(st, &L.dt_bias, sp.heads));
+    TL_TRY(dev_alloc(st, &L.a_log, sp.heads));
+    TL_TRY(dev_alloc(st, &L.dskip, sp.heads));
+    TL_TRY(dev_alloc(st, &L.onorm, L.od));
   } else if (sp.mixer == TL_MIXER_LINEAR) {
     TL_REQUIRE(sp.kv_heads == sp.heads && sp.dim <= 256 && sp.vdim <= 512,
                "tl_stack_create: layer %d: gated linear attention with %d / %d heads, sizes %d (at most 256) / %d (at most 512)", i,
@@ -428,7 +466,8 @@ int setup_layer(TlStack* st, int i, int* first_mix) {
   Layer& L = st->layers[i];
   const tl_layer_spec& sp = L.sp;
   const size_t W = cfg->width;
-  const bool dyt = cfg->norm == TL_NORM_DYT, lnorm = cfg->norm == TL_NORM_LAYER, rms = cfg->norm == TL_NORM_RMS;
+  const bool dyt = cfg->norm == TL_NORM_DYT, rms = cfg->norm == TL_NORM_RMS, lbias = cfg->norm == TL_NORM_LAYER;
+  const bool lnorm = lbias || cfg->norm == TL_NORM_LAYER_PLAIN;
   TL_REQUIRE((sp.block == TL_BLOCK_POST_NORM && !dyt && !lnorm && !rms) || (sp.block == TL_BLOCK_PARALLEL && dyt) ||
                  (sp.block == TL_BLOCK_PRE_NORM && (lnorm || rms)),
              "tl_stack_create: layer %d: block kind %d with norm kind %d (post-norm blocks take the one-plus RMS norm, parallel "
@@ -438,9 +477,10 @@ int setup_layer(TlStack* st, int i, int* first_mix) {
              "runs in parallel and pre-norm blocks only", i);
   TL_REQUIRE(sp.mlp != TL_MLP_UNIT || sp.block == TL_BLOCK_PRE_NORM,
              "tl_stack_create: layer %d: the plain up / activation / down unit runs in pre-norm blocks only", i);
-  TL_REQUIRE((sp.mixer != TL_MIXER_LATENT && sp.mixer != TL_MIXER_GDELTA && sp.mixer != TL_MIXER_LINEAR) || sp.block == TL_BLOCK_PRE_NORM,
-             "tl_stack_create: layer %d: latent attention, the generalized delta rule and gated linear attention run in "
-             "pre-norm blocks only", i);
+  TL_REQUIRE((sp.mixer != TL_MIXER_LATENT && sp.mixer != TL_MIXER_GDELTA && sp.mixer != TL_MIXER_LINEAR && sp.mixer != TL_MIXER_SSM) ||
+                 sp.block == TL_BLOCK_PRE_NORM,
+             "tl_stack_create: layer %d: latent attention, the generalized delta rule, gated linear attention and the state space "
+             "run in pre-norm blocks only", i);
   TL_REQUIRE(sp.mixer != TL_MIXER_DELTA || sp.block != TL_BLOCK_POST_NORM, "tl_stack_create: layer %d: the delta rule runs "
              "in parallel and pre-norm blocks only", i);
   TL_REQUIRE(sp.glu == TL_GLU_SWISH || sp.glu == TL_GLU_RELU, "tl_stack_create: layer %d: gated unit of kind %d", i, sp.glu);
@@ -480,7 +520,15 @@ int setup_layer(TlStack* st, int i, int* first_mix) {
     TL_TRY(dev_alloc(st, &L.norm1, W));
     TL_TRY(dev_alloc(st, &L.norm2, W));
     L.expect.insert("norm1");
-    if (lnorm) {
+    for (int q = 0; q < 2 && cfg->streams > 0; ++q) {
+      const size_t ns = cfg->streams;
+      const std::string p = q == 0 ? "hc1." : "hc2.";
+      (q == 0 || sp.mlp != TL_MLP_NONE ? L.expect : L.optional).insert({p + "in", p + "out", p + "mix"});
+      TL_TRY(dev_alloc(st, &L.hc_in[q], ns));
+      TL_TRY(dev_alloc(st, &L.hc_out[q], ns));
+      TL_TRY(dev_alloc(st, &L.hc_mix[q], ns * ns));
+    }
+    if (lbias) {
       TL_TRY(dev_alloc(st, &L.norm1_b, W));
       TL_TRY(dev_alloc(st, &L.norm2_b, W));
       L.expect.insert("norm1.b");
@@ -503,26 +551,29 @@ int setup_layer(TlStack* st, int i, int* first_mix) {
   }
   if (cfg->canon_taps > 1) st->cache_bytes += sizeof(float) * (size_t)(cfg->canon_taps - 1) * W * (sp.mlp != TL_MLP_NONE ? 2 : 1);
   // ---- feed-forward ----
-  const bool pre_rms = sp.block == TL_BLOCK_PRE_NORM && rms;
+  const bool pre = sp.block == TL_BLOCK_PRE_NORM;
   if (sp.mlp == TL_MLP_MOE) {
-    TL_REQUIRE(sp.block != TL_BLOCK_PRE_NORM || rms, "tl_stack_create: layer %d: routed experts behind a layer norm", i);
     TL_REQUIRE(sp.experts > 0 && sp.top > 0 && sp.top <= sp.experts && sp.expert_ff > 0 && sp.shared_ff >= 0,
                "tl_stack_create: layer %d: %d experts, top %d, sizes %d / %d", i, sp.experts, sp.top, sp.expert_ff, sp.shared_ff);
-    TL_REQUIRE(sp.route == TL_ROUTE_TOP_LOGITS ||
+    TL_REQUIRE(sp.route == TL_ROUTE_TOP_LOGITS || sp.route == TL_ROUTE_SOFTMAX ||
                    ((sp.route == TL_ROUTE_SOFTMAX_GROUPS || sp.route == TL_ROUTE_SIGMOID_GROUPS) && sp.route_groups > 0 &&
                     sp.experts % sp.route_groups == 0 && sp.route_keep > 0 && sp.route_keep <= sp.route_groups &&
                     (long long)sp.route_keep * (sp.experts / sp.route_groups) >= sp.top),
                "tl_stack_create: layer %d: router kind %d, %d experts in %d groups, %d kept, top %d", i, sp.route, sp.experts,
                sp.route_groups, sp.route_keep, sp.top);
     TL_REQUIRE(!sp.shared_gate || sp.shared_ff > 0, "tl_stack_create: layer %d: a gate without a shared expert", i);
-    TL_REQUIRE(!pre_rms || !sp.shared_gate, "tl_stack_create: layer %d: a gated shared expert runs in parallel blocks only", i);
+    TL_REQUIRE(!pre || !sp.shared_gate, "tl_stack_create: layer %d: a gated shared expert runs in parallel blocks only", i);
+    TL_REQUIRE(sp.act == TL_ACT_NONE || (sp.act == TL_ACT_GELU && sp.shared_ff == 0),
+               "tl_stack_create: layer %d: plain experts with activation kind %d and a shared expert of %d", i, sp.act, sp.shared_ff);
     if (own) {
-      if (sp.block == TL_BLOCK_POST_NORM || pre_rms) L.expect.insert("norm2");
+      if (sp.block == TL_BLOCK_POST_NORM || pre) L.expect.insert("norm2");
+      if (lbias) L.expect.insert("norm2.b");
       L.expect.insert("mlp.router");
       if (sp.route == TL_ROUTE_TOP_LOGITS) L.expect.insert("mlp.router.b");
       if (sp.route == TL_ROUTE_SIGMOID_GROUPS) L.expect.insert("mlp.correction");
       for (int e = 0; e < sp.experts; ++e)
-        for (const char* k : {"gate", "up", "down"}) L.expect.insert("mlp.e" + std::to_string(e) + "." + k);
+        for (const char* k : {"gate", "up", "down"})
+          if (k[0] != 'g' || sp.act == TL_ACT_NONE) L.expect.insert("mlp.e" + std::to_string(e) + "." + k);
       TL_TRY(dev_alloc(st, &L.router, (size_t)sp.experts * W));
       TL_TRY(dev_alloc(st, &L.router_b, sp.experts));
       TL_TRY(dev_alloc(st, &L.gu, (size_t)sp.experts * 2 * sp.expert_ff * W));
@@ -545,7 +596,7 @@ int setup_layer(TlStack* st, int i, int* first_mix) {
     TL_REQUIRE(sp.block != TL_BLOCK_PRE_NORM || rms, "tl_stack_create: layer %d: a gated unit behind a layer norm", i);
     TL_REQUIRE(sp.shared_ff > 0, "tl_stack_create: layer %d: a dense feed-forward of size %d", i, sp.shared_ff);
     if (own) {
-      if (pre_rms) L.expect.insert("norm2");
+      if (pre) L.expect.insert("norm2");
       L.expect.insert({"mlp.gate", "mlp.up", "mlp.down"});
       TL_TRY(dev_alloc(st, &L.sgu, (size_t)2 * sp.shared_ff * W));
       TL_TRY(dev_alloc(st, &L.sdown, W * sp.shared_ff));
@@ -553,10 +604,11 @@ int setup_layer(TlStack* st, int i, int* first_mix) {
     st->max_sff = sp.shared_ff > st->max_sff ? sp.shared_ff : st->max_sff;
   } else if (sp.mlp == TL_MLP_UNIT) {
     TL_REQUIRE(lnorm, "tl_stack_create: layer %d: the plain up / activation / down unit sits behind a layer norm", i);
-    TL_REQUIRE(sp.shared_ff > 0 && sp.act >= TL_ACT_NONE && sp.act <= TL_ACT_TANH,
+    TL_REQUIRE(sp.shared_ff > 0 && sp.act >= TL_ACT_NONE && sp.act <= TL_ACT_GELU,
                "tl_stack_create: layer %d: a feed-forward of size %d with activation kind %d", i, sp.shared_ff, sp.act);
     if (own) {
-      L.expect.insert({"norm2", "norm2.b", "mlp.up", "mlp.down"});
+      L.expect.insert({"norm2", "mlp.up", "mlp.down"});
+      if (lbias) L.expect.insert("norm2.b");
       if (sp.act == TL_ACT_XIELU) L.expect.insert("mlp.act");
       TL_TRY(dev_alloc(st, &L.sgu, (size_t)sp.shared_ff * W));
       TL_TRY(dev_alloc(st, &L.sdown, W * sp.shared_ff));
@@ -564,7 +616,7 @@ int setup_layer(TlStack* st, int i, int* first_mix) {
     st->max_sff = sp.shared_ff > st->max_sff ? sp.shared_ff : st->max_sff;
   } else if (own) {
     L.optional.insert("norm2");
-    if (lnorm) L.optional.insert("norm2.b");
+    if (lbias) L.optional.insert("norm2.b");
   }
   return 0;
 }
@@ -575,7 +627,12 @@ int tl_stack_create(const tl_stack_config* cfg, TlStack** out) {
   TL_REQUIRE(cfg && out && cfg->layers, "tl_stack_create: null argument");
   TL_REQUIRE(cfg->width > 0 && cfg->vocab > 0 && cfg->n_layers > 0 && cfg->max_positions > 0,
              "tl_stack_create: non-positive size in the configuration");
-  TL_REQUIRE(cfg->norm >= TL_NORM_RMS_ONE_PLUS && cfg->norm <= TL_NORM_RMS, "tl_stack_create: norm kind %d", cfg->norm);
+  TL_REQUIRE(cfg->norm >= TL_NORM_RMS_ONE_PLUS && cfg->norm <= TL_NORM_LAYER_PLAIN, "tl_stack_create: norm kind %d", cfg->norm);
+  const bool lnorm = cfg->norm == TL_NORM_LAYER || cfg->norm == TL_NORM_LAYER_PLAIN;
+  TL_REQUIRE(cfg->streams >= 0 && cfg->streams <= 16 && ((cfg->streams == 0 && cfg->residual_mult == 0.0f) || lnorm),
+             "tl_stack_create: %d residual streams (at most 16), residual factor %g: both belong to blocks behind a layer norm",
+             cfg->streams, cfg->residual_mult);
+  TL_REQUIRE(cfg->streams == 0 || !cfg->embed_norm, "tl_stack_create: an embedding norm with residual streams");
   TL_REQUIRE(cfg->canon_taps >= 0 && cfg->canon_taps <= 64 && (cfg->canon_taps == 0 || cfg->norm == TL_NORM_RMS),
              "tl_stack_create: %d taps on what the sublayers read (a convolution there follows the plain RMS norm)", cfg->canon_taps);
   TL_REQUIRE(cfg->norm != TL_NORM_RMS || !cfg->embed_norm, "tl_stack_create: an embedding norm with the plain RMS norm");
@@ -583,6 +640,7 @@ int tl_stack_create(const tl_stack_config* cfg, TlStack** out) {
   st->cfg = *cfg;
   st->layers.resize(cfg->n_layers);
   const size_t W = cfg->width;
+  if (const char* e = getenv("TL_STACK_CHUNK")) st->chunk = atoi(e) > 0 ? atoi(e) : st->chunk;
   int first_mix = -1;
   int rc = 0;
   auto fail = [&](int code) {
@@ -608,7 +666,6 @@ int tl_stack_create(const tl_stack_config* cfg, TlStack** out) {
     return fail(rc);
   st->need_globals = 1 | 2 | 8 | (cfg->embed_norm ? 4 : 0) | (cfg->norm == TL_NORM_DYT ? 16 | 32 : 0) |
                      (cfg->norm == TL_NORM_LAYER ? 16 | (cfg->embed_norm ? 64 : 0) : 0);
-  if (const char* e = getenv("TL_STACK_CHUNK")) st->chunk = atoi(e) > 0 ? atoi(e) : st->chunk;
   if (const char* e = getenv("TL_STACK_GEMV")) st->gemv_decode = atoi(e) != 0;
   if (const char* e = getenv("TL_STACK_FUSE_ROUTER")) st->fuse_router = atoi(e) != 0;
   if (const char* e = getenv("TL_STACK_FORK")) st->fork = atoi(e) != 0;
@@ -693,6 +750,27 @@ int tl_stack_set_tensor(TlStack* st, const char* name, int type, const long long
   if (r == "norm2.b") VECTOR(L.norm2_b, W);
   if (r == "canon1") MATRIX(L.canon1, W, st->cfg.canon_taps);
   if (r == "canon2") MATRIX(L.canon2, W, st->cfg.canon_taps);
+  for (int q = 0; q < 2 && st->cfg.streams > 0; ++q) {
+    const long long ns = st->cfg.streams;
+    const std::string p = q == 0 ? "hc1." : "hc2.";
+    if (r == p + "in") VECTOR(L.hc_in[q], ns);
+    if (r == p + "out") VECTOR(L.hc_out[q], ns);
+    if (r == p + "mix") {
+      TL_REQUIRE(shape_is(shape, ndim, ns, ns), "tl_stack_set_tensor: %s is not %lld x %lld", name, ns, ns);
+      return upload_as_f32(L.hc_mix[q], type, host, (size_t)(ns * ns), s);
+    }
+  }
+  if (sp.mixer == TL_MIXER_SSM) {
+    const long long ch = L.vd + L.kd + L.qd;
+    if (r == "mix.in") MATRIX(L.wqkv, L.pd, W);
+    if (r == "mix.conv") MATRIX(L.conv, ch, sp.conv_taps);
+    if (r == "mix.conv.b") VECTOR(L.conv_b, ch);
+    if (r == "mix.dt_bias") VECTOR(L.dt_bias, sp.heads);
+    if (r == "mix.A_log") VECTOR(L.a_log, sp.heads);
+    if (r == "mix.D") VECTOR(L.dskip, sp.heads);
+    if (r == "mix.norm") VECTOR(L.onorm, L.od);
+    if (r == "mix.o") MATRIX(L.wo, W, L.od);
+  }
   if (sp.mixer == TL_MIXER_LINEAR) {
     const long long hd = (long long)sp.heads * sp.dim;
     if (r == "mix.q") MATRIX(L.wqkv, hd, W);
@@ -747,7 +825,7 @@ int tl_stack_set_tensor(TlStack* st, const char* name, int type, const long long
     const long long qh = sp.dim + sp.rot_dim;
     if (r == "mix.dq") MATRIX(L.wqkv, sp.q_rank, W);
     if (r == "mix.dkv") MATRIX(L.wqkv + (size_t)sp.q_rank * W, L.kd, W);
-    if (r == "mix.g") MATRIX(L.wqkv + (size_t)L.gate_off * W, sp.heads, W);
+    if (r == "mix.g") MATRIX(L.wqkv + (size_t)L.gate_off * W, L.pd - L.gate_off, W);
     if (r == "mix.dq.norm") VECTOR(L.dq_norm, sp.q_rank);
     if (r == "mix.dkv.norm") VECTOR(L.dkv_norm, sp.kv_rank);
     if (r == "mix.uq") MATRIX(L.wuq, sp.heads * qh, sp.q_rank);
@@ -853,6 +931,7 @@ int tl_stack_set_tensor(TlStack* st, const char* name, int type, const long long
     if (sscanf(r.c_str(), "mlp.e%d.%n", &e, &u2) == 1 && u2 > 0 && e >= 0 && e < sp.experts) {
       const std::string k = r.substr(u2);
       uint16_t* gu = L.gu + (size_t)e * 2 * ff * W;
+      if (k == "up" && sp.act != TL_ACT_NONE) MATRIX(L.gu + (size_t)e * ff * W, ff, W);
       if (k == "gate") PAIRED(gu, ff, W);
       if (k == "up") PAIRED(gu + W, ff, W);
       if (k == "down") MATRIX(L.down + (size_t)e * W * ff, W, ff);
@@ -911,6 +990,11 @@ int tl_stack_finalize(TlStack* st, hipStream_t s) {
       } else {
         L.ckv = st->layers[L.kv_src].ckv;  // an earlier layer: already placed
       }
+    } else if (L.sp.mixer == TL_MIXER_SSM) {
+      L.state = p;
+      p += (size_t)L.sp.heads * L.sp.vdim * L.sp.dim;
+      L.hist = p;
+      p += (size_t)(L.sp.conv_taps - 1) * (L.qd + L.kd + L.vd);
     } else if (L.sp.mixer == TL_MIXER_GDELTA) {
       L.state = p;
       p += (size_t)L.sp.heads * L.sp.dim * L.sp.dim;
@@ -927,6 +1011,8 @@ int tl_stack_finalize(TlStack* st, hipStream_t s) {
   if (st->any_maps) TL_TRY(dev_alloc(st, &st->att2, C * st->max_od));
   if (st->any_pair) TL_TRY(dev_alloc(st, &st->proj2, C * W));
   if (st->cfg.canon_taps > 0) TL_TRY(dev_alloc(st, &st->hn, C * W));
+  if (st->cfg.streams > 0) TL_TRY(dev_alloc(st, &st->xs, C * W * st->cfg.streams));
+  if (st->max_gram) TL_TRY(dev_alloc(st, &st->gram, st->max_gram));
   TL_TRY(dev_alloc(st, &st->x, C * W));
   TL_TRY(dev_alloc(st, &st->h, C * W));
   TL_TRY(dev_alloc(st, &st->qkv, C * st->max_qkv));
@@ -972,7 +1058,7 @@ int tl_stack_finalize(TlStack* st, hipStream_t s) {
         if (L.sp.mixer != TL_MIXER_SWA && L.sp.mixer != TL_MIXER_LATENT) continue;
         const bool lat = L.sp.mixer == TL_MIXER_LATENT;
         const size_t n = tl_swa_ws_floats(T, L.sp.heads, lat ? L.sp.kv_rank : L.sp.vdim,
-                                          tl_swa_splits(T, lat ? 0 : L.sp.window, st->cfg.max_positions, lat ? 0 : L.sp.keep_first));
+                                          tl_swa_splits(T, L.sp.window, st->cfg.max_positions, lat ? 0 : L.sp.keep_first));
         ws = n > ws ? n : ws;
       }
     TL_TRY(dev_alloc(st, &st->swa_ws, ws));
@@ -1078,9 +1164,18 @@ void tl_stack_bytes_per_token(const TlStack* st, int pos, double* weight_bytes, 
     const tl_layer_spec& sp = L.sp;
     wb += 2.0 * W * (L.pd + L.od);
     if (sp.mlp == TL_MLP_UNIT) wb += 2.0 * W * 2.0 * sp.shared_ff;
+    if (sp.mlp == TL_MLP_MOE)
+      wb += 2.0 * W * (sp.experts + (sp.act != TL_ACT_NONE ? 2.0 : 3.0) * sp.expert_ff * sp.top + 3.0 * sp.shared_ff + (sp.shared_gate ? 1.0 : 0.0));
+    if (sp.mlp == TL_MLP_DENSE) wb += 2.0 * W * 3.0 * sp.shared_ff;
+    if (sp.mixer == TL_MIXER_SSM) {
+      wb += 2.0 * (double)(L.qd + L.kd + L.vd) * sp.conv_taps;
+      kb += 2.0 * 4.0 * ((double)sp.heads * sp.vdim * sp.dim + (double)(sp.conv_taps - 1) * (L.qd + L.kd + L.vd));
+      continue;
+    }
     if (sp.mixer == TL_MIXER_LATENT) {
       wb += 2.0 * ((double)L.qd * sp.q_rank + (double)sp.heads * sp.kv_rank * (sp.dim + sp.vdim));
-      kb += 4.0 * (pos + 2.0) * (sp.kv_rank + sp.rot_dim);  // every head reads the same rows: counted once
+      const double seen = sp.window > 0 && pos + 1 > sp.window ? sp.window : pos + 1.0;
+      kb += 4.0 * (seen + 1.0) * (sp.kv_rank + sp.rot_dim);  // every head reads the same rows: counted once
       continue;
     }
     if (sp.mixer == TL_MIXER_GDELTA) {
@@ -1088,9 +1183,6 @@ void tl_stack_bytes_per_token(const TlStack* st, int pos, double* weight_bytes, 
       kb += 2.0 * 4.0 * sp.heads * sp.dim * sp.dim;
       continue;
     }
-    if (sp.mlp == TL_MLP_MOE)
-      wb += 2.0 * W * (sp.experts + 3.0 * sp.expert_ff * sp.top + 3.0 * sp.shared_ff + (sp.shared_gate ? 1.0 : 0.0));
-    if (sp.mlp == TL_MLP_DENSE) wb += 2.0 * W * 3.0 * sp.shared_ff;
     if (sp.mixer == TL_MIXER_DELTA || sp.mixer == TL_MIXER_LINEAR) {
       wb += 2.0 * ((double)sp.heads * sp.dim * sp.decay_rank + (double)L.vd * sp.gate_rank);
       kb += 2.0 * 4.0 * sp.heads * sp.vdim * sp.dim;  // the state is read and written
@@ -1158,6 +1250,7 @@ int moe_experts(TlStack* st, const Layer& L, const Layer& Wt, const float* in, i
     d.alpha = sp.act_alpha;
     d.up_add = sp.glu_up_add;
     d.glu_kind = sp.glu;
+    d.unit_act = sp.act;
     d.sgate = sp.shared_gate ? st->sgate : nullptr;
     d.act = st->act_buf;
     d.y = one_token_out;
@@ -1166,7 +1259,7 @@ int moe_experts(TlStack* st, const Layer& L, const Layer& Wt, const float* in, i
   TL_TRY(tl_launch_moe_plan(st->ids, S, sp.experts, st->off, st->slot_of, s));
   DenseArgs g = {};  // gate | up of every slot, grouped by expert: item p reads token slot_of[p] / top
   g.w = Wt.gu;
-  g.rows = 2 * ff;
+  g.rows = sp.act != TL_ACT_NONE ? ff : 2 * ff;
   g.cols = W;
   g.x = in;
   g.ldx = W;
@@ -1178,11 +1271,12 @@ int moe_experts(TlStack* st, const Layer& L, const Layer& Wt, const float* in, i
   g.x_div = sp.top;
   g.groups = sp.experts;
   g.group_off = st->off;
-  g.glu = 1;
+  g.glu = sp.act == TL_ACT_NONE;
   g.glu_limit = sp.expert_limit;
   g.glu_alpha = sp.act_alpha;
   g.glu_up_add = sp.glu_up_add;
   g.glu_kind = sp.glu;
+  g.act = sp.act;  // plain experts: the activation of the up product
   TL_TRY(tl_launch_dense_gemm(g, s));
   DenseArgs d = {};  // down: item p writes the row of its slot, so that a token's choices lie side by side
   d.w = Wt.down;
@@ -1236,6 +1330,7 @@ RouterArgs router_args(TlStack* st, const Layer& L, const Layer& Wt, const float
   r.corr = sp.route == TL_ROUTE_SIGMOID_GROUPS ? Wt.router_b : nullptr;
   r.groups = sp.route_groups;
   r.keep = sp.route_keep;
+  r.scale = sp.route_scale;
   if (sp.shared_gate) {
     r.gate_w = Wt.sg;
     r.gate_out = st->sgate;
@@ -1571,6 +1666,8 @@ int latent_mixer(TlStack* st, Layer& L, const float* in, int T, int start_pos, c
   p.kv_norm = L.kd ? L.dkv_norm : nullptr;
   p.eps = c.norm_eps;
   p.rot_dims = sp.rot_dims;
+  p.halves = sp.rot_halves;
+  p.mscale = L.mscale;
   p.freq = L.freq;
   p.cache = L.kd ? L.ckv : nullptr;
   p.T = T;
@@ -1585,21 +1682,27 @@ int latent_mixer(TlStack* st, Layer& L, const float* in, int T, int start_pos, c
   q.heads = H;
   q.rot_dim = sp.rot_dim;
   q.rot_dims = sp.rot_dims;
+  q.halves = sp.rot_halves;
+  q.mscale = L.mscale;
   q.freq = L.freq;
   q.T = T;
   q.start_pos = start_pos;
   q.pos_dev = pos_dev;
   if (!pos_dev && st->latent_expand > 0 && T >= st->latent_expand) {
-    // A long chunk: keys [W_uk,n c | rotated part] and values W_uv,n c per head for the rows [0, start_pos + T), then ordinary
+    // A long chunk: keys [W_uk,n c | rotated part] and values W_uv,n c per head for the rows that its tokens can see (up to
+    // start_pos + T, from the window's start of the first token on; each at its own position in the buffers), then ordinary
     // attention with as many key heads as query heads (fewer products per query-key pair than over the latent rows).
-    const int P = start_pos + T;
+    const int lo = sp.window > 0 && start_pos - sp.window + 1 > 0 ? start_pos - sp.window + 1 : 0;
+    const int P = start_pos + T - lo;
+    const float* rows = L.ckv + (size_t)lo * ah;
+    float *lk = st->lk + (size_t)lo * H * qh, *lv = st->lv + (size_t)lo * H * sp.vdim;
     q.out = st->lq;  // the rotated query part in place
     q.out_stride = qh;
     q.out_off = sp.dim;
     TL_TRY(tl_launch_latent_query(q, s));
-    TL_TRY(project_heads(st, L.wuk, H, sp.dim, sp.kv_rank, L.ckv, ah, 0, st->lk, H * qh, qh, P, s));
-    TL_TRY(tl_launch_latent_spread(L.ckv, sp.kv_rank, sp.rot_dim, st->lk, H, sp.dim, P, s));
-    TL_TRY(project(st, L.wuv, H * sp.vdim, sp.kv_rank, L.ckv, ah, st->lv, H * sp.vdim, P, s));
+    TL_TRY(project_heads(st, L.wuk, H, sp.dim, sp.kv_rank, rows, ah, 0, lk, H * qh, qh, P, s));
+    TL_TRY(tl_launch_latent_spread(rows, sp.kv_rank, sp.rot_dim, lk, H, sp.dim, P, s));
+    TL_TRY(project(st, L.wuv, H * sp.vdim, sp.kv_rank, rows, ah, lv, H * sp.vdim, P, s));
     SwaArgs e = {};
     e.q = st->lq;
     e.ldq = H * qh;
@@ -1611,11 +1714,13 @@ int latent_mixer(TlStack* st, Layer& L, const float* in, int T, int start_pos, c
     e.kv_heads = H;
     e.dim = qh;
     e.vdim = sp.vdim;
+    e.window = sp.window;
     e.scale = sp.scale;
     e.start_pos = start_pos;
     e.nsplit = 1;
     TL_TRY(tl_launch_swa(e, s));
     if (sp.head_gate) TL_TRY(tl_launch_head_gate(st->att, st->qkv + L.gate_off, ld, T, H, sp.vdim, s));
+    if (sp.out_gate) TL_TRY(tl_launch_out_gate(st->att, st->qkv + L.gate_off, ld, T, L.od, s));
     return project(st, L.wo, W, L.od, st->att, L.od, st->proj, W, T, s);
   }
   // the plain part of head n's query through W_uk,n^T: scores against the cached latent itself
@@ -1637,16 +1742,18 @@ int latent_mixer(TlStack* st, Layer& L, const float* in, int T, int start_pos, c
   a.kv_heads = 1;
   a.dim = ah;
   a.vdim = sp.kv_rank;
+  a.window = sp.window;
   a.scale = sp.scale;
   a.start_pos = start_pos;
   a.pos_dev = pos_dev;
-  a.nsplit = tl_swa_splits(T, 0, c.max_positions, 0);
+  a.nsplit = tl_swa_splits(T, sp.window, c.max_positions, 0);
   a.ws = st->swa_ws;
   a.done_cnt = st->swa_cnt;
   TL_TRY(tl_launch_swa(a, s));
   // head n's weighted latent through W_uv,n (lq is free again)
   TL_TRY(project_heads(st, L.wuv, H, sp.vdim, sp.kv_rank, st->att, H * sp.kv_rank, sp.kv_rank, st->lq, L.od, sp.vdim, T, s));
   if (sp.head_gate) TL_TRY(tl_launch_head_gate(st->lq, st->qkv + L.gate_off, ld, T, H, sp.vdim, s));
+  if (sp.out_gate) TL_TRY(tl_launch_out_gate(st->lq, st->qkv + L.gate_off, ld, T, L.od, s));
   return project(st, L.wo, W, L.od, st->lq, L.od, st->proj, W, T, s);
 }
 
@@ -1693,6 +1800,79 @@ int gdelta_mixer(TlStack* st, Layer& L, const float* in, int T, hipStream_t s) {
   return project(st, L.wo, W, L.od, st->att, L.od, st->proj, W, T, s);
 }
 
+int ssm_mixer(TlStack* st, Layer& L, const float* in, int T, hipStream_t s) {
+  const tl_layer_spec& sp = L.sp;
+  const int W = st->cfg.width, ld = L.pd, ch = L.qd + L.kd + L.vd;
+  TL_TRY(project(st, L.wqkv, ld, W, in, W, st->qkv, ld, T, s));  // z | x | B | C | dt
+  const float* xbc = st->qkv + L.od;
+  PartNormArgs n = {};
+  n.x = st->att;
+  n.w = L.onorm;
+  n.T = T;
+  n.width = L.od;
+  n.parts = sp.norm_parts;
+  n.eps = st->cfg.norm_eps;
+  if (T == 1 && st->gemv_decode) {
+    SsmStepArgs a = {};
+    a.p = st->qkv;
+    a.conv = L.conv;
+    a.conv_b = L.conv_b;
+    a.taps = sp.conv_taps;
+    a.hist = L.hist;
+    a.dt_bias = L.dt_bias;
+    a.a_log = L.a_log;
+    a.d = L.dskip;
+    a.state = L.state;
+    a.y = st->att;
+    a.heads = sp.heads;
+    a.groups = sp.kv_heads;
+    a.state_n = sp.dim;
+    a.vdim = sp.vdim;
+    TL_TRY(tl_launch_ssm_step(a, s));
+    if (sp.conv_taps > 1) {
+      n.hist = L.hist;
+      n.hist_in = xbc;
+      n.taps = sp.conv_taps;
+      n.channels = ch;
+    }
+  } else {
+    ConvArgs cv = {};
+    cv.in = xbc;
+    cv.ldi = ld;
+    cv.C = ch;
+    cv.taps = sp.conv_taps;
+    cv.T = T;
+    cv.out_bias = L.conv_b;
+    cv.w = L.conv;
+    cv.hist = L.hist;
+    cv.act = 1;
+    cv.out = st->dq;
+    cv.ldo = ch;
+    TL_TRY(tl_launch_causal_conv(cv, s));
+    SsmScanArgs a = {};
+    a.xbc = st->dq;
+    a.ld = ch;
+    a.dt_raw = xbc + ch;
+    a.dt_ld = ld;
+    a.dt_bias = L.dt_bias;
+    a.a_log = L.a_log;
+    a.d = L.dskip;
+    a.z = st->qkv;
+    a.z_ld = ld;
+    a.state = L.state;
+    a.y = st->att;
+    a.gram = st->gram;
+    a.T = T;
+    a.heads = sp.heads;
+    a.groups = sp.kv_heads;
+    a.state_n = sp.dim;
+    a.vdim = sp.vdim;
+    TL_TRY(tl_launch_ssm_scan(a, s));
+  }
+  TL_TRY(tl_launch_part_norm(n, s));
+  return project(st, L.wo, W, L.od, st->att, L.od, st->proj, W, T, s);
+}
+
 LnParams ln1_of_layer(const Layer& Wt) { return LnParams{Wt.norm1, Wt.norm1_b}; }
 
 // The launch(es) that finish x in a pre-norm block: x += a_scale a + b_scale b + sum_j slot_w[j] slots[j], and the input of
@@ -1708,12 +1888,53 @@ struct Addends {
   const float* slot_w = nullptr;
   int top = 0;
 };
+// What reads the streams (or x) next, in the terms of the hyper launch: its input weights and norm, and, where asked for, its
+// router. next == NULL: nobody; the sum of the streams goes to st->x for the final norm.
+void hyper_next(TlStack* st, HyperArgs& r, Layer* next, int which, int T, bool* routed) {
+  const tl_stack_config& c = st->cfg;
+  r.x = c.streams > 0 ? st->xs : st->x;
+  r.streams = c.streams > 0 ? c.streams : 1;
+  r.T = T;
+  r.width = c.width;
+  r.eps = c.norm_eps;
+  r.h = st->h;
+  if (c.streams > 0 && (!next || st->hook)) r.sum = st->x;
+  if (!next) return;
+  const Layer& Wn = st->layers[next->wsrc];
+  r.in = Wn.hc_in[which - 1];
+  r.next = which == 1 ? ln1_of_layer(Wn) : LnParams{Wn.norm2, Wn.norm2_b};
+  if (routed && which == 2 && st->fuse_router && next->sp.mlp == TL_MLP_MOE && !next->sp.shared_gate) {
+    r.route = router_args(st, *next, Wn, nullptr, T);  // the router reads the row this launch has just finished
+    *routed = true;
+  }
+}
+
 // *routed (optional): set when the router of `next`'s feed-forward rode in the launch (the caller then launches none)
-int finish_x(TlStack* st, const Addends& add, Layer* next, int which, int T, hipStream_t s, bool* routed = nullptr) {
+// from: the layer whose sublayer `done` (1: mixer, 2: feed-forward) the addends come from (its own hyper-connection weights)
+int finish_x(TlStack* st, const Addends& add, Layer* next, int which, int T, hipStream_t s, bool* routed = nullptr,
+             const Layer* from = nullptr, int done = 1) {
   const tl_stack_config& c = st->cfg;
   const int W = c.width;
   const Layer* Wn = next ? &st->layers[next->wsrc] : nullptr;
-  if (c.norm == TL_NORM_LAYER) {
+  if (routed) *routed = false;
+  const bool lnorm = c.norm == TL_NORM_LAYER || c.norm == TL_NORM_LAYER_PLAIN;
+  if (lnorm && (c.streams > 0 || add.slots || c.residual_mult != 0.0f || (which == 2 && next && next->sp.mlp == TL_MLP_MOE))) {
+    TL_REQUIRE(!add.b && add.a_scale == 1.0f, "layer-list engine: a layer-norm block adds one sublayer output");
+    const Layer* Wf = from ? &st->layers[from->wsrc] : nullptr;
+    HyperArgs r = {};
+    hyper_next(st, r, next, which, T, routed);
+    r.a = add.a;
+    r.slots = add.slots;
+    r.slot_w = add.slot_w;
+    r.top = add.top;
+    r.mult = c.residual_mult != 0.0f ? c.residual_mult : 1.0f;
+    if (Wf) {
+      r.mix = Wf->hc_mix[done - 1];
+      r.out = Wf->hc_out[done - 1];
+    }
+    return tl_launch_hyper(r, s);
+  }
+  if (lnorm) {
     TL_REQUIRE(add.a && !add.b && !add.slots && add.a_scale == 1.0f, "layer-list engine: a layer-norm block adds one sublayer output");
     LnParams n = {};
     if (Wn) n = which == 1 ? ln1_of_layer(*Wn) : LnParams{Wn->norm2, Wn->norm2_b};
@@ -1769,6 +1990,7 @@ int run_mixer(TlStack* st, Layer& L, const Layer& Wt, int T, int start_pos, cons
     case TL_MIXER_SWA: return swa_mixer(st, L, Wt, st->h, T, start_pos, pos_dev, s, out, pre, pre_ld);
     case TL_MIXER_LATENT: return latent_mixer(st, L, st->h, T, start_pos, pos_dev, s);
     case TL_MIXER_GDELTA: return gdelta_mixer(st, L, st->h, T, s);
+    case TL_MIXER_SSM: return ssm_mixer(st, L, st->h, T, s);
     case TL_MIXER_LINEAR: return linear_mixer(st, L, Wt, st->h, T, s, out, pre, pre_ld);
     default: return delta_mixer(st, L, Wt, st->h, T, s, out, pre, pre_ld);
   }
@@ -1838,9 +2060,9 @@ int pre_norm_layer(TlStack* st, size_t li, int T, int start_pos, const int* pos_
     mix.b = st->proj2;
     mix.b_scale = sp.side_scale;
   }
-  if (sp.mlp == TL_MLP_NONE) return finish_x(st, mix, after, 1, T, s);
+  if (sp.mlp == TL_MLP_NONE) return finish_x(st, mix, after, 1, T, s, nullptr, &L, 1);
   bool routed = false;
-  TL_TRY(finish_x(st, mix, &L, 2, T, s, &routed));
+  TL_TRY(finish_x(st, mix, &L, 2, T, s, &routed, &L, 1));
   Addends ffo;
   if (sp.mlp == TL_MLP_UNIT) {
     const int ff = sp.shared_ff;
@@ -1862,7 +2084,7 @@ int pre_norm_layer(TlStack* st, size_t li, int T, int start_pos, const int* pos_
       if (sp.shared_ff) ffo.a = st->sout;
     }
   }
-  return finish_x(st, ffo, after, 1, T, s);
+  return finish_x(st, ffo, after, 1, T, s, nullptr, &L, 2);
 }
 
 DytParams dyt_of_layer(const Layer& Wt) { return DytParams{Wt.norm1_alpha, Wt.norm1, Wt.norm1_b}; }
@@ -1925,13 +2147,21 @@ int tl_stack_forward(TlStack* st, const int* tokens_dev, int T, int start_pos, c
   TL_REQUIRE(n_rows >= 0 && n_rows <= T && (n_rows == 0 || logits_dev), "tl_stack_forward: bad logits request");
   const tl_stack_config& c = st->cfg;
   const int W = c.width;
-  const bool dyt = c.norm == TL_NORM_DYT, lnorm = c.norm == TL_NORM_LAYER;
-  if (c.norm == TL_NORM_RMS) {
+  const bool dyt = c.norm == TL_NORM_DYT, lnorm = c.norm == TL_NORM_LAYER || c.norm == TL_NORM_LAYER_PLAIN;
+  if (lnorm && !c.embed_norm) {
+    HyperArgs r = {};  // every stream starts as the (scaled) embedding row
+    hyper_next(st, r, &st->layers[0], 1, T, nullptr);
+    r.table = st->embed;
+    r.tokens = tokens_dev;
+    r.vocab = c.vocab;
+    r.embed_scale = c.embed_scale != 0.0f ? c.embed_scale : 1.0f;
+    TL_TRY(tl_launch_hyper(r, s));
+  } else if (c.norm == TL_NORM_RMS) {
     TL_TRY(tl_launch_embed_rows(st->embed, c.vocab, W, tokens_dev, T, st->x, DytParams{}, st->h, s,
                                 c.embed_scale != 0.0f ? c.embed_scale : 1.0f));
     TL_TRY(finish_x(st, Addends{}, &st->layers[0], 1, T, s));
   } else if (lnorm) {
-    const LnParams emb = c.embed_norm ? LnParams{st->embed_norm, st->embed_norm_b} : LnParams{};
+    const LnParams emb = LnParams{st->embed_norm, c.norm == TL_NORM_LAYER ? st->embed_norm_b : nullptr};
     TL_TRY(tl_launch_embed_ln(st->embed, c.vocab, W, tokens_dev, T, emb, ln1_of_layer(st->layers[st->layers[0].wsrc]), c.norm_eps,
                               st->x, st->h, s));
   } else if (c.embed_norm) {
@@ -1980,7 +2210,7 @@ int tl_stack_forward(TlStack* st, const int* tokens_dev, int T, int start_pos, c
     if (!rows_dev && n_rows == 1) src = st->x + (size_t)last * W;
     TL_REQUIRE(rows_dev || n_rows == 1 || n_rows == T, "tl_stack_forward: %d rows without a list", n_rows);
     if (dyt) TL_TRY(tl_launch_dyt_rows(src, W, rows_dev, n_rows, DytParams{st->final_alpha, st->final_norm, st->final_b}, st->xn, s));
-    else if (lnorm) TL_TRY(tl_launch_ln_rows(src, W, rows_dev, n_rows, LnParams{st->final_norm, st->final_b}, c.norm_eps, st->xn, s));
+    else if (lnorm) TL_TRY(tl_launch_ln_rows(src, W, rows_dev, n_rows, LnParams{st->final_norm, c.norm == TL_NORM_LAYER ? st->final_b : nullptr}, c.norm_eps, st->xn, s));
     else TL_TRY(tl_launch_norm_rows(src, W, rows_dev, n_rows, st->final_norm, c.norm_eps, st->xn, s, c.norm != TL_NORM_RMS));
     TL_TRY(project(st, st->head, c.vocab, W, st->xn, W, logits_dev, c.vocab, n_rows, s, c.logit_softcap));
   }

@@ -557,6 +557,35 @@ def _potipel_spec(sp, i, L, sides):
             raise ValueError(f"layer {i}: unknown feed-forward kind {ml['kind']!r}")
 
 
+def _madudra_spec(sp, i, L):
+    mx, ml = L["mixer"], L.get("mlp")
+    sp.block = 2
+    if L["type"] == "latent_attention":
+        sp.mixer, sp.heads, sp.kv_heads, sp.dim, sp.vdim, sp.scale = 2, mx["heads"], mx["heads"], mx["dim"], mx["vdim"], float(mx["scale"])
+        sp.rot_dim, sp.q_rank, sp.kv_rank, sp.out_gate, sp.rot_halves = mx["rot_dim"], mx["q_rank"], mx["kv_rank"], 1, 1
+        sp.window = int((mx.get("mask") or {}).get("size", 0))
+        rot = mx.get("rot")
+        if rot:
+            sp.rot_dims, sp.rot_base = rot["dims"], float(rot["base"])
+            sc = rot.get("scaling")
+            if sc:
+                sp.rot_factor, sp.rot_original = float(sc["factor"]), float(sc["original"])
+                sp.rot_fast, sp.rot_slow = float(sc["fast"]), float(sc["slow"])
+        if mx.get("kv_from") is not None:
+            sp.kv_from = mx["kv_from"] + 1
+    elif L["type"] == "mamba2":
+        sp.mixer, sp.heads, sp.kv_heads, sp.dim, sp.vdim = 5, mx["heads"], mx["groups"], mx["state"], mx["vdim"]
+        sp.conv_taps, sp.norm_parts = mx["conv"], mx["norm_groups"]
+    else:
+        raise ValueError(f"layer {i}: unknown type {L['type']!r}")
+    if ml is not None:
+        if ml["kind"] != "moe":
+            raise ValueError(f"layer {i}: unknown feed-forward kind {ml['kind']!r}")
+        r = ml["router"]
+        sp.mlp, sp.route, sp.experts, sp.top, sp.route_scale = 1, 3, r["experts"], r["top"], float(r["scale"])
+        sp.act, sp.expert_ff = 3, ml["expert"]["ff"]
+
+
 def stack_config_struct(config, max_pos, tensors=None):
     """The ctypes form (tl_stack_config) of a layer-list configuration given as config.json's dictionary; returns
     (struct, the array it points into). The C++ host does the same from the file (host/tl_stack_config.cpp); this one
@@ -564,11 +593,13 @@ def stack_config_struct(config, max_pos, tensors=None):
     layers = config["layers"]
     arr = (capi.LayerSpec * len(layers))()
     madalorn, sogalix = config.get("architecture") == "Madalorn", config.get("architecture") == "Sogalix"
-    potipel = config.get("architecture") == "Potipel"
+    potipel, madudra = config.get("architecture") == "Potipel", config.get("architecture") == "Madudra"
     sides = (capi.LayerSpec * len(layers))()
     for i, L in enumerate(layers):
         if potipel:
             _potipel_spec(arr[i], i, L, sides)
+        elif madudra:
+            _madudra_spec(arr[i], i, L)
         elif madalorn:
             _madalorn_spec(arr[i], i, L, tensors or {}, layers)
         elif sogalix:
@@ -576,9 +607,12 @@ def stack_config_struct(config, max_pos, tensors=None):
         else:
             _ralasun_spec(arr[i], i, L)
     c = capi.StackConfig(config["width"], config["vocab"], len(layers), int(max_pos), float(config["norm"]["eps"]), arr,
-                         1 if madalorn else 2 if sogalix else 3 if potipel else 0, 0 if madalorn or potipel else 1,
+                         1 if madalorn else 2 if sogalix else 3 if potipel else 4 if madudra else 0,
+                         0 if madalorn or potipel or madudra else 1,
                          float(config.get("logit_softcap") or 0.0) if madalorn else 0.0,
-                         float(config["embedding"]["scale"]) if potipel else 0.0, int(config["canon"]["taps"]) if potipel else 0)
+                         float(config["embedding"]["scale"]) if potipel or madudra else 0.0,
+                         int(config["canon"]["taps"]) if potipel else 0, int(config["streams"]) if madudra else 0,
+                         float(config["residual_mult"]) if madudra else 0.0)
     return c, (arr, sides)
 
 

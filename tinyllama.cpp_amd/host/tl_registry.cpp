@@ -19,6 +19,7 @@ const std::vector<ModelFamily>& model_families() {
       {"Madalorn", "folder", load_stack_folder},
       {"Sogalix", "folder", load_stack_folder},
       {"Potipel", "folder", load_stack_folder},
+      {"Madudra", "folder", load_stack_folder},
   };
   return table;
 }

@@ -44,6 +44,16 @@
 //               "right": {"heads", "kv_heads", "dim", "vdim", "conv"}, "left_scale", "right_scale"},
 //     "mlp": null | {"kind": "dense", "ff"} | {"kind": "moe", "router": {"experts", "top", "groups": {"count", "keep"}},
 //     "expert": {"ff", "limit"}}}]}
+// Madudra   pre-norm blocks with layer norms (weight only) over several residual streams (hyper-connections), a factor on what a
+//           sublayer adds; the embedding row is scaled. Mixers: "latent_attention" = as Sogalix's, but windowed, rotated in
+//           halves with a context extension and gated per output column; "mamba2" = selective state space with one decay per
+//           head. Feed-forward: routed plain experts W_down gelu(W_up h), weights = softmax over all experts times a factor.
+//   {"architecture", "width", "vocab", "norm": {"eps"}, "embedding": {"scale"}, "streams", "residual_mult",
+//     "layers": [{"type": "latent_attention" | "mamba2",
+//     "mixer": {"heads", "dim", "rot_dim", "vdim", "q_rank", "kv_rank", "scale", "mask": {"size"},
+//               "rot": {"base", "dims", "scaling": {"factor", "original", "fast", "slow"}}, "kv_from": j} |
+//              {"heads", "vdim", "state", "groups", "conv", "norm_groups"},
+//     "mlp": null | {"kind": "moe", "router": {"experts", "top", "scale"}, "expert": {"ff"}}}]}
 #include <chrono>
 #include <cmath>
 #include <fstream>
@@ -118,6 +128,36 @@ int tensor_rows(const SafeTensorsFile& file, const std::string& name) {
   return (int)t->shape[0];
 }
 
+void read_rotation(const Json& mx, tl_layer_spec* sp) {
+  const Json* rot = present(mx, "rot");
+  if (!rot) return;
+  sp->rot_dims = geti(*rot, "dims");
+  sp->rot_base = getf(*rot, "base");
+  if (const Json* sc = present(*rot, "scaling")) {
+    sp->rot_factor = getf(*sc, "factor");
+    sp->rot_original = getf(*sc, "original");
+    sp->rot_fast = getf(*sc, "fast");
+    sp->rot_slow = getf(*sc, "slow");
+  }
+}
+
+void read_latent(const Json& mx, int index, const std::string& where, tl_layer_spec* sp) {
+  sp->mixer = TL_MIXER_LATENT;
+  sp->heads = sp->kv_heads = geti(mx, "heads");
+  sp->dim = geti(mx, "dim");
+  sp->vdim = geti(mx, "vdim");
+  sp->scale = getf(mx, "scale");
+  sp->rot_dim = geti(mx, "rot_dim");
+  sp->q_rank = geti(mx, "q_rank");
+  sp->kv_rank = geti(mx, "kv_rank");
+  read_rotation(mx, sp);
+  if (const Json* kf = present(mx, "kv_from")) {
+    const int j = (int)kf->as_int("kv_from");
+    if (j < 0 || j >= index) throw std::runtime_error(where + ": kv_from must name an earlier layer");
+    sp->kv_from = j + 1;
+  }
+}
+
 tl_layer_spec madalorn_layer(const Json& layers, int index, const SafeTensorsFile& file) {
   const Json& L = layers.arr[index];
   const std::string where = "layers[" + std::to_string(index) + "]";
@@ -153,16 +193,7 @@ tl_layer_spec madalorn_layer(const Json& layers, int index, const SafeTensorsFil
       sp.window = geti(*mask, "size");
       if (const Json* kf = present(*mask, "keep_first")) sp.keep_first = (int)kf->as_int("keep_first");
     }
-    if (const Json* rot = present(mx, "rot")) {
-      sp.rot_dims = geti(*rot, "dims");
-      sp.rot_base = getf(*rot, "base");
-      if (const Json* sc = present(*rot, "scaling")) {
-        sp.rot_factor = getf(*sc, "factor");
-        sp.rot_original = getf(*sc, "original");
-        sp.rot_fast = getf(*sc, "fast");
-        sp.rot_slow = getf(*sc, "slow");
-      }
-    }
+    read_rotation(mx, &sp);
   } else if (type == "channel_delta") {
     sp.mixer = TL_MIXER_DELTA;
     sp.conv_taps = geti(mx, "conv");
@@ -221,23 +252,8 @@ tl_layer_spec sogalix_layer(const Json& layers, int index, const SafeTensorsFile
       if (sp.q_temp_every <= 0) throw std::runtime_error(where + ": q_temp.every must be positive");
     }
   } else if (type == "latent_attention") {
-    sp.mixer = TL_MIXER_LATENT;
-    sp.kv_heads = sp.heads;
-    sp.vdim = geti(mx, "vdim");
-    sp.scale = getf(mx, "scale");
-    sp.rot_dim = geti(mx, "rot_dim");
-    sp.q_rank = geti(mx, "q_rank");
-    sp.kv_rank = geti(mx, "kv_rank");
+    read_latent(mx, index, where, &sp);
     sp.head_gate = 1;
-    if (const Json* rot = present(mx, "rot")) {
-      sp.rot_dims = geti(*rot, "dims");
-      sp.rot_base = getf(*rot, "base");
-    }
-    if (const Json* kf = present(mx, "kv_from")) {
-      const int j = (int)kf->as_int("kv_from");
-      if (j < 0 || j >= index) throw std::runtime_error(where + ": kv_from must name an earlier layer");
-      sp.kv_from = j + 1;
-    }
   } else if (type == "general_delta") {
     sp.mixer = TL_MIXER_GDELTA;
     sp.kv_heads = sp.heads;
@@ -253,6 +269,44 @@ tl_layer_spec sogalix_layer(const Json& layers, int index, const SafeTensorsFile
     sp.mlp = TL_MLP_UNIT;
     sp.act = TL_ACT_XIELU;
     sp.shared_ff = geti(*ml, "ff");
+  }
+  return sp;
+}
+
+tl_layer_spec madudra_layer(const Json& layers, int index) {
+  const Json& L = layers.arr[index];
+  const std::string where = "layers[" + std::to_string(index) + "]";
+  tl_layer_spec sp = {};
+  const std::string& type = L.at("type").as_string("type");
+  const Json& mx = L.at("mixer");
+  sp.block = TL_BLOCK_PRE_NORM;
+  if (type == "latent_attention") {
+    read_latent(mx, index, where, &sp);
+    if (const Json* mask = present(mx, "mask")) sp.window = geti(*mask, "size");
+    sp.rot_halves = 1;
+    sp.out_gate = 1;
+  } else if (type == "mamba2") {
+    sp.mixer = TL_MIXER_SSM;
+    sp.heads = geti(mx, "heads");
+    sp.kv_heads = geti(mx, "groups");
+    sp.vdim = geti(mx, "vdim");
+    sp.dim = geti(mx, "state");
+    sp.conv_taps = geti(mx, "conv");
+    sp.norm_parts = geti(mx, "norm_groups");
+  } else {
+    throw std::runtime_error(where + ": unknown layer type \"" + type + "\"");
+  }
+  if (const Json* ml = present(L, "mlp")) {
+    const std::string& kind = ml->at("kind").as_string("kind");
+    if (kind != "moe") throw std::runtime_error(where + ": unknown feed-forward kind \"" + kind + "\"");
+    const Json& r = ml->at("router");
+    sp.mlp = TL_MLP_MOE;
+    sp.route = TL_ROUTE_SOFTMAX;
+    sp.experts = geti(r, "experts");
+    sp.top = geti(r, "top");
+    sp.route_scale = getf(r, "scale");
+    sp.act = TL_ACT_GELU;
+    sp.expert_ff = geti(ml->at("expert"), "ff");
   }
   return sp;
 }
@@ -358,7 +412,8 @@ void load_stack_folder(const std::string& dir, int device, int max_context, Load
   const Json& layers = cfg.at("layers");
   if (layers.kind != Json::ARRAY || layers.arr.empty()) throw std::runtime_error("config.json: \"layers\" is empty");
   const std::string arch = cfg.at("architecture").as_string("architecture");
-  const bool madalorn = arch == "Madalorn", sogalix = arch == "Sogalix", potipel = arch == "Potipel";
+  const bool madalorn = arch == "Madalorn", sogalix = arch == "Sogalix", potipel = arch == "Potipel",
+             madudra = arch == "Madudra";
   SafeTensorsFile file;
   file.open(dir + "/model.safetensors");
   std::vector<tl_layer_spec> specs, sides(layers.arr.size());  // (sides: second mixers, addressed by the entries of specs)
@@ -366,6 +421,7 @@ void load_stack_folder(const std::string& dir, int device, int max_context, Load
     specs.push_back(madalorn  ? madalorn_layer(layers, (int)i, file)
                     : sogalix ? sogalix_layer(layers, (int)i, file)
                     : potipel ? potipel_layer(layers, (int)i, &sides[i])
+                    : madudra ? madudra_layer(layers, (int)i)
                               : ralasun_layer(layers.arr[i], (int)i, file));
   tl_stack_config sc = {};
   sc.width = geti(cfg, "width");
@@ -374,10 +430,15 @@ void load_stack_folder(const std::string& dir, int device, int max_context, Load
   sc.max_positions = max_context > 0 ? max_context : kDefaultContext;
   sc.norm_eps = (float)cfg.at("norm").at("eps").as_double("norm.eps");
   sc.layers = specs.data();
-  sc.norm = madalorn ? TL_NORM_DYT : sogalix ? TL_NORM_LAYER : potipel ? TL_NORM_RMS : TL_NORM_RMS_ONE_PLUS;
-  sc.embed_norm = madalorn || potipel ? 0 : 1;
+  sc.norm = madalorn ? TL_NORM_DYT : sogalix ? TL_NORM_LAYER : potipel ? TL_NORM_RMS : madudra ? TL_NORM_LAYER_PLAIN : TL_NORM_RMS_ONE_PLUS;
+  sc.embed_norm = madalorn || potipel || madudra ? 0 : 1;
+  if (potipel || madudra) sc.embed_scale = (float)cfg.at("embedding").at("scale").as_double("embedding.scale");
+  if (madudra) {
+    sc.streams = geti(cfg, "streams");
+    sc.residual_mult = getf(cfg, "residual_mult");
+    if (sc.streams < 1) throw std::runtime_error("config.json: \"streams\" must be at least 1");
+  }
   if (potipel) {
-    sc.embed_scale = (float)cfg.at("embedding").at("scale").as_double("embedding.scale");
     sc.canon_taps = (int)cfg.at("canon").at("taps").as_int("canon.taps");
   }
   if (madalorn)

@@ -644,6 +644,95 @@ def build_potipel(config, seed=0, gain=1.0):
     return t
 
 
+def madudra_latent(heads, dim, rot_dim, vdim, q_rank, kv_rank, window, base=10000.0, scaling=None, kv_from=None, scale=None):
+    """scaling: None or (factor, original, fast, slow)."""
+    rot = {"base": float(base), "dims": rot_dim}
+    if scaling is not None:
+        rot["scaling"] = dict(zip(("factor", "original", "fast", "slow"), scaling))
+    mixer = {"dim": dim, "heads": heads, "kv_rank": kv_rank, "q_rank": q_rank, "rot": rot, "rot_dim": rot_dim,
+             "scale": float(scale if scale is not None else (dim + rot_dim) ** -0.5), "vdim": vdim}
+    if window:
+        mixer["mask"] = {"size": int(window)}
+    if kv_from is not None:
+        mixer["kv_from"] = int(kv_from)
+    return mixer
+
+
+def madudra_mamba(heads, vdim, state, groups=1, conv=4, norm_groups=1):
+    return {"conv": conv, "groups": groups, "heads": heads, "norm_groups": norm_groups, "state": state, "vdim": vdim}
+
+
+def madudra_moe(experts, top, ff, scale=1.0):
+    return {"kind": "moe", "router": {"experts": experts, "top": top, "scale": float(scale)}, "expert": {"ff": ff}}
+
+
+def madudra_layer(kind, mixer, mlp=None):
+    return {"type": kind, "mixer": mixer, "mlp": mlp}
+
+
+def madudra_config(width, vocab, layers, streams=2, residual_mult=0.7, eps=1e-6, embed_scale=4.0):
+    return {"architecture": "Madudra", "embedding": {"scale": float(embed_scale)}, "layers": list(layers), "norm": {"eps": float(eps)},
+            "residual_mult": float(residual_mult), "streams": int(streams), "vocab": int(vocab), "width": int(width)}
+
+
+def build_madudra(config, seed=0, gain=1.0):
+    """Random tensors {checkpoint name: uint16 bf16 bits} of a Madudra configuration."""
+    rng = np.random.default_rng(seed)
+    W, V, ns = config["width"], config["vocab"], config["streams"]
+    t = {}
+
+    def mat(name, rows, cols, std=None):
+        t[name] = to_bf16(rng.standard_normal((rows, cols)).astype(np.float32) * (std or gain / np.sqrt(cols)))
+
+    def vec(name, n, centre, spread):
+        t[name] = to_bf16((centre + spread * rng.standard_normal(n)).astype(np.float32))
+
+    def streams(p):
+        vec(p + "in", ns, 1.0 / ns, 0.5)
+        vec(p + "out", ns, 1.0, 0.5)
+        t[p + "mix"] = to_bf16((0.7 * np.eye(ns) + 0.3 / ns + 0.15 * rng.standard_normal((ns, ns))).astype(np.float32))
+
+    mat("embed", V, W, 1.0 / config["embedding"]["scale"])
+    vec("final.norm", W, 1.0, 0.1)
+    mat("head", V, W, 4.0 / np.sqrt(W))
+    for i, L in enumerate(config["layers"]):
+        mx, ml, p = L["mixer"], L.get("mlp"), f"l{i}."
+        H, dv = mx["heads"], mx["vdim"]
+        vec(p + "norm1", W, 1.0, 0.1)
+        streams(p + "hc1.")
+        if L["type"] == "latent_attention":
+            d, rd, rq, rk = mx["dim"], mx["rot_dim"], mx["q_rank"], mx["kv_rank"]
+            mat(p + "mix.dq", rq, W)
+            vec(p + "mix.dq.norm", rq, 1.0, 0.1)
+            mat(p + "mix.uq", H * (d + rd), rq, 2.0 / np.sqrt(rq))
+            if mx.get("kv_from") is None:
+                mat(p + "mix.dkv", rk + rd, W)
+                vec(p + "mix.dkv.norm", rk, 1.0, 0.1)
+            mat(p + "mix.uk", H * d, rk, 2.0 / np.sqrt(rk))
+            mat(p + "mix.uv", H * dv, rk)
+            mat(p + "mix.g", H * dv, W, 2.0 / np.sqrt(W))
+            mat(p + "mix.o", W, H * dv)
+        else:
+            N, G, inner = mx["state"], mx["groups"], H * dv
+            mat(p + "mix.in", 2 * inner + 2 * G * N + H, W, 1.5 / np.sqrt(W))
+            mat(p + "mix.conv", inner + 2 * G * N, mx["conv"], 0.6)
+            vec(p + "mix.conv.b", inner + 2 * G * N, 0.0, 0.2)
+            vec(p + "mix.dt_bias", H, -1.5, 1.0)
+            vec(p + "mix.A_log", H, -0.5, 1.0)
+            vec(p + "mix.D", H, 1.0, 0.3)
+            vec(p + "mix.norm", inner, 1.0, 0.1)
+            mat(p + "mix.o", W, inner)
+        if ml is not None:
+            vec(p + "norm2", W, 1.0, 0.1)
+            streams(p + "hc2.")
+            E, ff = ml["router"]["experts"], ml["expert"]["ff"]
+            mat(p + "mlp.router", E, W, 3.0 / np.sqrt(W))
+            for e in range(E):
+                mat(f"{p}mlp.e{e}.up", ff, W, 2.0 / np.sqrt(W))
+                mat(f"{p}mlp.e{e}.down", W, ff)
+    return t
+
+
 def write_stack_dir(path, config, tensors):
     """config.json + model.safetensors (8-byte little-endian header length, JSON header, data) under `path`."""
     import json
