@@ -52,8 +52,9 @@ def parse():
     ap.add_argument("--prompt-len", type=int, default=4)
     ap.add_argument("--no-cpu-baseline", action="store_true")
     ap.add_argument("--cpu-layers", type=int, default=8, help="layers in the CPU-baseline sample")
-    ap.add_argument("--family", default=None, choices=[None, "ralasun", "madalorn", "sogalix", "potipel"],
-                    help="potipel: prefill / decode throughput of that layer-list design at --sizes beside a Madalorn model of "
+    ap.add_argument("--family", default=None, choices=[None, "ralasun", "madalorn", "sogalix", "potipel", "madudra"],
+                    help="madudra: prefill / decode throughput of that layer-list design at --sizes beside a Sogalix model of "
+                         "equal size (latent attention behind layer norms there too); potipel: prefill / decode throughput of that layer-list design at --sizes beside a Madalorn model of "
                          "equal size; sogalix: prefill / decode throughput of that layer-list design at --sizes beside a Madalorn model of "
                          "equal size; madalorn: prefill / decode throughput of that layer-list design at --sizes beside a Ralasun model of "
                          "equal size (the closest existing model: same engine, bf16 weights, window attention, routed experts); "
@@ -357,6 +358,67 @@ def _build_potipel(S, engine, z, max_pos, rng, pool):
     return m, per_tok / n
 
 
+def _build_madudra(S, engine, z, max_pos, rng, pool):
+    """State space, windowed latent attention, state space, latent attention on the cache of the one before, in turn; four residual
+    streams. State space: 2 x width channels in heads of 64, 128 state rows, 8 groups; latent sizes as in the Sogalix model. Every
+    layer has routed plain experts whose active columns add up to those of the other families' feed-forward at this size."""
+    W, V, H, d, n = z["width"], z["vocab"], z["heads"], z["dim"], z["layers"]
+    ff = (z["top"] * z["ff"] + z["shared_ff"]) // z["top"]
+    rq, rk, rd, ns, taps = W // 2, 4 * d, d // 2, 4, 4
+    hm, vm, N, G = 2 * W // 64, 64, 128, 8
+    inner, ch = hm * vm, hm * vm + 2 * G * N
+    moe = S.madudra_moe(z["experts"], z["top"], ff, scale=2.0)
+    layers = []
+    for i in range(n):
+        if i % 2 == 0:
+            layers.append(S.madudra_layer("mamba2", S.madudra_mamba(hm, vm, N, groups=G, conv=taps, norm_groups=G), moe))
+        else:
+            layers.append(S.madudra_layer("latent_attention", S.madudra_latent(
+                H, d, rd, d, rq, rk, z["window"], base=250000.0, scaling=(4.0, 4096, 32.0, 1.0), kv_from=i - 2 if i % 4 == 3 else None), moe))
+    m = engine.StackModel(S.madudra_config(W, V, layers, streams=ns, residual_mult=0.5, embed_scale=1.0), max_pos)
+
+    def mat(nm, r, c, std=None):
+        m.set_tensor(nm, _pool_bf16(S, r * c, std or 1.0 / np.sqrt(c), rng, pool).reshape(r, c))
+
+    def vec(nm, k, centre, spread=0.05):
+        m.set_tensor(nm, S.to_bf16((centre + spread * rng.standard_normal(k)).astype(np.float32)))
+
+    mat("embed", V, W, 1.0), mat("head", V, W), vec("final.norm", W, 1.0)
+    per_tok = 0
+    for i, L in enumerate(layers):
+        p, mx = f"l{i}.", L["mixer"]
+        for q in "12":
+            vec(p + "norm" + q, W, 1.0), vec(p + f"hc{q}.in", ns, 1.0 / ns), vec(p + f"hc{q}.out", ns, 1.0)
+            m.set_tensor(p + f"hc{q}.mix", S.to_bf16((0.7 * np.eye(ns) + 0.3 / ns).astype(np.float32)))
+        if L["type"] == "latent_attention":
+            own = mx.get("kv_from") is None
+            mat(p + "mix.dq", rq, W), vec(p + "mix.dq.norm", rq, 1.0), mat(p + "mix.uq", H * (d + rd), rq)
+            if own:
+                mat(p + "mix.dkv", rk + rd, W), vec(p + "mix.dkv.norm", rk, 1.0)
+            mat(p + "mix.uk", H * d, rk), mat(p + "mix.uv", H * d, rk), mat(p + "mix.g", H * d, W), mat(p + "mix.o", W, H * d)
+            per_tok += W * (rq + (rk + rd if own else 0) + H * d) + rq * H * (d + rd) + 2 * rk * H * d + H * d * W
+        else:
+            mat(p + "mix.in", inner + ch + hm, W), mat(p + "mix.conv", ch, taps, 0.5), vec(p + "mix.conv.b", ch, 0.0)
+            vec(p + "mix.dt_bias", hm, -2.0, 0.5), vec(p + "mix.A_log", hm, 0.0, 0.5), vec(p + "mix.D", hm, 1.0)
+            vec(p + "mix.norm", inner, 1.0), mat(p + "mix.o", W, inner)
+            per_tok += W * (inner + ch + hm) + inner * W
+        mat(p + "mlp.router", z["experts"], W)
+        for e in range(z["experts"]):
+            mat(p + f"mlp.e{e}.up", ff, W), mat(p + f"mlp.e{e}.down", W, ff)
+        per_tok += 2 * W * z["top"] * ff + W * z["experts"]
+    m.finalize()
+    return m, per_tok / n
+
+
+# family -> (builder, layers in words, the closest earlier family's name, its builder)
+FAMILIES = {
+    "madudra": (_build_madudra, "mamba2 / latent_attention / mamba2 / latent_attention (shared cache) in turn", "sogalix", _build_sogalix),
+    "potipel": (_build_potipel, "parallel (window attention | delta rule) / differential attention / hgrn2 in turn", "madalorn", _build_madalorn),
+    "sogalix": (_build_sogalix, "latent_attention / general_delta / attention / general_delta in turn", "madalorn", _build_madalorn),
+    "madalorn": (_build_madalorn, "attention / channel_delta in turn", "ralasun", _build_ralasun),
+}
+
+
 def stack_bench(args):
     from _pkg import load_package
     pkg = load_package()
@@ -371,54 +433,19 @@ def stack_bench(args):
         z = STACK_SIZES[name]
         W, V = z["width"], z["vocab"]
         max_pos = T + args.steps + args.warmup + 64
-        if args.family == "potipel":
+        if args.family in FAMILIES:
+            build, words, twin, build_twin = FAMILIES[args.family]
             z = dict(z, vdim=z["dim"])
             t0 = time.time()
-            m, per_tok = _build_potipel(S, engine, z, max_pos, rng, pool)
-            r = {"size": name, "shape": z, "layers": "parallel (window attention | delta rule) / differential attention / hgrn2 in turn",
-                 "load_s": round(time.time() - t0, 1)}
+            m, per_tok = build(S, engine, z, max_pos, rng, pool)
+            r = {"size": name, "shape": z, "layers": words, "load_s": round(time.time() - t0, 1)}
             got, toks, first = _time_stack_model(m, args, T, V, z["layers"], per_tok, rng)
             r.update(got)
             m.free()
             if not args.no_twin:
-                m, per_tok = _build_madalorn(S, engine, z, max_pos, rng, pool)
-                tw, _, _ = _time_stack_model(m, args, T, V, z["layers"], per_tok, rng)
+                m, per_tok = build_twin(S, engine, z, max_pos, rng, pool)
+                r[twin + "_twin"], _, _ = _time_stack_model(m, args, T, V, z["layers"], per_tok, rng)
                 m.free()
-                r["madalorn_twin"] = tw
-            results.append(r)
-            print(json.dumps(r), file=sys.stderr, flush=True)
-            continue
-        if args.family == "sogalix":
-            z = dict(z, vdim=z["dim"])
-            t0 = time.time()
-            m, per_tok = _build_sogalix(S, engine, z, max_pos, rng, pool)
-            r = {"size": name, "shape": z, "layers": "latent_attention / general_delta / attention / general_delta in turn",
-                 "load_s": round(time.time() - t0, 1)}
-            got, toks, first = _time_stack_model(m, args, T, V, z["layers"], per_tok, rng)
-            r.update(got)
-            m.free()
-            if not args.no_twin:
-                m, per_tok = _build_madalorn(S, engine, z, max_pos, rng, pool)
-                tw, _, _ = _time_stack_model(m, args, T, V, z["layers"], per_tok, rng)
-                m.free()
-                r["madalorn_twin"] = tw
-            results.append(r)
-            print(json.dumps(r), file=sys.stderr, flush=True)
-            continue
-        if args.family == "madalorn":
-            # the delta rule's value size equals its key size here, and the attention's values are its keys
-            z = dict(z, vdim=z["dim"])
-            t0 = time.time()
-            m, per_tok = _build_madalorn(S, engine, z, max_pos, rng, pool)
-            r = {"size": name, "shape": z, "layers": "attention / channel_delta in turn", "load_s": round(time.time() - t0, 1)}
-            got, toks, first = _time_stack_model(m, args, T, V, z["layers"], per_tok, rng)
-            r.update(got)
-            m.free()
-            if not args.no_twin:
-                m, per_tok = _build_ralasun(S, engine, z, max_pos, rng, pool)
-                tw, _, _ = _time_stack_model(m, args, T, V, z["layers"], per_tok, rng)
-                m.free()
-                r["ralasun_twin"] = tw
             results.append(r)
             print(json.dumps(r), file=sys.stderr, flush=True)
             continue
@@ -463,13 +490,9 @@ def stack_bench(args):
             r["llama_twin"] = tw
         results.append(r)
         print(json.dumps(r), file=sys.stderr, flush=True)
-    label = ("layer-list family (Potipel): prefill / decode tokens/s beside a Madalorn model of equal size"
-             if args.family == "potipel" else
-             "layer-list family (Sogalix): prefill / decode tokens/s beside a Madalorn model of equal size"
-             if args.family == "sogalix" else
-             "layer-list family (Madalorn): prefill / decode tokens/s beside a Ralasun model of equal size"
-             if args.family == "madalorn" else
-             "layer-list family (Ralasun): prefill / decode tokens/s beside a Llama model of equal size")
+    twin_name = FAMILIES[args.family][2] if args.family in FAMILIES else "llama"
+    label = (f"layer-list family ({args.family.capitalize()}): prefill / decode tokens/s beside a {twin_name.capitalize()} model of "
+             "equal size")
     print(json.dumps({"metric": label, "n_gpus": 1, "steps": args.steps, "warmup": args.warmup, "prefill_tokens": T,
                       "dtype": "bf16 weights, fp32 activations", "data": "synthetic", "results": results}))
     return 0

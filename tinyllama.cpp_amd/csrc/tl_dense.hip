@@ -317,7 +317,7 @@ extern "C" int tl_dense_matmul(const void* w_bf16_dev, int rows, int cols, const
 extern "C" int tl_dense_matmul_act(const void* w_bf16_dev, int rows, int cols, const float* x_dev, float* y_dev, int num_tokens,
                                    int terms, int act, float act_p, float act_q, int act_from, void* stream) {
   hipStream_t s = static_cast<hipStream_t>(stream);
-  TL_REQUIRE(act >= TL_ACT_NONE && act <= TL_ACT_TANH, "tl_dense_matmul_act: activation kind %d", act);
+  TL_REQUIRE(act >= TL_ACT_NONE && act <= TL_ACT_GELU, "tl_dense_matmul_act: activation kind %d", act);
   if (terms == 0) {
     TL_REQUIRE(num_tokens == 1, "tl_dense_matmul_act: terms 0 (FP32 GEMV) takes one token, not %d", num_tokens);
     return tl_launch_dense_gemv_act(static_cast<const uint16_t*>(w_bf16_dev), rows, cols, x_dev, y_dev,
