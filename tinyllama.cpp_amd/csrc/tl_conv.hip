@@ -76,6 +76,55 @@ __global__ __launch_bounds__(256) void conv4_kernel(const ConvArgs a) {
   *reinterpret_cast<float4*>(a.out + (size_t)t * a.ldo + c) = acc;
 }
 
+// grid (C / 4 in 256s, T in CONV_RUN s): the inputs a thread holds slide along, so a row is read once (and its last TAPS - 1 rows
+// once more by the next run)
+constexpr int CONV_RUN = 8;
+template <int TAPS>
+__global__ __launch_bounds__(256) void conv_run_kernel(const ConvArgs a) {
+  const int t0 = blockIdx.y * CONV_RUN, c = (blockIdx.x * 256 + threadIdx.x) * 4;
+  if (c >= a.C) return;
+  constexpr int H = TAPS - 1;
+  const float4 zero = make_float4(0.0f, 0.0f, 0.0f, 0.0f);
+  const float4 b = a.bias ? *reinterpret_cast<const float4*>(a.bias + c) : zero;
+  const float4 ob = a.out_bias ? *reinterpret_cast<const float4*>(a.out_bias + c) : zero;
+  float4 w[TAPS];
+#pragma unroll
+  for (int j = 0; j < TAPS; ++j) {
+    const unsigned short* wc = a.w + (size_t)c * TAPS + j;
+    w[j] = make_float4(tl_bf2f(wc[0]), tl_bf2f(wc[TAPS]), tl_bf2f(wc[2 * TAPS]), tl_bf2f(wc[3 * TAPS]));
+  }
+  float4 u[CONV_RUN + H];
+#pragma unroll
+  for (int i = 0; i < CONV_RUN + H; ++i) {
+    const int tt = t0 - H + i;  // token of this input, relative to the call
+    if (tt >= a.T) {
+      u[i] = zero;
+    } else if (tt >= 0) {
+      u[i] = *reinterpret_cast<const float4*>(a.in + (size_t)tt * a.ldi + c);
+      u[i].x += b.x, u[i].y += b.y, u[i].z += b.z, u[i].w += b.w;
+    } else {
+      u[i] = *reinterpret_cast<const float4*>(a.hist + (size_t)(H + tt) * a.C + c);
+    }
+  }
+#pragma unroll
+  for (int i = 0; i < CONV_RUN; ++i) {
+    if (t0 + i >= a.T) break;
+    float4 acc = ob;
+#pragma unroll
+    for (int j = 0; j < TAPS; ++j) {
+      acc.x += w[j].x * u[i + j].x, acc.y += w[j].y * u[i + j].y;
+      acc.z += w[j].z * u[i + j].z, acc.w += w[j].w * u[i + j].w;
+    }
+    if (a.act == 1) {
+      acc.x = acc.x / (1.0f + expf(-acc.x)), acc.y = acc.y / (1.0f + expf(-acc.y));
+      acc.z = acc.z / (1.0f + expf(-acc.z)), acc.w = acc.w / (1.0f + expf(-acc.w));
+    }
+    const float4 cur = u[i + H];
+    if (a.add_input) acc.x += cur.x, acc.y += cur.y, acc.z += cur.z, acc.w += cur.w;
+    *reinterpret_cast<float4*>(a.out + (size_t)(t0 + i) * a.ldo + c) = acc;
+  }
+}
+
 __global__ __launch_bounds__(256) void conv_history_rows_kernel(const ConvArgs a) {
   const int c = blockIdx.x * 256 + threadIdx.x, H = a.taps - 1;
   if (c >= a.C) return;
@@ -95,9 +144,14 @@ int tl_launch_causal_conv(const ConvArgs& a, hipStream_t s) {
   TL_REQUIRE(a.T == 1 || a.out + (size_t)a.T * a.ldo <= a.in || a.in + (size_t)a.T * a.ldi <= a.out,
              "causal_conv: output over input with more than one token");
   TL_REQUIRE(a.act == 0 || a.act == 1, "causal_conv: activation %d", a.act);
-  const bool vec = a.T > 1 && (a.C & 3) == 0 && a.ldi == a.C && (a.ldo & 3) == 0 && ((size_t)a.in & 15) == 0 &&
+  const bool al = a.T > 1 && (a.C & 3) == 0 && (a.ldi & 3) == 0 && (a.ldo & 3) == 0 && ((size_t)a.in & 15) == 0 &&
                    ((size_t)a.out & 15) == 0 && ((size_t)a.hist & 15) == 0 && ((size_t)a.bias & 15) == 0 && ((size_t)a.out_bias & 15) == 0;
-  if (vec) conv4_kernel<<<dim3((a.C / 4 + 255) / 256, a.T), 256, 0, s>>>(a);
+  const bool vec = al && a.ldi == a.C;
+  const dim3 runs((a.C / 4 + 255) / 256, (a.T + CONV_RUN - 1) / CONV_RUN);
+  if (al && a.T >= CONV_RUN && a.taps == 4) conv_run_kernel<4><<<runs, 256, 0, s>>>(a);
+  else if (al && a.T >= CONV_RUN && a.taps == 3) conv_run_kernel<3><<<runs, 256, 0, s>>>(a);
+  else if (al && a.T >= CONV_RUN && a.taps == 2) conv_run_kernel<2><<<runs, 256, 0, s>>>(a);
+  else if (vec) conv4_kernel<<<dim3((a.C / 4 + 255) / 256, a.T), 256, 0, s>>>(a);
   else conv_kernel<<<dim3((a.C + 255) / 256, a.T), 256, 0, s>>>(a);
   if (a.T > 1 && a.taps > 1) conv_history_rows_kernel<<<(a.C + 255) / 256, 256, 0, s>>>(a);
   TL_HIP(hipGetLastError());

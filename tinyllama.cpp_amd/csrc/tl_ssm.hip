@@ -12,7 +12,8 @@
 //     S_after = exp(c_last) S_before + sum_j exp(c_last - c_j) dt_j B_j x_j^T:
 //
 // the recurrence becomes three small matrix products per block; only S is handed on from block to block.
-//   ssm_gram    C_i . B_j of every block and GROUP (lower triangle of 64 x 64): heads / groups heads share it.
+//   ssm_gram    C_i . B_j of every block and GROUP (lower triangle of 64 x 64): heads / groups heads share it; and, per block and
+//               head, dt, c and the two exponentials that depend on one token only.
 //   ssm_walk    one workgroup of 4 waves per (32 value channels, head) walks the blocks in order. S lives in accumulator
 //               registers: wave w holds the state rows 32 (w + 4 k) .. + 31 of its 32 columns, in the layout in which the matrix
 //               instruction leaves a result -- which is also the operand layout its product with C needs (the order of a sum's
@@ -48,12 +49,39 @@ __device__ __forceinline__ ssm_f32x4 ssm_ld4(const float* p, int d, int n, bool 
   return v;
 }
 
-// grid (blocks, groups), 3 waves: the tiles (0,0), (1,0), (1,1) of the block's 64 x 64 products
+// What the walk needs of a block of tokens and a head besides x, B, C, and what it keeps in LDS of it
+struct SsmSteps {
+  double cum[SSM_Q];                    // c_i
+  float dt[SSM_Q], w[SSM_Q], e[SSM_Q];  // dt_j; exp(c_last - c_j) dt_j; exp(c_i)
+};
+constexpr int SSM_STEP_FLOATS = sizeof(SsmSteps) / sizeof(float);
+
+// grid (blocks, groups + heads in threes), 3 waves. blockIdx.y < groups: the tiles (0,0), (1,0), (1,1) of the block's 64 x 64
+// products of that group; otherwise a wave per head: its SsmSteps
 __global__ __launch_bounds__(192) void ssm_gram_kernel(const SsmScanArgs a, int vec) {
   const int wave = threadIdx.x >> 6, lane = threadIdx.x & 63, r = lane & 31, h = lane >> 5;
-  const int ti = wave == 0 ? 0 : 1, tj = wave == 2 ? 1 : 0;
   const int t0 = blockIdx.x * SSM_Q, g = blockIdx.y;
-  if (ti == 1 && t0 + 32 >= a.T) return;  // no token of the second half: nothing reads those tiles
+  float* grams = a.gram;
+  SsmSteps* steps = reinterpret_cast<SsmSteps*>(a.gram + (size_t)gridDim.x * a.groups * SSM_Q * SSM_Q);
+  if (g >= a.groups) {
+    const int head = (g - a.groups) * 3 + wave;
+    if (head >= a.heads) return;
+    const float dt = t0 + lane < a.T ? ssm_softplus(a.dt_raw[(size_t)(t0 + lane) * a.dt_ld + head] + a.dt_bias[head]) : 0.0f;
+    double c = -(double)(expf(a.a_log[head]) * dt);
+#pragma unroll
+    for (int o = 1; o < 64; o <<= 1) {
+      const double up = __shfl_up(c, o);
+      if (lane >= o) c += up;
+    }
+    const double tot = __shfl(c, 63);
+    SsmSteps* o = steps + (size_t)blockIdx.x * a.heads + head;
+    o->cum[lane] = c;
+    o->dt[lane] = dt;
+    o->w[lane] = dt * expf((float)(tot - c));
+    o->e[lane] = expf((float)c);
+    return;
+  }
+  const int ti = wave == 0 ? 0 : 1, tj = wave == 2 ? 1 : 0;
   const int N = a.state_n, inner = a.heads * a.vdim;
   auto row = [&](int t) { return t < a.T ? t : a.T - 1; };  // rows beyond the call carry weight 0 where they are used
   const float* bp = a.xbc + (size_t)row(t0 + tj * 32 + r) * a.ld + inner + (size_t)g * N;
@@ -66,33 +94,81 @@ __global__ __launch_bounds__(192) void ssm_gram_kernel(const SsmScanArgs a, int 
 #pragma unroll
     for (int c = 0; c < 4; ++c) acc = __builtin_amdgcn_mfma_f32_32x32x2f32(cv[c], bv[c], acc, 0, 0, 0);
   }
-  float* o = a.gram + ((size_t)blockIdx.x * a.groups + g) * SSM_Q * SSM_Q;
+  float* o = grams + ((size_t)blockIdx.x * a.groups + g) * SSM_Q * SSM_Q;
 #pragma unroll
   for (int e = 0; e < 16; ++e) o[(size_t)(ti * 32 + ssm_row(e, h)) * SSM_Q + tj * 32 + r] = acc[e];
 }
 
-struct SsmLds {  // dynamic LDS of ssm_walk_kernel
-  double cum[SSM_Q];                 // c_i
+struct SsmLds {  // dynamic LDS of ssm_walk_kernel; what a block's last readers may still read while the next one arrives is doubled
+  SsmSteps st[2];
+  float x[2][SSM_Q][SSM_LD];         // x of the block
   float p[SSM_Q][SSM_PLD];           // exp(c_i - c_j) dt_j (C_i . B_j), j <= i
-  float x[SSM_Q][SSM_LD];            // x of the block
   float part[4][SSM_Q][SSM_LD];      // the waves' partial Y
-  float dt[SSM_Q], w[SSM_Q], e[SSM_Q];  // dt_j; exp(c_last - c_j) dt_j; exp(c_i)
 };
 
-// NT state tiles of 32 rows per wave: state <= 128 NT
+// NT state tiles of 32 rows per wave: state <= 128 NT. Whatever comes from memory for a block is asked for while the block before
+// is worked on (B and C only with NT == 1: registers), since a workgroup is often alone on its CU.
 template <int NT>
-__global__ __launch_bounds__(256, 2) void ssm_walk_kernel(const SsmScanArgs a, int vec) {
+__global__ __launch_bounds__(256, NT == 1 ? 2 : 1) void ssm_walk_kernel(const SsmScanArgs a, int vec) {
   extern __shared__ __attribute__((aligned(16))) unsigned char ssm_lds_raw[];
   SsmLds& L = *reinterpret_cast<SsmLds*>(ssm_lds_raw);
+  constexpr bool PF = NT == 1;
   const int tid = threadIdx.x, wave = tid >> 6, lane = tid & 63, r = lane & 31, h = lane >> 5;
   const int v0 = blockIdx.x * 32, head = blockIdx.y, g = head / (a.heads / a.groups);
-  const int N = a.state_n, vdim = a.vdim, inner = a.heads * vdim;
+  const int N = a.state_n, vdim = a.vdim, inner = a.heads * vdim, last = a.T - 1;
+  const int blocks = (a.T + SSM_Q - 1) / SSM_Q;
   const bool vlive = v0 + r < vdim;
   const float* xp = a.xbc + (size_t)head * vdim + v0;
   const float* bp = a.xbc + inner + (size_t)g * N;
   const float* cp = bp + (size_t)a.groups * N;
-  const float rate = expf(a.a_log[head]), dtb = a.dt_bias[head], dskip = a.d[head];
+  const float* zp = a.z ? a.z + (size_t)head * vdim + v0 : nullptr;
+  const float dskip = a.d[head];
+  const float* stp = a.gram + (size_t)blocks * a.groups * SSM_Q * SSM_Q + (size_t)head * SSM_STEP_FLOATS;
   float* sp = a.state + (size_t)head * N * vdim + v0;
+  // (row offsets fit 32 bits: the launcher checks; rows beyond the call repeat its last row and carry weight 0)
+  auto row = [&](int t) __attribute__((always_inline)) { return (unsigned)(t < last ? t : last); };
+  // this thread's elements of a block: x and z (token i * 8 + tid / 32, column tid % 32), the products (row i * 4 + tid / 64)
+  const int xt = tid >> 5, xc = tid & 31;
+  const bool xlive = v0 + xc < vdim;
+  float xr[8], zr[8], gr[16], sr[2];
+  auto fetch_x = [&](int b) __attribute__((always_inline)) {
+#pragma unroll
+    for (int i = 0; i < 8; ++i) xr[i] = xlive ? xp[row(b * SSM_Q + i * 8 + xt) * (unsigned)a.ld + xc] : 0.0f;
+    const float* s = stp + (size_t)b * a.heads * SSM_STEP_FLOATS;
+    sr[0] = s[tid];
+    sr[1] = tid < SSM_STEP_FLOATS - 256 ? s[256 + tid] : 0.0f;
+  };
+  auto fetch_z = [&](int b) __attribute__((always_inline)) {
+    if (!zp) return;
+#pragma unroll
+    for (int i = 0; i < 8; ++i) zr[i] = xlive ? zp[row(b * SSM_Q + i * 8 + xt) * (unsigned)a.z_ld + xc] : 0.0f;
+  };
+  auto fetch_g = [&](int b) __attribute__((always_inline)) {
+    const float* gp = a.gram + ((size_t)b * a.groups + g) * SSM_Q * SSM_Q;
+#pragma unroll
+    for (int i = 0; i < 16; ++i) gr[i] = gp[i * 256 + tid];  // (never-written tiles are not used below)
+  };
+  ssm_f32x4 cr[PF ? 2 : 1][4];
+  auto fetch_c = [&](int b, int tt, int k, ssm_f32x4* to) __attribute__((always_inline)) {
+    const float* c = cp + row(b * SSM_Q + tt * 32 + r) * (unsigned)a.ld;
+#pragma unroll
+    for (int q = 0; q < 4; ++q) to[q] = ssm_ld4(c, 32 * (wave + 4 * k) + 8 * q + 4 * h, N, vec);
+  };
+  float br[PF ? 2 : 1][16];
+  auto fetch_b = [&](int b, int half, int k, float* to) __attribute__((always_inline)) {
+    const int n = 32 * (wave + 4 * k) + r;
+    const float* p = bp + (n < N ? n : N - 1);  // (rows beyond the state meet zeros of C and are not stored)
+    const unsigned t = b * SSM_Q + 32 * half + h;
+    if ((int)(t + 32) <= a.T) {
+      const unsigned o = t * (unsigned)a.ld;
+#pragma unroll
+      for (int s = 0; s < 16; ++s) to[s] = p[o + 2 * s * (unsigned)a.ld];
+    } else {
+#pragma unroll
+      for (int s = 0; s < 16; ++s) to[s] = p[row(t + 2 * s) * (unsigned)a.ld];
+    }
+  };
+  const bool mine = 32 * wave < N;  // this wave holds state rows at all
   ssm_f32x16 S[NT];
 #pragma unroll
   for (int k = 0; k < NT; ++k)
@@ -101,117 +177,127 @@ __global__ __launch_bounds__(256, 2) void ssm_walk_kernel(const SsmScanArgs a, i
       const int n = 32 * (wave + 4 * k) + ssm_row(e, h);
       S[k][e] = n < N && vlive ? sp[(size_t)n * vdim + r] : 0.0f;
     }
-  for (int t0 = 0; t0 < a.T; t0 += SSM_Q) {
-    const int nt = a.T - t0 < SSM_Q ? a.T - t0 : SSM_Q;
+  fetch_x(0);
+  fetch_g(0);
+  if (PF && mine) {
+#pragma unroll
+    for (int tt = 0; tt < 2; ++tt) fetch_c(0, tt, 0, cr[PF ? tt : 0]);
+#pragma unroll
+    for (int tt = 0; tt < 2; ++tt) fetch_b(0, tt, 0, br[PF ? tt : 0]);
+  }
+  fetch_z(0);
+  for (int b = 0; b < blocks; ++b) {
+    const int t0 = b * SSM_Q, nt = a.T - t0 < SSM_Q ? a.T - t0 : SSM_Q;
     const bool two = nt > 32;  // tokens in the second half of the block
-    auto row = [&](int t) { return (size_t)(t0 + (t < nt ? t : nt - 1)); };
-    if (wave == 0) {
-      const float dt = lane < nt ? ssm_softplus(a.dt_raw[(size_t)(t0 + lane) * a.dt_ld + head] + dtb) : 0.0f;
-      double c = -(double)(rate * dt);
+    const bool more = b + 1 < blocks;
+    SsmSteps& st = L.st[b & 1];
+    float (*x)[SSM_LD] = L.x[b & 1];
 #pragma unroll
-      for (int o = 1; o < 64; o <<= 1) {
-        const double up = __shfl_up(c, o);
-        if (lane >= o) c += up;
-      }
-      const double tot = __shfl(c, 63);
-      L.cum[lane] = c;
-      L.dt[lane] = dt;
-      L.w[lane] = dt * expf((float)(tot - c));
-      L.e[lane] = expf((float)c);
-    }
-#pragma unroll
-    for (int i = 0; i < SSM_Q * 32 / 256; ++i) {
-      const int idx = i * 256 + tid, t = idx >> 5, c = idx & 31;
-      L.x[t][c] = t < nt && v0 + c < vdim ? xp[(size_t)(t0 + t) * a.ld + c] : 0.0f;
-    }
-    // C S of the waves' state rows: the scores of the first product's operand come straight from the token's own row
+    for (int i = 0; i < 8; ++i) x[i * 8 + xt][xc] = t0 + i * 8 + xt < a.T ? xr[i] : 0.0f;
+    reinterpret_cast<float*>(&st)[tid] = sr[0];
+    if (tid < SSM_STEP_FLOATS - 256) reinterpret_cast<float*>(&st)[256 + tid] = sr[1];
+    __syncthreads();  // x and the steps of the block are in LDS
+    if (more) fetch_x(b + 1);
+    // C S over this wave's state rows
     ssm_f32x16 acc[2];
 #pragma unroll
     for (int tt = 0; tt < 2; ++tt)
 #pragma unroll
       for (int e = 0; e < 16; ++e) acc[tt][e] = 0.0f;
-#pragma unroll
-    for (int tt = 0; tt < 2; ++tt) {
-      if (tt == 1 && !two) break;
-      const float* cr = cp + row(tt * 32 + r) * a.ld;
-#pragma unroll
-      for (int k = 0; k < NT; ++k) {
-        const int n0 = 32 * (wave + 4 * k);
-        if (n0 >= N) break;
-        ssm_f32x4 cv[4];
-#pragma unroll
-        for (int q = 0; q < 4; ++q) cv[q] = ssm_ld4(cr, n0 + 8 * q + 4 * h, N, vec);
+    if (PF) {
+      if (mine) {
 #pragma unroll
         for (int q = 0; q < 4; ++q)
 #pragma unroll
-          for (int c = 0; c < 4; ++c) acc[tt] = __builtin_amdgcn_mfma_f32_32x32x2f32(cv[q][c], S[k][4 * q + c], acc[tt], 0, 0, 0);
+          for (int c = 0; c < 4; ++c)
+#pragma unroll
+            for (int tt = 0; tt < 2; ++tt)
+              acc[tt] = __builtin_amdgcn_mfma_f32_32x32x2f32(cr[PF ? tt : 0][q][c], S[0][4 * q + c], acc[tt], 0, 0, 0);
+        if (more) {
+#pragma unroll
+          for (int tt = 0; tt < 2; ++tt) fetch_c(b + 1, tt, 0, cr[PF ? tt : 0]);
+        }
+      }
+    } else {
+#pragma unroll
+      for (int tt = 0; tt < 2; ++tt) {
+        if (tt == 1 && !two) continue;
+#pragma unroll
+        for (int k = 0; k < NT; ++k) {
+          if (32 * (wave + 4 * k) >= N) continue;
+          fetch_c(b, tt, k, cr[0]);
+#pragma unroll
+          for (int q = 0; q < 4; ++q)
+#pragma unroll
+            for (int c = 0; c < 4; ++c)
+              acc[tt] = __builtin_amdgcn_mfma_f32_32x32x2f32(cr[0][q][c], S[k][4 * q + c], acc[tt], 0, 0, 0);
+        }
       }
     }
-    __syncthreads();  // dt, c_i and x of the block are in LDS
-    const float* gp = a.gram + ((size_t)(t0 / SSM_Q) * a.groups + g) * SSM_Q * SSM_Q;
+    {
+      const int tj = lane;  // (this thread's column of the products in every row it fills)
+      const double cj = st.cum[tj];
+      const float dj = st.dt[tj];
 #pragma unroll
-    for (int i = 0; i < SSM_Q * SSM_Q / 256; ++i) {
-      const int idx = i * 256 + tid, ti = idx >> 6, tj = idx & 63;
-      float v = 0.0f;
-      if (tj <= ti && ti < nt) v = gp[idx] * expf((float)(L.cum[ti] - L.cum[tj])) * L.dt[tj];
-      L.p[ti][tj] = v;
+      for (int i = 0; i < 16; ++i) {
+        const int ti = i * 4 + wave;
+        L.p[ti][tj] = tj <= ti && ti < nt ? gr[i] * expf((float)(st.cum[ti] - cj)) * dj : 0.0f;
+      }
     }
+    if (more) fetch_g(b + 1);
 #pragma unroll
     for (int tt = 0; tt < 2; ++tt)
 #pragma unroll
-      for (int e = 0; e < 16; ++e) acc[tt][e] *= L.e[tt * 32 + ssm_row(e, h)];
+      for (int e = 0; e < 16; ++e) acc[tt][e] *= st.e[tt * 32 + ssm_row(e, h)];
     __syncthreads();  // P is whole
     // P X: the first half's tokens look at 32 columns (8 a wave), the second half's at 64 (16 a wave)
     {
       const int j0 = 8 * wave + 4 * h;
       const ssm_f32x4 pv = *reinterpret_cast<const ssm_f32x4*>(&L.p[r][j0]);
 #pragma unroll
-      for (int c = 0; c < 4; ++c) acc[0] = __builtin_amdgcn_mfma_f32_32x32x2f32(pv[c], L.x[j0 + c][r], acc[0], 0, 0, 0);
-      if (two) {
+      for (int c = 0; c < 4; ++c) acc[0] = __builtin_amdgcn_mfma_f32_32x32x2f32(pv[c], x[j0 + c][r], acc[0], 0, 0, 0);
 #pragma unroll
-        for (int q = 0; q < 2; ++q) {
-          const int j1 = 16 * wave + 8 * q + 4 * h;
-          const ssm_f32x4 pw = *reinterpret_cast<const ssm_f32x4*>(&L.p[32 + r][j1]);
+      for (int q = 0; q < 2; ++q) {
+        const int j1 = 16 * wave + 8 * q + 4 * h;
+        const ssm_f32x4 pw = *reinterpret_cast<const ssm_f32x4*>(&L.p[32 + r][j1]);
 #pragma unroll
-          for (int c = 0; c < 4; ++c) acc[1] = __builtin_amdgcn_mfma_f32_32x32x2f32(pw[c], L.x[j1 + c][r], acc[1], 0, 0, 0);
+        for (int c = 0; c < 4; ++c) acc[1] = __builtin_amdgcn_mfma_f32_32x32x2f32(pw[c], x[j1 + c][r], acc[1], 0, 0, 0);
+      }
+    }
+    // S <- exp(c_last) S + B^T (w x)
+    const float decay = st.e[SSM_Q - 1];
+#pragma unroll
+    for (int k = 0; k < NT; ++k) {
+      if (32 * (wave + 4 * k) >= N) continue;
+#pragma unroll
+      for (int e = 0; e < 16; ++e) S[k][e] *= decay;
+#pragma unroll
+      for (int half = 0; half < 2; ++half) {
+        if (half == 1 && !two) continue;
+        float* bv = br[PF ? half : 0];
+        if (!PF) fetch_b(b, half, k, bv);
+#pragma unroll
+        for (int s = 0; s < 16; ++s) {
+          const int j = 32 * half + 2 * s + h;
+          S[k] = __builtin_amdgcn_mfma_f32_32x32x2f32(bv[s], st.w[j] * x[j][r], S[k], 0, 0, 0);
         }
+        if (PF && more) fetch_b(b + 1, half, 0, bv);
       }
     }
 #pragma unroll
     for (int tt = 0; tt < 2; ++tt)
 #pragma unroll
       for (int e = 0; e < 16; ++e) L.part[wave][tt * 32 + ssm_row(e, h)][r] = acc[tt][e];
-    // S <- exp(c_last) S + B^T (w x)
-    const float decay = L.e[SSM_Q - 1];
-#pragma unroll
-    for (int k = 0; k < NT; ++k) {
-      const int n = 32 * (wave + 4 * k) + r;
-      if (32 * (wave + 4 * k) >= N) break;
-#pragma unroll
-      for (int e = 0; e < 16; ++e) S[k][e] *= decay;
-#pragma unroll
-      for (int half = 0; half < 2; ++half) {
-        if (half == 1 && !two) break;
-        float bv[16];
-#pragma unroll
-        for (int s = 0; s < 16; ++s) bv[s] = n < N ? bp[row(32 * half + 2 * s + h) * a.ld + n] : 0.0f;
-#pragma unroll
-        for (int s = 0; s < 16; ++s) {
-          const int j = 32 * half + 2 * s + h;
-          S[k] = __builtin_amdgcn_mfma_f32_32x32x2f32(bv[s], L.w[j] * L.x[j][r], S[k], 0, 0, 0);
-        }
-      }
-    }
     __syncthreads();  // the partial Y are whole
 #pragma unroll
-    for (int i = 0; i < SSM_Q * 32 / 256; ++i) {
-      const int idx = i * 256 + tid, t = idx >> 5, c = idx & 31;
-      if (t >= nt || v0 + c >= vdim) continue;
-      float y = ((L.part[0][t][c] + L.part[1][t][c]) + (L.part[2][t][c] + L.part[3][t][c])) + dskip * L.x[t][c];
-      if (a.z) y *= ssm_silu(a.z[(size_t)(t0 + t) * a.z_ld + (size_t)head * vdim + v0 + c]);
-      a.y[(size_t)(t0 + t) * inner + (size_t)head * vdim + v0 + c] = y;
+    for (int i = 0; i < 8; ++i) {
+      const int t = i * 8 + xt;
+      if (t >= nt || !xlive) continue;
+      float y = ((L.part[0][t][xc] + L.part[1][t][xc]) + (L.part[2][t][xc] + L.part[3][t][xc])) + dskip * x[t][xc];
+      if (zp) y *= ssm_silu(zr[i]);
+      a.y[(size_t)(t0 + t) * inner + (size_t)head * vdim + v0 + xc] = y;
     }
-    __syncthreads();  // x and the partial Y may be overwritten
+    if (more) fetch_z(b + 1);
   }
 #pragma unroll
   for (int k = 0; k < NT; ++k)
@@ -352,7 +438,9 @@ int launch_walk(const SsmScanArgs& a, int vec, hipStream_t s) {
 
 }  // namespace
 
-size_t tl_ssm_gram_floats(int T, int groups) { return (size_t)((T + SSM_Q - 1) / SSM_Q) * groups * SSM_Q * SSM_Q; }
+size_t tl_ssm_gram_floats(int T, int heads, int groups) {
+  return (size_t)((T + SSM_Q - 1) / SSM_Q) * ((size_t)groups * SSM_Q * SSM_Q + (size_t)heads * SSM_STEP_FLOATS);
+}
 
 int tl_launch_ssm_scan(const SsmScanArgs& a, hipStream_t s) {
   TL_REQUIRE(a.xbc && a.dt_raw && a.dt_bias && a.a_log && a.d && a.state && a.y && a.gram && a.T > 0, "ssm_scan: bad arguments");
@@ -363,7 +451,9 @@ int tl_launch_ssm_scan(const SsmScanArgs& a, hipStream_t s) {
              "ssm_scan: row strides %d / %d / %d", a.ld, a.dt_ld, a.z_ld);
   // 16-byte pieces of B and C rows
   const int vec = (a.state_n & 3) == 0 && (a.ld & 3) == 0 && ((a.heads * a.vdim) & 3) == 0 && ((size_t)a.xbc & 15) == 0;
-  ssm_gram_kernel<<<dim3((a.T + SSM_Q - 1) / SSM_Q, a.groups), 192, 0, s>>>(a, vec);
+  TL_REQUIRE(a.T < (1 << 30) / (a.ld > a.z_ld ? a.ld : a.z_ld), "ssm_scan: %d tokens in rows of %d / %d", a.T, a.ld, a.z_ld);
+  TL_REQUIRE(((size_t)a.gram & 7) == 0, "ssm_scan: scratch not aligned");
+  ssm_gram_kernel<<<dim3((a.T + SSM_Q - 1) / SSM_Q, a.groups + (a.heads + 2) / 3), 192, 0, s>>>(a, vec);
   const int nt = (a.state_n + 127) / 128;
   if (nt <= 1) return launch_walk<1>(a, vec, s);
   if (nt <= 2) return launch_walk<2>(a, vec, s);
@@ -396,7 +486,7 @@ int tl_launch_part_norm(const PartNormArgs& a, hipStream_t s) {
 extern "C" int tl_state_space(const float* xbc_dev, int ld, const float* dt_raw_dev, int dt_ld, const float* dt_bias_dev,
                               const float* a_log_dev, const float* d_dev, const float* z_dev, int z_ld, float* state_dev,
                               float* y_dev, int num_tokens, int heads, int groups, int state, int vdim, void* stream) {
-  TL_REQUIRE(num_tokens > 0 && groups > 0, "tl_state_space: bad arguments");
+  TL_REQUIRE(num_tokens > 0 && groups > 0 && heads > 0, "tl_state_space: bad arguments");
   SsmScanArgs a = {};
   a.xbc = xbc_dev;
   a.ld = ld;
@@ -415,7 +505,7 @@ extern "C" int tl_state_space(const float* xbc_dev, int ld, const float* dt_raw_
   a.state_n = state;
   a.vdim = vdim;
   void* ws = nullptr;
-  TL_TRY(tl_scratch(TL_SCRATCH_SSM, sizeof(float) * tl_ssm_gram_floats(num_tokens, groups), &ws));
+  TL_TRY(tl_scratch(TL_SCRATCH_SSM, sizeof(float) * tl_ssm_gram_floats(num_tokens, heads, groups), &ws));
   a.gram = static_cast<float*>(ws);
   return tl_launch_ssm_scan(a, static_cast<hipStream_t>(stream));
 }

@@ -493,7 +493,7 @@ struct SsmScanArgs {
   float* gram;           // scratch, tl_ssm_gram_floats
   int T, heads, groups, state_n, vdim;
 };
-size_t tl_ssm_gram_floats(int T, int groups);
+size_t tl_ssm_gram_floats(int T, int heads, int groups);
 int tl_launch_ssm_scan(const SsmScanArgs& a, hipStream_t s);
 // one token with its convolution
 struct SsmStepArgs {

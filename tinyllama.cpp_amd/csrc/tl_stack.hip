@@ -391,7 +391,7 @@ int setup_mixer(TlStack* st, Layer& L, int i, bool own, int* first_mix) {
     const int ch = L.vd + L.kd + L.qd;   // channels of the convolution: x | B | C
     L.pd = L.od + ch + sp.heads;         // z | x | B | C | dt
     st->max_dc = ch > st->max_dc ? ch : st->max_dc;
-    const size_t gr = tl_ssm_gram_floats(st->chunk, sp.kv_heads);
+    const size_t gr = tl_ssm_gram_floats(st->chunk, sp.heads, sp.kv_heads);
     st->max_gram = gr > st->max_gram ? gr : st->max_gram;
     st->cache_bytes += sizeof(float) * ((size_t)sp.heads * sp.vdim * sp.dim + (size_t)(sp.conv_taps - 1) * ch);
     L.expect.insert({"mix.in", "mix.conv", "mix.conv.b", "mix.dt_bias", "mix.A_log", "mix.D", "mix.norm", "mix.o"});
