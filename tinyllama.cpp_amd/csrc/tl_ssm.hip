@@ -37,6 +37,15 @@ constexpr int SSM_LD = 36, SSM_PLD = 68;  // padded LDS rows of 32 / 64 floats (
 
 __device__ __forceinline__ float ssm_softplus(float z) { return z > 20.0f ? z : log1pf(expf(z)); }
 __device__ __forceinline__ float ssm_silu(float z) { return z / (1.0f + expf(-z)); }
+// the same from the hardware's exp2 and reciprocal: relative error near 1e-7 |z| where the result matters
+__device__ __forceinline__ float ssm_silu_fast(float z) { return z * __builtin_amdgcn_rcpf(1.0f + __expf(-z)); }
+// base (the same for the wave) + a lane's own element: one 32-bit offset register per load
+__device__ __forceinline__ float ssm_at(const float* base, unsigned e) {
+  return *reinterpret_cast<const float*>(reinterpret_cast<const char*>(base) + (size_t)(e * 4u));
+}
+__device__ __forceinline__ ssm_f32x4 ssm_at4(const float* base, unsigned e) {
+  return *reinterpret_cast<const ssm_f32x4*>(reinterpret_cast<const char*>(base) + (size_t)(e * 4u));
+}
 // row of a 32 x 32 result held in accumulator register e of lane half h
 __device__ __forceinline__ int ssm_row(int e, int h) { return (e & 3) + 8 * (e >> 2) + 4 * h; }
 
@@ -55,6 +64,7 @@ struct SsmSteps {
   float dt[SSM_Q], w[SSM_Q], e[SSM_Q];  // dt_j; exp(c_last - c_j) dt_j; exp(c_i)
 };
 constexpr int SSM_STEP_FLOATS = sizeof(SsmSteps) / sizeof(float);
+static_assert(SSM_STEP_FLOATS == 256 + 64, "ssm_walk_kernel copies 256 + 64 floats");
 
 // grid (blocks, groups + heads in threes), 3 waves. blockIdx.y < groups: the tiles (0,0), (1,0), (1,1) of the block's 64 x 64
 // products of that group; otherwise a wave per head: its SsmSteps
@@ -108,20 +118,22 @@ struct SsmLds {  // dynamic LDS of ssm_walk_kernel; what a block's last readers 
 
 // NT state tiles of 32 rows per wave: state <= 128 NT. Whatever comes from memory for a block is asked for while the block before
 // is worked on (B and C only with NT == 1: registers), since a workgroup is often alone on its CU.
-template <int NT>
+// EVEN: state and vdim are multiples of 32, the tokens whole blocks, and B, C rows can be read in 16-byte pieces.
+template <int NT, bool EVEN>
 __global__ __launch_bounds__(256, NT == 1 ? 2 : 1) void ssm_walk_kernel(const SsmScanArgs a, int vec) {
   extern __shared__ __attribute__((aligned(16))) unsigned char ssm_lds_raw[];
   SsmLds& L = *reinterpret_cast<SsmLds*>(ssm_lds_raw);
   constexpr bool PF = NT == 1;
-  const int tid = threadIdx.x, wave = tid >> 6, lane = tid & 63, r = lane & 31, h = lane >> 5;
+  const int tid = threadIdx.x, lane = tid & 63, r = lane & 31, h = lane >> 5;
+  const int wave = __builtin_amdgcn_readfirstlane(tid >> 6);
   const int v0 = blockIdx.x * 32, head = blockIdx.y, g = head / (a.heads / a.groups);
   const int N = a.state_n, vdim = a.vdim, inner = a.heads * vdim, last = a.T - 1;
   const int blocks = (a.T + SSM_Q - 1) / SSM_Q;
-  const bool vlive = v0 + r < vdim;
-  const float* xp = a.xbc + (size_t)head * vdim + v0;
+  const bool vlive = EVEN || v0 + r < vdim;
+  const float* xp = a.xbc + (size_t)head * vdim;
   const float* bp = a.xbc + inner + (size_t)g * N;
   const float* cp = bp + (size_t)a.groups * N;
-  const float* zp = a.z ? a.z + (size_t)head * vdim + v0 : nullptr;
+  const float* zp = a.z ? a.z + (size_t)head * vdim : nullptr;
   const float dskip = a.d[head];
   const float* stp = a.gram + (size_t)blocks * a.groups * SSM_Q * SSM_Q + (size_t)head * SSM_STEP_FLOATS;
   float* sp = a.state + (size_t)head * N * vdim + v0;
@@ -129,43 +141,60 @@ __global__ __launch_bounds__(256, NT == 1 ? 2 : 1) void ssm_walk_kernel(const Ss
   auto row = [&](int t) __attribute__((always_inline)) { return (unsigned)(t < last ? t : last); };
   // this thread's elements of a block: x and z (token i * 8 + tid / 32, column tid % 32), the products (row i * 4 + tid / 64)
   const int xt = tid >> 5, xc = tid & 31;
-  const bool xlive = v0 + xc < vdim;
+  const bool xlive = EVEN || v0 + xc < vdim;
+  const unsigned xv = xlive ? v0 + xc : vdim - 1;  // (a column beyond vdim repeats the last one and is not stored)
   float xr[8], zr[8], gr[16], sr[2];
-  auto fetch_x = [&](int b) __attribute__((always_inline)) {
+  // a block that the call fills: a pointer per row that the wave shares, one offset per lane for the whole kernel
+  const unsigned ld = a.ld, zld = a.z_ld;
+  const unsigned xo = xt * ld + xv, zo = xt * zld + xv;
+  auto rows8 = [&](const float* p, unsigned stride, unsigned off, int b, float* to) __attribute__((always_inline)) {
+    if (EVEN) {
+      const float* q = p + (size_t)b * SSM_Q * stride;
 #pragma unroll
-    for (int i = 0; i < 8; ++i) xr[i] = xlive ? xp[row(b * SSM_Q + i * 8 + xt) * (unsigned)a.ld + xc] : 0.0f;
+      for (int i = 0; i < 8; ++i) to[i] = ssm_at(q + (size_t)(8 * i) * stride, off);
+    } else {
+#pragma unroll
+      for (int i = 0; i < 8; ++i) to[i] = ssm_at(p, row(b * SSM_Q + i * 8 + xt) * stride + xv);
+    }
+  };
+  auto fetch_x = [&](int b) __attribute__((always_inline)) {
+    rows8(xp, ld, xo, b, xr);
     const float* s = stp + (size_t)b * a.heads * SSM_STEP_FLOATS;
-    sr[0] = s[tid];
-    sr[1] = tid < SSM_STEP_FLOATS - 256 ? s[256 + tid] : 0.0f;
+    sr[0] = ssm_at(s, tid);
+    sr[1] = ssm_at(s, 256 + (tid & 63));
   };
   auto fetch_z = [&](int b) __attribute__((always_inline)) {
-    if (!zp) return;
-#pragma unroll
-    for (int i = 0; i < 8; ++i) zr[i] = xlive ? zp[row(b * SSM_Q + i * 8 + xt) * (unsigned)a.z_ld + xc] : 0.0f;
+    if (zp) rows8(zp, zld, zo, b, zr);
   };
   auto fetch_g = [&](int b) __attribute__((always_inline)) {
     const float* gp = a.gram + ((size_t)b * a.groups + g) * SSM_Q * SSM_Q;
 #pragma unroll
-    for (int i = 0; i < 16; ++i) gr[i] = gp[i * 256 + tid];  // (never-written tiles are not used below)
+    for (int i = 0; i < 16; ++i) gr[i] = ssm_at(gp + i * 256, tid);  // (never-written tiles are not used below)
   };
   ssm_f32x4 cr[PF ? 2 : 1][4];
   auto fetch_c = [&](int b, int tt, int k, ssm_f32x4* to) __attribute__((always_inline)) {
-    const float* c = cp + row(b * SSM_Q + tt * 32 + r) * (unsigned)a.ld;
+    const int n0 = 32 * (wave + 4 * k);
+    if (EVEN) {
+      const float* c = cp + (size_t)(b * SSM_Q + tt * 32) * ld + n0;
 #pragma unroll
-    for (int q = 0; q < 4; ++q) to[q] = ssm_ld4(c, 32 * (wave + 4 * k) + 8 * q + 4 * h, N, vec);
+      for (int q = 0; q < 4; ++q) to[q] = ssm_at4(c + 8 * q, r * ld + 4 * h);
+    } else {
+      const float* c = cp + (size_t)row(b * SSM_Q + tt * 32 + r) * ld;
+#pragma unroll
+      for (int q = 0; q < 4; ++q) to[q] = ssm_ld4(c, n0 + 8 * q + 4 * h, N, vec);
+    }
   };
   float br[PF ? 2 : 1][16];
   auto fetch_b = [&](int b, int half, int k, float* to) __attribute__((always_inline)) {
     const int n = 32 * (wave + 4 * k) + r;
-    const float* p = bp + (n < N ? n : N - 1);  // (rows beyond the state meet zeros of C and are not stored)
-    const unsigned t = b * SSM_Q + 32 * half + h;
-    if ((int)(t + 32) <= a.T) {
-      const unsigned o = t * (unsigned)a.ld;
+    const unsigned nn = EVEN || n < N ? n : N - 1;  // (rows beyond the state meet zeros of C and are not stored)
+    if (EVEN) {
+      const float* p = bp + (size_t)(b * SSM_Q + 32 * half) * ld;
 #pragma unroll
-      for (int s = 0; s < 16; ++s) to[s] = p[o + 2 * s * (unsigned)a.ld];
+      for (int s = 0; s < 16; ++s) to[s] = ssm_at(p + (size_t)(2 * s) * ld, h * ld + nn);
     } else {
 #pragma unroll
-      for (int s = 0; s < 16; ++s) to[s] = p[row(t + 2 * s) * (unsigned)a.ld];
+      for (int s = 0; s < 16; ++s) to[s] = ssm_at(bp, row(b * SSM_Q + 32 * half + 2 * s + h) * ld + nn);
     }
   };
   const bool mine = 32 * wave < N;  // this wave holds state rows at all
@@ -187,17 +216,17 @@ __global__ __launch_bounds__(256, NT == 1 ? 2 : 1) void ssm_walk_kernel(const Ss
   }
   fetch_z(0);
   for (int b = 0; b < blocks; ++b) {
-    const int t0 = b * SSM_Q, nt = a.T - t0 < SSM_Q ? a.T - t0 : SSM_Q;
-    const bool two = nt > 32;  // tokens in the second half of the block
-    const bool more = b + 1 < blocks;
+    const int nb = b + 1 < blocks ? b + 1 : b;  // (after the last block its own values are read once more: no branch)
+    const int t0 = b * SSM_Q, nt = EVEN || a.T - t0 > SSM_Q ? SSM_Q : a.T - t0;
+    const bool two = EVEN || nt > 32;  // tokens in the second half of the block
     SsmSteps& st = L.st[b & 1];
     float (*x)[SSM_LD] = L.x[b & 1];
 #pragma unroll
-    for (int i = 0; i < 8; ++i) x[i * 8 + xt][xc] = t0 + i * 8 + xt < a.T ? xr[i] : 0.0f;
+    for (int i = 0; i < 8; ++i) x[i * 8 + xt][xc] = EVEN || t0 + i * 8 + xt < a.T ? xr[i] : 0.0f;
     reinterpret_cast<float*>(&st)[tid] = sr[0];
-    if (tid < SSM_STEP_FLOATS - 256) reinterpret_cast<float*>(&st)[256 + tid] = sr[1];
+    reinterpret_cast<float*>(&st)[256 + (tid & 63)] = sr[1];  // (four writers of one value)
     __syncthreads();  // x and the steps of the block are in LDS
-    if (more) fetch_x(b + 1);
+    fetch_x(nb);
     // C S over this wave's state rows
     ssm_f32x16 acc[2];
 #pragma unroll
@@ -213,10 +242,8 @@ __global__ __launch_bounds__(256, NT == 1 ? 2 : 1) void ssm_walk_kernel(const Ss
 #pragma unroll
             for (int tt = 0; tt < 2; ++tt)
               acc[tt] = __builtin_amdgcn_mfma_f32_32x32x2f32(cr[PF ? tt : 0][q][c], S[0][4 * q + c], acc[tt], 0, 0, 0);
-        if (more) {
 #pragma unroll
-          for (int tt = 0; tt < 2; ++tt) fetch_c(b + 1, tt, 0, cr[PF ? tt : 0]);
-        }
+        for (int tt = 0; tt < 2; ++tt) fetch_c(nb, tt, 0, cr[PF ? tt : 0]);
       }
     } else {
 #pragma unroll
@@ -241,10 +268,12 @@ __global__ __launch_bounds__(256, NT == 1 ? 2 : 1) void ssm_walk_kernel(const Ss
 #pragma unroll
       for (int i = 0; i < 16; ++i) {
         const int ti = i * 4 + wave;
-        L.p[ti][tj] = tj <= ti && ti < nt ? gr[i] * expf((float)(st.cum[ti] - cj)) * dj : 0.0f;
+        const float d = fminf((float)(st.cum[ti] - cj), 0.0f);
+        const float v = gr[i] * __expf(d) * dj;  // (hardware exp2: its error is 1e-7 of the largest weight, 1)
+        L.p[ti][tj] = tj <= ti && ti < nt ? v : 0.0f;
       }
     }
-    if (more) fetch_g(b + 1);
+    fetch_g(nb);
 #pragma unroll
     for (int tt = 0; tt < 2; ++tt)
 #pragma unroll
@@ -276,12 +305,12 @@ __global__ __launch_bounds__(256, NT == 1 ? 2 : 1) void ssm_walk_kernel(const Ss
         if (half == 1 && !two) continue;
         float* bv = br[PF ? half : 0];
         if (!PF) fetch_b(b, half, k, bv);
+        float xw[16];
 #pragma unroll
-        for (int s = 0; s < 16; ++s) {
-          const int j = 32 * half + 2 * s + h;
-          S[k] = __builtin_amdgcn_mfma_f32_32x32x2f32(bv[s], st.w[j] * x[j][r], S[k], 0, 0, 0);
-        }
-        if (PF && more) fetch_b(b + 1, half, 0, bv);
+        for (int s = 0; s < 16; ++s) xw[s] = st.w[32 * half + 2 * s + h] * x[32 * half + 2 * s + h][r];
+#pragma unroll
+        for (int s = 0; s < 16; ++s) S[k] = __builtin_amdgcn_mfma_f32_32x32x2f32(bv[s], xw[s], S[k], 0, 0, 0);
+        if (PF) fetch_b(nb, half, 0, bv);
       }
     }
 #pragma unroll
@@ -289,15 +318,26 @@ __global__ __launch_bounds__(256, NT == 1 ? 2 : 1) void ssm_walk_kernel(const Ss
 #pragma unroll
       for (int e = 0; e < 16; ++e) L.part[wave][tt * 32 + ssm_row(e, h)][r] = acc[tt][e];
     __syncthreads();  // the partial Y are whole
+    float y[8];
 #pragma unroll
     for (int i = 0; i < 8; ++i) {
       const int t = i * 8 + xt;
-      if (t >= nt || !xlive) continue;
-      float y = ((L.part[0][t][xc] + L.part[1][t][xc]) + (L.part[2][t][xc] + L.part[3][t][xc])) + dskip * x[t][xc];
-      if (zp) y *= ssm_silu(zr[i]);
-      a.y[(size_t)(t0 + t) * inner + (size_t)head * vdim + v0 + xc] = y;
+      y[i] = ((L.part[0][t][xc] + L.part[1][t][xc]) + (L.part[2][t][xc] + L.part[3][t][xc])) + dskip * x[t][xc];
     }
-    if (more) fetch_z(b + 1);
+    if (zp) {
+#pragma unroll
+      for (int i = 0; i < 8; ++i) y[i] *= ssm_silu_fast(zr[i]);
+    }
+    float* yp = a.y + (size_t)t0 * inner + (size_t)head * vdim + v0;
+    if (EVEN) {
+#pragma unroll
+      for (int i = 0; i < 8; ++i) yp[(size_t)(8 * i + xt) * inner + xc] = y[i];
+    } else {
+#pragma unroll
+      for (int i = 0; i < 8; ++i)
+        if (i * 8 + xt < nt && xlive) yp[(size_t)(8 * i + xt) * inner + xc] = y[i];
+    }
+    fetch_z(nb);
   }
 #pragma unroll
   for (int k = 0; k < NT; ++k)
@@ -427,11 +467,12 @@ __global__ __launch_bounds__(256) void part_norm_kernel(const PartNormArgs a) {
   for (int c = tid; c < n; c += 256) x[c] = x[c] * inv * w[c];
 }
 
-template <int NT>
+template <int NT, bool EVEN>
 int launch_walk(const SsmScanArgs& a, int vec, hipStream_t s) {
   static TlDeviceOnce lds_raised;  // per instantiation, per device
-  TL_TRY(tl_raise_lds_limit(ssm_walk_kernel<NT>, 160 * 1024, lds_raised));
-  ssm_walk_kernel<NT><<<dim3((a.vdim + 31) / 32, a.heads), 256, sizeof(SsmLds), s>>>(a, vec);
+  auto kernel = ssm_walk_kernel<NT, EVEN>;
+  TL_TRY(tl_raise_lds_limit(kernel, 160 * 1024, lds_raised));
+  kernel<<<dim3((a.vdim + 31) / 32, a.heads), 256, sizeof(SsmLds), s>>>(a, vec);
   TL_HIP(hipGetLastError());
   return 0;
 }
@@ -453,11 +494,24 @@ int tl_launch_ssm_scan(const SsmScanArgs& a, hipStream_t s) {
   const int vec = (a.state_n & 3) == 0 && (a.ld & 3) == 0 && ((a.heads * a.vdim) & 3) == 0 && ((size_t)a.xbc & 15) == 0;
   TL_REQUIRE(a.T < (1 << 30) / (a.ld > a.z_ld ? a.ld : a.z_ld), "ssm_scan: %d tokens in rows of %d / %d", a.T, a.ld, a.z_ld);
   TL_REQUIRE(((size_t)a.gram & 7) == 0, "ssm_scan: scratch not aligned");
+  const bool even = vec && (a.state_n & 31) == 0 && (a.vdim & 31) == 0;
+  if (even && a.T > SSM_Q && a.T % SSM_Q) {  // whole blocks on the even kernel, the rest as a call of its own
+    SsmScanArgs w = a, rest = a;
+    w.T = a.T - a.T % SSM_Q;
+    rest.T = a.T - w.T;
+    rest.xbc += (size_t)w.T * a.ld;
+    rest.dt_raw += (size_t)w.T * a.dt_ld;
+    if (a.z) rest.z += (size_t)w.T * a.z_ld;
+    rest.y += (size_t)w.T * a.heads * a.vdim;
+    TL_TRY(tl_launch_ssm_scan(w, s));
+    return tl_launch_ssm_scan(rest, s);
+  }
   ssm_gram_kernel<<<dim3((a.T + SSM_Q - 1) / SSM_Q, a.groups + (a.heads + 2) / 3), 192, 0, s>>>(a, vec);
+  const bool fast = even && a.T % SSM_Q == 0;
   const int nt = (a.state_n + 127) / 128;
-  if (nt <= 1) return launch_walk<1>(a, vec, s);
-  if (nt <= 2) return launch_walk<2>(a, vec, s);
-  return launch_walk<4>(a, vec, s);
+  if (nt <= 1) return fast ? launch_walk<1, true>(a, vec, s) : launch_walk<1, false>(a, vec, s);
+  if (nt <= 2) return fast ? launch_walk<2, true>(a, vec, s) : launch_walk<2, false>(a, vec, s);
+  return fast ? launch_walk<4, true>(a, vec, s) : launch_walk<4, false>(a, vec, s);
 }
 
 int tl_launch_ssm_step(const SsmStepArgs& a, hipStream_t s) {
