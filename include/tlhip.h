@@ -490,7 +490,8 @@ int tl_moe_route_sigmoid_groups(const float* x_dev, int num_tokens, int width, c
 /* softmax window attention with the score options of TL_MIXER_SWA: heads of a query / key row q_hstride / k_hstride floats
  * apart (0: dim), rows ldq / k_ld / v_ld apart (0: packed); score = (q . k) scale, capped by softcap tanh(. / softcap) when
  * softcap > 0, minus r1[head] ln(1 + r2[head] (i - j)) when r1_dev is set; sink != 0: exp(sink_dev[head]) (exp(0) without
- * sink_dev) joins the denominator */
+ * sink_dev) joins the denominator. One key/value head whose rows are the values as well (v_cache_dev == k_cache_dev, k_ld == v_ld),
+ * at least 8 query heads and at most 4 tokens, no option: the heads' products over a tile of rows run together */
 int tl_window_attention_opts(const float* q_dev, int ldq, int q_hstride, const float* k_cache_dev, int k_ld, int k_hstride,
                              const float* v_cache_dev, int v_ld, float* out_dev, int num_tokens, int start_pos, int heads,
                              int kv_heads, int dim, int vdim, int window, float scale, float softcap, const float* r1_dev,

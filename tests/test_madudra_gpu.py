@@ -431,13 +431,14 @@ def test_far_keys_and_window_edges_decide_the_logits(env, expand):
     m.free()
 
 
-def test_one_key_just_inside_and_just_outside_the_window(env):
+@pytest.mark.parametrize("heads", [3, 11])
+def test_one_key_just_inside_and_just_outside_the_window(env, heads):
     """Attention over latent rows (one key/value head, keys the whole row, values its first columns): one row with a score far
     above the rest is copied by positions up to window - 1 behind it and not seen one further, in a prompt and for single
     tokens, with the row at the edges of the kernels' 32- and 64-key pieces. Rows outside the window hold NaN."""
     capi, orc = env["capi"], env["oracle"]
     rng = np.random.default_rng(3)
-    heads, rank, rd, P = 3, 16, 8, 420
+    rank, rd, P = 16, 8, 420
     dim = rank + rd
     for window in (5, 40, 64, 65, 129):
         for star in (0, 31, 63, 64, 200):
@@ -458,6 +459,35 @@ def test_one_key_just_inside_and_just_outside_the_window(env):
                 call(env, "tl_window_attention_opts", qd.ptr, heads * dim, 0, kd.ptr, dim, 0, kd.ptr, dim, od.ptr, T, start, heads, 1, dim,
                      rank, window, 1.0, 0.0, None, None, 0, None)
                 assert np.allclose(od.to_numpy(np.float32, (T, heads, rank)), want[start:start + T], rtol=1e-5, atol=1e-5), (window, star)
+
+
+@pytest.mark.parametrize("heads,rank,rd,window", [(32, 512, 64, 300), (8, 16, 8, 0), (40, 128, 40, 65), (70, 260, 4, 1), (9, 64, 700 - 64, 33),
+                                                  (16, 40, 20, 1000)])
+def test_latent_rows_shared_by_many_heads(env, heads, rank, rd, window):
+    """Single tokens and portions of up to four over one row of keys and values for all heads, near the start and far into a
+    cache: fewer tiles than splits, splits of several tiles, head tiles that are not full. Rows that a position may not see are
+    NaN; one far row dominates for some heads."""
+    orc = env["oracle"]
+    rng = np.random.default_rng(heads + rank)
+    dim, P = rank + rd, 2700
+    rows = rng.standard_normal((P, dim)).astype(np.float32)
+    scale = 2.0 / math.sqrt(dim)
+    for start, T in ((0, 1), (1, 1), (31, 2), (32, 1), (63, 4), (600, 3), (P - 1, 1)):
+        q = rng.standard_normal((T, heads, dim)).astype(np.float32)
+        kc = rows.copy()
+        far = max(0, start - (window or P) + T) if window != 1 else start
+        q[:, ::3] = (10.0 * rows[far])[None, None] / np.linalg.norm(rows[far])
+        kc[start + T:] = np.nan
+        if window > 0:
+            kc[:max(0, start - window + 1)] = np.nan
+        qd, kd = dev(env, q), dev(env, kc)
+        od = env["engine"].DeviceBuffer(4 * T * heads * rank)
+        call(env, "tl_window_attention_opts", qd.ptr, heads * dim, 0, kd.ptr, dim, 0, kd.ptr, dim, od.ptr, T, start, heads, 1, dim, rank,
+             window, scale, 0.0, None, None, 0, None)
+        want = orc.softmax_attention(q.astype(np.float64), np.broadcast_to(rows[:, None], (P, heads, dim)).astype(np.float64),
+                                     np.broadcast_to(rows[:, None, :rank], (P, heads, rank)).astype(np.float64), scale,
+                                     np.arange(start, start + T), window)
+        assert np.allclose(od.to_numpy(np.float32, (T, heads, rank)), want, rtol=3e-5, atol=3e-6), (start, T)
 
 
 def test_first_tokens_of_a_sequence(env):

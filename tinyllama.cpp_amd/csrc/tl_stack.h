@@ -112,9 +112,13 @@ struct SwaArgs {
   const float* dist_r1;     // optional [heads] (with dist_r2): score <- score - r1 ln(1 + r2 (i - j)), after the cap
   const float* dist_r2;
   const float* sink_val;    // with sink: the sink's score per head (NULL: 0)
+  // 1: every query head reads the same key rows, which are the values as well (kv_heads == 1, vc == kc, plain softmax, few
+  // tokens): the heads' products over a tile of rows run together. nsplit = tl_swa_shared_splits (> 0), ws set
+  int shared;
 };
 int tl_launch_swa(const SwaArgs& a, hipStream_t s);
 int tl_swa_splits(int T, int window, int max_pos, int keep_first = 0);  // splits worth having for T tokens over a cache of max_pos rows
+int tl_swa_shared_splits(const SwaArgs& a, int max_pos);
 size_t tl_swa_ws_floats(int T, int heads, int vdim, int nsplit);
 
 // ---- tl_norm.hip -------------------------------------------------------------------------------------------------------

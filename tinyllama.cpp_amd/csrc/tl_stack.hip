@@ -1057,8 +1057,9 @@ int tl_stack_finalize(TlStack* st, hipStream_t s) {
         const Layer& L = *Lp;
         if (L.sp.mixer != TL_MIXER_SWA && L.sp.mixer != TL_MIXER_LATENT) continue;
         const bool lat = L.sp.mixer == TL_MIXER_LATENT;
-        const size_t n = tl_swa_ws_floats(T, L.sp.heads, lat ? L.sp.kv_rank : L.sp.vdim,
-                                          tl_swa_splits(T, L.sp.window, st->cfg.max_positions, lat ? 0 : L.sp.keep_first));
+        const int splits = tl_swa_splits(T, L.sp.window, st->cfg.max_positions, lat ? 0 : L.sp.keep_first);
+        // (latent rows: the shared-row kernel may cut finer, up to 64)
+        const size_t n = tl_swa_ws_floats(T, L.sp.heads, lat ? L.sp.kv_rank : L.sp.vdim, lat ? 64 : splits);
         ws = n > ws ? n : ws;
       }
     TL_TRY(dev_alloc(st, &st->swa_ws, ws));
@@ -1746,7 +1747,9 @@ int latent_mixer(TlStack* st, Layer& L, const float* in, int T, int start_pos, c
   a.scale = sp.scale;
   a.start_pos = start_pos;
   a.pos_dev = pos_dev;
-  a.nsplit = tl_swa_splits(T, sp.window, c.max_positions, 0);
+  a.nsplit = tl_swa_shared_splits(a, c.max_positions);
+  a.shared = a.nsplit > 0;
+  if (!a.shared) a.nsplit = tl_swa_splits(T, sp.window, c.max_positions, 0);
   a.ws = st->swa_ws;
   a.done_cnt = st->swa_cnt;
   TL_TRY(tl_launch_swa(a, s));

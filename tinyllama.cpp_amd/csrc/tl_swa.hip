@@ -256,6 +256,196 @@ __global__ __launch_bounds__(256) void swa_kernel(const SwaArgs a) {
 
 __global__ __launch_bounds__(64) void swa_combine_kernel(const SwaArgs a) { swa_merge_records(a, blockIdx.x, blockIdx.y, threadIdx.x); }
 
+// ---- few tokens, many query heads over ONE head of keys whose rows are the values as well (a latent cache) ------------------
+// All heads read the same rows, so a workgroup takes a tile of 32 keys for 32 heads at once: the rows go into LDS once, and both
+// products run on the FP32 matrix instruction.
+//   S^T[key][head]: the key size is dealt to the eight waves (a lane's query piece stays in registers), the partial sums meet
+//   in LDS; softmax with 16 lanes per head; O[head][column] += P V with the value columns dealt to the waves, V read from the
+//   rows that are in LDS already. A workgroup walks the tiles of its split with a running maximum and leaves a record as
+//   swa_kernel does; swa_shared_combine_kernel merges the records, 64 columns of a head per workgroup.
+typedef float swa_f32x4 __attribute__((ext_vector_type(4)));
+typedef float swa_f32x16 __attribute__((ext_vector_type(16)));
+constexpr int SH_WAVES = 8, SH_LD = 36;
+constexpr int SH_MAX_K = 12;  // 64-value pieces of a key row: dim <= 768
+__host__ __device__ inline int swa_shared_dp(int dim) { return (dim + 63) & ~63; }
+__host__ __device__ inline size_t swa_shared_lds_floats(int dim) {
+  return (size_t)32 * (swa_shared_dp(dim) + 4) + (SH_WAVES + 1) * 32 * SH_LD + 32;
+}
+
+template <int NC>  // 32-column pieces of a value row per wave: vdim <= 256 NC
+__global__ __launch_bounds__(512) void swa_shared_kernel(const SwaArgs a) {
+  extern __shared__ __attribute__((aligned(16))) float lds[];
+  const int dp = swa_shared_dp(a.dim), ts = dp + 4, kw = dp / SH_WAVES, ki = dp / 64;
+  float* tile = lds;                              // [32 keys][dp + 4]
+  float* part = tile + 32 * ts;                   // [waves][32 keys][SH_LD heads]
+  float* ps = part + SH_WAVES * 32 * SH_LD;       // [32 heads][SH_LD keys]
+  float* sm_c = ps + 32 * SH_LD;                  // [32] a head's factor on what it has summed so far
+  const int tid = threadIdx.x, lane = tid & 63, r = lane & 31, h = lane >> 5;
+  const int wave = __builtin_amdgcn_readfirstlane(tid >> 6);
+  const int t = blockIdx.x, h0 = blockIdx.y * 32;
+  const int i = (a.pos_dev ? *a.pos_dev : a.start_pos) + t;
+  const int jlo = (a.window > 0 && i - a.window + 1 > 0) ? i - a.window + 1 : 0;
+  const int tiles = (i - jlo + 32) >> 5, per = (tiles + a.nsplit - 1) / a.nsplit;
+  const int c_lo = blockIdx.z * per, c_hi = c_lo + per < tiles ? c_lo + per : tiles;
+  const int my_head = tid >> 4, my_key = tid & 15;  // softmax: 16 lanes per head, keys my_key and my_key + 16
+  float m = -INFINITY, l = 0.0f;
+  swa_f32x16 o[NC];
+#pragma unroll
+  for (int n = 0; n < NC; ++n)
+#pragma unroll
+    for (int e = 0; e < 16; ++e) o[n][e] = 0.0f;
+  swa_f32x4 q[SH_MAX_K];
+  if (c_lo < c_hi) {
+    const bool live = h0 + r < a.heads;
+    const float* qp = a.q + (size_t)t * a.ldq + (size_t)(live ? h0 + r : h0) * a.dim;
+#pragma unroll
+    for (int u = 0; u < SH_MAX_K; ++u)
+      if (u < ki) {
+        const int d = wave * kw + 8 * u + 4 * h;
+        q[u] = live && d < a.dim ? *reinterpret_cast<const swa_f32x4*>(qp + d) : swa_f32x4{0.0f, 0.0f, 0.0f, 0.0f};
+      }
+  }
+  for (int c = c_lo; c < c_hi; ++c) {
+    const int j0 = jlo + c * 32;
+    {  // four rows a wave, all their 16-byte pieces in flight
+      swa_f32x4 v[4][3];
+#pragma unroll
+      for (int u = 0; u < 4; ++u) {
+        const int j = j0 + wave + SH_WAVES * u < i ? j0 + wave + SH_WAVES * u : i;  // (beyond the last key: its row again, weight 0)
+        const float* kp = a.kc + (size_t)j * a.kld;
+#pragma unroll
+        for (int w = 0; w < 3; ++w) {
+          const int d = 4 * lane + 256 * w;
+          v[u][w] = d < a.dim ? *reinterpret_cast<const swa_f32x4*>(kp + d) : swa_f32x4{0.0f, 0.0f, 0.0f, 0.0f};
+        }
+      }
+#pragma unroll
+      for (int u = 0; u < 4; ++u)
+#pragma unroll
+        for (int w = 0; w < 3; ++w)
+          if (4 * lane + 256 * w < dp) *reinterpret_cast<swa_f32x4*>(tile + (wave + SH_WAVES * u) * ts + 4 * lane + 256 * w) = v[u][w];
+    }
+    __syncthreads();
+    swa_f32x16 s;
+#pragma unroll
+    for (int e = 0; e < 16; ++e) s[e] = 0.0f;
+#pragma unroll
+    for (int u = 0; u < SH_MAX_K; ++u)
+      if (u < ki) {
+        const swa_f32x4 kv = *reinterpret_cast<const swa_f32x4*>(tile + r * ts + wave * kw + 8 * u + 4 * h);
+#pragma unroll
+        for (int d = 0; d < 4; ++d) s = __builtin_amdgcn_mfma_f32_32x32x2f32(kv[d], q[u][d], s, 0, 0, 0);
+      }
+#pragma unroll
+    for (int e = 0; e < 16; ++e) part[(wave * 32 + (e & 3) + 8 * (e >> 2) + 4 * h) * SH_LD + r] = s[e];
+    __syncthreads();
+    {
+      float sc[2];
+#pragma unroll
+      for (int u = 0; u < 2; ++u) {
+        float acc = 0.0f;
+#pragma unroll
+        for (int w = 0; w < SH_WAVES; ++w) acc += part[(w * 32 + my_key + 16 * u) * SH_LD + my_head];
+        sc[u] = j0 + my_key + 16 * u <= i ? acc * a.scale : -INFINITY;
+      }
+      float cm = fmaxf(sc[0], sc[1]);
+#pragma unroll
+      for (int w = 8; w >= 1; w >>= 1) cm = fmaxf(cm, __shfl_xor(cm, w));
+      const float mn = fmaxf(m, cm);  // finite: a tile's first key is visible
+      const float corr = expf(m - mn), p0 = expf(sc[0] - mn), p1 = expf(sc[1] - mn);
+      float sum = p0 + p1;
+#pragma unroll
+      for (int w = 8; w >= 1; w >>= 1) sum += __shfl_xor(sum, w);
+      l = l * corr + sum;
+      m = mn;
+      ps[my_head * SH_LD + my_key] = p0;
+      ps[my_head * SH_LD + my_key + 16] = p1;
+      if (my_key == 0) sm_c[my_head] = corr;
+    }
+    __syncthreads();
+    if (c > c_lo) {
+#pragma unroll
+      for (int e = 0; e < 16; ++e) {
+        const float f = sm_c[(e & 3) + 8 * (e >> 2) + 4 * h];
+#pragma unroll
+        for (int n = 0; n < NC; ++n) o[n][e] *= f;
+      }
+    }
+#pragma unroll
+    for (int u = 0; u < 4; ++u) {
+      const swa_f32x4 pv = *reinterpret_cast<const swa_f32x4*>(ps + r * SH_LD + 8 * u + 4 * h);
+#pragma unroll
+      for (int n = 0; n < NC; ++n) {
+        const int col = (wave * NC + n) * 32;
+        if (col >= a.vdim) continue;
+#pragma unroll
+        for (int d = 0; d < 4; ++d)  // (columns beyond vdim are the row's other columns, or zeros: not stored)
+          o[n] = __builtin_amdgcn_mfma_f32_32x32x2f32(pv[d], tile[(8 * u + 4 * h + d) * ts + col + r], o[n], 0, 0, 0);
+      }
+    }
+    __syncthreads();  // the tile may be overwritten
+  }
+  const int rs = a.vdim + 2;
+  float* rec = a.ws + ((size_t)t * a.heads * a.nsplit + blockIdx.z) * rs;  // + head * nsplit * rs
+  if (my_key == 0 && h0 + my_head < a.heads) {  // (a split without a tile leaves -inf and 0; its values are not read)
+    rec[(size_t)(h0 + my_head) * a.nsplit * rs] = m;
+    rec[(size_t)(h0 + my_head) * a.nsplit * rs + 1] = l;
+  }
+  if (c_lo >= c_hi) return;
+#pragma unroll
+  for (int n = 0; n < NC; ++n) {
+    const int col = (wave * NC + n) * 32 + r;
+#pragma unroll
+    for (int e = 0; e < 16; ++e) {
+      const int head = h0 + (e & 3) + 8 * (e >> 2) + 4 * h;
+      if (col < a.vdim && head < a.heads) rec[(size_t)head * a.nsplit * rs + 2 + col] = o[n][e];
+    }
+  }
+}
+
+// grid (T * heads, vdim in 64s), 4 waves: each sums every fourth record
+__global__ __launch_bounds__(256) void swa_shared_combine_kernel(const SwaArgs a) {
+  __shared__ float sum[4][64];
+  const int lane = threadIdx.x & 63, wave = threadIdx.x >> 6, d = blockIdx.y * 64 + lane, rs = a.vdim + 2;
+  const float* rec = a.ws + (size_t)blockIdx.x * a.nsplit * rs;
+  const float mz = lane < a.nsplit ? rec[(size_t)lane * rs] : -INFINITY;
+  const float lz = lane < a.nsplit ? rec[(size_t)lane * rs + 1] : 0.0f;
+  float M = mz;
+#pragma unroll
+  for (int o = 32; o >= 1; o >>= 1) M = fmaxf(M, __shfl_xor(M, o));
+  const float fz = mz == -INFINITY ? 0.0f : expf(mz - M);
+  float L = lz * fz;
+#pragma unroll
+  for (int o = 32; o >= 1; o >>= 1) L += __shfl_xor(L, o);
+  float acc = 0.0f;
+  for (int z0 = wave; z0 < a.nsplit; z0 += 32) {  // eight records' values in flight together
+    float v[8];
+#pragma unroll
+    for (int u = 0; u < 8; ++u) {
+      const int z = z0 + 4 * u < a.nsplit ? z0 + 4 * u : z0;
+      v[u] = d < a.vdim ? rec[(size_t)z * rs + 2 + d] : 0.0f;
+    }
+#pragma unroll
+    for (int u = 0; u < 8; ++u) {
+      const float f = __shfl(fz, (z0 + 4 * u) & 63);
+      acc += z0 + 4 * u < a.nsplit && f != 0.0f ? v[u] * f : 0.0f;
+    }
+  }
+  sum[wave][lane] = acc;
+  __syncthreads();
+  if (wave == 0 && d < a.vdim) a.out[(size_t)blockIdx.x * a.vdim + d] = ((sum[0][lane] + sum[1][lane]) + (sum[2][lane] + sum[3][lane])) / L;
+}
+
+template <int NC>
+int launch_swa_shared(const SwaArgs& a, hipStream_t s) {
+  static TlDeviceOnce lds_raised;  // per instantiation, per device
+  TL_TRY(tl_raise_lds_limit(swa_shared_kernel<NC>, 160 * 1024, lds_raised));
+  swa_shared_kernel<NC><<<dim3(a.T, (a.heads + 31) / 32, a.nsplit), 512, sizeof(float) * swa_shared_lds_floats(a.dim), s>>>(a);
+  swa_shared_combine_kernel<<<dim3(a.T * a.heads, (a.vdim + 63) / 64), 256, 0, s>>>(a);
+  TL_HIP(hipGetLastError());
+  return 0;
+}
+
 // ---- prompt chunks on the FP32 matrix instruction (v_mfma_f32_32x32x2_f32: exact FP32 products, FP32 accumulation) --------
 // One workgroup of 4 waves per (32-query tile, head). The key tiles of 32 positions that any query of the tile can see
 // (from the first query's window start to the last query's position) are dealt round-robin to the waves; each wave walks its
@@ -264,9 +454,6 @@ __global__ __launch_bounds__(64) void swa_combine_kernel(const SwaArgs a) { swa_
 //     order of a sum does not matter to the instruction), B = the query tile in LDS, zero-padded to a multiple of 8.
 //   The result has the query on the lane and 16 keys in registers; those registers are the A operand of O += P V as they
 //     stand (the result layout puts the key index where the next product's k index lives); V rows are read 128 B per half wave.
-typedef float swa_f32x4 __attribute__((ext_vector_type(4)));
-typedef float swa_f32x16 __attribute__((ext_vector_type(16)));
-
 // key (row of the 32x32 result) held in accumulator register e of lane half h
 __device__ __forceinline__ int swa_acc_row(int e, int h) { return (e & 3) + 8 * (e >> 2) + 4 * h; }
 
@@ -523,6 +710,23 @@ static bool swa_mfma_wanted(const SwaArgs& a) {
   return on && a.T >= 16 && db <= 4 && sizeof(float) * swa_mfma_lds_floats(a.dim, db) <= 160 * 1024;
 }
 
+// splits of the shared-row kernel for tokens that see at most `window` of max_pos positions; 0: the shapes are not its own
+// (TL_SWA_SHARED=0: never)
+int tl_swa_shared_splits(const SwaArgs& a, int max_pos) {
+  static const bool on = [] {
+    const char* e = getenv("TL_SWA_SHARED");
+    return !e || atoi(e) != 0;
+  }();
+  if (!on || a.T > 4 || a.kv_heads != 1 || a.heads < 8 || a.kc != a.vc || a.kld != a.vld || a.kld <= 0 || a.sigmoid || a.sink ||
+      a.softcap > 0.0f || a.dist_r1 || a.keep_first || a.q_hstride || a.k_hstride || a.vdim > a.dim || a.vdim > 512 ||
+      a.dim > 64 * SH_MAX_K || (a.dim & 3) || (a.kld & 3) || (a.ldq & 3) || ((size_t)a.kc & 15) || ((size_t)a.q & 15) ||
+      sizeof(float) * swa_shared_lds_floats(a.dim) > 160 * 1024)
+    return 0;
+  const int keys = a.window > 0 && a.window < max_pos ? a.window : max_pos;
+  const int tiles = (keys + 31) / 32;
+  return tiles < 64 ? tiles : 64;
+}
+
 int tl_launch_swa(const SwaArgs& a, hipStream_t s) {
   TL_REQUIRE(a.q && a.kc && a.vc && a.out && a.T > 0, "swa: bad arguments");
   TL_REQUIRE(a.heads > 0 && a.kv_heads > 0 && a.heads % a.kv_heads == 0, "swa: %d heads over %d key/value heads", a.heads,
@@ -540,6 +744,10 @@ int tl_launch_swa(const SwaArgs& a, hipStream_t s) {
              "swa: head strides %d / %d below the key size %d", a.q_hstride, a.k_hstride, a.dim);
   TL_REQUIRE((a.kld == 0 || a.kld >= (a.kv_heads - 1) * (a.k_hstride > 0 ? a.k_hstride : a.dim) + a.dim) && (a.vld == 0 || a.vld >= a.kv_heads * a.vdim),
              "swa: cache rows %d / %d shorter than the heads they hold", a.kld, a.vld);
+  if (a.shared) {
+    TL_REQUIRE(a.ws && a.nsplit >= 1 && a.nsplit <= 64 && tl_swa_shared_splits(a, 1) > 0, "swa: not shapes of the shared-row kernel");
+    return a.vdim <= 256 ? launch_swa_shared<1>(a, s) : launch_swa_shared<2>(a, s);
+  }
   if (swa_mfma_wanted(a)) {
     switch ((a.vdim + 31) / 32) {
       case 1: return launch_swa_mfma<1>(a, s);
@@ -688,8 +896,10 @@ extern "C" int tl_window_attention_opts(const float* q_dev, int ldq, int q_hstri
   a.sink = sink;
   a.sink_val = sink_dev;
   a.start_pos = start_pos;
-  a.nsplit = tl_swa_splits(num_tokens, window, start_pos + num_tokens, 0);
-  if (a.nsplit > 1) {
+  a.nsplit = tl_swa_shared_splits(a, start_pos + num_tokens);
+  a.shared = a.nsplit > 0;
+  if (!a.shared) a.nsplit = tl_swa_splits(num_tokens, window, start_pos + num_tokens, 0);
+  if (a.nsplit > 1 || a.shared) {
     void* ws = nullptr;
     TL_TRY(tl_scratch(TL_SCRATCH_ATTN, sizeof(float) * tl_swa_ws_floats(num_tokens, heads, vdim, a.nsplit), &ws));
     a.ws = static_cast<float*>(ws);
