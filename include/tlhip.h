@@ -402,7 +402,8 @@ typedef struct tl_stack_config {
                                all the embedding row at first; sublayer q (1: mixer, 2: feed-forward) reads norm(sum_s in[s] x_s)
                                and, its output being y, x_t <- sum_s mix[s][t] x_s + residual_mult out[t] y (tensors l<i>.hc<q>.in
                                and .out [streams], .mix [streams][streams], from x to). The final norm reads the streams' sum */
-  float residual_mult;      /* != 0 (pre-norm blocks behind a layer norm): factor on what a sublayer adds to the residual */
+  float residual_mult;      /* pre-norm blocks behind a layer norm: factor on what a sublayer adds to the residual (without streams, 0
+                               stands for 1) */
 } tl_stack_config;
 /* the operators such a model is built from, callable on their own (all FP32 in and out, weights bf16 [rows][cols]):
  * Y[T][rows] = X[T][cols] W^T; terms 1 / 3 = MFMA GEMM with bf16-rounded / three-term-split activations, 0 = FP32 GEMV (T = 1) */

@@ -1930,7 +1930,7 @@ int finish_x(TlStack* st, const Addends& add, Layer* next, int which, int T, hip
     r.slots = add.slots;
     r.slot_w = add.slot_w;
     r.top = add.top;
-    r.mult = c.residual_mult != 0.0f ? c.residual_mult : 1.0f;
+    r.mult = c.streams > 0 || c.residual_mult != 0.0f ? c.residual_mult : 1.0f;
     if (Wf) {
       r.mix = Wf->hc_mix[done - 1];
       r.out = Wf->hc_out[done - 1];
