@@ -6,10 +6,11 @@
 //   tl_dense.hip  bf16 weight matrices [rows][cols]: GEMV (one token) and MFMA GEMM (a chunk of tokens, optionally grouped
 //                 by expert with gathered input rows / scattered output rows); FP32 activations and accumulation
 //   tl_swa.hip    sliding-window attention without rotation, key and value sizes independent, over a flat FP32 cache
+//                 (decode over rows that all heads share, keys and values at once: the heads' products run together)
 //   tl_moe.hip    router (top-k, softmax over the chosen logits), grouping plan, clamped gated activation, decode GEMVs
 //   tl_norm.hip   RMS norms with zero-centred weights: embedding gather + norm, whole-projection q/k norm + value mixing +
 //                 cache write, residual += norm(sublayer output), row-gathering norm in front of the head; layer norms of
-//                 pre-norm blocks (residual sum + the norm of the sublayer that follows)
+//                 pre-norm blocks (residual sum + the norm of the sublayer that follows), also over several residual streams
 //   tl_rope.hip   rotary positions, per-head unit norm;  tl_delta.hip  two delta-rule recurrences with their preparation
 //   tl_conv.hip   a short causal convolution over time per channel with its history (sublayer inputs; projected q, k, v)
 //   tl_latent.hip latent attention: norms of the latents, the rotated shared key part, cache rows, output gates
