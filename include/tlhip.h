@@ -254,11 +254,17 @@ enum tl_mixer_kind {
   TL_MIXER_LINEAR = 4,      /* gated linear attention whose forget gate also decides what is written (no keys):
                                q = silu(W_q h), f = l + (1 - l) sigmoid(W_f h + b), S <- diag(f) S + (1 - f) v^T, o = S^T q,
                                RMS norm per head with one plain weight [vdim] */
-  TL_MIXER_SSM = 5          /* selective state space with one decay per head and token (Mamba-2's form): z | x | B | C | dt =
+  TL_MIXER_SSM = 5,         /* selective state space with one decay per head and token (Mamba-2's form): z | x | B | C | dt =
                                W_in h with x [heads][vdim], B and C [kv_heads][dim] (kv_heads = groups of heads that share B
                                and C, dim = state size), dt [heads]; x, B, C through a causal convolution per channel + bias +
                                silu (conv_taps); dt <- softplus(dt + dt_bias); S <- exp(-exp(A_log) dt) S + dt B x^T,
                                y = S^T C + D x; y silu(z), RMS norm in norm_parts equal parts of the row, weights; W_o */
+  TL_MIXER_GLA = 6,         /* gated linear attention with a decay per key channel: q = W_q h dim^-1/2, k = W_k h, v = W_v h,
+                               alpha = sigmoid(W_a2 (W_a1 h) + b)^(1 / decay_tau); S <- diag(alpha) S + k v^T, o = S^T q; RMS norm
+                               per head with one plain weight [vdim], times silu(W_g h); W_o. decay_rank = rows of a1 */
+  TL_MIXER_LIGHTNING = 7    /* linear attention with one constant decay per head (decay): q, k, v = silu(W h),
+                               S <- decay S + k v^T, o = S^T q; the concatenated heads RMS-normed together with a plain weight
+                               [heads * vdim], times sigmoid(W_g h); W_o */
 };
 enum tl_mlp_kind {
   TL_MLP_NONE = 0,
@@ -271,7 +277,9 @@ enum tl_act_kind {
   TL_ACT_XIELU = 1,         /* z > 0: P z^2 + z / 2; z <= 0: Q (e^z - 1 - z) + z / 2, with P = softplus(p), Q = 1/2 + softplus(q)
                                from the two numbers of the tensor mlp.act */
   TL_ACT_TANH = 2,
-  TL_ACT_GELU = 3           /* z Phi(z) = z / 2 (1 + erf(z / sqrt 2)) */
+  TL_ACT_GELU = 3,          /* z Phi(z) = z / 2 (1 + erf(z / sqrt 2)) */
+  TL_ACT_SILU = 4,          /* z sigmoid(z) */
+  TL_ACT_SIGMOID_POWER = 5  /* sigmoid(z)^P, formed as exp(-P softplus(-z)) */
 };
 enum tl_glu_kind {
   TL_GLU_SWISH = 0,         /* g sigmoid(act_alpha g) (u + glu_up_add), g = min(gate, limit), u = clamp(up, -limit, limit) */
@@ -280,7 +288,8 @@ enum tl_glu_kind {
 enum tl_block_kind {
   TL_BLOCK_POST_NORM = 0,   /* x += N1(mixer(x)); x += N2(ff(x)): the sublayers read x, the norm is on their output */
   TL_BLOCK_PARALLEL = 1,    /* h = N1(x); x += mixer(h) + ff(h): one norm, both sublayers read its output */
-  TL_BLOCK_PRE_NORM = 2     /* x += mixer(N1(x)); x += ff(N2(x)): a norm in front of each sublayer */
+  TL_BLOCK_PRE_NORM = 2,    /* x += mixer(N1(x)); x += ff(N2(x)): a norm in front of each sublayer */
+  TL_BLOCK_PARALLEL_NORMS = 3 /* x += mixer(N1(x)) + ff(N2(x)): both sublayers read the same x, each behind its own norm */
 };
 enum tl_norm_kind {
   TL_NORM_RMS_ONE_PLUS = 0, /* y / sqrt(mean(y^2) + eps) * (1 + w) */
@@ -301,6 +310,13 @@ enum tl_qk_norm {
   TL_QK_NORM_HEAD_UNIT = 2, /* per head, after the rotation: x / sqrt(mean(x^2) + eps), no weights */
   TL_QK_NORM_HEAD_RMS = 3   /* per head (and score map): RMS norm over dim with one plain weight [dim] for all heads
                                (mix.q.norm, mix.k.norm) */
+};
+enum tl_rot_scaling {       /* what rot_factor (> 0) does to the rotary frequencies */
+  TL_ROT_BLEND = 0,         /* blending by pair index (rot_factor below) */
+  TL_ROT_LINEAR = 1,        /* every f_i divided by rot_factor */
+  TL_ROT_WAVELENGTH = 2     /* by wavelength l = 2 pi / f: f where l < rot_original / rot_fast, f / rot_factor where
+                               l > rot_original / rot_slow, between the two (1 - s) f / rot_factor + s f with
+                               s = (rot_original / l - rot_slow) / (rot_fast - rot_slow) */
 };
 enum tl_route_kind {
   TL_ROUTE_TOP_LOGITS = 0,  /* the `top` largest logits (+ bias); weights = softmax over the chosen logits */
@@ -356,7 +372,8 @@ typedef struct tl_layer_spec {
                                shared by all heads); rot_dims <= rot_dim of them turn */
   int kv_from;              /* TL_MIXER_LATENT: 1 + index of an EARLIER latent layer (with a projection of its own and the same
                                kv_rank, rot_dim and rotation) whose cached latent and rotated key part this layer reads; 0: its own */
-  int head_gate;            /* TL_MIXER_LATENT: 1: head n's output is multiplied by sigmoid(W_g h)_n (mix.g, one row per head) */
+  int head_gate;            /* TL_MIXER_LATENT, TL_MIXER_SWA: 1: head n's output is multiplied by sigmoid(W_g h)_n (mix.g, one row
+                               per head) */
   float decay_scale;        /* TL_MIXER_GDELTA: decay = exp(-decay_scale * sigmoid(W_w2 tanh(W_w1 h) + w0)); decay_rank = rows of w1 */
   int act;                  /* TL_MLP_UNIT: tl_act_kind. TL_MLP_MOE: TL_ACT_NONE: the experts are gated units (glu); otherwise an
                                expert is W_down act(W_up h) (tensors mlp.e<j>.{up,down}) */
@@ -382,9 +399,16 @@ typedef struct tl_layer_spec {
           weights_of are the layer's). The first mixer's tensors are then l<i>.mix.left.*, the second's l<i>.mix.right.* ---- */
   const struct tl_layer_spec* side;
   float mix_scale, side_scale;
-  int rot_halves;           /* 1: dimension i turns with dimension i + rot_dims / 2 (0: 2i with 2i + 1); TL_MIXER_LATENT */
+  int rot_halves;           /* 1: dimension i turns with dimension i + rot_dims / 2 (0: 2i with 2i + 1); TL_MIXER_LATENT, TL_MIXER_SWA */
   float route_scale;        /* TL_ROUTE_SOFTMAX: factor on the weights */
   int norm_parts;           /* TL_MIXER_SSM: equal parts of the row, each normed by its own root mean square */
+  int rot_scaling;          /* tl_rot_scaling */
+  int chunk;                /* TL_MIXER_SWA: > 0: position i sees j <= i only where floor(i / chunk) == floor(j / chunk), counted from
+                               position 0 of the sequence */
+  float decay_tau;          /* TL_MIXER_GLA */
+  const double* decay;      /* TL_MIXER_LIGHTNING: one factor in [0, 1] per head, read when the model is created */
+  int side_norm;            /* two mixers side by side: 1: each output is RMS-normed over the width with a plain weight of its own
+                               (mix.left.out, mix.right.out) before it is scaled and summed */
 } tl_layer_spec;
 typedef struct tl_stack_config {
   int width, vocab, n_layers;
@@ -404,6 +428,7 @@ typedef struct tl_stack_config {
                                and .out [streams], .mix [streams][streams], from x to). The final norm reads the streams' sum */
   float residual_mult;      /* pre-norm blocks behind a layer norm: factor on what a sublayer adds to the residual (without streams, 0
                                stands for 1) */
+  float logit_scale;        /* != 0: the logits are multiplied by it (in front of the cap) */
 } tl_stack_config;
 /* the operators such a model is built from, callable on their own (all FP32 in and out, weights bf16 [rows][cols]):
  * Y[T][rows] = X[T][cols] W^T; terms 1 / 3 = MFMA GEMM with bf16-rounded / three-term-split activations, 0 = FP32 GEMV (T = 1) */
@@ -540,6 +565,42 @@ int tl_hyper_connect(float* x_dev, const float* y_dev, const float* mix_dev, con
 int tl_rotary_halves(float* x_dev, int num_tokens, int start_pos, int heads, int dim, int rot_dims, float rot_base,
                      float rot_factor, float rot_original, float rot_fast, float rot_slow, void* stream);
 
+/* what precedes the scores of a rotated attention: per head an RMS norm over dim with the plain weight norm_dev [dim] (NULL: none),
+ * then the rotation of tl_rotary_heads / tl_rotary_halves (halves != 0) with frequencies scaled as scaling (tl_rot_scaling) says */
+int tl_rotary_normed(float* x_dev, int num_tokens, int start_pos, int heads, int dim, int rot_dims, float rot_base, int scaling,
+                     float rot_factor, float rot_original, float rot_fast, float rot_slow, int halves, const float* norm_dev,
+                     float eps, void* stream);
+/* tl_swa_attention inside chunks of `chunk` positions (<= 0: every j <= i); gate_dev (optional, rows gate_ld apart): head h's
+ * output is multiplied by sigmoid(gate[t][h]) */
+int tl_chunk_attention(const float* q_dev, const float* k_cache_dev, const float* v_cache_dev, float* out_dev, int num_tokens,
+                       int start_pos, int heads, int kv_heads, int dim, int vdim, int chunk, float scale, const float* gate_dev,
+                       int gate_ld, void* stream);
+/* Y[T][rows] = act(X W^T + bias): bias (optional) on every output feature, act (tl_act_kind) on the features act_from <= r <
+ * act_to. terms as tl_dense_matmul */
+int tl_dense_matmul_bias(const void* w_bf16_dev, int rows, int cols, const float* x_dev, float* y_dev, int num_tokens, int terms,
+                         const float* bias_dev, int act, float act_p, float act_q, int act_from, int act_to, void* stream);
+/* the recurrence of TL_MIXER_GLA: q, k (heads * dim each) and v (heads * vdim) at columns q_off, k_off, v_off of rows ld apart,
+ * alpha [T][heads * dim]; S <- diag(alpha) S + k v^T, o = q_scale S^T q. state_dev [heads][vdim][dim], updated in place */
+int tl_channel_decay_attention(const float* p_dev, int ld, int q_off, int k_off, int v_off, const float* alpha_dev, float q_scale,
+                               float* state_dev, float* o_dev, int num_tokens, int heads, int dim, int vdim, void* stream);
+/* one token of TL_MIXER_GLA between its two products: alpha = sigmoid(W_a2 a1 + a2_bias)^power, the recurrence, RMS norm per head with
+ * norm_dev [vdim], times silu(gate): p_dev holds q | k | v | gate | a1 (heads * dim, heads * dim, heads * vdim, heads * vdim, rank) */
+int tl_channel_decay_step(const float* p_dev, const void* a2_bf16_dev, const float* a2_bias_dev, int rank, float power, float q_scale,
+                          const float* norm_dev, float eps, float* state_dev, float* o_dev, int heads, int dim, int vdim,
+                          void* stream);
+/* the recurrence of TL_MIXER_LIGHTNING: v (heads * vdim) | k | q (heads * dim each) in rows ld apart, log_decay_dev [heads] (double);
+ * several tokens are walked in blocks on the matrix cores. state_dev [heads][dim][vdim], updated in place */
+int tl_constant_decay_attention(const float* vkq_dev, int ld, const double* log_decay_dev, float* state_dev, float* o_dev,
+                                int num_tokens, int heads, int dim, int vdim, void* stream);
+/* rows of x RMS-normed whole with the plain weight [width], times sigmoid(gate) (rows gate_ld apart); in place */
+int tl_gated_row_norm(float* x_dev, const float* weight_dev, const float* gate_dev, int gate_ld, int num_tokens, int width, float eps,
+                      void* stream);
+/* x[t] += a_scale A + b_scale B + c with A = a / rms(a) * a_weight (a_weight NULL: A = a), B likewise; a, b, c may be NULL. Then
+ * h1 = x / rms(x) * weight1 and h2 = x / rms(x) * weight2 (either weight may be NULL). Rows of `width` floats */
+int tl_resid_two_norms(float* x_dev, const float* a_dev, float a_scale, const float* a_weight_dev, const float* b_dev, float b_scale,
+                       const float* b_weight_dev, const float* c_dev, const float* weight1_dev, float* h1_dev,
+                       const float* weight2_dev, float* h2_dev, int num_tokens, int width, float eps, void* stream);
+
 int tl_model_create_stack(const tl_stack_config* cfg, tl_model** out);
 /* tensors by checkpoint name: embed, embed.norm, final.norm, head, l<i>.norm1, l<i>.norm2, l<i>.mix.{q,k,v,o,q.norm,k.norm,vmix,pb},
  * l<i>.mix.{q,k,v}.conv, l<i>.mix.{b,a1,a2,g1,g2,A_log,dt_bias,norm}, l<i>.mlp.router, l<i>.mlp.router.b,
@@ -548,7 +609,8 @@ int tl_model_create_stack(const tl_stack_config* cfg, tl_model** out);
  * l<i>.mix.left.* and l<i>.mix.right.*; latent attention
  * l<i>.mix.{dq,dq.norm,uq,dkv,dkv.norm,uk,uv,g,o}; state space l<i>.mix.{in,conv,conv.b,dt_bias,A_log,D,norm,o};
  * hyper-connections l<i>.hc{1,2}.{in,out,mix}; generalized delta rule l<i>.mix.{r,k,v,g,a,a.b,w1,w2,w0,norm,o}; a Dynamic
- * Tanh norm <n> also has <n>.alpha and <n>.b, a layer norm <n>.b. type: TL_BF16 (matrices and vectors) or TL_F32 (vectors). */
+ * Tanh norm <n> also has <n>.alpha and <n>.b, a layer norm <n>.b; channel-decay linear attention l<i>.mix.{q,k,v,g,a1,a2,a2.b,norm,o},
+ * constant-decay linear attention l<i>.mix.{q,k,v,g,norm,o}; normed pairs l<i>.mix.{left,right}.out. type: TL_BF16 (matrices and vectors) or TL_F32 (vectors). */
 int tl_model_set_tensor_named(tl_model* m, const char* name, int type, const long long* shape, int ndim, const void* host_data);
 /* a prompt, or a portion of one, at positions start_pos..: logits of the token rows listed in rows_host (ascending; NULL: the
  * last token when n_rows == 1, all tokens when n_rows == num_tokens) -> logits_host[n_rows][vocab]. The cache keeps what

@@ -43,14 +43,16 @@ LayerSpec._fields_ = [("mixer", C.c_int), ("heads", C.c_int), ("kv_heads", C.c_i
                 ("glu", C.c_int), ("score_maps", C.c_int), ("diff_init", C.c_float), ("out_gate", C.c_int),
                 ("qkv_bias", C.c_int), ("qkv_conv", C.c_int), ("score_softcap", C.c_float), ("dist_bias", C.c_int),
                 ("decay_per_head", C.c_int), ("side", C.POINTER(LayerSpec)), ("mix_scale", C.c_float),
-                ("side_scale", C.c_float), ("rot_halves", C.c_int), ("route_scale", C.c_float), ("norm_parts", C.c_int)]
+                ("side_scale", C.c_float), ("rot_halves", C.c_int), ("route_scale", C.c_float), ("norm_parts", C.c_int),
+                ("rot_scaling", C.c_int), ("chunk", C.c_int), ("decay_tau", C.c_float), ("decay", C.POINTER(C.c_double)),
+                ("side_norm", C.c_int)]
 
 
 class StackConfig(C.Structure):
     _fields_ = [("width", C.c_int), ("vocab", C.c_int), ("n_layers", C.c_int), ("max_positions", C.c_int),
                 ("norm_eps", C.c_float), ("layers", C.POINTER(LayerSpec)), ("norm", C.c_int), ("embed_norm", C.c_int),
                 ("logit_softcap", C.c_float), ("embed_scale", C.c_float), ("canon_taps", C.c_int), ("streams", C.c_int),
-                ("residual_mult", C.c_float)]
+                ("residual_mult", C.c_float), ("logit_scale", C.c_float)]
 
 
 BF16 = 30
@@ -168,6 +170,18 @@ SIGNATURES = {
     "tl_hyper_connect": [_fp, _fp, _fp, _fp, C.c_float, _fp, _fp, _fp, C.c_float, _fp, _fp, C.c_int, C.c_int, C.c_int, _vp],
     "tl_rotary_halves": [_fp, C.c_int, C.c_int, C.c_int, C.c_int, C.c_int, C.c_float, C.c_float, C.c_float, C.c_float, C.c_float,
                          _vp],
+    "tl_rotary_normed": [_fp, C.c_int, C.c_int, C.c_int, C.c_int, C.c_int, C.c_float, C.c_int, C.c_float, C.c_float, C.c_float,
+                         C.c_float, C.c_int, _fp, C.c_float, _vp],
+    "tl_chunk_attention": [_fp, _fp, _fp, _fp, C.c_int, C.c_int, C.c_int, C.c_int, C.c_int, C.c_int, C.c_int, C.c_float, _fp, C.c_int,
+                           _vp],
+    "tl_dense_matmul_bias": [_vp, C.c_int, C.c_int, _fp, _fp, C.c_int, C.c_int, _fp, C.c_int, C.c_float, C.c_float, C.c_int, C.c_int,
+                             _vp],
+    "tl_channel_decay_attention": [_fp, C.c_int, C.c_int, C.c_int, C.c_int, _fp, C.c_float, _fp, _fp, C.c_int, C.c_int, C.c_int,
+                                   C.c_int, _vp],
+    "tl_channel_decay_step": [_fp, _vp, _fp, C.c_int, C.c_float, C.c_float, _fp, C.c_float, _fp, _fp, C.c_int, C.c_int, C.c_int, _vp],
+    "tl_constant_decay_attention": [_fp, C.c_int, _vp, _fp, _fp, C.c_int, C.c_int, C.c_int, C.c_int, _vp],
+    "tl_gated_row_norm": [_fp, _fp, _fp, C.c_int, C.c_int, C.c_int, C.c_float, _vp],
+    "tl_resid_two_norms": [_fp, _fp, C.c_float, _fp, _fp, C.c_float, _fp, _fp, _fp, _fp, _fp, _fp, C.c_int, C.c_int, C.c_float, _vp],
     "tl_general_delta": [_fp, C.c_int, _fp, _fp, _fp, C.c_float, _fp, _fp, _fp, C.c_int, C.c_int, C.c_int, _vp],
 }
 

@@ -15,6 +15,8 @@
 //                the next token's operands in flight. The three dot products a token needs -- (g s) . k, (g s) . q and k . q,
 //                since o = (g s) . q + u (k . q) -- are reduced together over the sixteen lanes with row-local lane swaps, so a
 //                token costs one reduction latency, not two. A decode step is the same kernel with one token.
+//                With plain_write nothing is removed before the write: linear attention with a decay per key channel. gla_step is
+//                its one-token form with everything between the two products around it (decay projection, head norm, gate).
 //   gated norm   o / rms(o) * w * sigmoid(gate) per head, in front of the output projection.
 //
 // A second recurrence lives here beside it, the generalized delta rule: a decay w and a removal rate a per head and key
@@ -136,6 +138,7 @@ __global__ __launch_bounds__(256) void delta_scan_kernel(const DeltaScanArgs a) 
   const int kvh = h / (a.heads / a.kv_heads);
   const bool live = col < a.vdim;           // lanes of a column beyond vdim compute on zeros and store nothing
   const int d0 = sub * E;
+  const float oscale = a.q_scale != 0.0f ? a.q_scale : 1.0f;
   float* sp = a.state + ((size_t)h * a.vdim + (live ? col : 0)) * a.dim;
   float s[E];
 #pragma unroll
@@ -201,7 +204,7 @@ __global__ __launch_bounds__(256) void delta_scan_kernel(const DeltaScanArgs a) 
       const float u = a.plain_write ? bc * vc : bc * (vc - sk);
 #pragma unroll
       for (int e = 0; e < E; ++e) s[e] += kc[e] * u;
-      if (live && sub == 0) a.o[(size_t)(t0 + tt) * a.heads * a.vdim + (size_t)h * a.vdim + col] = sq + u * kq;
+      if (live && sub == 0) a.o[(size_t)(t0 + tt) * a.heads * a.vdim + (size_t)h * a.vdim + col] = (sq + u * kq) * oscale;
     }
     if (more) stash(b ^ 1);  // the other buffer: its last readers passed the barrier at the end of the stage before
     __syncthreads();
@@ -211,6 +214,101 @@ __global__ __launch_bounds__(256) void delta_scan_kernel(const DeltaScanArgs a) 
     for (int e = 0; e < E; ++e)
       if (d0 + e < a.dim) sp[d0 + e] = s[e];
   }
+}
+
+// grid (heads), 1024 threads: 64 columns of S at a time, sixteen lanes a column (E key channels each, dim <= 16 E). The state is
+// asked for first, the decay of the head's key channels (eight lanes a channel) is formed under its round trip.
+template <int E>
+__global__ __launch_bounds__(1024) void gla_step_kernel(const GlaStepArgs a, int vec) {
+  extern __shared__ __attribute__((aligned(16))) float sl[];  // k | q | alpha (16 E each) | v | o (vdim each) | a1
+  __shared__ float red[16];
+  constexpr int DP = 16 * E, P = E >= 16 ? 1 : 16 / E;  // column passes in flight together
+  float *sk = sl, *sq = sl + DP, *sa = sl + 2 * DP, *sv = sl + 3 * DP, *so = sv + a.vdim, *s1 = so + a.vdim;
+  const int tid = threadIdx.x, sub = tid & 15, cl = tid >> 4, h = blockIdx.x, d0 = sub * E;
+  const int hd = a.heads * a.dim, vd = a.heads * a.vdim;
+  float* S = a.state + (size_t)h * a.vdim * a.dim;
+  float s[P][E];
+  auto load = [&](int col, float* to) __attribute__((always_inline)) {
+    const float* p = S + (size_t)(col < a.vdim ? col : 0) * a.dim + d0;
+    if (vec && E >= 4) {
+#pragma unroll
+      for (int e = 0; e + 4 <= E; e += 4) {
+        const float4 f = *reinterpret_cast<const float4*>(p + e);
+        to[e] = f.x, to[e + (E > 1 ? 1 : 0)] = f.y, to[e + (E > 2 ? 2 : 0)] = f.z, to[e + (E > 3 ? 3 : 0)] = f.w;
+      }
+    } else {
+#pragma unroll
+      for (int e = 0; e < E; ++e) to[e] = d0 + e < a.dim ? p[e] : 0.0f;
+    }
+  };
+#pragma unroll
+  for (int i = 0; i < P; ++i) load(cl + 64 * i, s[i]);
+  for (int i = tid; i < DP; i += 1024) {
+    sk[i] = i < a.dim ? a.p[hd + h * a.dim + i] : 0.0f;
+    sq[i] = i < a.dim ? a.p[h * a.dim + i] : 0.0f;
+  }
+  for (int i = tid; i < a.vdim; i += 1024) sv[i] = a.p[2 * hd + h * a.vdim + i];
+  for (int i = tid; i < a.rank; i += 1024) s1[i] = a.p[2 * hd + 2 * vd + i];
+  __syncthreads();
+  for (int c0 = 0; c0 < DP; c0 += 128) {  // (every lane stays in the loop: the sum below crosses lanes)
+    const int c = c0 + (tid >> 3);
+    float z = 0.0f;
+    if (c < a.dim) {
+      const unsigned short* w = a.a2 + ((size_t)h * a.dim + c) * a.rank;
+      for (int r = tid & 7; r < a.rank; r += 8) z += tl_bf2f(w[r]) * s1[r];
+    }
+    z += __shfl_xor(z, 1);
+    z += __shfl_xor(z, 2);
+    z += __shfl_xor(z, 4);
+    if ((tid & 7) == 0 && c < DP) sa[c] = c < a.dim ? tl_act_apply(TL_ACT_SIGMOID_POWER, z + a.a2_b[h * a.dim + c], a.power, 0.0f) : 0.0f;
+  }
+  __syncthreads();
+  float kc[E], qc[E], ac[E];
+#pragma unroll
+  for (int e = 0; e < E; ++e) kc[e] = sk[d0 + e], qc[e] = sq[d0 + e], ac[e] = sa[d0 + e];
+  for (int b = 0; b < a.vdim; b += 64 * P) {
+    if (b > 0) {
+#pragma unroll
+      for (int i = 0; i < P; ++i) load(b + cl + 64 * i, s[i]);
+    }
+#pragma unroll
+    for (int i = 0; i < P; ++i) {
+      const int col = b + cl + 64 * i;
+      const bool live = col < a.vdim;
+      const float v = live ? sv[col] : 0.0f;
+      float o = 0.0f;
+#pragma unroll
+      for (int e = 0; e < E; ++e) {
+        s[i][e] = ac[e] * s[i][e] + kc[e] * v;
+        o += s[i][e] * qc[e];
+      }
+      o = row16_sum(o);
+      if (!live) continue;
+      if (sub == 0) so[col] = o * a.q_scale;
+      float* p = S + (size_t)col * a.dim + d0;
+      if (vec && E >= 4) {
+#pragma unroll
+        for (int e = 0; e + 4 <= E; e += 4)
+          *reinterpret_cast<float4*>(p + e) = make_float4(s[i][e], s[i][e + (E > 1 ? 1 : 0)], s[i][e + (E > 2 ? 2 : 0)], s[i][e + (E > 3 ? 3 : 0)]);
+      } else {
+#pragma unroll
+        for (int e = 0; e < E; ++e)
+          if (d0 + e < a.dim) p[e] = s[i][e];
+      }
+    }
+  }
+  __syncthreads();
+  float ss = 0.0f;
+  for (int c = tid; c < a.vdim; c += 1024) ss += so[c] * so[c];
+  ss = tl_wave_sum(ss);
+  if ((tid & 63) == 0) red[tid >> 6] = ss;
+  __syncthreads();
+  ss = 0.0f;
+#pragma unroll
+  for (int w = 0; w < 16; ++w) ss += red[w];
+  const float inv = 1.0f / sqrtf(ss / (float)a.vdim + a.eps);
+  const float* gp = a.p + 2 * hd + vd + h * a.vdim;
+  for (int c = tid; c < a.vdim; c += 1024) a.o[h * a.vdim + c] = so[c] * inv * a.norm[c] * (gp[c] * sigmoidf_(gp[c]));
 }
 
 // a wave per (token, head); gate rows gate_ld floats apart; weights of its own for every head or one vector for all
@@ -428,6 +526,25 @@ int tl_launch_delta_scan(const DeltaScanArgs& a, hipStream_t s) {
   return 0;
 }
 
+bool tl_gla_step_fits(int dim, int vdim, int rank) { return dim <= 256 && vdim <= 2048 && rank <= 4096; }
+
+int tl_launch_gla_step(const GlaStepArgs& a, hipStream_t s) {
+  TL_REQUIRE(a.p && a.a2 && a.a2_b && a.norm && a.state && a.o && a.rank > 0 && a.heads > 0 && a.dim > 0 && a.vdim > 0, "gla_step: bad arguments");
+  TL_REQUIRE(tl_gla_step_fits(a.dim, a.vdim, a.rank), "gla_step: sizes %d / %d, inner size %d", a.dim, a.vdim, a.rank);
+  const int e = (a.dim + 15) / 16, ep = e <= 1 ? 1 : e <= 2 ? 2 : e <= 4 ? 4 : e <= 8 ? 8 : 16;
+  const int vec = a.dim == 16 * ep && ((size_t)a.state & 15) == 0;
+  const size_t lds = sizeof(float) * (3 * 16 * (size_t)ep + 2 * (size_t)a.vdim + a.rank);
+  switch (ep) {
+    case 1: gla_step_kernel<1><<<a.heads, 1024, lds, s>>>(a, vec); break;
+    case 2: gla_step_kernel<2><<<a.heads, 1024, lds, s>>>(a, vec); break;
+    case 4: gla_step_kernel<4><<<a.heads, 1024, lds, s>>>(a, vec); break;
+    case 8: gla_step_kernel<8><<<a.heads, 1024, lds, s>>>(a, vec); break;
+    default: gla_step_kernel<16><<<a.heads, 1024, lds, s>>>(a, vec); break;
+  }
+  TL_HIP(hipGetLastError());
+  return 0;
+}
+
 int tl_launch_gated_head_norm_rows(float* o, const float* gate, int gate_ld, const float* w, int w_per_head, int T, int heads,
                                    int vdim, float eps, hipStream_t s) {
   TL_REQUIRE(o && gate && w, "gated_head_norm: bad arguments");
@@ -636,4 +753,49 @@ extern "C" int tl_gated_linear_attention(const float* p_dev, int ld, const float
   d.vdim = vdim;
   d.plain_write = 1;
   return tl_launch_delta_scan(d, s);
+}
+
+extern "C" int tl_channel_decay_attention(const float* p_dev, int ld, int q_off, int k_off, int v_off, const float* alpha_dev,
+                                          float q_scale, float* state_dev, float* o_dev, int num_tokens, int heads, int dim, int vdim,
+                                          void* stream) {
+  TL_REQUIRE(p_dev && q_off >= 0 && k_off >= 0 && v_off >= 0 && q_off + heads * dim <= ld && k_off + heads * dim <= ld &&
+                 v_off + heads * vdim <= ld,
+             "tl_channel_decay_attention: columns outside rows of %d", ld);
+  DeltaScanArgs d = {};
+  d.q = p_dev + q_off;
+  d.k = p_dev + k_off;
+  d.ldq = ld;
+  d.v = p_dev + v_off;
+  d.ldv = ld;
+  d.g = alpha_dev;
+  d.state = state_dev;
+  d.o = o_dev;
+  d.T = num_tokens;
+  d.heads = heads;
+  d.kv_heads = heads;
+  d.dim = dim;
+  d.vdim = vdim;
+  d.plain_write = 1;
+  d.q_scale = q_scale;
+  return tl_launch_delta_scan(d, static_cast<hipStream_t>(stream));
+}
+
+extern "C" int tl_channel_decay_step(const float* p_dev, const void* a2_bf16_dev, const float* a2_bias_dev, int rank, float power,
+                                     float q_scale, const float* norm_dev, float eps, float* state_dev, float* o_dev, int heads, int dim,
+                                     int vdim, void* stream) {
+  GlaStepArgs a = {};
+  a.p = p_dev;
+  a.a2 = static_cast<const uint16_t*>(a2_bf16_dev);
+  a.a2_b = a2_bias_dev;
+  a.rank = rank;
+  a.power = power;
+  a.q_scale = q_scale;
+  a.norm = norm_dev;
+  a.eps = eps;
+  a.state = state_dev;
+  a.o = o_dev;
+  a.heads = heads;
+  a.dim = dim;
+  a.vdim = vdim;
+  return tl_launch_gla_step(a, static_cast<hipStream_t>(stream));
 }

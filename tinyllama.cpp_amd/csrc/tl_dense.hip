@@ -166,6 +166,7 @@ __global__ __launch_bounds__(256) void dense_gemm_kernel(const DenseArgs a) {
   }
   // C layout: lane holds token (lane & 31) of a 32 x 32 product, features (e / 4) * 8 + (lane >> 5) * 4 + (e & 3)
   const bool v4 = (a.ldy & 3) == 0 && ((size_t)Y & 15) == 0;
+  const int act_to = a.act_to > 0 ? a.act_to : a.rows;
 #pragma unroll
   for (int j = 0; j < WN; ++j) {
     const int it = t0 + (wn * WN + j) * 32 + (lane & 31);
@@ -184,6 +185,11 @@ __global__ __launch_bounds__(256) void dense_gemm_kernel(const DenseArgs a) {
               yr[(f >> 1) + e] = tl_glu_apply(a.glu_kind, acc[i][j][gq * 4 + 2 * e], acc[i][j][gq * 4 + 2 * e + 1], a.glu_limit, a.glu_alpha, a.glu_up_add);
           continue;
         }
+        if (a.bias) {
+#pragma unroll
+          for (int e = 0; e < 4; ++e)
+            if (f + e < a.rows) acc[i][j][gq * 4 + e] += a.bias[f + e];
+        }
         if (a.softcap > 0.0f) {
 #pragma unroll
           for (int e = 0; e < 4; ++e) acc[i][j][gq * 4 + e] = a.softcap * tanhf(acc[i][j][gq * 4 + e] / a.softcap);
@@ -191,7 +197,7 @@ __global__ __launch_bounds__(256) void dense_gemm_kernel(const DenseArgs a) {
         if (a.act) {
 #pragma unroll
           for (int e = 0; e < 4; ++e)
-            if (f + e >= a.act_from) acc[i][j][gq * 4 + e] = tl_act_apply(a.act, acc[i][j][gq * 4 + e], a.act_p, a.act_q);
+            if (f + e >= a.act_from && f + e < act_to) acc[i][j][gq * 4 + e] = tl_act_apply(a.act, acc[i][j][gq * 4 + e], a.act_p, a.act_q);
         }
         if (v4 && f + 4 <= a.rows) {
           *reinterpret_cast<float4*>(yr + f) =
@@ -224,8 +230,9 @@ __global__ __launch_bounds__(256) void dense_gemv_kernel(const unsigned short* _
 #pragma unroll
     for (int r = 0; r < RW; ++r)
       if (row0 + r < rows) {
+        if (act.bias) out[r] += act.bias[row0 + r];
         float v = softcap > 0.0f ? softcap * tanhf(out[r] / softcap) : out[r];
-        if (act.act && row0 + r >= act.act_from) v = tl_act_apply(act.act, v, act.act_p, act.act_q);
+        if (act.act && row0 + r >= act.act_from && (act.act_to <= 0 || row0 + r < act.act_to)) v = tl_act_apply(act.act, v, act.act_p, act.act_q);
         y[row0 + r] = v;
       }
   }
@@ -242,6 +249,7 @@ int tl_launch_dense_gemm(const DenseArgs& a, hipStream_t s) {
   TL_REQUIRE(groups == 1 || a.group_off || (a.x_gstride >= 0 && a.y_gstride > 0 && !a.x_rows && !a.y_rows),
              "dense gemm: groups without group_off or per-head column strides");
   TL_REQUIRE(!a.act || !a.glu, "dense gemm: an activation and a gated unit in one epilogue");
+  TL_REQUIRE(!a.bias || (!a.glu && groups == 1), "dense gemm: a bias with a gated unit or several matrices");
   // 128 x 128 tiles when there is enough of both sides to fill them (grouped launches: tokens per group on average)
   const long long per_group = a.group_off ? (long long)a.T / groups : a.T;
   // Measured at width 4096, chunks of 512 tokens: a dense launch has too few 128 x 128 tiles to fill 256 CUs (6144 x 512:
@@ -321,7 +329,7 @@ extern "C" int tl_dense_matmul_act(const void* w_bf16_dev, int rows, int cols, c
   if (terms == 0) {
     TL_REQUIRE(num_tokens == 1, "tl_dense_matmul_act: terms 0 (FP32 GEMV) takes one token, not %d", num_tokens);
     return tl_launch_dense_gemv_act(static_cast<const uint16_t*>(w_bf16_dev), rows, cols, x_dev, y_dev,
-                                    GemvActArgs{act, act_from, act_p, act_q}, s);
+                                    GemvActArgs{act, act_from, act_p, act_q, 0, nullptr}, s);
   }
   DenseArgs a = {};
   a.w = static_cast<const uint16_t*>(w_bf16_dev);
@@ -335,6 +343,35 @@ extern "C" int tl_dense_matmul_act(const void* w_bf16_dev, int rows, int cols, c
   a.terms = terms;
   a.act = act;
   a.act_from = act_from;
+  a.act_p = act_p;
+  a.act_q = act_q;
+  return tl_launch_dense_gemm(a, s);
+}
+
+extern "C" int tl_dense_matmul_bias(const void* w_bf16_dev, int rows, int cols, const float* x_dev, float* y_dev, int num_tokens,
+                                    int terms, const float* bias_dev, int act, float act_p, float act_q, int act_from, int act_to,
+                                    void* stream) {
+  hipStream_t s = static_cast<hipStream_t>(stream);
+  TL_REQUIRE(act >= TL_ACT_NONE && act <= TL_ACT_SIGMOID_POWER, "tl_dense_matmul_bias: activation kind %d", act);
+  if (terms == 0) {
+    TL_REQUIRE(num_tokens == 1, "tl_dense_matmul_bias: terms 0 (FP32 GEMV) takes one token, not %d", num_tokens);
+    return tl_launch_dense_gemv_act(static_cast<const uint16_t*>(w_bf16_dev), rows, cols, x_dev, y_dev,
+                                    GemvActArgs{act, act_from, act_p, act_q, act_to, bias_dev}, s);
+  }
+  DenseArgs a = {};
+  a.w = static_cast<const uint16_t*>(w_bf16_dev);
+  a.rows = rows;
+  a.cols = cols;
+  a.x = x_dev;
+  a.ldx = cols;
+  a.y = y_dev;
+  a.ldy = rows;
+  a.T = num_tokens;
+  a.terms = terms;
+  a.bias = bias_dev;
+  a.act = act;
+  a.act_from = act_from;
+  a.act_to = act_to;
   a.act_p = act_p;
   a.act_q = act_q;
   return tl_launch_dense_gemm(a, s);

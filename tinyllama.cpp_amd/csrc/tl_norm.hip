@@ -437,6 +437,104 @@ void launch_hyper(const HyperArgs& a, size_t lds, hipStream_t s) {
   }
 }
 
+// ---- two sublayers that read the same x: both outputs (normed on the way in, if asked for) join the residual, and the norms of the
+// two sublayers that read x next share one set of statistics. A thread holds its columns (PER pieces of V) in registers ----------
+__device__ __forceinline__ void block_sum2(float& p, float& q, float* red) {  // red: 2 kMaxWaves floats
+#pragma unroll
+  for (int o = 32; o >= 1; o >>= 1) {
+    p += __shfl_xor(p, o);
+    q += __shfl_xor(q, o);
+  }
+  if ((threadIdx.x & 63) == 0) {
+    red[threadIdx.x >> 6] = p;
+    red[kMaxWaves + (threadIdx.x >> 6)] = q;
+  }
+  __syncthreads();
+  p = q = 0.0f;
+  for (int w = 0; w < (int)(blockDim.x >> 6); ++w) {
+    p += red[w];
+    q += red[kMaxWaves + w];
+  }
+}
+
+template <int V, int PER>
+__global__ __launch_bounds__(1024) void resid_norms_kernel(const ResidNormsArgs a) {
+  __shared__ float red[2 * kMaxWaves], red2[kMaxWaves];
+  const size_t r0 = (size_t)blockIdx.x * a.width;
+  const int step = blockDim.x * V, c0 = threadIdx.x * V;
+  HyperVec<V> x[PER], ya[PER], yb[PER];
+  float sa = 0.0f, sb = 0.0f;
+#pragma unroll
+  for (int i = 0; i < PER; ++i) {
+    const int c = c0 + i * step;
+#pragma unroll
+    for (int e = 0; e < V; ++e) x[i].v[e] = ya[i].v[e] = yb[i].v[e] = 0.0f;
+    if (c >= a.width) continue;
+    x[i].load(a.x + r0 + c);
+    if (a.a) ya[i].load(a.a + r0 + c);
+    if (a.b) yb[i].load(a.b + r0 + c);
+    if (a.c) {
+      HyperVec<V> yc;
+      yc.load(a.c + r0 + c);
+#pragma unroll
+      for (int e = 0; e < V; ++e) x[i].v[e] += yc.v[e];
+    }
+#pragma unroll
+    for (int e = 0; e < V; ++e) {
+      sa += ya[i].v[e] * ya[i].v[e];
+      sb += yb[i].v[e] * yb[i].v[e];
+    }
+  }
+  float fa = a.a_scale, fb = a.b_scale;
+  if (a.a_w || a.b_w) {
+    block_sum2(sa, sb, red);
+    if (a.a_w) fa *= 1.0f / sqrtf(sa / (float)a.width + a.eps);
+    if (a.b_w) fb *= 1.0f / sqrtf(sb / (float)a.width + a.eps);
+  }
+  float ss = 0.0f;
+#pragma unroll
+  for (int i = 0; i < PER; ++i) {
+    const int c = c0 + i * step;
+    if (c >= a.width) continue;
+    if (a.a) {
+      HyperVec<V> w;
+#pragma unroll
+      for (int e = 0; e < V; ++e) w.v[e] = 1.0f;
+      if (a.a_w) w.load(a.a_w + c);
+#pragma unroll
+      for (int e = 0; e < V; ++e) x[i].v[e] += ya[i].v[e] * fa * w.v[e];
+    }
+    if (a.b) {
+      HyperVec<V> w;
+#pragma unroll
+      for (int e = 0; e < V; ++e) w.v[e] = 1.0f;
+      if (a.b_w) w.load(a.b_w + c);
+#pragma unroll
+      for (int e = 0; e < V; ++e) x[i].v[e] += yb[i].v[e] * fb * w.v[e];
+    }
+    if (a.a || a.b || a.c) x[i].store(a.x + r0 + c);
+#pragma unroll
+    for (int e = 0; e < V; ++e) ss += x[i].v[e] * x[i].v[e];
+  }
+  if (!a.w1 && !a.w2) return;
+  const float inv = 1.0f / sqrtf(block_sum(ss, red2) / (float)a.width + a.eps);
+#pragma unroll
+  for (int i = 0; i < PER; ++i) {
+    const int c = c0 + i * step;
+    if (c >= a.width) continue;
+#pragma unroll
+    for (int k = 0; k < 2; ++k) {
+      const float* wp = k == 0 ? a.w1 : a.w2;
+      if (!wp) continue;
+      HyperVec<V> w;
+      w.load(wp + c);
+#pragma unroll
+      for (int e = 0; e < V; ++e) w.v[e] *= x[i].v[e] * inv;
+      w.store((k == 0 ? a.h1 : a.h2) + r0 + c);
+    }
+  }
+}
+
 __device__ __forceinline__ float dyt_of(float x, float alpha, float w, float b) { return tanhf(alpha * x) * w + b; }
 
 // grid (column blocks of 256, T)
@@ -600,6 +698,53 @@ int tl_launch_resid_rms(const ResidRmsArgs& a, hipStream_t s) {
   resid_rms_kernel<<<a.T, row_threads(a.T), lds, s>>>(a);
   TL_HIP(hipGetLastError());
   return 0;
+}
+
+int tl_launch_resid_norms(const ResidNormsArgs& a, hipStream_t s) {
+  TL_REQUIRE(a.x && a.T > 0 && (a.w1 || a.w2 || a.a || a.b || a.c), "resid_norms: bad arguments");
+  TL_REQUIRE(a.width > 0 && a.width <= kMaxRowFloats, "resid_norms: width %d outside (0, %d]", a.width, kMaxRowFloats);
+  TL_REQUIRE((!a.w1 || a.h1) && (!a.w2 || a.h2), "resid_norms: a norm without its output");
+  TL_REQUIRE((!a.a_w || a.a) && (!a.b_w || a.b), "resid_norms: norm weights without a sublayer output");
+  bool v4 = (a.width & 3) == 0;
+  for (const float* p : {(const float*)a.x, a.a, a.a_w, a.b, a.b_w, a.c, a.w1, a.w2, (const float*)a.h1, (const float*)a.h2})
+    v4 = v4 && ((size_t)p & 15) == 0;
+  const int pieces = v4 ? a.width / 4 : a.width, most = v4 ? 4 : 16;
+  int th = row_threads(a.T);
+  while (th < 1024 && (pieces + th - 1) / th > most) th *= 2;
+  const int per = (pieces + th - 1) / th;
+  if (v4) {
+    if (per <= 1) resid_norms_kernel<4, 1><<<a.T, th, 0, s>>>(a);
+    else if (per <= 2) resid_norms_kernel<4, 2><<<a.T, th, 0, s>>>(a);
+    else resid_norms_kernel<4, 4><<<a.T, th, 0, s>>>(a);
+  } else {
+    if (per <= 4) resid_norms_kernel<1, 4><<<a.T, th, 0, s>>>(a);
+    else resid_norms_kernel<1, 16><<<a.T, th, 0, s>>>(a);
+  }
+  TL_HIP(hipGetLastError());
+  return 0;
+}
+
+extern "C" int tl_resid_two_norms(float* x_dev, const float* a_dev, float a_scale, const float* a_weight_dev, const float* b_dev,
+                                  float b_scale, const float* b_weight_dev, const float* c_dev, const float* weight1_dev,
+                                  float* h1_dev, const float* weight2_dev, float* h2_dev, int num_tokens, int width, float eps,
+                                  void* stream) {
+  ResidNormsArgs a = {};
+  a.x = x_dev;
+  a.T = num_tokens;
+  a.width = width;
+  a.a = a_dev;
+  a.a_w = a_weight_dev;
+  a.a_scale = a_scale;
+  a.b = b_dev;
+  a.b_w = b_weight_dev;
+  a.b_scale = b_scale;
+  a.c = c_dev;
+  a.w1 = weight1_dev;
+  a.w2 = weight2_dev;
+  a.h1 = h1_dev;
+  a.h2 = h2_dev;
+  a.eps = eps;
+  return tl_launch_resid_norms(a, static_cast<hipStream_t>(stream));
 }
 
 int tl_launch_norm_rows(const float* x, int width, const int* rows_dev, int n, const float* w, float eps, float* out,

@@ -20,7 +20,9 @@
 //               terms is free as long as both operands agree), so S never moves. The waves' partial Y meet in LDS.
 //   ssm_step    one token: a workgroup per (32 value channels, head) forms the convolution of the channels it needs itself
 //               (history read, not written: other workgroups read it too), updates its piece of S and reads it out.
-//   part_norm   RMS norm of a row in equal parts, in place; for one token it also shifts the convolution's history, whose
+//   With log_decay the same walk is linear attention with one CONSTANT decay per head, S <- decay S + k v^T, o = S^T q: x = v, B = k,
+//   C = q, dt = 1, no skip (lightning_step: its one-token form).
+//   part_norm   RMS norm of a row in equal parts, in place, optionally times a sigmoid gate; for one token it also shifts the convolution's history, whose
 //               readers are done by then.
 #include <math.h>
 
@@ -76,8 +78,9 @@ __global__ __launch_bounds__(192) void ssm_gram_kernel(const SsmScanArgs a, int 
   if (g >= a.groups) {
     const int head = (g - a.groups) * 3 + wave;
     if (head >= a.heads) return;
-    const float dt = t0 + lane < a.T ? ssm_softplus(a.dt_raw[(size_t)(t0 + lane) * a.dt_ld + head] + a.dt_bias[head]) : 0.0f;
-    double c = -(double)(expf(a.a_log[head]) * dt);
+    const bool in = t0 + lane < a.T;
+    const float dt = !in ? 0.0f : a.log_decay ? 1.0f : ssm_softplus(a.dt_raw[(size_t)(t0 + lane) * a.dt_ld + head] + a.dt_bias[head]);
+    double c = !in ? 0.0 : a.log_decay ? a.log_decay[head] : -(double)(expf(a.a_log[head]) * dt);
 #pragma unroll
     for (int o = 1; o < 64; o <<= 1) {
       const double up = __shfl_up(c, o);
@@ -134,7 +137,7 @@ __global__ __launch_bounds__(256, NT == 1 ? 2 : 1) void ssm_walk_kernel(const Ss
   const float* bp = a.xbc + inner + (size_t)g * N;
   const float* cp = bp + (size_t)a.groups * N;
   const float* zp = a.z ? a.z + (size_t)head * vdim : nullptr;
-  const float dskip = a.d[head];
+  const float dskip = a.d ? a.d[head] : 0.0f;
   const float* stp = a.gram + (size_t)blocks * a.groups * SSM_Q * SSM_Q + (size_t)head * SSM_STEP_FLOATS;
   float* sp = a.state + (size_t)head * N * vdim + v0;
   // (row offsets fit 32 bits: the launcher checks; rows beyond the call repeat its last row and carry weight 0)
@@ -464,7 +467,86 @@ __global__ __launch_bounds__(256) void part_norm_kernel(const PartNormArgs a) {
   if ((tid & 63) == 0) red[tid >> 6] = ss;
   __syncthreads();
   const float inv = 1.0f / sqrtf(((red[0] + red[1]) + (red[2] + red[3])) / (float)n + a.eps);
-  for (int c = tid; c < n; c += 256) x[c] = x[c] * inv * w[c];
+  const float* gt = a.gate ? a.gate + (size_t)t * a.gate_ld + (size_t)part * n : nullptr;
+  for (int c = tid; c < n; c += 256) x[c] = x[c] * inv * w[c] * (gt ? 1.0f / (1.0f + expf(-gt[c])) : 1.0f);
+}
+
+// grid (value channels in 32s, heads), 256 threads: 8 column quads x 32 state rows, the state in passes of 32 rows
+__global__ __launch_bounds__(256) void lightning_step_kernel(const LightningStepArgs a, int vec) {
+  extern __shared__ __attribute__((aligned(16))) float sl[];  // k [dim] | q [dim]
+  __shared__ float red[4][32];
+  const int tid = threadIdx.x, cq = tid & 7, rg = tid >> 3;
+  const int v0 = blockIdx.x * 32, head = blockIdx.y, N = a.dim, vdim = a.vdim;
+  const float* vp = a.vkq + (size_t)head * vdim + v0 + 4 * cq;
+  const float* kp = a.vkq + (size_t)a.heads * vdim + (size_t)head * N;
+  const float* qp = kp + (size_t)a.heads * N;
+  float* sp = a.state + (size_t)head * N * vdim + v0 + 4 * cq;
+  const int left = vdim - v0 - 4 * cq;  // columns of this thread's quad that exist (<= 0: none)
+  auto load4 = [&](const float* p, bool wide) __attribute__((always_inline)) {
+    float4 v = make_float4(0.0f, 0.0f, 0.0f, 0.0f);
+    if (left <= 0) return v;
+    if (wide) return *reinterpret_cast<const float4*>(p);
+    v.x = p[0];
+    if (left > 1) v.y = p[1];
+    if (left > 2) v.z = p[2];
+    if (left > 3) v.w = p[3];
+    return v;
+  };
+  constexpr int PF = 4;  // passes whose state is in flight together
+  const float4 v4 = load4(vp, false);
+  const float decay = (float)exp(a.log_decay[head]);
+  for (int i = tid; i < N; i += 256) {
+    sl[i] = kp[i];
+    sl[N + i] = qp[i];
+  }
+  float4 y = make_float4(0.0f, 0.0f, 0.0f, 0.0f);
+  for (int n0 = 0; n0 < N; n0 += 32 * PF) {
+    float4 st[PF];
+#pragma unroll
+    for (int i = 0; i < PF; ++i) {
+      const int n = n0 + rg + 32 * i;
+      st[i] = n < N ? load4(sp + (size_t)n * vdim, vec != 0) : make_float4(0.0f, 0.0f, 0.0f, 0.0f);
+    }
+    if (n0 == 0) __syncthreads();
+#pragma unroll
+    for (int i = 0; i < PF; ++i) {
+      const int n = n0 + rg + 32 * i;
+      if (n >= N || left <= 0) continue;
+      const float k = sl[n], q = sl[N + n];
+      float4 s = st[i];
+      s.x = decay * s.x + k * v4.x;
+      s.y = decay * s.y + k * v4.y;
+      s.z = decay * s.z + k * v4.z;
+      s.w = decay * s.w + k * v4.w;
+      y.x += q * s.x;
+      y.y += q * s.y;
+      y.z += q * s.z;
+      y.w += q * s.w;
+      float* p = sp + (size_t)n * vdim;
+      if (vec) {
+        *reinterpret_cast<float4*>(p) = s;
+      } else {
+        p[0] = s.x;
+        if (left > 1) p[1] = s.y;
+        if (left > 2) p[2] = s.z;
+        if (left > 3) p[3] = s.w;
+      }
+    }
+  }
+#pragma unroll
+  for (int o = 8; o < 64; o <<= 1) {  // the eight state rows a wave works on side by side
+    y.x += __shfl_xor(y.x, o);
+    y.y += __shfl_xor(y.y, o);
+    y.z += __shfl_xor(y.z, o);
+    y.w += __shfl_xor(y.w, o);
+  }
+  if ((tid & 63) < 8) {
+    float* o = &red[tid >> 6][4 * cq];
+    o[0] = y.x, o[1] = y.y, o[2] = y.z, o[3] = y.w;
+  }
+  __syncthreads();
+  if (tid < 32 && v0 + tid < vdim)
+    a.y[(size_t)head * vdim + v0 + tid] = (red[0][tid] + red[1][tid]) + (red[2][tid] + red[3][tid]);
 }
 
 template <int NT, bool EVEN>
@@ -484,11 +566,12 @@ size_t tl_ssm_gram_floats(int T, int heads, int groups) {
 }
 
 int tl_launch_ssm_scan(const SsmScanArgs& a, hipStream_t s) {
-  TL_REQUIRE(a.xbc && a.dt_raw && a.dt_bias && a.a_log && a.d && a.state && a.y && a.gram && a.T > 0, "ssm_scan: bad arguments");
+  TL_REQUIRE(a.xbc && (a.log_decay || (a.dt_raw && a.dt_bias && a.a_log && a.d)) && a.state && a.y && a.gram && a.T > 0,
+             "ssm_scan: bad arguments");
   TL_REQUIRE(a.heads > 0 && a.heads <= 65535 && a.groups > 0 && a.groups <= 65535 && a.heads % a.groups == 0 && a.vdim > 0,
              "ssm_scan: %d heads in %d groups, value size %d", a.heads, a.groups, a.vdim);
   TL_REQUIRE(a.state_n > 0 && a.state_n <= 512, "ssm_scan: state size %d outside (0, 512]", a.state_n);
-  TL_REQUIRE(a.ld >= a.heads * a.vdim + 2 * a.groups * a.state_n && a.dt_ld >= a.heads && (!a.z || a.z_ld >= a.heads * a.vdim),
+  TL_REQUIRE(a.ld >= a.heads * a.vdim + 2 * a.groups * a.state_n && (a.log_decay || a.dt_ld >= a.heads) && (!a.z || a.z_ld >= a.heads * a.vdim),
              "ssm_scan: row strides %d / %d / %d", a.ld, a.dt_ld, a.z_ld);
   // 16-byte pieces of B and C rows
   const int vec = (a.state_n & 3) == 0 && (a.ld & 3) == 0 && ((a.heads * a.vdim) & 3) == 0 && ((size_t)a.xbc & 15) == 0;
@@ -500,7 +583,7 @@ int tl_launch_ssm_scan(const SsmScanArgs& a, hipStream_t s) {
     w.T = a.T - a.T % SSM_Q;
     rest.T = a.T - w.T;
     rest.xbc += (size_t)w.T * a.ld;
-    rest.dt_raw += (size_t)w.T * a.dt_ld;
+    if (a.dt_raw) rest.dt_raw += (size_t)w.T * a.dt_ld;
     if (a.z) rest.z += (size_t)w.T * a.z_ld;
     rest.y += (size_t)w.T * a.heads * a.vdim;
     TL_TRY(tl_launch_ssm_scan(w, s));
@@ -526,9 +609,19 @@ int tl_launch_ssm_step(const SsmStepArgs& a, hipStream_t s) {
   return 0;
 }
 
+int tl_launch_lightning_step(const LightningStepArgs& a, hipStream_t s) {
+  TL_REQUIRE(a.vkq && a.log_decay && a.state && a.y && a.heads > 0 && a.heads <= 65535 && a.dim > 0 && a.dim <= 4096 && a.vdim > 0,
+             "lightning_step: bad arguments");
+  const int vec = (a.vdim & 3) == 0 && ((size_t)a.state & 15) == 0;
+  lightning_step_kernel<<<dim3((a.vdim + 31) / 32, a.heads), 256, sizeof(float) * 2 * (size_t)a.dim, s>>>(a, vec);
+  TL_HIP(hipGetLastError());
+  return 0;
+}
+
 int tl_launch_part_norm(const PartNormArgs& a, hipStream_t s) {
   TL_REQUIRE(a.x && a.w && a.T > 0 && a.parts > 0 && a.width > 0 && a.width % a.parts == 0, "part_norm: %d channels in %d parts",
              a.width, a.parts);
+  TL_REQUIRE(!a.gate || a.gate_ld >= a.width, "part_norm: gate rows of %d for %d channels", a.gate_ld, a.width);
   TL_REQUIRE(!a.hist || (a.T == 1 && a.hist_in && a.taps > 1 && a.channels > 0), "part_norm: a history rides along for one token");
   const long long blocks = (long long)a.T * a.parts + (a.hist ? (a.channels + 255) / 256 : 0);
   TL_REQUIRE(blocks <= 0x7fffffffLL, "part_norm: launch too large");
@@ -598,5 +691,40 @@ extern "C" int tl_part_norm(float* x_dev, const float* weight_dev, int num_token
   a.hist_in = in_dev;
   a.taps = taps;
   a.channels = channels;
+  return tl_launch_part_norm(a, static_cast<hipStream_t>(stream));
+}
+
+extern "C" int tl_constant_decay_attention(const float* vkq_dev, int ld, const double* log_decay_dev, float* state_dev, float* o_dev,
+                                           int num_tokens, int heads, int dim, int vdim, void* stream) {
+  TL_REQUIRE(num_tokens > 0 && heads > 0 && dim > 0 && vdim > 0, "tl_constant_decay_attention: bad arguments");
+  hipStream_t s = static_cast<hipStream_t>(stream);
+  if (num_tokens == 1) return tl_launch_lightning_step(LightningStepArgs{vkq_dev, log_decay_dev, state_dev, o_dev, heads, dim, vdim}, s);
+  SsmScanArgs a = {};
+  a.xbc = vkq_dev;
+  a.ld = ld;
+  a.log_decay = log_decay_dev;
+  a.state = state_dev;
+  a.y = o_dev;
+  a.T = num_tokens;
+  a.heads = a.groups = heads;
+  a.state_n = dim;
+  a.vdim = vdim;
+  void* ws = nullptr;
+  TL_TRY(tl_scratch(TL_SCRATCH_SSM, sizeof(float) * tl_ssm_gram_floats(num_tokens, heads, heads), &ws));
+  a.gram = static_cast<float*>(ws);
+  return tl_launch_ssm_scan(a, s);
+}
+
+extern "C" int tl_gated_row_norm(float* x_dev, const float* weight_dev, const float* gate_dev, int gate_ld, int num_tokens, int width,
+                                 float eps, void* stream) {
+  PartNormArgs a = {};
+  a.x = x_dev;
+  a.w = weight_dev;
+  a.T = num_tokens;
+  a.width = width;
+  a.parts = 1;
+  a.eps = eps;
+  a.gate = gate_dev;
+  a.gate_ld = gate_ld;
   return tl_launch_part_norm(a, static_cast<hipStream_t>(stream));
 }

@@ -15,7 +15,7 @@
 //   tl_conv.hip   a short causal convolution over time per channel with its history (sublayer inputs; projected q, k, v)
 //   tl_latent.hip latent attention: norms of the latents, the rotated shared key part, cache rows, output gates
 //   tl_ssm.hip    selective state space (one decay per head and token): blocks of a prompt on the matrix cores, one-token step,
-//                 RMS norm of a row in equal parts
+//                 RMS norm of a row in equal parts; linear attention with a constant decay per head on the same block walk
 #pragma once
 #include "tl_internal.h"
 
@@ -45,6 +45,8 @@ struct DenseArgs {
   // act_q = 1/2 + softplus(q))
   int act, act_from;
   float act_p, act_q;
+  int act_to;            // > 0: ... and in front of act_to
+  const float* bias;     // optional [rows] (not with glu, not per head): added to the product, in front of the activation
   // groups > 1 without group_off: one product per head over ALL items -- group g multiplies matrix g with the columns
   // x[.][g * x_gstride ..] (0: every head reads the same columns) and writes y[.][g * y_gstride ..]
   int x_gstride, y_gstride;
@@ -55,6 +57,8 @@ int tl_launch_dense_gemv(const uint16_t* w, int rows, int cols, const float* x, 
 struct GemvActArgs {
   int act, act_from;     // as DenseArgs
   float act_p, act_q;
+  int act_to;
+  const float* bias;
 };
 int tl_launch_dense_gemv_act(const uint16_t* w, int rows, int cols, const float* x, float* y, const GemvActArgs& act, hipStream_t s);
 // one token, one product per head: y[g * y_stride + r] = W[g][r] . x[g * x_stride ..]
@@ -65,6 +69,8 @@ __host__ __device__ inline float tl_act_apply(int act, float z, float p, float q
   if (act == TL_ACT_XIELU) return z > 0.0f ? p * z * z + 0.5f * z : q * (expm1f(z) - z) + 0.5f * z;
   if (act == TL_ACT_TANH) return tanhf(z);
   if (act == TL_ACT_GELU) return 0.5f * z * (1.0f + erff(z * 0.70710678118654752f));
+  if (act == TL_ACT_SILU) return z / (1.0f + expf(-z));
+  if (act == TL_ACT_SIGMOID_POWER) return expf(-p * (fmaxf(-z, 0.0f) + log1pf(expf(-fabsf(z)))));
   return z;
 }
 
@@ -116,6 +122,10 @@ struct SwaArgs {
   // 1: every query head reads the same key rows, which are the values as well (kv_heads == 1, vc == kc, plain softmax, few
   // tokens): the heads' products over a tile of rows run together. nsplit = tl_swa_shared_splits (> 0), ws set
   int shared;
+  // > 0: position i sees j <= i only inside its own chunk of so many positions, counted from position 0 (also under a window)
+  int chunk;
+  const float* gate;  // optional, token t at gate + t * gate_ld (not with shared): head h's output is multiplied by sigmoid(gate[h])
+  int gate_ld;
 };
 int tl_launch_swa(const SwaArgs& a, hipStream_t s);
 int tl_swa_splits(int T, int window, int max_pos, int keep_first = 0);  // splits worth having for T tokens over a cache of max_pos rows
@@ -208,6 +218,21 @@ struct ResidRmsArgs {
   RouterArgs route;
 };
 int tl_launch_resid_rms(const ResidRmsArgs& a, hipStream_t s);
+// blocks whose two sublayers read the same x behind a norm each: x[t] += a_scale A + b_scale B + c, A = a[t] / rms(a[t]) * a_w (a_w NULL:
+// a itself), B likewise; then h1 = x / rms(x) * w1 and h2 = x / rms(x) * w2 for the sublayers that read x next (either may be absent)
+struct ResidNormsArgs {
+  float* x;              // [T][width]
+  int T, width;
+  const float *a, *a_w;  // optional [T][width], [width]
+  float a_scale;
+  const float *b, *b_w;
+  float b_scale;
+  const float* c;        // optional [T][width]
+  const float *w1, *w2;  // optional [width]
+  float *h1, *h2;        // [T][width]
+  float eps;
+};
+int tl_launch_resid_norms(const ResidNormsArgs& a, hipStream_t s);
 // ---- norm-first blocks: Dynamic Tanh (elementwise, no statistics) and the plain residual sum ------------------------------
 struct DytParams {
   const float* alpha;    // device scalar (NULL: no norm asked for)
@@ -365,11 +390,13 @@ int tl_launch_moe_decode(const MoeDecodeArgs& a, hipStream_t s);
 // ---- tl_rope.hip -------------------------------------------------------------------------------------------------------
 // f[i] (i < rot_dims / 2) and the factor on cos / sin of a layer's rotary positions (tl_layer_spec: rot_*), computed in double
 void tl_rotary_frequencies(int rot_dims, double base, double factor, double original, double fast, double slow, double* f,
-                           float* mscale);
+                           float* mscale, int scaling = TL_ROT_BLEND);
 struct RotaryArgs {
   float* qk;             // [T][ld]: q heads (heads * dim) | k heads (kv_heads * dim) of a token, updated in place
   int ld, heads, kv_heads, dim;
   int rot_dims;          // the first rot_dims dimensions of a head rotate: (2i, 2i + 1) by position * freq[i]
+  int halves;            // 1: the pairs are (i, i + rot_dims / 2)
+  const float *q_norm, *k_norm;  // optional plain weights [dim]: an RMS norm per head in FRONT of the rotation (eps below)
   const double* freq;    // device [rot_dims / 2], double: position * frequency is formed and reduced to [-pi, pi] in double
   float mscale;          // on cos and sin
   int unit_norm;         // 1: after the rotation a head is divided by its root mean square (eps inside the root)
@@ -422,6 +449,7 @@ struct DeltaScanArgs {
   // plain_write != 0: nothing is removed before the write, u = beta v (a gated linear recurrence S <- diag(g) S + k v^T);
   // beta may then be NULL (1)
   int plain_write;
+  float q_scale;         // != 0: o is multiplied by it
 };
 int tl_launch_delta_scan(const DeltaScanArgs& a, hipStream_t s);
 // o[t][h] <- o / sqrt(mean(o^2) + eps) * w * sigmoid(gate[t][h]) per head (w [vdim] shared by the heads); in place
@@ -446,6 +474,21 @@ struct HeadNormArgs {
 int tl_launch_head_norm(const HeadNormArgs& a, hipStream_t s);
 // what precedes the gated linear recurrence of TL_MIXER_LINEAR: p [T][ld] = q | f (heads * dim each) | ...;
 // qk [T][2 * heads * dim] = silu(q) | 1 - f, g [T][heads * dim] = f, f = lower + (1 - lower) sigmoid(p_f + f_bias)
+// one token of TL_MIXER_GLA between its products, a workgroup per head: p = q | k | v | gate | a1 as projected
+struct GlaStepArgs {
+  const float* p;
+  const uint16_t* a2;    // bf16 [heads * dim][rank]
+  const float* a2_b;     // [heads * dim]
+  int rank;
+  float power, q_scale;  // alpha = sigmoid(a2 a1 + a2_b)^power
+  const float* norm;     // [vdim]
+  float eps;
+  float* state;          // [heads][vdim][dim]
+  float* o;              // [heads * vdim]
+  int heads, dim, vdim;
+};
+bool tl_gla_step_fits(int dim, int vdim, int rank);
+int tl_launch_gla_step(const GlaStepArgs& a, hipStream_t s);
 struct LinearPreArgs {
   const float* p;
   int ld, T, heads, dim;
@@ -497,6 +540,9 @@ struct SsmScanArgs {
   float* y;              // [T][heads * vdim]
   float* gram;           // scratch, tl_ssm_gram_floats
   int T, heads, groups, state_n, vdim;
+  // log_decay [heads] set: linear attention with a constant decay, S <- e^log_decay S + B x^T (dt = 1, no skip; dt_raw, dt_bias,
+  // a_log, d are not read)
+  const double* log_decay;
 };
 size_t tl_ssm_gram_floats(int T, int heads, int groups);
 int tl_launch_ssm_scan(const SsmScanArgs& a, hipStream_t s);
@@ -513,6 +559,15 @@ struct SsmStepArgs {
   int heads, groups, state_n, vdim;
 };
 int tl_launch_ssm_step(const SsmStepArgs& a, hipStream_t s);
+// one token of the constant-decay form: S <- e^log_decay S + k v^T, y = S^T q; vkq = v (heads * vdim) | k | q (heads * dim each)
+struct LightningStepArgs {
+  const float* vkq;
+  const double* log_decay;  // [heads]
+  float* state;             // [heads][dim][vdim]
+  float* y;                 // [heads * vdim]
+  int heads, dim, vdim;
+};
+int tl_launch_lightning_step(const LightningStepArgs& a, hipStream_t s);
 // every row of x [T][width] in `parts` equal parts, each divided by its root mean square, times w [width]; in place. hist (one
 // row): a convolution's history [taps - 1][channels] drops its oldest row and gains hist_in [channels]
 struct PartNormArgs {
@@ -523,6 +578,8 @@ struct PartNormArgs {
   float* hist;
   const float* hist_in;
   int taps, channels;
+  const float* gate;     // optional, token t at gate + t * gate_ld: the normed row is multiplied by sigmoid(gate)
+  int gate_ld;
 };
 int tl_launch_part_norm(const PartNormArgs& a, hipStream_t s);
 

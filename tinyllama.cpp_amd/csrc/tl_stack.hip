@@ -8,6 +8,8 @@
 //                             finishes x also writes the norm of whatever reads x next (norm2, or the next layer's norm1)
 //         TL_BLOCK_PARALLEL   h = norm1(x); x += mixer(h) + ff(h)       -- one Dynamic Tanh norm, both sublayers read its output;
 //                             the norm of the NEXT block rides in the launch that finishes x (it is elementwise)
+//         TL_BLOCK_PARALLEL_NORMS  x += mixer(norm1(x)) + ff(norm2(x)) -- a norm each over the same x: one launch finishes x and writes
+//                             both norms for the block that follows (tl_norm.hip: resid_norms)
 // Mixers  TL_MIXER_SWA    q | k (| v) = W h in one product; either the whole-projection q/k RMS norm with optional value mixing
 //                         (tl_norm.hip), or rotary positions + per-head unit norm, values optionally the keys as projected
 //                         (tl_rope.hip); k, v -> cache; windowed attention with softmax or sigmoid weights, optionally with
@@ -26,12 +28,19 @@
 //         TL_MIXER_SSM    z | x | B | C | dt = W h in one product; several tokens: convolution, the blocks' C B^T, the walk over the
 //                         blocks with the state in registers (it applies D, the gate silu(z)), RMS norm in parts; one token: convolution,
 //                         state update and read-out in one launch, then the norm, which also shifts the convolution's history; W_o
-//         TL_MIXER_SWA with its options: two score maps per head over the same values (differential attention: one attention
+//         TL_MIXER_GLA    linear attention with a decay per key channel: q | k | v | gate | a1 = W h in one product; several tokens: a2
+//                         behind a1 with the decay in its epilogue, the delta rule's scan without its removal step, gated head norm;
+//                         one token: all of that in one launch (gla_step); W_o
+//         TL_MIXER_LIGHTNING linear attention with a constant decay per head: gate | v | k | q = W h in one product (silu on v, k, q in its
+//                         epilogue); the state space's walk over blocks with a constant decay, or lightning_step; RMS norm of the whole
+//                         row times the gate; W_o
+//         TL_MIXER_SWA with its options: chunks instead of a window, an RMS norm per head in front of the rotation, biases in the first
+//                         product, a gate per head where a head's output is finished; two score maps per head over the same values (differential attention: one attention
 //                         launch per map, then (a1 - lambda a2) / rms (1 - diff) sigmoid(gate)), a norm per head and map, biases
 //                         and a causal convolution on q, k, v (tl_conv.hip), capped scores, a logarithmic distance bias, a learned
 //                         sink per head; TL_MIXER_DELTA with one decay per head and direct projections for decay and gate
 //         Two mixers side by side (tl_layer_spec::side): both read the same input, their first products are one product, the
-//                         layer's mixer output is mix_scale * first + side_scale * second
+//                         layer's mixer output is mix_scale * first + side_scale * second, optionally behind an RMS norm of each
 //         Pre-norm blocks behind a layer norm may keep several residual streams (hyper-connections, tl_stack_config::streams): the
 //                         launch that finishes a sublayer mixes the old streams, adds its output to each, sums the next sublayer's
 //                         input from the new ones and norms it (tl_norm.hip: hyper). Without streams the same launch adds experts'
@@ -50,7 +59,7 @@
 // flat by absolute position; a window only bounds what attention reads. Delta layers: S [heads][vdim][dim] and the
 // convolution's last taps - 1 inputs (linear attention: S only; attention with a convolution on q, k, v: that history too;
 // every layer: the histories of the convolutions on what its sublayers read); latent layers with a projection of their
-// own: rows [max_positions][kv_rank + rot_dim]; generalized delta layers: S [heads][dim][dim]; state-space layers: S
+// own: rows [max_positions][kv_rank + rot_dim]; constant-decay linear attention: S [heads][dim][vdim]; generalized delta layers: S [heads][dim][dim]; state-space layers: S
 // [heads][state][vdim] and the convolution's history. tl_stack_reset gives everything back (one sequence at a time): zeros are the state of
 // an empty sequence.
 #include <math.h>
@@ -110,6 +119,9 @@ struct Layer {
   float *conv_b = nullptr, *dskip = nullptr;
   // hyper-connections of the two sublayers: in [streams], out [streams], mix [streams][streams]
   float *hc_in[2] = {nullptr, nullptr}, *hc_out[2] = {nullptr, nullptr}, *hc_mix[2] = {nullptr, nullptr};
+  float* prod_b = nullptr;                   // biases of the first product (zeros where a column has none); a pair shares one row
+  double* log_decay = nullptr;               // constant-decay linear attention [heads]; this layer's own, also when it borrows tensors
+  float* out_norm = nullptr;                 // a mixer of a normed pair: the RMS norm of its output [width]
   std::unique_ptr<Layer> side;               // the second mixer of a pair: its mixer fields, tensors and state only
   std::set<std::string> expect, optional;    // tensor names (without the "l<i>." prefix) still missing / accepted and ignored
 };
@@ -133,6 +145,7 @@ struct TlStack {
   int exact_below = 64;     // portions shorter than this always multiply with three terms (TL_STACK_EXACT_BELOW; at least 2)
   bool gemv_decode = true;
   bool fuse_router = true;  // TL_STACK_FUSE_ROUTER=0: the router as a launch of its own (A/B, tests)
+  bool fuse_steps = true;   // TL_STACK_FUSE_STEPS=0: one token of a recurrence in as many launches as a chunk takes (A/B, tests)
   bool fuse_canon = true;   // TL_STACK_FUSE_CANON=0: the convolution on what a sublayer reads as a launch of its own also for one token
   // One token through a parallel block: mixer and feed-forward read the same h and meet only in the residual sum, so the
   // feed-forward's launches go to a second stream (forked and joined by events; under capture they become a parallel branch
@@ -146,6 +159,7 @@ struct TlStack {
   float* hn = nullptr;      // the norm of x before the convolution on what a sublayer reads
   bool any_pair = false, any_maps = false;
   float* h = nullptr;       // norm-first blocks: the normalised input both sublayers read
+  float* h2 = nullptr;      // TL_BLOCK_PARALLEL_NORMS: what the feed-forward reads
   float *dq = nullptr, *da = nullptr, *dg = nullptr, *dbeta = nullptr, *ddecay = nullptr;  // delta rule
   float *lq = nullptr, *lqa = nullptr;      // latent attention: up-projected queries, absorbed queries
   float* xs = nullptr;                      // residual streams [chunk][streams][width] (x then holds their sum)
@@ -180,7 +194,7 @@ int dev_alloc(TlStack* st, T** p, size_t n) {
   return 0;
 }
 
-int upload_as_f32(float* dst, int type, const void* host, size_t n, hipStream_t s) {
+int upload_as_f32(float* dst, int type, const void* host, size_t n, hipStream_t s, float factor = 1.0f) {
   std::vector<float> wide(n);
   if (type == TL_BF16) {
     const uint16_t* b = static_cast<const uint16_t*>(host);
@@ -191,6 +205,8 @@ int upload_as_f32(float* dst, int type, const void* host, size_t n, hipStream_t 
   } else {
     memcpy(wide.data(), host, n * 4);
   }
+  if (factor != 1.0f)
+    for (float& v : wide) v *= factor;
   TL_HIP(hipMemcpyAsync(dst, wide.data(), n * 4, hipMemcpyHostToDevice, s));
   TL_HIP(hipStreamSynchronize(s));
   return 0;
@@ -222,6 +238,12 @@ bool shape_is(const long long* shape, int ndim, long long a, long long b = -1) {
 
 namespace {
 
+// keys that a position can see at most: the smaller of window and chunk (0: no bound)
+int swa_bound(const tl_layer_spec& sp) {
+  if (sp.chunk > 0 && (sp.window <= 0 || sp.chunk < sp.window)) return sp.chunk;
+  return sp.window > 0 ? sp.window : 0;
+}
+
 int upload_frequencies(TlStack* st, Layer& L, const std::vector<double>& f) {
   TL_TRY(dev_alloc(st, &L.freq, f.size()));
   TL_HIP(hipMemcpy(L.freq, f.data(), sizeof(double) * f.size(), hipMemcpyHostToDevice));
@@ -232,12 +254,16 @@ int upload_frequencies(TlStack* st, Layer& L, const std::vector<double>& f) {
 // the layer holds tensors of its own) and its share of the cache. first_mix: the first value-mixing layer so far.
 int setup_mixer(TlStack* st, Layer& L, int i, bool own, int* first_mix) {
   const tl_stack_config* cfg = &st->cfg;
+  const double* const decay = L.sp.decay;
+  L.sp.decay = nullptr;  // (the caller's array: read here, once)
   const tl_layer_spec& sp = L.sp;
   const size_t W = cfg->width;
-  TL_REQUIRE(sp.mixer >= TL_MIXER_SWA && sp.mixer <= TL_MIXER_SSM,
+  TL_REQUIRE(sp.mixer >= TL_MIXER_SWA && sp.mixer <= TL_MIXER_LIGHTNING,
              "tl_stack_create: layer %d has mixer kind %d; this engine has windowed attention (%d), the gated delta rule (%d), "
-             "latent attention (%d), the generalized delta rule (%d), gated linear attention (%d) and the state space (%d)",
-             i, sp.mixer, TL_MIXER_SWA, TL_MIXER_DELTA, TL_MIXER_LATENT, TL_MIXER_GDELTA, TL_MIXER_LINEAR, TL_MIXER_SSM);
+             "latent attention (%d), the generalized delta rule (%d), gated linear attention (%d), the state space (%d) and linear "
+             "attention with a decay per channel (%d) or a constant one (%d)",
+             i, sp.mixer, TL_MIXER_SWA, TL_MIXER_DELTA, TL_MIXER_LATENT, TL_MIXER_GDELTA, TL_MIXER_LINEAR, TL_MIXER_SSM, TL_MIXER_GLA,
+             TL_MIXER_LIGHTNING);
   TL_REQUIRE(sp.heads > 0 && sp.kv_heads > 0 && sp.heads % sp.kv_heads == 0 && sp.dim > 0 && sp.vdim > 0,
              "tl_stack_create: layer %d: %d heads / %d key-value heads / sizes %d, %d", i, sp.heads, sp.kv_heads, sp.dim, sp.vdim);
   if (sp.mixer == TL_MIXER_SWA) {
@@ -249,10 +275,19 @@ int setup_mixer(TlStack* st, Layer& L, int i, bool own, int* first_mix) {
                "tl_stack_create: layer %d: attention weights of kind %d, query temperature every %d", i, sp.attn_weight,
                sp.q_temp_every);
     L.rotary_path = sp.rot_dims > 0 || sp.qk_norm == TL_QK_NORM_HEAD_UNIT || sp.values_are_keys;
-    TL_REQUIRE(!L.rotary_path || (sp.qk_norm != TL_QK_NORM_WHOLE && sp.qk_norm != TL_QK_NORM_HEAD_RMS && !sp.v_mix &&
-                                  sp.q_temp_every == 0 && sp.score_maps <= 1 && !sp.qkv_conv && !sp.qkv_bias),
-               "tl_stack_create: layer %d: rotation / per-head unit norm / values-are-keys do not combine with the weighted q/k "
-               "norms, value mixing, a query temperature, score maps or a convolution on q, k, v", i);
+    TL_REQUIRE(!L.rotary_path || (sp.qk_norm != TL_QK_NORM_WHOLE && !sp.v_mix && sp.q_temp_every == 0 && sp.score_maps <= 1 &&
+                                  !sp.qkv_conv),
+               "tl_stack_create: layer %d: rotation / per-head unit norm / values-are-keys do not combine with a norm over the whole "
+               "q / k, value mixing, a query temperature, score maps or a convolution on q, k, v", i);
+    TL_REQUIRE(sp.rot_scaling >= TL_ROT_BLEND && sp.rot_scaling <= TL_ROT_WAVELENGTH &&
+                   (sp.rot_scaling != TL_ROT_WAVELENGTH || sp.rot_factor <= 0.0f || (sp.rot_original > 0.0f && sp.rot_fast > 0.0f && sp.rot_slow > 0.0f)),
+               "tl_stack_create: layer %d: frequency scaling of kind %d (factor %g, original %g, fast %g, slow %g)", i, sp.rot_scaling,
+               sp.rot_factor, sp.rot_original, sp.rot_fast, sp.rot_slow);
+    TL_REQUIRE(sp.chunk >= 0 && (sp.chunk == 0 || sp.keep_first == 0), "tl_stack_create: layer %d: chunks of %d, %d kept first keys", i,
+               sp.chunk, sp.keep_first);
+    TL_REQUIRE(!sp.head_gate || (!sp.out_gate && sp.score_maps <= 1), "tl_stack_create: layer %d: a gate per head beside one per output "
+               "column or with two score maps", i);
+    TL_REQUIRE(!sp.qkv_bias || !sp.values_are_keys, "tl_stack_create: layer %d: biases with values that are keys", i);
     TL_REQUIRE(sp.qk_norm >= TL_QK_NORM_NONE && sp.qk_norm <= TL_QK_NORM_HEAD_RMS, "tl_stack_create: layer %d: q/k norm %d", i, sp.qk_norm);
     TL_REQUIRE(sp.score_maps == 0 || sp.score_maps == 1 || sp.score_maps == 2, "tl_stack_create: layer %d: %d score maps", i, sp.score_maps);
     const int maps = sp.score_maps == 2 ? 2 : 1;
@@ -261,15 +296,15 @@ int setup_mixer(TlStack* st, Layer& L, int i, bool own, int* first_mix) {
     TL_REQUIRE(!sp.out_gate || maps == 2, "tl_stack_create: layer %d: the output gate rides in the combination of two score maps", i);
     TL_REQUIRE(sp.qk_norm != TL_QK_NORM_HEAD_RMS || (!sp.v_mix && sp.q_temp_every == 0),
                "tl_stack_create: layer %d: the per-head q/k norm does not combine with value mixing or a query temperature", i);
-    TL_REQUIRE(sp.qkv_conv >= 0 && sp.qkv_conv <= 64 && (!sp.qkv_bias || sp.qkv_conv > 0) && (!sp.qkv_conv || !sp.v_mix),
-               "tl_stack_create: layer %d: %d taps on q, k, v (biases ride in that convolution)", i, sp.qkv_conv);
+    TL_REQUIRE(sp.qkv_conv >= 0 && sp.qkv_conv <= 64 && (!sp.qkv_conv || !sp.v_mix),
+               "tl_stack_create: layer %d: %d taps on q, k, v", i, sp.qkv_conv);
     TL_REQUIRE(sp.score_softcap >= 0.0f, "tl_stack_create: layer %d: score cap %g", i, sp.score_softcap);
     L.qd = sp.heads * sp.dim * maps;
     L.kd = sp.kv_heads * sp.dim * maps;
     L.vd = sp.kv_heads * sp.vdim;
     L.od = sp.heads * sp.vdim;
     L.gate_off = L.qd + L.kd + (sp.values_are_keys ? 0 : L.vd);
-    L.pd = L.gate_off + (sp.out_gate ? L.od : 0);
+    L.pd = L.gate_off + (sp.out_gate ? L.od : sp.head_gate ? sp.heads : 0);
     if (maps == 2) st->any_maps = true;
     if (sp.v_mix) {
       if (*first_mix < 0) {
@@ -297,7 +332,7 @@ int setup_mixer(TlStack* st, Layer& L, int i, bool own, int* first_mix) {
       if (sp.attn_weight == TL_ATTN_SIGMOID) L.expect.insert("mix.pb");
       if (sp.attn_weight == TL_ATTN_SOFTMAX_LEARNED_SINK) L.expect.insert("mix.sink");
       if (maps == 2) L.expect.insert({"mix.lq1", "mix.lk1", "mix.lq2", "mix.lk2"});
-      if (sp.out_gate) L.expect.insert("mix.g");
+      if (sp.out_gate || sp.head_gate) L.expect.insert("mix.g");
       if (sp.qkv_bias) L.expect.insert({"mix.q.b", "mix.k.b", "mix.v.b"});
       if (sp.qkv_conv > 0) L.expect.insert({"mix.q.conv", "mix.k.conv", "mix.v.conv"});
       if (sp.dist_bias) L.expect.insert({"mix.r1", "mix.r2"});
@@ -308,11 +343,12 @@ int setup_mixer(TlStack* st, Layer& L, int i, bool own, int* first_mix) {
       TL_TRY(dev_alloc(st, &L.sinkv, sp.heads));
       TL_TRY(dev_alloc(st, &L.r1, sp.heads));
       TL_TRY(dev_alloc(st, &L.r2, sp.heads));
-      if (sp.qkv_bias) TL_TRY(dev_alloc(st, &L.qkv_b, (size_t)L.qd + L.kd + L.vd));
+      if (sp.qkv_bias && sp.qkv_conv > 0) TL_TRY(dev_alloc(st, &L.qkv_b, (size_t)L.qd + L.kd + L.vd));
       if (sp.qkv_conv > 0) TL_TRY(dev_alloc(st, &L.conv, (size_t)(L.qd + L.kd + L.vd) * sp.qkv_conv));
       if (sp.rot_dims > 0) {
         std::vector<double> f(sp.rot_dims / 2);
-        tl_rotary_frequencies(sp.rot_dims, sp.rot_base, sp.rot_factor, sp.rot_original, sp.rot_fast, sp.rot_slow, f.data(), &L.mscale);
+        tl_rotary_frequencies(sp.rot_dims, sp.rot_base, sp.rot_factor, sp.rot_original, sp.rot_fast, sp.rot_slow, f.data(), &L.mscale,
+                              sp.rot_scaling);
         TL_TRY(upload_frequencies(st, L, f));
       }
     }
@@ -401,6 +437,46 @@ int setup_mixer(TlStack* st, Layer& L, int i, bool own, int* first_mix) {
     TL_TRY(dev_alloc(st, &L.a_log, sp.heads));
     TL_TRY(dev_alloc(st, &L.dskip, sp.heads));
     TL_TRY(dev_alloc(st, &L.onorm, L.od));
+  } else if (sp.mixer == TL_MIXER_GLA) {
+    TL_REQUIRE(sp.kv_heads == sp.heads && sp.dim <= 256 && sp.vdim <= 512 && sp.decay_rank > 0 && sp.decay_tau > 0.0f,
+               "tl_stack_create: layer %d: channel-decay linear attention with %d / %d heads, sizes %d (at most 256) / %d (at most 512), "
+               "inner size %d, tau %g", i, sp.heads, sp.kv_heads, sp.dim, sp.vdim, sp.decay_rank, sp.decay_tau);
+    const int hd = sp.heads * sp.dim;
+    L.qd = L.kd = hd;
+    L.vd = L.od = sp.heads * sp.vdim;
+    L.gate_off = 2 * hd + L.vd;
+    L.pd = L.gate_off + L.vd + sp.decay_rank;  // q | k | v | gate | a1
+    st->max_da = hd > st->max_da ? hd : st->max_da;
+    st->cache_bytes += sizeof(float) * (size_t)sp.heads * sp.vdim * sp.dim;
+    if (own) {
+      L.expect.insert({"mix.q", "mix.k", "mix.v", "mix.g", "mix.a1", "mix.a2", "mix.a2.b", "mix.norm", "mix.o"});
+      TL_TRY(dev_alloc(st, &L.wa2, (size_t)hd * sp.decay_rank));
+      TL_TRY(dev_alloc(st, &L.a_bias, hd));
+      TL_TRY(dev_alloc(st, &L.onorm, sp.vdim));
+    }
+  } else if (sp.mixer == TL_MIXER_LIGHTNING) {
+    TL_REQUIRE(sp.kv_heads == sp.heads && sp.dim <= 512 && decay,
+               "tl_stack_create: layer %d: constant-decay linear attention with %d / %d heads, key size %d (at most 512)%s", i, sp.heads,
+               sp.kv_heads, sp.dim, decay ? "" : ", without its decays");
+    const int hd = sp.heads * sp.dim;
+    L.qd = L.kd = hd;
+    L.vd = L.od = sp.heads * sp.vdim;
+    L.pd = 2 * L.vd + 2 * hd;  // gate | v | k | q
+    const size_t gr = tl_ssm_gram_floats(st->chunk, sp.heads, sp.heads);
+    st->max_gram = gr > st->max_gram ? gr : st->max_gram;
+    st->cache_bytes += sizeof(float) * (size_t)sp.heads * sp.vdim * sp.dim;
+    std::vector<double> ld(sp.heads);
+    for (int n = 0; n < sp.heads; ++n) {
+      TL_REQUIRE(decay[n] >= 0.0 && decay[n] <= 1.0, "tl_stack_create: layer %d: head %d decays by %g", i, n, decay[n]);
+      ld[n] = decay[n] > 0.0 ? log(decay[n]) : -1e4;  // (e^-10000 is 0 in every arithmetic used here)
+      if (ld[n] < -1e4) ld[n] = -1e4;
+    }
+    TL_TRY(dev_alloc(st, &L.log_decay, ld.size()));
+    TL_HIP(hipMemcpy(L.log_decay, ld.data(), sizeof(double) * ld.size(), hipMemcpyHostToDevice));
+    if (own) {
+      L.expect.insert({"mix.q", "mix.k", "mix.v", "mix.g", "mix.norm", "mix.o"});
+      TL_TRY(dev_alloc(st, &L.onorm, L.od));
+    }
   } else if (sp.mixer == TL_MIXER_LINEAR) {
     TL_REQUIRE(sp.kv_heads == sp.heads && sp.dim <= 256 && sp.vdim <= 512,
                "tl_stack_create: layer %d: gated linear attention with %d / %d heads, sizes %d (at most 256) / %d (at most 512)", i,
@@ -468,23 +544,29 @@ int setup_layer(TlStack* st, int i, int* first_mix) {
   const size_t W = cfg->width;
   const bool dyt = cfg->norm == TL_NORM_DYT, rms = cfg->norm == TL_NORM_RMS, lbias = cfg->norm == TL_NORM_LAYER;
   const bool lnorm = lbias || cfg->norm == TL_NORM_LAYER_PLAIN;
+  const bool two = sp.block == TL_BLOCK_PARALLEL_NORMS, first = sp.block == TL_BLOCK_PRE_NORM || two;
   TL_REQUIRE((sp.block == TL_BLOCK_POST_NORM && !dyt && !lnorm && !rms) || (sp.block == TL_BLOCK_PARALLEL && dyt) ||
-                 (sp.block == TL_BLOCK_PRE_NORM && (lnorm || rms)),
+                 (sp.block == TL_BLOCK_PRE_NORM && (lnorm || rms)) || (two && rms),
              "tl_stack_create: layer %d: block kind %d with norm kind %d (post-norm blocks take the one-plus RMS norm, parallel "
-             "blocks the Dynamic Tanh norm, pre-norm blocks the layer norm or the plain RMS norm)", i, sp.block, cfg->norm);
+             "blocks the Dynamic Tanh norm or, with a norm for each sublayer, the plain RMS norm, pre-norm blocks the layer norm or the "
+             "plain RMS norm)", i, sp.block, cfg->norm);
+  TL_REQUIRE(!two || cfg->canon_taps == 0, "tl_stack_create: layer %d: a convolution on what the sublayers read runs in pre-norm blocks only", i);
+  TL_REQUIRE(two == (cfg->layers[0].block == TL_BLOCK_PARALLEL_NORMS), "tl_stack_create: layer %d: parallel blocks with a norm for each "
+             "sublayer do not mix with other blocks", i);
+  TL_REQUIRE(!two || sp.mlp == TL_MLP_NONE || sp.mlp == TL_MLP_DENSE, "tl_stack_create: layer %d: a feed-forward of kind %d in a parallel "
+             "block with a norm for each sublayer", i, sp.mlp);
   TL_REQUIRE(sp.mlp >= TL_MLP_NONE && sp.mlp <= TL_MLP_UNIT, "tl_stack_create: layer %d has feed-forward kind %d", i, sp.mlp);
   TL_REQUIRE(sp.mlp != TL_MLP_DENSE || sp.block != TL_BLOCK_POST_NORM, "tl_stack_create: layer %d: a dense feed-forward "
              "runs in parallel and pre-norm blocks only", i);
   TL_REQUIRE(sp.mlp != TL_MLP_UNIT || sp.block == TL_BLOCK_PRE_NORM,
              "tl_stack_create: layer %d: the plain up / activation / down unit runs in pre-norm blocks only", i);
-  TL_REQUIRE((sp.mixer != TL_MIXER_LATENT && sp.mixer != TL_MIXER_GDELTA && sp.mixer != TL_MIXER_LINEAR && sp.mixer != TL_MIXER_SSM) ||
-                 sp.block == TL_BLOCK_PRE_NORM,
-             "tl_stack_create: layer %d: latent attention, the generalized delta rule, gated linear attention and the state space "
-             "run in pre-norm blocks only", i);
+  TL_REQUIRE(sp.mixer == TL_MIXER_SWA || sp.mixer == TL_MIXER_DELTA || first,
+             "tl_stack_create: layer %d: latent attention, the generalized delta rule, linear attention and the state space run in "
+             "blocks with a norm in front of each sublayer only", i);
   TL_REQUIRE(sp.mixer != TL_MIXER_DELTA || sp.block != TL_BLOCK_POST_NORM, "tl_stack_create: layer %d: the delta rule runs "
              "in parallel and pre-norm blocks only", i);
   TL_REQUIRE(sp.glu == TL_GLU_SWISH || sp.glu == TL_GLU_RELU, "tl_stack_create: layer %d: gated unit of kind %d", i, sp.glu);
-  TL_REQUIRE(!L.side || sp.block == TL_BLOCK_PRE_NORM, "tl_stack_create: layer %d: two mixers side by side run in pre-norm blocks only", i);
+  TL_REQUIRE(!L.side || first, "tl_stack_create: layer %d: two mixers side by side run in blocks with a norm in front of each sublayer only", i);
   L.wsrc = i;
   if (sp.weights_of > 0) {
     TL_REQUIRE(sp.weights_of - 1 < i, "tl_stack_create: layer %d takes its tensors from layer %d, which is not an earlier "
@@ -494,25 +576,47 @@ int setup_layer(TlStack* st, int i, int* first_mix) {
     tl_layer_spec a = sp, b = O.sp;
     a.weights_of = b.weights_of = 0;
     a.side = b.side = nullptr;
+    a.decay = b.decay = nullptr;  // (a constant decay is the layer's own)
     bool same = memcmp(&a, &b, sizeof(a)) == 0 && !L.side == !O.side;
-    if (same && L.side) same = memcmp(&L.side->sp, &O.side->sp, sizeof(a)) == 0;
+    if (same && L.side) {
+      tl_layer_spec sa = L.side->sp, sb = O.side->sp;
+      sa.decay = sb.decay = nullptr;
+      same = memcmp(&sa, &sb, sizeof(sa)) == 0;
+    }
     TL_REQUIRE(same, "tl_stack_create: layer %d differs from layer %d whose tensors it uses", i, L.wsrc);
   }
   const bool own = L.wsrc == i;
   TL_TRY(setup_mixer(st, L, i, own, first_mix));
   if (L.side) {
-    TL_REQUIRE(L.side->sp.mixer == TL_MIXER_SWA || L.side->sp.mixer == TL_MIXER_DELTA || L.side->sp.mixer == TL_MIXER_LINEAR,
-               "tl_stack_create: layer %d: a second mixer of kind %d", i, L.side->sp.mixer);
+    for (const Layer* m : {(const Layer*)&L, (const Layer*)L.side.get()})
+      TL_REQUIRE(m->sp.mixer == TL_MIXER_SWA || m->sp.mixer == TL_MIXER_DELTA || m->sp.mixer == TL_MIXER_LINEAR || m->sp.mixer == TL_MIXER_GLA ||
+                     m->sp.mixer == TL_MIXER_LIGHTNING,
+                 "tl_stack_create: layer %d: a mixer of kind %d in a pair", i, m->sp.mixer);
+    TL_REQUIRE(sp.mixer != TL_MIXER_LIGHTNING || L.side->sp.mixer != TL_MIXER_LIGHTNING,
+               "tl_stack_create: layer %d: two constant-decay mixers in a pair (their products carry an activation)", i);
+    TL_REQUIRE(!sp.side_norm || (cfg->norm == TL_NORM_RMS && cfg->canon_taps == 0),
+               "tl_stack_create: layer %d: norms on the outputs of a pair stand beside plain RMS norms without a convolution", i);
     TL_REQUIRE(!L.side->sp.v_mix && !sp.v_mix, "tl_stack_create: layer %d: value mixing inside a pair of mixers", i);
     L.side->wsrc = L.wsrc;
     TL_TRY(setup_mixer(st, *L.side, i, own, first_mix));
     st->any_pair = true;
+    if (sp.side_norm && own)
+      for (Layer* m : {&L, L.side.get()}) {
+        m->expect.insert("mix.out");
+        TL_TRY(dev_alloc(st, &m->out_norm, W));
+      }
   }
   {  // the first product's matrix; two mixers side by side share one, the second mixer's rows behind the first's: one product
     const int rows = L.pd + (L.side ? L.side->pd : 0);
     if (own) {
       TL_TRY(dev_alloc(st, &L.wqkv, (size_t)rows * W));
       if (L.side) L.side->wqkv = L.wqkv + (size_t)L.pd * W;
+      auto biased = [](const Layer& m) { return m.sp.mixer == TL_MIXER_SWA && m.sp.qkv_bias && m.sp.qkv_conv == 0; };
+      if (biased(L) || (L.side && biased(*L.side))) {
+        TL_TRY(dev_alloc(st, &L.prod_b, rows));
+        TL_HIP(hipMemset(L.prod_b, 0, sizeof(float) * rows));
+        if (L.side) L.side->prod_b = L.prod_b + L.pd;
+      }
     }
     st->max_qkv = rows > st->max_qkv ? rows : st->max_qkv;
   }
@@ -551,7 +655,7 @@ int setup_layer(TlStack* st, int i, int* first_mix) {
   }
   if (cfg->canon_taps > 1) st->cache_bytes += sizeof(float) * (size_t)(cfg->canon_taps - 1) * W * (sp.mlp != TL_MLP_NONE ? 2 : 1);
   // ---- feed-forward ----
-  const bool pre = sp.block == TL_BLOCK_PRE_NORM;
+  const bool pre = first;
   if (sp.mlp == TL_MLP_MOE) {
     TL_REQUIRE(sp.experts > 0 && sp.top > 0 && sp.top <= sp.experts && sp.expert_ff > 0 && sp.shared_ff >= 0,
                "tl_stack_create: layer %d: %d experts, top %d, sizes %d / %d", i, sp.experts, sp.top, sp.expert_ff, sp.shared_ff);
@@ -636,6 +740,8 @@ int tl_stack_create(const tl_stack_config* cfg, TlStack** out) {
   TL_REQUIRE(cfg->canon_taps >= 0 && cfg->canon_taps <= 64 && (cfg->canon_taps == 0 || cfg->norm == TL_NORM_RMS),
              "tl_stack_create: %d taps on what the sublayers read (a convolution there follows the plain RMS norm)", cfg->canon_taps);
   TL_REQUIRE(cfg->norm != TL_NORM_RMS || !cfg->embed_norm, "tl_stack_create: an embedding norm with the plain RMS norm");
+  TL_REQUIRE(cfg->logit_scale == 0.0f || cfg->norm == TL_NORM_RMS, "tl_stack_create: a factor on the logits rides in the final norm's "
+             "weights, which takes the plain RMS norm");
   TlStack* st = new TlStack();
   st->cfg = *cfg;
   st->layers.resize(cfg->n_layers);
@@ -669,6 +775,7 @@ int tl_stack_create(const tl_stack_config* cfg, TlStack** out) {
   if (const char* e = getenv("TL_STACK_GEMV")) st->gemv_decode = atoi(e) != 0;
   if (const char* e = getenv("TL_STACK_FUSE_ROUTER")) st->fuse_router = atoi(e) != 0;
   if (const char* e = getenv("TL_STACK_FORK")) st->fork = atoi(e) != 0;
+  if (const char* e = getenv("TL_STACK_FUSE_STEPS")) st->fuse_steps = atoi(e) != 0;
   if (const char* e = getenv("TL_STACK_FUSE_CANON")) st->fuse_canon = atoi(e) != 0;
   if (const char* e = getenv("TL_STACK_LEAD")) st->lead = atoi(e) > 0 ? atoi(e) : 0;
   if (const char* e = getenv("TL_STACK_EXACT_BELOW")) st->exact_below = atoi(e) > 2 ? atoi(e) : 2;
@@ -718,6 +825,11 @@ int tl_stack_set_tensor(TlStack* st, const char* name, int type, const long long
   if (n == "head") { st->got_globals |= 2; MATRIX(st->head, V, W); }
   if (n == "embed.norm") { st->got_globals |= 4; VECTOR(st->embed_norm, W); }
   if (n == "embed.norm.b") { st->got_globals |= 64; VECTOR(st->embed_norm_b, W); }
+  if (n == "final.norm" && st->cfg.logit_scale != 0.0f) {  // logits = scale head N(x): the factor joins the norm's weights
+    TL_REQUIRE(shape_is(shape, ndim, W), "tl_stack_set_tensor: %s does not have %lld elements", name, W);
+    st->got_globals |= 8;
+    return upload_as_f32(st->final_norm, type, host, (size_t)W, s, st->cfg.logit_scale);
+  }
   if (n == "final.norm") { st->got_globals |= 8; VECTOR(st->final_norm, W); }
   if (n == "final.norm.b") { st->got_globals |= 16; VECTOR(st->final_b, W); }
   if (n == "final.norm.alpha") { st->got_globals |= 32; VECTOR(st->final_alpha, 1); }
@@ -760,6 +872,23 @@ int tl_stack_set_tensor(TlStack* st, const char* name, int type, const long long
       return upload_as_f32(L.hc_mix[q], type, host, (size_t)(ns * ns), s);
     }
   }
+  if (r == "mix.out") VECTOR(L.out_norm, W);
+  if (sp.mixer == TL_MIXER_GLA) {
+    const long long hd = L.qd;
+    if (r == "mix.g") MATRIX(L.wqkv + (size_t)L.gate_off * W, L.vd, W);
+    if (r == "mix.a1") MATRIX(L.wqkv + (size_t)(L.gate_off + L.vd) * W, sp.decay_rank, W);
+    if (r == "mix.a2") MATRIX(L.wa2, hd, sp.decay_rank);
+    if (r == "mix.a2.b") VECTOR(L.a_bias, hd);
+    if (r == "mix.norm") VECTOR(L.onorm, sp.vdim);
+  }
+  if (sp.mixer == TL_MIXER_LIGHTNING) {
+    const long long hd = L.qd, vd = L.vd;
+    if (r == "mix.g") MATRIX(L.wqkv, vd, W);
+    if (r == "mix.v") MATRIX(L.wqkv + (size_t)vd * W, vd, W);
+    if (r == "mix.k") MATRIX(L.wqkv + (size_t)(2 * vd) * W, hd, W);
+    if (r == "mix.q") MATRIX(L.wqkv + (size_t)(2 * vd + hd) * W, hd, W);
+    if (r == "mix.norm") VECTOR(L.onorm, L.od);
+  }
   if (sp.mixer == TL_MIXER_SSM) {
     const long long ch = L.vd + L.kd + L.qd;
     if (r == "mix.in") MATRIX(L.wqkv, L.pd, W);
@@ -787,10 +916,11 @@ int tl_stack_set_tensor(TlStack* st, const char* name, int type, const long long
       if (r == "mix.q.norm") VECTOR(L.q_norm, hd);
       if (r == "mix.k.norm") VECTOR(L.k_norm, hd);
     }
-    if (r == "mix.g") MATRIX(L.wqkv + (size_t)L.gate_off * W, L.od, W);
-    if (r == "mix.q.b") VECTOR(L.qkv_b, L.qd);
-    if (r == "mix.k.b") VECTOR(L.qkv_b + L.qd, L.kd);
-    if (r == "mix.v.b") VECTOR(L.qkv_b + L.qd + L.kd, L.vd);
+    if (r == "mix.g") MATRIX(L.wqkv + (size_t)L.gate_off * W, sp.head_gate ? sp.heads : L.od, W);
+    float* const qb = taps > 0 ? L.qkv_b : L.prod_b;  // in front of the convolution, or in the product itself
+    if (r == "mix.q.b") VECTOR(qb, L.qd);
+    if (r == "mix.k.b") VECTOR(qb + L.qd, L.kd);
+    if (r == "mix.v.b") VECTOR(qb + L.qd + L.kd, L.vd);
     if (r == "mix.q.conv") MATRIX(L.conv, L.qd, taps);
     if (r == "mix.k.conv") MATRIX(L.conv + (size_t)L.qd * taps, L.kd, taps);
     if (r == "mix.v.conv") MATRIX(L.conv + (size_t)(L.qd + L.kd) * taps, L.vd, taps);
@@ -980,7 +1110,7 @@ int tl_stack_finalize(TlStack* st, hipStream_t s) {
         L.hist = p;
         p += (size_t)(L.sp.qkv_conv - 1) * (L.qd + L.kd + L.vd);
       }
-    } else if (L.sp.mixer == TL_MIXER_LINEAR) {
+    } else if (L.sp.mixer == TL_MIXER_LINEAR || L.sp.mixer == TL_MIXER_GLA || L.sp.mixer == TL_MIXER_LIGHTNING) {
       L.state = p;
       p += (size_t)L.sp.heads * L.sp.vdim * L.sp.dim;
     } else if (L.sp.mixer == TL_MIXER_LATENT) {
@@ -1015,12 +1145,13 @@ int tl_stack_finalize(TlStack* st, hipStream_t s) {
   if (st->max_gram) TL_TRY(dev_alloc(st, &st->gram, st->max_gram));
   TL_TRY(dev_alloc(st, &st->x, C * W));
   TL_TRY(dev_alloc(st, &st->h, C * W));
+  if (st->layers[0].sp.block == TL_BLOCK_PARALLEL_NORMS) TL_TRY(dev_alloc(st, &st->h2, C * W));
   TL_TRY(dev_alloc(st, &st->qkv, C * st->max_qkv));
   TL_TRY(dev_alloc(st, &st->att, C * st->max_od));
   TL_TRY(dev_alloc(st, &st->proj, C * W));
   TL_TRY(dev_alloc(st, &st->v_first, C * st->max_vd));
   TL_TRY(dev_alloc(st, &st->xn, C * W));
-  if (st->max_dc) {
+  if (st->max_dc || st->max_da) {
     TL_TRY(dev_alloc(st, &st->dq, C * st->max_dc));
     if (st->max_da > st->max_gd) st->max_gd = st->max_da;  // one buffer serves both recurrences' decay pre-activations
     TL_TRY(dev_alloc(st, &st->ddecay, C * st->max_da));
@@ -1057,7 +1188,7 @@ int tl_stack_finalize(TlStack* st, hipStream_t s) {
         const Layer& L = *Lp;
         if (L.sp.mixer != TL_MIXER_SWA && L.sp.mixer != TL_MIXER_LATENT) continue;
         const bool lat = L.sp.mixer == TL_MIXER_LATENT;
-        const int splits = tl_swa_splits(T, L.sp.window, st->cfg.max_positions, lat ? 0 : L.sp.keep_first);
+        const int splits = tl_swa_splits(T, swa_bound(L.sp), st->cfg.max_positions, lat ? 0 : L.sp.keep_first);
         // (latent rows: the shared-row kernel may cut finer, up to 64)
         const size_t n = tl_swa_ws_floats(T, L.sp.heads, lat ? L.sp.kv_rank : L.sp.vdim, lat ? 64 : splits);
         ws = n > ws ? n : ws;
@@ -1082,7 +1213,8 @@ int tl_stack_finalize(TlStack* st, hipStream_t s) {
     if (st->max_sff) TL_TRY(dev_alloc(st, &st->sact, C * st->max_sff));
   }
   bool any_parallel = false;
-  for (const Layer& L : st->layers) any_parallel |= L.sp.block == TL_BLOCK_PARALLEL && L.sp.mlp != TL_MLP_NONE;
+  for (const Layer& L : st->layers)
+    any_parallel |= (L.sp.block == TL_BLOCK_PARALLEL || L.sp.block == TL_BLOCK_PARALLEL_NORMS) && L.sp.mlp != TL_MLP_NONE;
   if (st->fork && any_parallel) {
     TL_HIP(hipStreamCreateWithFlags(&st->side, hipStreamNonBlocking));
     TL_HIP(hipEventCreateWithFlags(&st->ev_fork, hipEventDisableTiming));
@@ -1144,6 +1276,7 @@ int tl_stack_cache_ptr(TlStack* st, int which, int layer, void** out) {
   }
   const Layer& L = *Lp;
   // attention: 0 keys, 1 values; delta rule and linear attention: 0 the state S [heads][vdim][dim], 1 the convolution's history
+  // channel-decay linear attention: 0 the state [heads][vdim][dim]; constant decay: 0 the state [heads][dim][vdim]
   // latent attention: 0 the rows [max_pos][kv_rank + rot_dim] this layer reads; generalized delta rule: 0 the state
   if (L.sp.mixer == TL_MIXER_SWA) *out = which == 0 ? L.kc : L.vc;
   else if (L.sp.mixer == TL_MIXER_LATENT) *out = L.ckv;
@@ -1184,11 +1317,12 @@ void tl_stack_bytes_per_token(const TlStack* st, int pos, double* weight_bytes, 
       kb += 2.0 * 4.0 * sp.heads * sp.dim * sp.dim;
       continue;
     }
-    if (sp.mixer == TL_MIXER_DELTA || sp.mixer == TL_MIXER_LINEAR) {
+    if (sp.mixer == TL_MIXER_DELTA || sp.mixer == TL_MIXER_LINEAR || sp.mixer == TL_MIXER_GLA || sp.mixer == TL_MIXER_LIGHTNING) {
       wb += 2.0 * ((double)sp.heads * sp.dim * sp.decay_rank + (double)L.vd * sp.gate_rank);
       kb += 2.0 * 4.0 * sp.heads * sp.vdim * sp.dim;  // the state is read and written
     } else {
       double seen = sp.window > 0 && pos + 1 > sp.window ? sp.window : pos + 1;
+      if (sp.chunk > 0 && pos % sp.chunk + 1 < seen) seen = pos % sp.chunk + 1;
       if (sp.window > 0 && sp.keep_first > 0 && pos + 1 > sp.window)
         seen += sp.keep_first < pos + 1 - sp.window ? sp.keep_first : pos + 1 - sp.window;
       kb += 4.0 * (seen + 1.0) * (L.kd + L.vd);
@@ -1224,6 +1358,47 @@ int project(TlStack* st, const uint16_t* w, int rows, int cols, const float* x, 
   d.terms = terms_for(st, T);
   d.softcap = softcap;
   return tl_launch_dense_gemm(d, s);
+}
+
+// y = act(W x + bias) on a range of the rows (GemvActArgs); terms 0: what the engine uses for T tokens
+int project_act(TlStack* st, const uint16_t* w, int rows, int cols, const float* x, int ldx, float* y, int ldy, int T,
+                const GemvActArgs& act, hipStream_t s, int terms = 0) {
+  if (T == 1 && st->gemv_decode) return tl_launch_dense_gemv_act(w, rows, cols, x, y, act, s);
+  DenseArgs d = {};
+  d.w = w;
+  d.rows = rows;
+  d.cols = cols;
+  d.x = x;
+  d.ldx = ldx;
+  d.y = y;
+  d.ldy = ldy;
+  d.T = T;
+  d.terms = terms ? terms : terms_for(st, T);
+  d.act = act.act;
+  d.act_from = act.act_from;
+  d.act_to = act.act_to;
+  d.act_p = act.act_p;
+  d.act_q = act.act_q;
+  d.bias = act.bias;
+  return tl_launch_dense_gemm(d, s);
+}
+
+// The first product of a layer's mixer, or of both mixers of a pair (their matrices lie one behind the other), into st->qkv:
+// with the biases of its columns and the activation of a constant-decay mixer's
+int first_product(TlStack* st, const Layer& L, const Layer& Wt, const float* in, int T, hipStream_t s) {
+  const int W = st->cfg.width, rows = L.pd + (L.side ? L.side->pd : 0);
+  GemvActArgs act = {};
+  act.bias = Wt.prod_b;
+  if (L.sp.mixer == TL_MIXER_LIGHTNING) {
+    act.act = TL_ACT_SILU;
+    act.act_from = L.vd;
+    act.act_to = L.pd;
+  } else if (L.side && L.side->sp.mixer == TL_MIXER_LIGHTNING) {
+    act.act = TL_ACT_SILU;
+    act.act_from = L.pd + L.side->vd;
+    act.act_to = rows;
+  }
+  return project_act(st, Wt.wqkv, rows, W, in, W, st->qkv, rows, T, act, s);
 }
 
 // The routed experts (and the shared expert) of layer L on the rows of `in` (x itself for a post-norm block, the normalised
@@ -1377,7 +1552,7 @@ int swa_mixer(TlStack* st, Layer& L, const Layer& Wt, const float* in, int T, in
   float* const row0 = qkv;  // the product's rows (the gate columns stay there when q | k | v move on)
   const int ld0 = ld;
   if (!out) out = st->proj;
-  if (!pre) TL_TRY(project(st, Wt.wqkv, ld, W, in, W, st->qkv, ld, T, s));
+  if (!pre) TL_TRY(first_product(st, L, Wt, in, T, s));
   if (sp.qkv_conv > 0) {  // q | k | v (+ their biases) through a convolution over time; the rest of the row is not touched
     ConvArgs cv = {};
     cv.in = qkv;
@@ -1405,6 +1580,11 @@ int swa_mixer(TlStack* st, Layer& L, const Layer& Wt, const float* in, int T, in
     r.freq = Wt.freq;
     r.mscale = Wt.mscale;
     r.unit_norm = sp.qk_norm == TL_QK_NORM_HEAD_UNIT;
+    r.halves = sp.rot_halves;
+    if (sp.qk_norm == TL_QK_NORM_HEAD_RMS) {
+      r.q_norm = Wt.q_norm;
+      r.k_norm = Wt.k_norm;
+    }
     r.eps = c.norm_eps;
     r.kc = L.kc;
     if (sp.values_are_keys) {
@@ -1465,7 +1645,12 @@ int swa_mixer(TlStack* st, Layer& L, const Layer& Wt, const float* in, int T, in
   a.softcap = sp.score_softcap;
   a.dist_r1 = sp.dist_bias ? Wt.r1 : nullptr;
   a.dist_r2 = sp.dist_bias ? Wt.r2 : nullptr;
-  a.nsplit = tl_swa_splits(T, sp.window, c.max_positions, sp.keep_first);
+  a.chunk = sp.chunk;
+  if (sp.head_gate) {
+    a.gate = row0 + L.gate_off;
+    a.gate_ld = ld0;
+  }
+  a.nsplit = tl_swa_splits(T, swa_bound(sp), c.max_positions, sp.keep_first);
   a.ws = st->swa_ws;
   a.done_cnt = st->swa_cnt;
   if (sp.score_maps == 2) {
@@ -1611,6 +1796,106 @@ int linear_mixer(TlStack* st, Layer& L, const Layer& Wt, const float* in, int T,
   return project(st, Wt.wo, W, L.od, st->att, L.od, out, W, T, s);
 }
 
+// linear attention with a decay per key channel: q | k | v | gate | a1 = W h; alpha = sigmoid(W_a2 a1 + b)^(1 / tau) in the epilogue
+// of its product, the scan, gated head norm -- or, for one token, all of it in one launch; W_o
+int gla_mixer(TlStack* st, Layer& L, const Layer& Wt, const float* in, int T, hipStream_t s, float* out = nullptr,
+              float* pre = nullptr, int pre_ld = 0) {
+  const tl_layer_spec& sp = L.sp;
+  const int W = st->cfg.width, ld = pre ? pre_ld : L.pd, hd = L.qd, rank = sp.decay_rank;
+  float* const P = pre ? pre : st->qkv;
+  if (!out) out = st->proj;
+  if (!pre) TL_TRY(first_product(st, L, Wt, in, T, s));
+  const float power = (float)(1.0 / (double)sp.decay_tau), q_scale = (float)(1.0 / sqrt((double)sp.dim));
+  if (T == 1 && st->gemv_decode && st->fuse_steps && tl_gla_step_fits(sp.dim, sp.vdim, rank)) {
+    GlaStepArgs a = {};
+    a.p = P;
+    a.a2 = Wt.wa2;
+    a.a2_b = Wt.a_bias;
+    a.rank = rank;
+    a.power = power;
+    a.q_scale = q_scale;
+    a.norm = Wt.onorm;
+    a.eps = st->cfg.norm_eps;
+    a.state = L.state;
+    a.o = st->att;
+    a.heads = sp.heads;
+    a.dim = sp.dim;
+    a.vdim = sp.vdim;
+    TL_TRY(tl_launch_gla_step(a, s));
+    return project(st, Wt.wo, W, L.od, st->att, L.od, out, W, T, s);
+  }
+  // (the inner size is small: FP32-grade products cost nothing there, and what enters the recurrence stays exact)
+  TL_TRY(project_act(st, Wt.wa2, hd, rank, P + L.gate_off + L.vd, ld, st->ddecay, hd, T,
+                     GemvActArgs{TL_ACT_SIGMOID_POWER, 0, power, 0.0f, 0, Wt.a_bias}, s, 3));
+  DeltaScanArgs d = {};
+  d.q = P;
+  d.k = P + hd;
+  d.ldq = ld;
+  d.v = P + 2 * hd;
+  d.ldv = ld;
+  d.g = st->ddecay;
+  d.state = L.state;
+  d.o = st->att;
+  d.T = T;
+  d.heads = sp.heads;
+  d.kv_heads = sp.heads;
+  d.dim = sp.dim;
+  d.vdim = sp.vdim;
+  d.plain_write = 1;
+  d.q_scale = q_scale;
+  TL_TRY(tl_launch_delta_scan(d, s));
+  HeadNormArgs hn = {};
+  hn.o = st->att;
+  hn.gate = P + L.gate_off;
+  hn.gate_ld = ld;
+  hn.gate_act = 1;
+  hn.w = Wt.onorm;
+  hn.out_scale = 1.0f;
+  hn.T = T;
+  hn.heads = sp.heads;
+  hn.vdim = sp.vdim;
+  hn.eps = st->cfg.norm_eps;
+  TL_TRY(tl_launch_head_norm(hn, s));
+  return project(st, Wt.wo, W, L.od, st->att, L.od, out, W, T, s);
+}
+
+// linear attention with a constant decay per head: gate | silu(v | k | q) = W h; the recurrence; RMS norm of the row times the gate; W_o
+int lightning_mixer(TlStack* st, Layer& L, const Layer& Wt, const float* in, int T, hipStream_t s, float* out = nullptr,
+                    float* pre = nullptr, int pre_ld = 0) {
+  const tl_layer_spec& sp = L.sp;
+  const int W = st->cfg.width, ld = pre ? pre_ld : L.pd;
+  float* const P = pre ? pre : st->qkv;
+  if (!out) out = st->proj;
+  if (!pre) TL_TRY(first_product(st, L, Wt, in, T, s));
+  if (T == 1 && st->gemv_decode) {
+    TL_TRY(tl_launch_lightning_step(LightningStepArgs{P + L.vd, L.log_decay, L.state, st->att, sp.heads, sp.dim, sp.vdim}, s));
+  } else {
+    SsmScanArgs a = {};
+    a.xbc = P + L.vd;
+    a.ld = ld;
+    a.log_decay = L.log_decay;
+    a.state = L.state;
+    a.y = st->att;
+    a.gram = st->gram;
+    a.T = T;
+    a.heads = a.groups = sp.heads;
+    a.state_n = sp.dim;
+    a.vdim = sp.vdim;
+    TL_TRY(tl_launch_ssm_scan(a, s));
+  }
+  PartNormArgs n = {};
+  n.x = st->att;
+  n.w = Wt.onorm;
+  n.T = T;
+  n.width = L.od;
+  n.parts = 1;
+  n.eps = st->cfg.norm_eps;
+  n.gate = P;
+  n.gate_ld = ld;
+  TL_TRY(tl_launch_part_norm(n, s));
+  return project(st, Wt.wo, W, L.od, st->att, L.od, out, W, T, s);
+}
+
 // one product per head: y[t][n * y_stride ..] = W[n] x[t][n * x_stride ..]
 int project_heads(TlStack* st, const uint16_t* w, int heads, int rows, int cols, const float* x, int ldx, int x_stride, float* y,
                   int ldy, int y_stride, int T, hipStream_t s) {
@@ -1628,27 +1913,6 @@ int project_heads(TlStack* st, const uint16_t* w, int heads, int rows, int cols,
   d.groups = heads;
   d.x_gstride = x_stride;
   d.y_gstride = y_stride;
-  return tl_launch_dense_gemm(d, s);
-}
-
-// y = act(W x) on the rows from act_from on
-int project_act(TlStack* st, const uint16_t* w, int rows, int cols, const float* x, int ldx, float* y, int ldy, int T, int act,
-                int act_from, float act_p, float act_q, hipStream_t s) {
-  if (T == 1 && st->gemv_decode) return tl_launch_dense_gemv_act(w, rows, cols, x, y, GemvActArgs{act, act_from, act_p, act_q}, s);
-  DenseArgs d = {};
-  d.w = w;
-  d.rows = rows;
-  d.cols = cols;
-  d.x = x;
-  d.ldx = ldx;
-  d.y = y;
-  d.ldy = ldy;
-  d.T = T;
-  d.terms = terms_for(st, T);
-  d.act = act;
-  d.act_from = act_from;
-  d.act_p = act_p;
-  d.act_q = act_q;
   return tl_launch_dense_gemm(d, s);
 }
 
@@ -1764,7 +2028,7 @@ int gdelta_mixer(TlStack* st, Layer& L, const float* in, int T, hipStream_t s) {
   const tl_layer_spec& sp = L.sp;
   const int W = st->cfg.width, ld = L.pd, hd = sp.heads * sp.dim;
   // r | k | v | gate | a | tanh(w1 h)
-  TL_TRY(project_act(st, L.wqkv, ld, W, in, W, st->qkv, ld, T, TL_ACT_TANH, 5 * hd, 0.0f, 0.0f, s));
+  TL_TRY(project_act(st, L.wqkv, ld, W, in, W, st->qkv, ld, T, GemvActArgs{TL_ACT_TANH, 5 * hd, 0.0f, 0.0f, 0, nullptr}, s));
   TL_TRY(project(st, L.wa2, hd, sp.decay_rank, st->qkv + 5 * hd, ld, st->da, hd, T, s));
   GDeltaPreArgs p = {};
   p.p = st->qkv;
@@ -1887,6 +2151,7 @@ struct Addends {
   float a_scale = 1.0f;
   const float* b = nullptr;
   float b_scale = 1.0f;
+  const float *a_w = nullptr, *b_w = nullptr;  // RMS norms of a and b in front of their factors
   const float* slots = nullptr;
   const float* slot_w = nullptr;
   int top = 0;
@@ -1944,6 +2209,23 @@ int finish_x(TlStack* st, const Addends& add, Layer* next, int which, int T, hip
     return tl_launch_resid_ln(st->x, add.a, T, W, n, c.norm_eps, st->h, s);
   }
   const bool canon = c.canon_taps > 0 && Wn;
+  if (add.a_w) {  // a normed pair (no convolution on what the sublayers read beside it)
+    TL_REQUIRE(!canon && !add.slots, "layer-list engine: a normed pair with experts' outputs or a convolution");
+    ResidNormsArgs n = {};
+    n.x = st->x;
+    n.T = T;
+    n.width = W;
+    n.a = add.a;
+    n.a_w = add.a_w;
+    n.a_scale = add.a_scale;
+    n.b = add.b;
+    n.b_w = add.b_w;
+    n.b_scale = add.b_scale;
+    n.w1 = Wn ? (which == 1 ? Wn->norm1 : Wn->norm2) : nullptr;
+    n.h1 = st->h;
+    n.eps = c.norm_eps;
+    return tl_launch_resid_norms(n, s);
+  }
   ResidRmsArgs r = {};
   r.x = st->x;
   r.T = T;
@@ -1995,6 +2277,8 @@ int run_mixer(TlStack* st, Layer& L, const Layer& Wt, int T, int start_pos, cons
     case TL_MIXER_GDELTA: return gdelta_mixer(st, L, st->h, T, s);
     case TL_MIXER_SSM: return ssm_mixer(st, L, st->h, T, s);
     case TL_MIXER_LINEAR: return linear_mixer(st, L, Wt, st->h, T, s, out, pre, pre_ld);
+    case TL_MIXER_GLA: return gla_mixer(st, L, Wt, st->h, T, s, out, pre, pre_ld);
+    case TL_MIXER_LIGHTNING: return lightning_mixer(st, L, Wt, st->h, T, s, out, pre, pre_ld);
     default: return delta_mixer(st, L, Wt, st->h, T, s, out, pre, pre_ld);
   }
 }
@@ -2037,6 +2321,24 @@ int dense_unit(TlStack* st, const Layer& L, const Layer& Wt, const float* in, in
   return project(st, Wt.sdown, W, ff, st->sact, ff, st->sout, W, T, s);
 }
 
+// The mixer of a layer, or both mixers of a pair, on st->h: what they add to the residual
+int run_mixers(TlStack* st, Layer& L, const Layer& Wt, int T, int start_pos, const int* pos_dev, hipStream_t s, Addends* add) {
+  add->a = st->proj;
+  if (!L.side) return run_mixer(st, L, Wt, T, start_pos, pos_dev, s, st->proj);
+  const int ld = L.pd + L.side->pd;  // one first product; each mixer then works on its columns
+  TL_TRY(first_product(st, L, Wt, st->h, T, s));
+  TL_TRY(run_mixer(st, L, Wt, T, start_pos, pos_dev, s, st->proj, st->qkv, ld));
+  TL_TRY(run_mixer(st, *L.side, *Wt.side, T, start_pos, pos_dev, s, st->proj2, st->qkv + L.pd, ld));
+  add->a_scale = L.sp.mix_scale;
+  add->b = st->proj2;
+  add->b_scale = L.sp.side_scale;
+  if (L.sp.side_norm) {
+    add->a_w = Wt.out_norm;
+    add->b_w = Wt.side->out_norm;
+  }
+  return 0;
+}
+
 // h = the input of the mixer is already in st->h. x += mixer(h) (two mixers side by side: the weighted sum of both); then,
 // with a feed-forward, h = its input from the new x, x += ff(h). The launch that finishes x prepares the input of whatever
 // reads it next.
@@ -2044,32 +2346,17 @@ int pre_norm_layer(TlStack* st, size_t li, int T, int start_pos, const int* pos_
   Layer& L = st->layers[li];
   const Layer& Wt = st->layers[L.wsrc];
   const tl_layer_spec& sp = L.sp;
-  const tl_stack_config& c = st->cfg;
-  const int W = c.width;
+  const int W = st->cfg.width;
   Layer* after = li + 1 < st->layers.size() ? &st->layers[li + 1] : nullptr;
   Addends mix;
-  mix.a = st->proj;
-  if (L.side) {
-    // both mixers' first products as one (their matrices lie one behind the other); each then works on its columns
-    const int ld = L.pd + L.side->pd;
-    TL_TRY(project(st, Wt.wqkv, ld, W, st->h, W, st->qkv, ld, T, s));
-    TL_TRY(run_mixer(st, L, Wt, T, start_pos, pos_dev, s, st->proj, st->qkv, ld));
-    TL_TRY(run_mixer(st, *L.side, *Wt.side, T, start_pos, pos_dev, s, st->proj2, st->qkv + L.pd, ld));
-  } else {
-    TL_TRY(run_mixer(st, L, Wt, T, start_pos, pos_dev, s, st->proj, nullptr, 0));
-  }
-  if (L.side) {
-    mix.a_scale = sp.mix_scale;
-    mix.b = st->proj2;
-    mix.b_scale = sp.side_scale;
-  }
+  TL_TRY(run_mixers(st, L, Wt, T, start_pos, pos_dev, s, &mix));
   if (sp.mlp == TL_MLP_NONE) return finish_x(st, mix, after, 1, T, s, nullptr, &L, 1);
   bool routed = false;
   TL_TRY(finish_x(st, mix, &L, 2, T, s, &routed, &L, 1));
   Addends ffo;
   if (sp.mlp == TL_MLP_UNIT) {
     const int ff = sp.shared_ff;
-    TL_TRY(project_act(st, Wt.sgu, ff, W, st->h, W, st->sact, ff, T, sp.act, 0, Wt.act_p, Wt.act_q, s));
+    TL_TRY(project_act(st, Wt.sgu, ff, W, st->h, W, st->sact, ff, T, GemvActArgs{sp.act, 0, Wt.act_p, Wt.act_q, 0, nullptr}, s));
     TL_TRY(project(st, Wt.sdown, W, ff, st->sact, ff, st->sout, W, T, s));
     ffo.a = st->sout;
   } else if (sp.mlp == TL_MLP_DENSE) {
@@ -2088,6 +2375,50 @@ int pre_norm_layer(TlStack* st, size_t li, int T, int start_pos, const int* pos_
     }
   }
   return finish_x(st, ffo, after, 1, T, s, nullptr, &L, 2);
+}
+
+// what finishes x in front of a parallel block with a norm for each sublayer: x += add + ff, then both norms of `next` (NULL: none)
+int finish_two(TlStack* st, const Addends& add, const float* ff, const Layer* next, int T, hipStream_t s) {
+  ResidNormsArgs n = {};
+  n.x = st->x;
+  n.T = T;
+  n.width = st->cfg.width;
+  n.a = add.a;
+  n.a_w = add.a_w;
+  n.a_scale = add.a_scale;
+  n.b = add.b;
+  n.b_w = add.b_w;
+  n.b_scale = add.b_scale;
+  n.c = ff;
+  n.eps = st->cfg.norm_eps;
+  if (next) {
+    const Layer& Wn = st->layers[next->wsrc];
+    n.w1 = Wn.norm1;
+    n.h1 = st->h;
+    if (next->sp.mlp != TL_MLP_NONE) {
+      n.w2 = Wn.norm2;
+      n.h2 = st->h2;
+    }
+  }
+  return tl_launch_resid_norms(n, s);
+}
+
+// h = norm1(x), h2 = norm2(x) (already in st->h, st->h2); x += mixer(h) + ff(h2), and the next block's norms in the same launch. One
+// token: the feed-forward on the second stream, as in parallel_layer
+int parallel_norms_layer(TlStack* st, size_t li, int T, int start_pos, const int* pos_dev, hipStream_t s) {
+  Layer& L = st->layers[li];
+  const Layer& Wt = st->layers[L.wsrc];
+  const bool ff = L.sp.mlp != TL_MLP_NONE, forked = st->fork && T == 1 && ff;
+  if (forked) {
+    TL_HIP(hipEventRecord(st->ev_fork, s));
+    TL_HIP(hipStreamWaitEvent(st->side, st->ev_fork, 0));
+  }
+  if (ff) TL_TRY(dense_unit(st, L, Wt, st->h2, T, forked ? st->side : s));
+  if (forked) TL_HIP(hipEventRecord(st->ev_join, st->side));
+  Addends mix;
+  TL_TRY(run_mixers(st, L, Wt, T, start_pos, pos_dev, s, &mix));
+  if (forked) TL_HIP(hipStreamWaitEvent(s, st->ev_join, 0));
+  return finish_two(st, mix, ff ? st->sout : nullptr, li + 1 < st->layers.size() ? &st->layers[li + 1] : nullptr, T, s);
 }
 
 DytParams dyt_of_layer(const Layer& Wt) { return DytParams{Wt.norm1_alpha, Wt.norm1, Wt.norm1_b}; }
@@ -2162,7 +2493,8 @@ int tl_stack_forward(TlStack* st, const int* tokens_dev, int T, int start_pos, c
   } else if (c.norm == TL_NORM_RMS) {
     TL_TRY(tl_launch_embed_rows(st->embed, c.vocab, W, tokens_dev, T, st->x, DytParams{}, st->h, s,
                                 c.embed_scale != 0.0f ? c.embed_scale : 1.0f));
-    TL_TRY(finish_x(st, Addends{}, &st->layers[0], 1, T, s));
+    if (st->layers[0].sp.block == TL_BLOCK_PARALLEL_NORMS) TL_TRY(finish_two(st, Addends{}, nullptr, &st->layers[0], T, s));
+    else TL_TRY(finish_x(st, Addends{}, &st->layers[0], 1, T, s));
   } else if (lnorm) {
     const LnParams emb = LnParams{st->embed_norm, c.norm == TL_NORM_LAYER ? st->embed_norm_b : nullptr};
     TL_TRY(tl_launch_embed_ln(st->embed, c.vocab, W, tokens_dev, T, emb, ln1_of_layer(st->layers[st->layers[0].wsrc]), c.norm_eps,
@@ -2179,6 +2511,8 @@ int tl_stack_forward(TlStack* st, const int* tokens_dev, int T, int start_pos, c
     const tl_layer_spec& sp = L.sp;
     if (sp.block == TL_BLOCK_PARALLEL) {
       TL_TRY(parallel_layer(st, li, T, start_pos, pos_dev, s));
+    } else if (sp.block == TL_BLOCK_PARALLEL_NORMS) {
+      TL_TRY(parallel_norms_layer(st, li, T, start_pos, pos_dev, s));
     } else if (sp.block == TL_BLOCK_PRE_NORM) {
       TL_TRY(pre_norm_layer(st, li, T, start_pos, pos_dev, s));
     } else {

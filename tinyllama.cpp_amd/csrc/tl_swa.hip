@@ -6,6 +6,8 @@
 // With a sink the softmax's denominator has one more term exp(0): where partial (max, sum) pairs are merged, the maximum is
 // taken together with 0 and exp(-max) joins the sum once. The rows of the caches may be further apart than a row is wide
 // (kld, vld): a cache of latent rows is read as keys over its whole row and as values over its first vdim columns.
+// With chunk > 0 a position sees only the keys of its own chunk of so many positions (counted from position 0); with gate set a
+// head's output is multiplied by the sigmoid of one number where it is finished.
 // Sigmoid mode runs through the softmax machinery with the running maximum pinned to 0: every correction factor is exp(0) = 1,
 // the partial sums of waves and splits are simply added, and the final division falls away.
 //
@@ -37,6 +39,20 @@ __device__ __forceinline__ float swa_cap(float sc, float cap, float inv_cap) {
 }
 __device__ __forceinline__ float swa_dist(float r1, float r2, int d) { return r1 * __logf(1.0f + r2 * (float)d); }
 
+// first position that position i sees (kept first keys aside)
+__device__ __forceinline__ int swa_first_key(const SwaArgs& a, int i) {
+  int lo = a.window > 0 && i - a.window + 1 > 0 ? i - a.window + 1 : 0;
+  if (a.chunk > 0) {
+    const int c = i - i % a.chunk;
+    lo = c > lo ? c : lo;
+  }
+  return lo;
+}
+// the factor on the finished output of a (token, head)
+__device__ __forceinline__ float swa_out_factor(const SwaArgs& a, int t, int h) {
+  return a.gate ? 1.0f / (1.0f + expf(-a.gate[(size_t)t * a.gate_ld + h])) : 1.0f;
+}
+
 __device__ __forceinline__ void swa_st_agent(float* p, float v) {
   __hip_atomic_store(p, v, __ATOMIC_RELAXED, __HIP_MEMORY_SCOPE_AGENT);
 }
@@ -60,6 +76,7 @@ __device__ __forceinline__ void swa_merge_records(const SwaArgs& a, int t, int h
   float L = a.sink ? expf(sv - M) : 0.0f;
   for (int z = 0; z < a.nsplit; ++z) L += __shfl(lz * fz, z);  // in split order
   float* op = a.out + (size_t)t * a.heads * a.vdim + (size_t)h * a.vdim;
+  const float of = swa_out_factor(a, t, h);
   for (int d0 = 0; d0 < a.vdim; d0 += 64) {  // every lane stays in the loop: a shuffle reads nothing from a lane that has left
     const int d = d0 + lane;
     float acc = 0.0f;
@@ -78,7 +95,7 @@ __device__ __forceinline__ void swa_merge_records(const SwaArgs& a, int t, int h
 #pragma unroll
       for (int u = 0; u < 8; ++u) acc += v[u] * f[u];  // in split order
     }
-    if (d < a.vdim) op[d] = a.sigmoid ? acc : acc / L;
+    if (d < a.vdim) op[d] = (a.sigmoid ? acc : acc / L) * of;
   }
 }
 
@@ -91,7 +108,7 @@ __global__ __launch_bounds__(256) void swa_kernel(const SwaArgs a) {
   const int tid = threadIdx.x, wave = tid >> 6, lane = tid & 63;
   const int i = (a.pos_dev ? *a.pos_dev : a.start_pos) + t;
   const int g = h / (a.heads / a.kv_heads);
-  const int jlo = (a.window > 0 && i - a.window + 1 > 0) ? i - a.window + 1 : 0;
+  const int jlo = swa_first_key(a, i);
   const int n = i - jlo + 1;
   // kept first keys that lie before the window: pieces [0, pf) walk them, pieces [pf, pieces) the window
   const int nf = a.keep_first > 0 ? (a.keep_first < jlo ? a.keep_first : jlo) : 0;
@@ -246,11 +263,12 @@ __global__ __launch_bounds__(256) void swa_kernel(const SwaArgs a) {
     return;
   }
   float* op = a.out + (size_t)t * a.heads * a.vdim + (size_t)h * a.vdim;
+  const float of = swa_out_factor(a, t, h);
   for (int d = tid; d < a.vdim; d += 256) {
     float acc = 0.0f;
 #pragma unroll
     for (int w = 0; w < SWA_WAVES; ++w) acc += f[w] == 0.0f ? 0.0f : ow[w * a.vdim + d] * f[w];
-    op[d] = a.sigmoid ? acc : acc / L;
+    op[d] = (a.sigmoid ? acc : acc / L) * of;
   }
 }
 
@@ -485,7 +503,7 @@ __global__ __launch_bounds__(256, 2) void swa_mfma_kernel(const SwaArgs a) {  //
   const int last_i = q0 + 31 < a.T ? q0 + 31 : a.T - 1;
   const int qpos = start + (q0 + r < a.T ? q0 + r : a.T - 1);  // rows beyond the chunk repeat its last query; never stored
   const int last_q = start + last_i;
-  const int klo = a.window > 0 && start + q0 - a.window + 1 > 0 ? start + q0 - a.window + 1 : 0;
+  const int klo = swa_first_key(a, start + q0), qlo = swa_first_key(a, qpos);
   const int t_lo = klo >> 5, t_hi = last_q >> 5;
   // kept first keys: their tiles of 32 positions below the window's first tile are walked before the window's tiles
   // (virtual tile vt < tf is tile vt, vt >= tf is tile t_lo + vt - tf)
@@ -592,7 +610,7 @@ __global__ __launch_bounds__(256, 2) void swa_mfma_kernel(const SwaArgs a) {  //
 #pragma unroll
     for (int e = 0; e < 16; ++e) {
       const int p = p0 + swa_acc_row(e, h);
-      const bool seen = p <= qpos && (a.window <= 0 || qpos - p < a.window || p < a.keep_first);
+      const bool seen = p <= qpos && (p >= qlo || p < a.keep_first);
       float sc = s[e] * a.scale;
       if (a.softcap > 0.0f) sc = swa_cap(sc, a.softcap, inv_cap);
       if (a.dist_r1) sc -= swa_dist(r1, r2, seen ? qpos - p : 0);
@@ -651,7 +669,7 @@ __global__ __launch_bounds__(256, 2) void swa_mfma_kernel(const SwaArgs a) {  //
         const float m2 = sm_m[w * 32 + r];
         L += m2 == -INFINITY ? 0.0f : sm_l[w * 32 + r] * expf(m2 - M);
       }
-      sm_inv[r] = a.sigmoid ? 1.0f : 1.0f / L;
+      sm_inv[r] = (a.sigmoid ? 1.0f : 1.0f / L) * (q0 + r < a.T ? swa_out_factor(a, q0 + r, head) : 1.0f);
     }
   }
   __syncthreads();
@@ -718,7 +736,7 @@ int tl_swa_shared_splits(const SwaArgs& a, int max_pos) {
     return !e || atoi(e) != 0;
   }();
   if (!on || a.T > 4 || a.kv_heads != 1 || a.heads < 8 || a.kc != a.vc || a.kld != a.vld || a.kld <= 0 || a.sigmoid || a.sink ||
-      a.softcap > 0.0f || a.dist_r1 || a.keep_first || a.q_hstride || a.k_hstride || a.vdim > a.dim || a.vdim > 512 ||
+      a.softcap > 0.0f || a.dist_r1 || a.keep_first || a.chunk || a.gate || a.q_hstride || a.k_hstride || a.vdim > a.dim || a.vdim > 512 ||
       a.dim > 64 * SH_MAX_K || (a.dim & 3) || (a.kld & 3) || (a.ldq & 3) || ((size_t)a.kc & 15) || ((size_t)a.q & 15) ||
       sizeof(float) * swa_shared_lds_floats(a.dim) > 160 * 1024)
     return 0;
@@ -738,6 +756,7 @@ int tl_launch_swa(const SwaArgs& a, hipStream_t s) {
   TL_REQUIRE(a.keep_first >= 0, "swa: negative number of kept first keys");
   TL_REQUIRE(!a.sink || !a.sigmoid, "swa: a sink belongs to a softmax");
   TL_REQUIRE(!a.sink_val || a.sink, "swa: sink scores without a sink");
+  TL_REQUIRE(a.chunk >= 0 && (!a.gate || a.gate_ld >= a.heads), "swa: chunks of %d, gate rows of %d for %d heads", a.chunk, a.gate_ld, a.heads);
   TL_REQUIRE(!a.dist_r1 == !a.dist_r2, "swa: the distance bias needs both of its vectors");
   TL_REQUIRE(a.q_hstride >= 0 && a.k_hstride >= 0 && (a.q_hstride == 0 || a.q_hstride >= a.dim) &&
                  (a.k_hstride == 0 || a.k_hstride >= a.dim),
@@ -900,6 +919,34 @@ extern "C" int tl_window_attention_opts(const float* q_dev, int ldq, int q_hstri
   a.shared = a.nsplit > 0;
   if (!a.shared) a.nsplit = tl_swa_splits(num_tokens, window, start_pos + num_tokens, 0);
   if (a.nsplit > 1 || a.shared) {
+    void* ws = nullptr;
+    TL_TRY(tl_scratch(TL_SCRATCH_ATTN, sizeof(float) * tl_swa_ws_floats(num_tokens, heads, vdim, a.nsplit), &ws));
+    a.ws = static_cast<float*>(ws);
+  }
+  return tl_launch_swa(a, static_cast<hipStream_t>(stream));
+}
+
+extern "C" int tl_chunk_attention(const float* q_dev, const float* k_cache_dev, const float* v_cache_dev, float* out_dev,
+                                  int num_tokens, int start_pos, int heads, int kv_heads, int dim, int vdim, int chunk,
+                                  float scale, const float* gate_dev, int gate_ld, void* stream) {
+  SwaArgs a = {};
+  a.q = q_dev;
+  a.ldq = heads * dim;
+  a.kc = k_cache_dev;
+  a.vc = v_cache_dev;
+  a.out = out_dev;
+  a.T = num_tokens;
+  a.heads = heads;
+  a.kv_heads = kv_heads;
+  a.dim = dim;
+  a.vdim = vdim;
+  a.chunk = chunk > 0 ? chunk : 0;
+  a.scale = scale;
+  a.gate = gate_dev;
+  a.gate_ld = gate_ld;
+  a.start_pos = start_pos;
+  a.nsplit = tl_swa_splits(num_tokens, chunk, start_pos + num_tokens);
+  if (a.nsplit > 1) {
     void* ws = nullptr;
     TL_TRY(tl_scratch(TL_SCRATCH_ATTN, sizeof(float) * tl_swa_ws_floats(num_tokens, heads, vdim, a.nsplit), &ws));
     a.ws = static_cast<float*>(ws);

@@ -586,6 +586,52 @@ def _madudra_spec(sp, i, L):
         sp.act, sp.expert_ff = 3, ml["expert"]["ff"]
 
 
+def _ratuzen_spec(sp, i, L, sides, tensors):
+    """Fills entry i; a pair's second mixer goes to sides[i]. Returns what has to outlive the model's creation."""
+    mx, ml, keep = L["mixer"], L.get("mlp"), None
+    sp.block = 3
+
+    def sizes(m, to):
+        to.heads, to.kv_heads, to.dim, to.vdim = m["heads"], m.get("kv_heads", m["heads"]), m["dim"], m.get("vdim", m["dim"])
+
+    if L["type"] == "delta":
+        sp.mixer, sp.conv_taps, sp.decay_per_head = 1, mx["conv"], 1
+        sizes(mx, sp)
+    elif L["type"] in ("parallel", "parallel_2"):
+        lt, rt, r = mx["left"], mx["right"], sides[i]
+        sp.mixer, sp.scale = 0, float(lt["scale"])
+        sizes(lt, sp)
+        sizes(rt, r)
+        rot = lt.get("rot")
+        if rot:
+            sp.rot_dims, sp.rot_base = rot["dims"], float(rot["base"])
+            sc = rot.get("scaling")
+            if sc:
+                sp.rot_factor, sp.rot_scaling = float(sc["factor"]), 1
+                if "original" in sc:
+                    sp.rot_scaling, sp.rot_original = 2, float(sc["original"])
+                    sp.rot_fast, sp.rot_slow = float(sc["high"]), float(sc["low"])
+        if L["type"] == "parallel":
+            sp.qkv_bias, sp.chunk = 1, int((lt.get("mask") or {}).get("size", 0))
+            keep = (C.c_double * len(rt["decay"]))(*rt["decay"])
+            if len(keep) != r.heads:
+                raise ValueError(f"layer {i}: {len(keep)} decays for {r.heads} heads")
+            r.mixer, r.decay = 7, C.cast(keep, C.POINTER(C.c_double))
+        else:
+            sp.qk_norm, sp.rot_halves, sp.head_gate = 3, 1, 1
+            r.mixer, r.decay_tau, r.decay_rank = 6, float(rt["tau"]), int(np.shape(tensors[f"l{i}.mix.right.a1"])[0])
+        r.block = 3
+        sp.side = C.pointer(r)
+        sp.mix_scale, sp.side_scale, sp.side_norm = 0.5, 0.5, 1
+    else:
+        raise ValueError(f"layer {i}: unknown type {L['type']!r}")
+    if ml is not None:
+        if ml["kind"] != "dense":
+            raise ValueError(f"layer {i}: unknown feed-forward kind {ml['kind']!r}")
+        sp.mlp, sp.shared_ff, sp.shared_limit, sp.act_alpha, sp.glu_up_add = 2, ml["ff"], float(ml["limit"]), 1.702, 1.0
+    return keep
+
+
 def stack_config_struct(config, max_pos, tensors=None):
     """The ctypes form (tl_stack_config) of a layer-list configuration given as config.json's dictionary; returns
     (struct, the array it points into). The C++ host does the same from the file (host/tl_stack_config.cpp); this one
@@ -594,12 +640,16 @@ def stack_config_struct(config, max_pos, tensors=None):
     arr = (capi.LayerSpec * len(layers))()
     madalorn, sogalix = config.get("architecture") == "Madalorn", config.get("architecture") == "Sogalix"
     potipel, madudra = config.get("architecture") == "Potipel", config.get("architecture") == "Madudra"
+    ratuzen = config.get("architecture") == "Ratuzen"
+    keep = []
     sides = (capi.LayerSpec * len(layers))()
     for i, L in enumerate(layers):
         if potipel:
             _potipel_spec(arr[i], i, L, sides)
         elif madudra:
             _madudra_spec(arr[i], i, L)
+        elif ratuzen:
+            keep.append(_ratuzen_spec(arr[i], i, L, sides, tensors or {}))
         elif madalorn:
             _madalorn_spec(arr[i], i, L, tensors or {}, layers)
         elif sogalix:
@@ -607,13 +657,14 @@ def stack_config_struct(config, max_pos, tensors=None):
         else:
             _ralasun_spec(arr[i], i, L)
     c = capi.StackConfig(config["width"], config["vocab"], len(layers), int(max_pos), float(config["norm"]["eps"]), arr,
-                         1 if madalorn else 2 if sogalix else 3 if potipel else 4 if madudra else 0,
-                         0 if madalorn or potipel or madudra else 1,
+                         1 if madalorn else 2 if sogalix else 3 if potipel or ratuzen else 4 if madudra else 0,
+                         0 if madalorn or potipel or madudra or ratuzen else 1,
                          float(config.get("logit_softcap") or 0.0) if madalorn else 0.0,
                          float(config["embedding"]["scale"]) if potipel or madudra else 0.0,
                          int(config["canon"]["taps"]) if potipel else 0, int(config["streams"]) if madudra else 0,
-                         float(config["residual_mult"]) if madudra else 0.0)
-    return c, (arr, sides)
+                         float(config["residual_mult"]) if madudra else 0.0,
+                         float(config["logit_scale"]) if ratuzen else 0.0)
+    return c, (arr, sides, keep)
 
 
 class StackModel(Model):

@@ -20,6 +20,7 @@ const std::vector<ModelFamily>& model_families() {
       {"Sogalix", "folder", load_stack_folder},
       {"Potipel", "folder", load_stack_folder},
       {"Madudra", "folder", load_stack_folder},
+      {"Ratuzen", "folder", load_stack_folder},
   };
   return table;
 }

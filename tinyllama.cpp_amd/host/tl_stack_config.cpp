@@ -54,6 +54,17 @@
 //               "rot": {"base", "dims", "scaling": {"factor", "original", "fast", "slow"}}, "kv_from": j} |
 //              {"heads", "vdim", "state", "groups", "conv", "norm_groups"},
 //     "mlp": null | {"kind": "moe", "router": {"experts", "top", "scale"}, "expert": {"ff"}}}]}
+// Ratuzen   parallel blocks whose two sublayers read the same residual behind a plain RMS norm each; three mixers: "parallel" = rotated
+//           softmax attention inside chunks (biases on q, k, v, frequencies scaled by wavelength) beside linear attention with one constant
+//           decay per head; "parallel_2" = causal softmax attention (q/k RMS norms per head in front of a rotation in halves with linearly
+//           scaled frequencies, a gate per head) beside linear attention with a decay per key channel; both pairs are half the sum of the
+//           RMS-normed outputs; "delta" = gated delta rule with one decay per head. Feed-forward: a clamped 1.702-swish unit. Scaled logits.
+//   {"architecture", "width", "vocab", "norm": {"eps"}, "logit_scale", "layers": [{"type": "parallel" | "parallel_2" | "delta",
+//     "mixer": {"left": {"heads", "kv_heads", "dim", "vdim", "scale", "mask": {"size"},
+//                        "rot": {"base", "dims", "scaling": {"factor"} | {"factor", "low", "high", "original"}}},
+//               "right": {"heads", "dim", "vdim", "decay": [..]} | {"heads", "dim", "vdim", "tau"}} |
+//              {"heads", "kv_heads", "dim", "vdim", "conv"},
+//     "mlp": null | {"kind": "dense", "ff", "limit"}}]}
 #include <chrono>
 #include <cmath>
 #include <fstream>
@@ -138,6 +149,24 @@ void read_rotation(const Json& mx, tl_layer_spec* sp) {
     sp->rot_original = getf(*sc, "original");
     sp->rot_fast = getf(*sc, "fast");
     sp->rot_slow = getf(*sc, "slow");
+  }
+}
+
+// a window-less rotation whose scaling is by wavelength when it names low / high / original, else by the factor alone
+void read_scaled_rotation(const Json& mx, tl_layer_spec* sp) {
+  const Json* rot = present(mx, "rot");
+  if (!rot) return;
+  sp->rot_dims = geti(*rot, "dims");
+  sp->rot_base = getf(*rot, "base");
+  const Json* sc = present(*rot, "scaling");
+  if (!sc) return;
+  sp->rot_factor = getf(*sc, "factor");
+  sp->rot_scaling = TL_ROT_LINEAR;
+  if (present(*sc, "original")) {
+    sp->rot_scaling = TL_ROT_WAVELENGTH;
+    sp->rot_original = getf(*sc, "original");
+    sp->rot_fast = getf(*sc, "high");
+    sp->rot_slow = getf(*sc, "low");
   }
 }
 
@@ -400,6 +429,71 @@ tl_layer_spec potipel_layer(const Json& layers, int index, tl_layer_spec* side) 
   return sp;
 }
 
+// `side` receives the second mixer of a pair, `decay` its constant decays (the entries point at both)
+tl_layer_spec ratuzen_layer(const Json& layers, int index, const SafeTensorsFile& file, tl_layer_spec* side, std::vector<double>* decay) {
+  const Json& L = layers.arr[index];
+  const std::string where = "layers[" + std::to_string(index) + "]";
+  tl_layer_spec sp = {};
+  const std::string& type = L.at("type").as_string("type");
+  const Json& mx = L.at("mixer");
+  auto head_sizes = [](const Json& m, tl_layer_spec* to) {
+    to->heads = geti(m, "heads");
+    to->kv_heads = present(m, "kv_heads") ? geti(m, "kv_heads") : to->heads;
+    to->dim = geti(m, "dim");
+    to->vdim = present(m, "vdim") ? geti(m, "vdim") : to->dim;
+  };
+  if (type == "delta") {
+    sp.mixer = TL_MIXER_DELTA;
+    head_sizes(mx, &sp);
+    sp.conv_taps = geti(mx, "conv");
+    sp.decay_per_head = 1;
+  } else if (type == "parallel" || type == "parallel_2") {
+    const bool first = type == "parallel";
+    const Json &lt = mx.at("left"), &rt = mx.at("right");
+    sp.mixer = TL_MIXER_SWA;
+    head_sizes(lt, &sp);
+    sp.scale = getf(lt, "scale");
+    read_scaled_rotation(lt, &sp);
+    tl_layer_spec r = {};
+    head_sizes(rt, &r);
+    if (first) {
+      sp.qkv_bias = 1;
+      if (const Json* mask = present(lt, "mask")) sp.chunk = geti(*mask, "size");
+      r.mixer = TL_MIXER_LIGHTNING;
+      for (const Json& d : rt.at("decay").arr) decay->push_back(d.as_double("decay"));
+      if ((int)decay->size() != r.heads)
+        throw std::runtime_error(where + ": " + std::to_string(decay->size()) + " decays for " + std::to_string(r.heads) + " heads");
+      r.decay = decay->data();
+    } else {
+      sp.qk_norm = TL_QK_NORM_HEAD_RMS;
+      sp.rot_halves = 1;
+      sp.head_gate = 1;
+      r.mixer = TL_MIXER_GLA;
+      r.decay_tau = getf(rt, "tau");
+      r.decay_rank = tensor_rows(file, "l" + std::to_string(index) + ".mix.right.a1");
+    }
+    r.block = TL_BLOCK_PARALLEL_NORMS;
+    *side = r;
+    sp.side = side;
+    sp.mix_scale = sp.side_scale = 0.5f;
+    sp.side_norm = 1;
+  } else {
+    throw std::runtime_error(where + ": unknown layer type \"" + type + "\"");
+  }
+  sp.block = TL_BLOCK_PARALLEL_NORMS;
+  if (const Json* ml = present(L, "mlp")) {
+    const std::string& kind = ml->at("kind").as_string("kind");
+    if (kind != "dense") throw std::runtime_error(where + ": unknown feed-forward kind \"" + kind + "\"");
+    sp.mlp = TL_MLP_DENSE;
+    sp.glu = TL_GLU_SWISH;
+    sp.act_alpha = kGateAlpha;
+    sp.glu_up_add = 1.0f;
+    sp.shared_ff = geti(*ml, "ff");
+    sp.shared_limit = getf(*ml, "limit");
+  }
+  return sp;
+}
+
 }  // namespace
 
 void load_stack_folder(const std::string& dir, int device, int max_context, LoadedModel* out) {
@@ -413,15 +507,17 @@ void load_stack_folder(const std::string& dir, int device, int max_context, Load
   if (layers.kind != Json::ARRAY || layers.arr.empty()) throw std::runtime_error("config.json: \"layers\" is empty");
   const std::string arch = cfg.at("architecture").as_string("architecture");
   const bool madalorn = arch == "Madalorn", sogalix = arch == "Sogalix", potipel = arch == "Potipel",
-             madudra = arch == "Madudra";
+             madudra = arch == "Madudra", ratuzen = arch == "Ratuzen";
   SafeTensorsFile file;
   file.open(dir + "/model.safetensors");
   std::vector<tl_layer_spec> specs, sides(layers.arr.size());  // (sides: second mixers, addressed by the entries of specs)
+  std::vector<std::vector<double>> decays(layers.arr.size());
   for (size_t i = 0; i < layers.arr.size(); ++i)
     specs.push_back(madalorn  ? madalorn_layer(layers, (int)i, file)
                     : sogalix ? sogalix_layer(layers, (int)i, file)
                     : potipel ? potipel_layer(layers, (int)i, &sides[i])
                     : madudra ? madudra_layer(layers, (int)i)
+                    : ratuzen ? ratuzen_layer(layers, (int)i, file, &sides[i], &decays[i])
                               : ralasun_layer(layers.arr[i], (int)i, file));
   tl_stack_config sc = {};
   sc.width = geti(cfg, "width");
@@ -430,8 +526,13 @@ void load_stack_folder(const std::string& dir, int device, int max_context, Load
   sc.max_positions = max_context > 0 ? max_context : kDefaultContext;
   sc.norm_eps = (float)cfg.at("norm").at("eps").as_double("norm.eps");
   sc.layers = specs.data();
-  sc.norm = madalorn ? TL_NORM_DYT : sogalix ? TL_NORM_LAYER : potipel ? TL_NORM_RMS : madudra ? TL_NORM_LAYER_PLAIN : TL_NORM_RMS_ONE_PLUS;
-  sc.embed_norm = madalorn || potipel || madudra ? 0 : 1;
+  sc.norm = madalorn ? TL_NORM_DYT
+            : sogalix ? TL_NORM_LAYER
+            : potipel || ratuzen ? TL_NORM_RMS
+            : madudra ? TL_NORM_LAYER_PLAIN
+                      : TL_NORM_RMS_ONE_PLUS;
+  sc.embed_norm = madalorn || potipel || madudra || ratuzen ? 0 : 1;
+  if (ratuzen) sc.logit_scale = getf(cfg, "logit_scale");
   if (potipel || madudra) sc.embed_scale = (float)cfg.at("embedding").at("scale").as_double("embedding.scale");
   if (madudra) {
     sc.streams = geti(cfg, "streams");

@@ -733,6 +733,109 @@ def build_madudra(config, seed=0, gain=1.0):
     return t
 
 
+def ratuzen_chunked(heads, kv_heads, dim, vdim, chunk, right_heads, right_dim, right_vdim, decay, base=10000.0, rot_dims=None,
+                    scaling=None, scale=None):
+    """Mixer of a "parallel" layer. scaling: None or (factor, low, high, original)."""
+    rot = {"base": float(base), "dims": rot_dims if rot_dims is not None else dim}
+    if scaling is not None:
+        rot["scaling"] = dict(zip(("factor", "low", "high", "original"), scaling))
+    left = {"heads": heads, "kv_heads": kv_heads, "dim": dim, "vdim": vdim, "rot": rot,
+            "scale": float(scale if scale is not None else dim ** -0.5)}
+    if chunk:
+        left["mask"] = {"size": int(chunk)}
+    return {"left": left, "right": {"heads": right_heads, "dim": right_dim, "vdim": right_vdim, "decay": [float(d) for d in decay]}}
+
+
+def ratuzen_causal(heads, kv_heads, dim, vdim, right_heads, right_dim, right_vdim, tau=16.0, base=10000.0, rot_dims=None, factor=None,
+                   scale=None):
+    """Mixer of a "parallel_2" layer. factor: of the linear frequency scaling."""
+    rot = {"base": float(base), "dims": rot_dims if rot_dims is not None else dim}
+    if factor is not None:
+        rot["scaling"] = {"factor": float(factor)}
+    return {"left": {"heads": heads, "kv_heads": kv_heads, "dim": dim, "vdim": vdim, "rot": rot,
+                     "scale": float(scale if scale is not None else dim ** -0.5)},
+            "right": {"heads": right_heads, "dim": right_dim, "vdim": right_vdim, "tau": float(tau)}}
+
+
+def ratuzen_delta(heads, kv_heads, dim, vdim, conv=4):
+    return {"heads": heads, "kv_heads": kv_heads, "dim": dim, "vdim": vdim, "conv": conv}
+
+
+def ratuzen_layer(kind, mixer, ff=None, limit=1.5):
+    """kind: "parallel" | "parallel_2" | "delta"; ff: None or the gated unit's size."""
+    return {"type": kind, "mixer": mixer, "mlp": None if ff is None else {"kind": "dense", "ff": ff, "limit": float(limit)}}
+
+
+def ratuzen_config(width, vocab, layers, eps=1e-6, logit_scale=1.5):
+    return {"architecture": "Ratuzen", "layers": list(layers), "logit_scale": float(logit_scale), "norm": {"eps": float(eps)},
+            "vocab": int(vocab), "width": int(width)}
+
+
+def build_ratuzen(config, seed=0, gain=1.0, rank=8):
+    """Random tensors {checkpoint name: uint16 bf16 bits} of a Ratuzen configuration; rank: rows of the decay's inner projection."""
+    rng = np.random.default_rng(seed)
+    W, V = config["width"], config["vocab"]
+    t = {}
+
+    def mat(name, rows, cols, std=None):
+        t[name] = to_bf16(rng.standard_normal((rows, cols)).astype(np.float32) * (std or gain / np.sqrt(cols)))
+
+    def vec(name, n, centre, spread):
+        t[name] = to_bf16((centre + spread * rng.standard_normal(n)).astype(np.float32))
+
+    mat("embed", V, W, 1.0)
+    vec("final.norm", W, 1.0, 0.1)
+    mat("head", V, W, 4.0 / np.sqrt(W))
+    for i, L in enumerate(config["layers"]):
+        mx, ml, p = L["mixer"], L.get("mlp"), f"l{i}."
+        vec(p + "norm1", W, 1.0, 0.1)
+        if L["type"] == "delta":
+            q, H, G, d, dv = p + "mix.", mx["heads"], mx["kv_heads"], mx["dim"], mx["vdim"]
+            for n, rows in (("q", G * d), ("k", G * d), ("v", H * dv)):
+                mat(q + n, rows, W, 2.0 / np.sqrt(W))
+                mat(q + n + ".conv", rows, mx["conv"], 0.5)
+            mat(q + "b", H, W, 2.0 / np.sqrt(W))
+            mat(q + "a", H, W, 2.0 / np.sqrt(W))
+            vec(q + "A_log", H, -1.0, 1.0)
+            vec(q + "dt_bias", H, 0.0, 1.0)
+            vec(q + "norm", dv, 1.0, 0.1)
+            mat(q + "g", H * dv, W, 2.0 / np.sqrt(W))
+            mat(q + "o", W, H * dv)
+        else:
+            lt, rt, q = mx["left"], mx["right"], p + "mix.left."
+            H, G, d, dv = lt["heads"], lt["kv_heads"], lt["dim"], lt["vdim"]
+            for n, rows in (("q", H * d), ("k", G * d), ("v", G * dv)):
+                mat(q + n, rows, W, 2.0 / np.sqrt(W))
+                if L["type"] == "parallel":
+                    vec(q + n + ".b", rows, 0.0, 0.3)
+            if L["type"] == "parallel_2":
+                vec(q + "q.norm", d, 1.5, 0.3)
+                vec(q + "k.norm", d, 1.5, 0.3)
+                mat(q + "g", H, W, 2.0 / np.sqrt(W))
+            mat(q + "o", W, H * dv)
+            vec(q + "out", W, 1.0, 0.1)
+            q = p + "mix.right."
+            H, d, dv = rt["heads"], rt["dim"], rt["vdim"]
+            for n, rows in (("q", H * d), ("k", H * d), ("v", H * dv)):
+                mat(q + n, rows, W, 2.0 / np.sqrt(W))
+            mat(q + "g", H * dv, W, 2.0 / np.sqrt(W))
+            if L["type"] == "parallel_2":
+                mat(q + "a1", rank, W, 2.0 / np.sqrt(W))
+                mat(q + "a2", H * d, rank, 2.0 / np.sqrt(rank))
+                vec(q + "a2.b", H * d, 0.0, 1.0)
+                vec(q + "norm", dv, 1.0, 0.1)
+            else:
+                vec(q + "norm", H * dv, 1.0, 0.1)
+            mat(q + "o", W, H * dv)
+            vec(q + "out", W, 1.0, 0.1)
+        if ml is not None:
+            vec(p + "norm2", W, 1.0, 0.1)
+            mat(p + "mlp.gate", ml["ff"], W, 2.0 / np.sqrt(W))
+            mat(p + "mlp.up", ml["ff"], W, 2.0 / np.sqrt(W))
+            mat(p + "mlp.down", W, ml["ff"])
+    return t
+
+
 def write_stack_dir(path, config, tensors):
     """config.json + model.safetensors (8-byte little-endian header length, JSON header, data) under `path`."""
     import json
