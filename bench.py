@@ -52,8 +52,10 @@ def parse():
     ap.add_argument("--prompt-len", type=int, default=4)
     ap.add_argument("--no-cpu-baseline", action="store_true")
     ap.add_argument("--cpu-layers", type=int, default=8, help="layers in the CPU-baseline sample")
-    ap.add_argument("--family", default=None, choices=[None, "ralasun", "madalorn", "sogalix", "potipel", "madudra"],
-                    help="madudra: prefill / decode throughput of that layer-list design at --sizes beside a Sogalix model of "
+    ap.add_argument("--family", default=None, choices=[None, "ralasun", "madalorn", "sogalix", "potipel", "madudra", "ratuzen"],
+                    help="ratuzen: prefill / decode throughput of that layer-list design at --sizes beside a Potipel model of equal size "
+                         "(pairs of mixers behind plain RMS norms there too); "
+                         "madudra: prefill / decode throughput of that layer-list design at --sizes beside a Sogalix model of "
                          "equal size (latent attention behind layer norms there too); potipel: prefill / decode throughput of that layer-list design at --sizes beside a Madalorn model of "
                          "equal size; sogalix: prefill / decode throughput of that layer-list design at --sizes beside a Madalorn model of "
                          "equal size; madalorn: prefill / decode throughput of that layer-list design at --sizes beside a Ralasun model of "
@@ -410,8 +412,70 @@ def _build_madudra(S, engine, z, max_pos, rng, pool):
     return m, per_tok / n
 
 
+def _build_ratuzen(S, engine, z, max_pos, rng, pool):
+    """Pair with causal attention and channel-decay linear attention, delta rule, pair with chunked attention (chunks as long as the
+    other families' windows) and constant-decay linear attention, in turn; every linear mixer has as many heads of the same size as
+    the attention beside it. Every layer has one gated unit with as many columns as the other families' feed-forward uses per token."""
+    W, V, H, G, d, n = z["width"], z["vocab"], z["heads"], z["kv_heads"], z["dim"], z["layers"]
+    F, rank = z["top"] * z["ff"] + z["shared_ff"], 16
+    layers = []
+    for i in range(n):
+        if i % 3 == 0:
+            layers.append(S.ratuzen_layer("parallel_2", S.ratuzen_causal(H, G, d, d, H, d, d, tau=16.0, base=500000.0, factor=4.0), F, 7.0))
+        elif i % 3 == 1:
+            layers.append(S.ratuzen_layer("delta", S.ratuzen_delta(H, G, d, d, conv=4), F, 7.0))
+        else:
+            layers.append(S.ratuzen_layer("parallel", S.ratuzen_chunked(H, G, d, d, z["window"], H, d, d, np.exp(-np.linspace(0.5, 0.002, H)),
+                                                                        base=50000.0, scaling=(4.0, 1.0, 4.0, 4096)), F, 7.0))
+    cfg = S.ratuzen_config(W, V, layers, logit_scale=1.0)
+    shapes = {f"l{i}.mix.right.a1": np.empty((rank, W), np.uint16) for i, L in enumerate(layers) if L["type"] == "parallel_2"}
+    m = engine.StackModel(cfg, max_pos, tensors=shapes)
+
+    def mat(nm, r, c, std=None):
+        m.set_tensor(nm, _pool_bf16(S, r * c, std or 1.0 / np.sqrt(c), rng, pool).reshape(r, c))
+
+    def vec(nm, k, centre, spread=0.05):
+        m.set_tensor(nm, S.to_bf16((centre + spread * rng.standard_normal(k)).astype(np.float32)))
+
+    mat("embed", V, W, 1.0), mat("head", V, W), vec("final.norm", W, 1.0)
+    per_tok = 0
+    for i, L in enumerate(layers):
+        p = f"l{i}."
+        vec(p + "norm1", W, 1.0), vec(p + "norm2", W, 1.0)
+        if L["type"] == "delta":
+            q = p + "mix."
+            for nm, rows in (("q", G * d), ("k", G * d), ("v", H * d)):
+                mat(q + nm, rows, W), mat(q + nm + ".conv", rows, 4, 0.5)
+            mat(q + "b", H, W), mat(q + "a", H, W), mat(q + "g", H * d, W), mat(q + "o", W, H * d)
+            vec(q + "A_log", H, -1.0, 0.3), vec(q + "dt_bias", H, -1.0, 0.3), vec(q + "norm", d, 1.0)
+            per_tok += (2 * G * d + 3 * H * d + 2 * H) * W
+        else:
+            two = L["type"] == "parallel_2"
+            q = p + "mix.left."
+            for nm, rows in (("q", H * d), ("k", G * d), ("v", G * d)):
+                mat(q + nm, rows, W)
+                if not two:
+                    vec(q + nm + ".b", rows, 0.0)
+            if two:
+                vec(q + "q.norm", d, 1.0), vec(q + "k.norm", d, 1.0), mat(q + "g", H, W)
+            mat(q + "o", W, H * d), vec(q + "out", W, 1.0)
+            q = p + "mix.right."
+            for nm in "qkvg":
+                mat(q + nm, H * d, W)
+            mat(q + "o", W, H * d), vec(q + "out", W, 1.0), vec(q + "norm", d if two else H * d, 1.0)
+            if two:
+                mat(q + "a1", rank, W), mat(q + "a2", H * d, rank), vec(q + "a2.b", H * d, 1.0, 0.5)
+            per_tok += (2 * H * d + 2 * G * d + 5 * H * d) * W + (H * W + rank * (W + H * d) if two else 0)
+        mat(p + "mlp.gate", F, W), mat(p + "mlp.up", F, W), mat(p + "mlp.down", W, F)
+        per_tok += 3 * W * F
+    m.finalize()
+    return m, per_tok / n
+
+
 # family -> (builder, layers in words, the closest earlier family's name, its builder)
 FAMILIES = {
+    "ratuzen": (_build_ratuzen, "parallel_2 (causal attention | channel decay) / delta / parallel (chunked attention | constant decay) in turn",
+                "potipel", _build_potipel),
     "madudra": (_build_madudra, "mamba2 / latent_attention / mamba2 / latent_attention (shared cache) in turn", "sogalix", _build_sogalix),
     "potipel": (_build_potipel, "parallel (window attention | delta rule) / differential attention / hgrn2 in turn", "madalorn", _build_madalorn),
     "sogalix": (_build_sogalix, "latent_attention / general_delta / attention / general_delta in turn", "madalorn", _build_madalorn),

@@ -173,7 +173,7 @@ class RatuzenOracle:
         q = rotate(q.reshape(T, H, d), pos, f, False)
         k = self.append(i, "k", rotate(k.reshape(T, G, d), pos, f, False))
         v = self.append(i, "v", v.reshape(T, G, vd))
-        o = softmax_attention(q, k, v, mx["scale"], pos, mx["mask"]["size"])
+        o = softmax_attention(q, k, v, mx["scale"], pos, (mx.get("mask") or {}).get("size", 0))
         return o.reshape(T, -1) @ w[p + "o"].T
 
     def normed_attention(self, i, mx, p, h, pos):
