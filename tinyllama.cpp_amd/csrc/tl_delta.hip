@@ -31,6 +31,8 @@
 //                together, so a token again costs one reduction latency.
 #include <math.h>
 
+#include <type_traits>
+
 #include "tl_bf16.h"
 #include "tl_stack.h"
 
@@ -126,7 +128,8 @@ __device__ __forceinline__ float row16_sum(float x) {
 // The operands of 16 (8 for the largest key size) tokens at a time (k, q, g of the head; v of the workgroup's 16 columns; beta) are staged in LDS by
 // all threads together, the next stage's global loads in flight while the tokens of the stage in hand are walked: a token
 // then waits for an LDS read, not for a round trip to memory.
-template <int E>
+// PLAIN (plain_write): s <- g s + k u does not wait for any sum over the state, and o = s . q afterwards is the only one
+template <int E, bool PLAIN>
 __global__ __launch_bounds__(256) void delta_scan_kernel(const DeltaScanArgs a) {
   constexpr int DELTA_TB = E == 16 ? 8 : 16;  // tokens per stage (48 KB of LDS at most)
   constexpr int DP = 16 * E;                 // padded key size
@@ -191,6 +194,17 @@ __global__ __launch_bounds__(256) void delta_scan_kernel(const DeltaScanArgs a) 
       }
       const float vc = sv_[b][tt][cl], bc = sb_[b][tt];
       float sk = 0.0f, sq = 0.0f, kq = 0.0f;
+      if (PLAIN) {
+        const float u = bc * vc;
+#pragma unroll
+        for (int e = 0; e < E; ++e) {
+          s[e] = s[e] * gc[e] + kc[e] * u;
+          sq += s[e] * qc[e];
+        }
+        sq = row16_sum(sq);
+        if (live && sub == 0) a.o[(size_t)(t0 + tt) * a.heads * a.vdim + (size_t)h * a.vdim + col] = sq * oscale;
+        continue;
+      }
 #pragma unroll
       for (int e = 0; e < E; ++e) {
         s[e] *= gc[e];
@@ -201,7 +215,7 @@ __global__ __launch_bounds__(256) void delta_scan_kernel(const DeltaScanArgs a) 
       sk = row16_sum(sk);
       sq = row16_sum(sq);
       kq = row16_sum(kq);
-      const float u = a.plain_write ? bc * vc : bc * (vc - sk);
+      const float u = bc * (vc - sk);
 #pragma unroll
       for (int e = 0; e < E; ++e) s[e] += kc[e] * u;
       if (live && sub == 0) a.o[(size_t)(t0 + tt) * a.heads * a.vdim + (size_t)h * a.vdim + col] = (sq + u * kq) * oscale;
@@ -517,11 +531,16 @@ int tl_launch_delta_scan(const DeltaScanArgs& a, hipStream_t s) {
   TL_REQUIRE(a.dim <= 256, "delta_scan: key size %d above 256", a.dim);
   const dim3 grid((a.vdim + 15) / 16, a.heads);
   const int e = (a.dim + 15) / 16;
-  if (e <= 1) delta_scan_kernel<1><<<grid, 256, 0, s>>>(a);
-  else if (e <= 2) delta_scan_kernel<2><<<grid, 256, 0, s>>>(a);
-  else if (e <= 4) delta_scan_kernel<4><<<grid, 256, 0, s>>>(a);
-  else if (e <= 8) delta_scan_kernel<8><<<grid, 256, 0, s>>>(a);
-  else delta_scan_kernel<16><<<grid, 256, 0, s>>>(a);
+  auto launch = [&](auto plain) {
+    constexpr bool P = decltype(plain)::value;
+    if (e <= 1) delta_scan_kernel<1, P><<<grid, 256, 0, s>>>(a);
+    else if (e <= 2) delta_scan_kernel<2, P><<<grid, 256, 0, s>>>(a);
+    else if (e <= 4) delta_scan_kernel<4, P><<<grid, 256, 0, s>>>(a);
+    else if (e <= 8) delta_scan_kernel<8, P><<<grid, 256, 0, s>>>(a);
+    else delta_scan_kernel<16, P><<<grid, 256, 0, s>>>(a);
+  };
+  if (a.plain_write) launch(std::true_type{});
+  else launch(std::false_type{});
   TL_HIP(hipGetLastError());
   return 0;
 }

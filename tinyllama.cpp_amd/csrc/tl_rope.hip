@@ -74,7 +74,21 @@ __global__ __launch_bounds__(256) void rotary_kernel(const RotaryArgs a) {
   const double dpos = (double)pos;
   const int kd = a.kv_heads * a.dim;
   const int half = a.rot_dims >> 1;
-  // a wave per head: workgroup y of a token takes heads 4 y .. 4 y + 3 (one token of a decode step still fills several CUs)
+  // the angles are the same for every head: formed once
+  float sns[kMaxPairs], css[kMaxPairs];
+#pragma unroll
+  for (int r = 0; r < kMaxPairs; ++r) {
+    const int i = lane + 64 * r;
+    sns[r] = 0.0f, css[r] = a.mscale;
+    if (i < half) {
+      const double full = dpos * a.freq[i];
+      const float ang = (float)(full - 6.283185307179586476925 * rint(full * 0.159154943091895335769));
+      sincosf(ang, &sns[r], &css[r]);
+      sns[r] *= a.mscale;
+      css[r] *= a.mscale;
+    }
+  }
+  // a wave per head: workgroup y of a token takes heads 4 y .. 4 y + 3, then those 4 gridDim.y further on (one token of a decode step still fills several CUs)
   for (int hh = blockIdx.y * 4 + (threadIdx.x >> 6); hh < a.heads + a.kv_heads; hh += 4 * gridDim.y) {
     float* x = a.qk + (size_t)t * a.ld + (size_t)hh * a.dim;
     const bool is_k = hh >= a.heads;
@@ -113,12 +127,7 @@ __global__ __launch_bounds__(256) void rotary_kernel(const RotaryArgs a) {
     for (int r = 0; r < kMaxPairs; ++r) {
       const int i = lane + 64 * r;
       if (i < half) {
-        const double full = dpos * a.freq[i];
-        const float ang = (float)(full - 6.283185307179586476925 * rint(full * 0.159154943091895335769));
-        float sn, cs;
-        sincosf(ang, &sn, &cs);
-        sn *= a.mscale;
-        cs *= a.mscale;
+        const float sn = sns[r], cs = css[r];
         const float nu = u[r] * cs - v[r] * sn, nv = v[r] * cs + u[r] * sn;
         u[r] = nu;
         v[r] = nv;
@@ -162,7 +171,9 @@ int tl_launch_rotary(const RotaryArgs& a, hipStream_t s) {
   TL_REQUIRE(a.pos_dev || a.start_pos >= 0, "rotary: negative start position");
   TL_REQUIRE(!a.v_src || (a.v_dst && a.vd > 0), "rotary: a value row without its cache");
   TL_REQUIRE(!a.q_norm == !a.k_norm || a.heads == 0 || a.kv_heads == 0, "rotary: a norm on queries or keys alone");
-  const int per_token = (a.heads + a.kv_heads + 3) / 4;
+  // heads per wave: one for few tokens, up to five where there are workgroups enough anyway
+  int per_token = (a.heads + a.kv_heads + 3) / 4;
+  if (a.T >= 256) per_token = (per_token + 4) / 5;
   rotary_kernel<<<dim3(a.T, per_token < 65535 ? per_token : 65535), 256, 0, s>>>(a);
   TL_HIP(hipGetLastError());
   return 0;

@@ -447,12 +447,13 @@ __global__ __launch_bounds__(256) void ssm_step_kernel(const SsmStepArgs a, int 
   }
 }
 
-// grid (T * parts (+ the history's channels in 256s)), 256 threads a part
-__global__ __launch_bounds__(256) void part_norm_kernel(const PartNormArgs a) {
-  __shared__ float red[4];
-  const int tid = threadIdx.x, units = a.T * a.parts;
+// grid (T * parts (+ the history's channels in blockDim.x s)), a workgroup a part: 256 threads, or 1024 where a launch is a few long
+// rows and nothing but round trips to memory
+__global__ __launch_bounds__(1024) void part_norm_kernel(const PartNormArgs a) {
+  __shared__ float red[16];
+  const int tid = threadIdx.x, units = a.T * a.parts, step = blockDim.x;
   if ((int)blockIdx.x >= units) {
-    const int c = ((int)blockIdx.x - units) * 256 + tid, H = a.taps - 1;
+    const int c = ((int)blockIdx.x - units) * step + tid, H = a.taps - 1;
     if (c >= a.channels) return;
     for (int j = 0; j + 1 < H; ++j) a.hist[(size_t)j * a.channels + c] = a.hist[(size_t)(j + 1) * a.channels + c];
     a.hist[(size_t)(H - 1) * a.channels + c] = a.hist_in[c];
@@ -462,13 +463,15 @@ __global__ __launch_bounds__(256) void part_norm_kernel(const PartNormArgs a) {
   float* x = a.x + (size_t)t * a.width + (size_t)part * n;
   const float* w = a.w + (size_t)part * n;
   float ss = 0.0f;
-  for (int c = tid; c < n; c += 256) ss += x[c] * x[c];
+  for (int c = tid; c < n; c += step) ss += x[c] * x[c];
   ss = tl_wave_sum(ss);
   if ((tid & 63) == 0) red[tid >> 6] = ss;
   __syncthreads();
-  const float inv = 1.0f / sqrtf(((red[0] + red[1]) + (red[2] + red[3])) / (float)n + a.eps);
+  ss = 0.0f;
+  for (int w = 0; w < step >> 6; ++w) ss += red[w];
+  const float inv = 1.0f / sqrtf(ss / (float)n + a.eps);
   const float* gt = a.gate ? a.gate + (size_t)t * a.gate_ld + (size_t)part * n : nullptr;
-  for (int c = tid; c < n; c += 256) x[c] = x[c] * inv * w[c] * (gt ? 1.0f / (1.0f + expf(-gt[c])) : 1.0f);
+  for (int c = tid; c < n; c += step) x[c] = x[c] * inv * w[c] * (gt ? 1.0f / (1.0f + expf(-gt[c])) : 1.0f);
 }
 
 // grid (value channels in 32s, heads), 256 threads: 8 column quads x 32 state rows, the state in passes of 32 rows
@@ -623,9 +626,10 @@ int tl_launch_part_norm(const PartNormArgs& a, hipStream_t s) {
              a.width, a.parts);
   TL_REQUIRE(!a.gate || a.gate_ld >= a.width, "part_norm: gate rows of %d for %d channels", a.gate_ld, a.width);
   TL_REQUIRE(!a.hist || (a.T == 1 && a.hist_in && a.taps > 1 && a.channels > 0), "part_norm: a history rides along for one token");
-  const long long blocks = (long long)a.T * a.parts + (a.hist ? (a.channels + 255) / 256 : 0);
+  const int th = (long long)a.T * a.parts <= 64 && a.width / a.parts >= 1024 ? 1024 : 256;
+  const long long blocks = (long long)a.T * a.parts + (a.hist ? (a.channels + th - 1) / th : 0);
   TL_REQUIRE(blocks <= 0x7fffffffLL, "part_norm: launch too large");
-  part_norm_kernel<<<(unsigned)blocks, 256, 0, s>>>(a);
+  part_norm_kernel<<<(unsigned)blocks, th, 0, s>>>(a);
   TL_HIP(hipGetLastError());
   return 0;
 }

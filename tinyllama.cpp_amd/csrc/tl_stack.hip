@@ -2322,11 +2322,17 @@ int dense_unit(TlStack* st, const Layer& L, const Layer& Wt, const float* in, in
 }
 
 // The mixer of a layer, or both mixers of a pair, on st->h: what they add to the residual
+// (in two steps: mixers_product, after which other work may be forked off, and run_mixers)
+bool takes_product(const Layer& L) {
+  return L.sp.mixer != TL_MIXER_LATENT && L.sp.mixer != TL_MIXER_GDELTA && L.sp.mixer != TL_MIXER_SSM;
+}
+int mixers_product(TlStack* st, Layer& L, const Layer& Wt, int T, hipStream_t s) {
+  return takes_product(L) ? first_product(st, L, Wt, st->h, T, s) : 0;
+}
 int run_mixers(TlStack* st, Layer& L, const Layer& Wt, int T, int start_pos, const int* pos_dev, hipStream_t s, Addends* add) {
   add->a = st->proj;
-  if (!L.side) return run_mixer(st, L, Wt, T, start_pos, pos_dev, s, st->proj);
-  const int ld = L.pd + L.side->pd;  // one first product; each mixer then works on its columns
-  TL_TRY(first_product(st, L, Wt, st->h, T, s));
+  const int ld = L.pd + (L.side ? L.side->pd : 0);  // each mixer works on its columns of the product
+  if (!L.side) return run_mixer(st, L, Wt, T, start_pos, pos_dev, s, st->proj, takes_product(L) ? st->qkv : nullptr, ld);
   TL_TRY(run_mixer(st, L, Wt, T, start_pos, pos_dev, s, st->proj, st->qkv, ld));
   TL_TRY(run_mixer(st, *L.side, *Wt.side, T, start_pos, pos_dev, s, st->proj2, st->qkv + L.pd, ld));
   add->a_scale = L.sp.mix_scale;
@@ -2349,6 +2355,7 @@ int pre_norm_layer(TlStack* st, size_t li, int T, int start_pos, const int* pos_
   const int W = st->cfg.width;
   Layer* after = li + 1 < st->layers.size() ? &st->layers[li + 1] : nullptr;
   Addends mix;
+  TL_TRY(mixers_product(st, L, Wt, T, s));
   TL_TRY(run_mixers(st, L, Wt, T, start_pos, pos_dev, s, &mix));
   if (sp.mlp == TL_MLP_NONE) return finish_x(st, mix, after, 1, T, s, nullptr, &L, 1);
   bool routed = false;
@@ -2404,11 +2411,13 @@ int finish_two(TlStack* st, const Addends& add, const float* ff, const Layer* ne
 }
 
 // h = norm1(x), h2 = norm2(x) (already in st->h, st->h2); x += mixer(h) + ff(h2), and the next block's norms in the same launch. One
-// token: the feed-forward on the second stream, as in parallel_layer
+// token: the feed-forward on the second stream, as in parallel_layer, from the mixers' product on: that product is bound by the
+// bytes of its matrix and would only share them, what follows it is a chain of small launches that leaves the memory idle
 int parallel_norms_layer(TlStack* st, size_t li, int T, int start_pos, const int* pos_dev, hipStream_t s) {
   Layer& L = st->layers[li];
   const Layer& Wt = st->layers[L.wsrc];
   const bool ff = L.sp.mlp != TL_MLP_NONE, forked = st->fork && T == 1 && ff;
+  TL_TRY(mixers_product(st, L, Wt, T, s));
   if (forked) {
     TL_HIP(hipEventRecord(st->ev_fork, s));
     TL_HIP(hipStreamWaitEvent(st->side, st->ev_fork, 0));
