@@ -70,6 +70,7 @@
 #include <memory>
 #include <set>
 #include <string>
+#include <utility>
 #include <vector>
 
 #include "tl_stack.h"
@@ -155,6 +156,7 @@ struct TlStack {
   hipEvent_t ev_fork = nullptr, ev_join = nullptr;
   // workspaces for one chunk
   float *x = nullptr, *qkv = nullptr, *att = nullptr, *proj = nullptr, *v_first = nullptr, *xn = nullptr;
+  float* att_side = nullptr;                // one token of a pair's second mixer on the second stream
   float *att2 = nullptr, *proj2 = nullptr;  // the second score map of differential attention; the second mixer of a pair
   float* hn = nullptr;      // the norm of x before the convolution on what a sublayer reads
   bool any_pair = false, any_maps = false;
@@ -1139,7 +1141,10 @@ int tl_stack_finalize(TlStack* st, hipStream_t s) {
   TL_REQUIRE((size_t)(p - static_cast<float*>(st->cache_base)) * sizeof(float) == st->cache_bytes,
              "tl_stack_finalize: the cache layout does not add up to its allocation");
   if (st->any_maps) TL_TRY(dev_alloc(st, &st->att2, C * st->max_od));
-  if (st->any_pair) TL_TRY(dev_alloc(st, &st->proj2, C * W));
+  if (st->any_pair) {
+    TL_TRY(dev_alloc(st, &st->proj2, C * W));
+    TL_TRY(dev_alloc(st, &st->att_side, st->max_od));
+  }
   if (st->cfg.canon_taps > 0) TL_TRY(dev_alloc(st, &st->hn, C * W));
   if (st->cfg.streams > 0) TL_TRY(dev_alloc(st, &st->xs, C * W * st->cfg.streams));
   if (st->max_gram) TL_TRY(dev_alloc(st, &st->gram, st->max_gram));
@@ -1214,7 +1219,7 @@ int tl_stack_finalize(TlStack* st, hipStream_t s) {
   }
   bool any_parallel = false;
   for (const Layer& L : st->layers)
-    any_parallel |= (L.sp.block == TL_BLOCK_PARALLEL || L.sp.block == TL_BLOCK_PARALLEL_NORMS) && L.sp.mlp != TL_MLP_NONE;
+    any_parallel |= (L.sp.block == TL_BLOCK_PARALLEL || L.sp.block == TL_BLOCK_PARALLEL_NORMS) && (L.sp.mlp != TL_MLP_NONE || L.side);
   if (st->fork && any_parallel) {
     TL_HIP(hipStreamCreateWithFlags(&st->side, hipStreamNonBlocking));
     TL_HIP(hipEventCreateWithFlags(&st->ev_fork, hipEventDisableTiming));
@@ -2329,12 +2334,18 @@ bool takes_product(const Layer& L) {
 int mixers_product(TlStack* st, Layer& L, const Layer& Wt, int T, hipStream_t s) {
   return takes_product(L) ? first_product(st, L, Wt, st->h, T, s) : 0;
 }
-int run_mixers(TlStack* st, Layer& L, const Layer& Wt, int T, int start_pos, const int* pos_dev, hipStream_t s, Addends* add) {
+// ss: the stream of a pair's second mixer. Where it is not s (one token) that mixer's rows go through a buffer of its own; a mixer
+// with a key/value cache or a convolution shares more than that with the first one and stays on s.
+int run_mixers(TlStack* st, Layer& L, const Layer& Wt, int T, int start_pos, const int* pos_dev, hipStream_t s, Addends* add,
+               hipStream_t ss) {
   add->a = st->proj;
   const int ld = L.pd + (L.side ? L.side->pd : 0);  // each mixer works on its columns of the product
   if (!L.side) return run_mixer(st, L, Wt, T, start_pos, pos_dev, s, st->proj, takes_product(L) ? st->qkv : nullptr, ld);
   TL_TRY(run_mixer(st, L, Wt, T, start_pos, pos_dev, s, st->proj, st->qkv, ld));
-  TL_TRY(run_mixer(st, *L.side, *Wt.side, T, start_pos, pos_dev, s, st->proj2, st->qkv + L.pd, ld));
+  if (ss != s) std::swap(st->att, st->att_side);
+  const int rc = run_mixer(st, *L.side, *Wt.side, T, start_pos, pos_dev, ss, st->proj2, st->qkv + L.pd, ld);
+  if (ss != s) std::swap(st->att, st->att_side);
+  TL_TRY(rc);
   add->a_scale = L.sp.mix_scale;
   add->b = st->proj2;
   add->b_scale = L.sp.side_scale;
@@ -2356,7 +2367,7 @@ int pre_norm_layer(TlStack* st, size_t li, int T, int start_pos, const int* pos_
   Layer* after = li + 1 < st->layers.size() ? &st->layers[li + 1] : nullptr;
   Addends mix;
   TL_TRY(mixers_product(st, L, Wt, T, s));
-  TL_TRY(run_mixers(st, L, Wt, T, start_pos, pos_dev, s, &mix));
+  TL_TRY(run_mixers(st, L, Wt, T, start_pos, pos_dev, s, &mix, s));
   if (sp.mlp == TL_MLP_NONE) return finish_x(st, mix, after, 1, T, s, nullptr, &L, 1);
   bool routed = false;
   TL_TRY(finish_x(st, mix, &L, 2, T, s, &routed, &L, 1));
@@ -2411,21 +2422,30 @@ int finish_two(TlStack* st, const Addends& add, const float* ff, const Layer* ne
 }
 
 // h = norm1(x), h2 = norm2(x) (already in st->h, st->h2); x += mixer(h) + ff(h2), and the next block's norms in the same launch. One
-// token: the feed-forward on the second stream, as in parallel_layer, from the mixers' product on: that product is bound by the
-// bytes of its matrix and would only share them, what follows it is a chain of small launches that leaves the memory idle
+// token: the feed-forward on the second stream, as in parallel_layer, but from the mixers' product on: that product is bound by the
+// bytes of its matrix and would only share them, what follows it is a chain of small launches that leaves the memory idle. A pair's
+// linear mixer goes there, too, behind a feed-forward of many bytes and in front of a small one (tokens/s: one stream for both mixers
+// 2351 / 1307 / 1298 at widths 1024 / 2048 / 4096, the mixer first 3074 / 1494 / 1391, the feed-forward first 2773 / 1545 / 1424, a
+// third stream 2507 / 1446 / 1379)
+constexpr size_t kFeedForwardFirstBytes = 32u << 20;
 int parallel_norms_layer(TlStack* st, size_t li, int T, int start_pos, const int* pos_dev, hipStream_t s) {
   Layer& L = st->layers[li];
   const Layer& Wt = st->layers[L.wsrc];
-  const bool ff = L.sp.mlp != TL_MLP_NONE, forked = st->fork && T == 1 && ff;
+  const bool ff = L.sp.mlp != TL_MLP_NONE;
+  const bool linear = L.side && (L.side->sp.mixer == TL_MIXER_LIGHTNING || (L.side->sp.mixer == TL_MIXER_GLA && L.sp.mixer == TL_MIXER_SWA));
+  const bool forked = st->fork && T == 1 && (ff || linear);
+  const bool ff_first = !linear || 6 * (size_t)st->cfg.width * L.sp.shared_ff > kFeedForwardFirstBytes;
+  hipStream_t fs = forked ? st->side : s;
   TL_TRY(mixers_product(st, L, Wt, T, s));
   if (forked) {
     TL_HIP(hipEventRecord(st->ev_fork, s));
     TL_HIP(hipStreamWaitEvent(st->side, st->ev_fork, 0));
   }
-  if (ff) TL_TRY(dense_unit(st, L, Wt, st->h2, T, forked ? st->side : s));
-  if (forked) TL_HIP(hipEventRecord(st->ev_join, st->side));
   Addends mix;
-  TL_TRY(run_mixers(st, L, Wt, T, start_pos, pos_dev, s, &mix));
+  if (ff && ff_first) TL_TRY(dense_unit(st, L, Wt, st->h2, T, fs));
+  TL_TRY(run_mixers(st, L, Wt, T, start_pos, pos_dev, s, &mix, linear ? fs : s));
+  if (ff && !ff_first) TL_TRY(dense_unit(st, L, Wt, st->h2, T, fs));
+  if (forked) TL_HIP(hipEventRecord(st->ev_join, st->side));
   if (forked) TL_HIP(hipStreamWaitEvent(s, st->ev_join, 0));
   return finish_two(st, mix, ff ? st->sout : nullptr, li + 1 < st->layers.size() ? &st->layers[li + 1] : nullptr, T, s);
 }
