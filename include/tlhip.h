@@ -429,6 +429,8 @@ typedef struct tl_stack_config {
   float residual_mult;      /* pre-norm blocks behind a layer norm: factor on what a sublayer adds to the residual (without streams, 0
                                stands for 1) */
   float logit_scale;        /* != 0: the logits are multiplied by it (in front of the cap) */
+  int exact_first;          /* > 0 (at most 32): where a chunk's products round activations to bf16, so many tokens at the start of a
+                               sequence keep 16 mantissa bits (recurrences that norm their read-out are sensitive at an empty state) */
 } tl_stack_config;
 /* the operators such a model is built from, callable on their own (all FP32 in and out, weights bf16 [rows][cols]):
  * Y[T][rows] = X[T][cols] W^T; terms 1 / 3 = MFMA GEMM with bf16-rounded / three-term-split activations, 0 = FP32 GEMV (T = 1) */

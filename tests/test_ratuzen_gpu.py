@@ -415,9 +415,29 @@ def test_residual_stream_after_every_layer(env, variant):
         m.reset_kv()
         got = f64(m.prefill_rows(toks, 0))
         err = np.sqrt(((got - want) ** 2).mean(-1)) / np.sqrt((want * want).mean())
-        # (the first token's linear read-outs are +-v / rms(v): where k . q is small its sign hangs on the rounding)
-        assert np.median(err) < BF16_TOL, err
+        assert err.max() < BF16_TOL, err
     m.free()
+
+
+def test_first_token_of_a_long_prompt_keeps_more_bits_in_bf16_mode(env):
+    """A recurrence's first read-out is v (k . q), normed: where k . q is small its sign hangs on the last bits of the layer's input.
+    So a sequence's first token keeps 16 bits of its activations where the chunk products round them to 8."""
+    cfg = small_config(env["synth"], "wide")
+    m, tensors, orc = make(env, cfg, seed=3, exact=False)
+    loose, _, _ = make(env, cfg, tensors=tensors, exact=False, TL_STACK_EXACT_FIRST=0)
+    rng = np.random.default_rng(12)
+    worst = [0.0, 0.0]
+    for _ in range(12):
+        toks = rng.integers(0, cfg["vocab"], 80).astype(np.int32)
+        orc.reset()
+        want = orc.forward(list(toks[:3]))
+        for j, mm in enumerate((m, loose)):
+            mm.reset_kv()
+            worst[j] = max(worst[j], rel_rms(mm.prefill_rows(toks, 0, np.array([0, 79], np.int32))[:1], want[:1]))
+    print(worst)
+    assert worst[0] < 1e-3 and worst[1] > 5 * worst[0], worst
+    m.free()
+    loose.free()
 
 
 @pytest.mark.parametrize("variant", VARIANTS)

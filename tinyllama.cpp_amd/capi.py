@@ -52,7 +52,7 @@ class StackConfig(C.Structure):
     _fields_ = [("width", C.c_int), ("vocab", C.c_int), ("n_layers", C.c_int), ("max_positions", C.c_int),
                 ("norm_eps", C.c_float), ("layers", C.POINTER(LayerSpec)), ("norm", C.c_int), ("embed_norm", C.c_int),
                 ("logit_softcap", C.c_float), ("embed_scale", C.c_float), ("canon_taps", C.c_int), ("streams", C.c_int),
-                ("residual_mult", C.c_float), ("logit_scale", C.c_float)]
+                ("residual_mult", C.c_float), ("logit_scale", C.c_float), ("exact_first", C.c_int)]
 
 
 BF16 = 30

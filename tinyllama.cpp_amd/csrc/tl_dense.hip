@@ -41,11 +41,15 @@ constexpr int BK = 32, LDK = 40;  // LDK: padded row of a tile in LDS (80 B, kee
 
 // A workgroup of 4 waves (2 x 2) owns a (64 WM)-feature x (64 WN)-token tile; a wave WM x WN products of 32 x 32. The next
 // k-block's weights and activations are asked for (into registers) before the products of the block in LDS start.
-template <int TERMS, int WM, int WN>
+// FIRST: the first 32 items are multiplied with two terms (terms == 1 otherwise): the second terms of those rows have a place of their
+// own in LDS, and the waves that own the 32 items add their products. (All three terms doubled those waves' products and cost 6 % of a
+// prompt of 2048 tokens at width 4096, since a launch of one round ends with its slowest workgroup; the second one alone costs 2 %.)
+template <int TERMS, int WM, int WN, bool FIRST = false>
 __global__ __launch_bounds__(256) void dense_gemm_kernel(const DenseArgs a) {
   constexpr int BM = 64 * WM, BN = 64 * WN;
   __shared__ __attribute__((aligned(16))) unsigned short Ws[BM][LDK];
   __shared__ __attribute__((aligned(16))) unsigned short Xs[TERMS][BN][LDK];
+  __shared__ __attribute__((aligned(16))) unsigned short Xe[FIRST ? 32 : 1][LDK];
   __shared__ int xrow[BN];
   const int tid = threadIdx.x, g = blockIdx.z;
   int lo = 0, hi = a.T;
@@ -67,6 +71,7 @@ __global__ __launch_bounds__(256) void dense_gemm_kernel(const DenseArgs a) {
   }
   __syncthreads();
   const int wave = tid >> 6, lane = tid & 63, wm = wave & 1, wn = wave >> 1;
+  const bool lead = FIRST && blockIdx.y == 0;
   const int lr = tid >> 2, lk = (tid & 3) * 8;  // this thread stages 8 consecutive k of rows lr + 64 i of both tiles
   const int K = a.cols;
   const bool vec = (K & 7) == 0 && (a.ldx & 3) == 0 && ((size_t)X & 15) == 0 && ((size_t)W & 15) == 0;
@@ -143,6 +148,15 @@ __global__ __launch_bounds__(256) void dense_gemm_kernel(const DenseArgs a) {
         p.z = h[4] | ((unsigned)h[5] << 16); p.w = h[6] | ((unsigned)h[7] << 16);
         *reinterpret_cast<uint4*>(&Xs[t][lr + 64 * j][lk]) = p;
       }
+      if (FIRST && j == 0 && lead && lr < 32) {
+        unsigned short h[8];
+#pragma unroll
+        for (int e = 0; e < 8; ++e) h[e] = f2bf(xreg[j][e]);
+        uint4 p;
+        p.x = h[0] | ((unsigned)h[1] << 16); p.y = h[2] | ((unsigned)h[3] << 16);
+        p.z = h[4] | ((unsigned)h[5] << 16); p.w = h[6] | ((unsigned)h[7] << 16);
+        *reinterpret_cast<uint4*>(&Xe[FIRST ? lr : 0][lk]) = p;
+      }
     }
     __syncthreads();
     if (k0 + BK < K) fetch(k0 + BK);  // in flight while the products below run
@@ -160,6 +174,17 @@ __global__ __launch_bounds__(256) void dense_gemm_kernel(const DenseArgs a) {
 #pragma unroll
           for (int i = 0; i < WM; ++i) acc[i][j] = __builtin_amdgcn_mfma_f32_32x32x8bf16_1k(af[i], bfr, acc[i][j], 0, 0, 0);
         }
+      }
+    }
+    if (FIRST && lead && wn == 0) {  // (a loop of its own: the one above keeps its schedule)
+#pragma unroll
+      for (int ks = 0; ks < BK / 8; ++ks) {
+        const int kk = ks * 8 + (lane >> 5) * 4;
+        const bf16x4 bfr = *reinterpret_cast<const bf16x4*>(&Xe[FIRST ? lane & 31 : 0][kk]);
+#pragma unroll
+        for (int i = 0; i < WM; ++i)
+          acc[i][0] = __builtin_amdgcn_mfma_f32_32x32x8bf16_1k(
+              *reinterpret_cast<const bf16x4*>(&Ws[(wm * WM + i) * 32 + (lane & 31)][kk]), bfr, acc[i][0], 0, 0, 0);
       }
     }
     __syncthreads();
@@ -244,6 +269,8 @@ int tl_launch_dense_gemm(const DenseArgs& a, hipStream_t s) {
   TL_REQUIRE(a.w && a.x && a.y && a.rows > 0 && a.cols > 0 && a.T > 0, "dense gemm: bad arguments");
   TL_REQUIRE(a.terms == 1 || a.terms == 3, "dense gemm: terms must be 1 or 3 (got %d)", a.terms);
   TL_REQUIRE(!a.x_rows || a.x_div >= 1, "dense gemm: x_div must be >= 1");
+  TL_REQUIRE(a.exact_items <= 0 || (a.exact_items <= 32 && !a.group_off && a.groups <= 1 && !a.x_rows),
+             "dense gemm: %d first items with two terms (at most 32, one matrix)", a.exact_items);
   TL_REQUIRE(!a.glu || (a.rows & 1) == 0, "dense gemm: gated pairs need an even number of rows (got %d)", a.rows);
   const int groups = a.groups > 0 ? a.groups : 1;
   TL_REQUIRE(groups == 1 || a.group_off || (a.x_gstride >= 0 && a.y_gstride > 0 && !a.x_rows && !a.y_rows),
@@ -262,11 +289,14 @@ int tl_launch_dense_gemm(const DenseArgs& a, hipStream_t s) {
   const int BM = big ? 128 : 64, BN = big ? 128 : 64;
   dim3 grid((a.rows + BM - 1) / BM, (a.T + BN - 1) / BN, groups);
   TL_REQUIRE(grid.y <= 65535 && grid.z <= 65535, "dense gemm: launch too large");
+  const bool first = a.exact_items > 0 && a.terms == 1;
   if (big) {
-    if (a.terms == 1) dense_gemm_kernel<1, 2, 2><<<grid, 256, 0, s>>>(a);
+    if (first) dense_gemm_kernel<1, 2, 2, true><<<grid, 256, 0, s>>>(a);
+    else if (a.terms == 1) dense_gemm_kernel<1, 2, 2><<<grid, 256, 0, s>>>(a);
     else dense_gemm_kernel<3, 2, 2><<<grid, 256, 0, s>>>(a);
   } else {
-    if (a.terms == 1) dense_gemm_kernel<1, 1, 1><<<grid, 256, 0, s>>>(a);
+    if (first) dense_gemm_kernel<1, 1, 1, true><<<grid, 256, 0, s>>>(a);
+    else if (a.terms == 1) dense_gemm_kernel<1, 1, 1><<<grid, 256, 0, s>>>(a);
     else dense_gemm_kernel<3, 1, 1><<<grid, 256, 0, s>>>(a);
   }
   TL_HIP(hipGetLastError());

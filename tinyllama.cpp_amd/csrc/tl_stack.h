@@ -28,6 +28,7 @@ struct DenseArgs {
   float* y;              // outputs, row r at y + r * ldy
   int ldy;
   int T;                 // items (tokens); with group_off: upper bound of the items of one group
+  int exact_items;       // terms == 1, one matrix: > 0 (at most 32): the first so many items keep two terms (16 mantissa bits)
   int terms;             // bf16 MFMAs per product: 1 = activations rounded to bf16, 3 = FP32-grade (hi + mid + lo split)
   const int* x_rows;     // optional (device): item i reads activation row x_rows[i] / x_div
   int x_div;

@@ -144,6 +144,13 @@ struct TlStack {
   int chunk = 2048;
   int lead = 1;             // tokens of tl_stack_lead_tokens (TL_STACK_LEAD; 0: none)
   int exact_below = 64;     // portions shorter than this always multiply with three terms (TL_STACK_EXACT_BELOW; at least 2)
+  // Behind a recurrence whose read-out is normed per head, a linear mixer's or a delta rule's, the first token reads v (k . q): where
+  // k . q is small its SIGN hangs on the last bits of the layer's input, as it does behind the generalized delta rule (see
+  // tl_stack_lead_tokens). A model with such mixers may ask for its first tokens to keep two terms inside their chunk
+  // (tl_stack_config::exact_first; measured on a model of such layers: position 0 of a long prompt up to 19 % of the logits' spread
+  // off where later positions stay below 2 %). TL_STACK_EXACT_FIRST=0: not.
+  int exact_first = 0;
+  int exact_items = 0;      // ... of the forward call that is being enqueued
   bool gemv_decode = true;
   bool fuse_router = true;  // TL_STACK_FUSE_ROUTER=0: the router as a launch of its own (A/B, tests)
   bool fuse_steps = true;   // TL_STACK_FUSE_STEPS=0: one token of a recurrence in as many launches as a chunk takes (A/B, tests)
@@ -742,6 +749,7 @@ int tl_stack_create(const tl_stack_config* cfg, TlStack** out) {
   TL_REQUIRE(cfg->canon_taps >= 0 && cfg->canon_taps <= 64 && (cfg->canon_taps == 0 || cfg->norm == TL_NORM_RMS),
              "tl_stack_create: %d taps on what the sublayers read (a convolution there follows the plain RMS norm)", cfg->canon_taps);
   TL_REQUIRE(cfg->norm != TL_NORM_RMS || !cfg->embed_norm, "tl_stack_create: an embedding norm with the plain RMS norm");
+  TL_REQUIRE(cfg->exact_first >= 0 && cfg->exact_first <= 32, "tl_stack_create: %d first tokens multiplied with two terms", cfg->exact_first);
   TL_REQUIRE(cfg->logit_scale == 0.0f || cfg->norm == TL_NORM_RMS, "tl_stack_create: a factor on the logits rides in the final norm's "
              "weights, which takes the plain RMS norm");
   TlStack* st = new TlStack();
@@ -779,6 +787,8 @@ int tl_stack_create(const tl_stack_config* cfg, TlStack** out) {
   if (const char* e = getenv("TL_STACK_FORK")) st->fork = atoi(e) != 0;
   if (const char* e = getenv("TL_STACK_FUSE_STEPS")) st->fuse_steps = atoi(e) != 0;
   if (const char* e = getenv("TL_STACK_FUSE_CANON")) st->fuse_canon = atoi(e) != 0;
+  st->exact_first = cfg->exact_first;
+  if (const char* e = getenv("TL_STACK_EXACT_FIRST")) st->exact_first = atoi(e) > 0 && atoi(e) <= 32 ? atoi(e) : 0;
   if (const char* e = getenv("TL_STACK_LEAD")) st->lead = atoi(e) > 0 ? atoi(e) : 0;
   if (const char* e = getenv("TL_STACK_EXACT_BELOW")) st->exact_below = atoi(e) > 2 ? atoi(e) : 2;
   if (const char* e = getenv("TL_STACK_LATENT_EXPAND")) st->latent_expand = atoi(e) > 0 ? atoi(e) : 0;
@@ -1361,6 +1371,7 @@ int project(TlStack* st, const uint16_t* w, int rows, int cols, const float* x, 
   d.ldy = ldy;
   d.T = T;
   d.terms = terms_for(st, T);
+  d.exact_items = st->exact_items;
   d.softcap = softcap;
   return tl_launch_dense_gemm(d, s);
 }
@@ -1379,6 +1390,7 @@ int project_act(TlStack* st, const uint16_t* w, int rows, int cols, const float*
   d.ldy = ldy;
   d.T = T;
   d.terms = terms ? terms : terms_for(st, T);
+  d.exact_items = st->exact_items;
   d.act = act.act;
   d.act_from = act.act_from;
   d.act_to = act.act_to;
@@ -2317,6 +2329,7 @@ int dense_unit(TlStack* st, const Layer& L, const Layer& Wt, const float* in, in
   u.ldy = ff;
   u.T = T;
   u.terms = terms_for(st, T);
+  u.exact_items = st->exact_items;
   u.glu = 1;
   u.glu_limit = sp.shared_limit;
   u.glu_alpha = sp.act_alpha;
@@ -2511,6 +2524,7 @@ int tl_stack_forward(TlStack* st, const int* tokens_dev, int T, int start_pos, c
   const tl_stack_config& c = st->cfg;
   const int W = c.width;
   const bool dyt = c.norm == TL_NORM_DYT, lnorm = c.norm == TL_NORM_LAYER || c.norm == TL_NORM_LAYER_PLAIN;
+  st->exact_items = !pos_dev && start_pos == 0 ? st->exact_first : 0;
   if (lnorm && !c.embed_norm) {
     HyperArgs r = {};  // every stream starts as the (scaled) embedding row
     hyper_next(st, r, &st->layers[0], 1, T, nullptr);
@@ -2570,6 +2584,7 @@ int tl_stack_forward(TlStack* st, const int* tokens_dev, int T, int start_pos, c
       st->hook(st->hook_ctx, (int)li, st->x, T, W);
     }
   }
+  st->exact_items = 0;
   if (n_rows > 0) {
     const int last = T - 1;
     const float* src = st->x;

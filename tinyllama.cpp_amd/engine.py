@@ -663,7 +663,7 @@ def stack_config_struct(config, max_pos, tensors=None):
                          float(config["embedding"]["scale"]) if potipel or madudra else 0.0,
                          int(config["canon"]["taps"]) if potipel else 0, int(config["streams"]) if madudra else 0,
                          float(config["residual_mult"]) if madudra else 0.0,
-                         float(config["logit_scale"]) if ratuzen else 0.0)
+                         float(config["logit_scale"]) if ratuzen else 0.0, 1 if ratuzen else 0)
     return c, (arr, sides, keep)
 
 

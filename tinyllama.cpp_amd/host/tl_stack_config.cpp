@@ -532,7 +532,10 @@ void load_stack_folder(const std::string& dir, int device, int max_context, Load
             : madudra ? TL_NORM_LAYER_PLAIN
                       : TL_NORM_RMS_ONE_PLUS;
   sc.embed_norm = madalorn || potipel || madudra || ratuzen ? 0 : 1;
-  if (ratuzen) sc.logit_scale = getf(cfg, "logit_scale");
+  if (ratuzen) {
+    sc.logit_scale = getf(cfg, "logit_scale");
+    sc.exact_first = 1;  // every mixer of the design norms what it reads from its state
+  }
   if (potipel || madudra) sc.embed_scale = (float)cfg.at("embedding").at("scale").as_double("embedding.scale");
   if (madudra) {
     sc.streams = geti(cfg, "streams");
