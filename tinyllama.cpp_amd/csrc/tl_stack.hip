@@ -147,8 +147,8 @@ struct TlStack {
   // Behind a recurrence whose read-out is normed per head, a linear mixer's or a delta rule's, the first token reads v (k . q): where
   // k . q is small its SIGN hangs on the last bits of the layer's input, as it does behind the generalized delta rule (see
   // tl_stack_lead_tokens). A model with such mixers may ask for its first tokens to keep two terms inside their chunk
-  // (tl_stack_config::exact_first; measured on a model of such layers: position 0 of a long prompt up to 19 % of the logits' spread
-  // off where later positions stay below 2 %). TL_STACK_EXACT_FIRST=0: not.
+  // (tl_stack_config::exact_first; position 0 of a long prompt is otherwise now and then ten times as far off as later positions).
+  // TL_STACK_EXACT_FIRST=0: not.
   int exact_first = 0;
   int exact_items = 0;      // ... of the forward call that is being enqueued
   bool gemv_decode = true;
@@ -2339,8 +2339,8 @@ int dense_unit(TlStack* st, const Layer& L, const Layer& Wt, const float* in, in
   return project(st, Wt.sdown, W, ff, st->sact, ff, st->sout, W, T, s);
 }
 
-// The mixer of a layer, or both mixers of a pair, on st->h: what they add to the residual
-// (in two steps: mixers_product, after which other work may be forked off, and run_mixers)
+// The mixer of a layer, or both mixers of a pair, on st->h, in two steps: mixers_product, after which other work may be forked off,
+// and run_mixers, which says what they add to the residual
 bool takes_product(const Layer& L) {
   return L.sp.mixer != TL_MIXER_LATENT && L.sp.mixer != TL_MIXER_GDELTA && L.sp.mixer != TL_MIXER_SSM;
 }
